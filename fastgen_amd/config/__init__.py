@@ -12,6 +12,7 @@ from . import buderax as _buderax  # registers Buderax
 from . import gisodra as _gisodra  # registers Gisodra
 from . import zudisun as _zudisun  # registers Zudisun
 from . import sodotar as _sodotar  # registers Sodotar
+from . import ropelix as _ropelix  # registers Ropelix
 
 __all__ = [
     "Architecture",

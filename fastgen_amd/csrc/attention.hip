@@ -11,7 +11,8 @@
 // Semantics (fastgen/forward.py:176-258): query at position p of sequence b
 // sees keys 0..p of b through block_table[b]; scores (q.k)*scale, softmax in
 // fp32, o = P.V; query head h reads kv head h / (H/KV).  With window > 0 only
-// keys p-window+1..p are seen.
+// keys p-window+1..p are seen.  With `dist` (r1, r2 per query head) a score loses r1 * ln(1 + r2 * n) for a key n
+// tokens back.
 #include "common.h"
 #include "kv_layout.h"
 
@@ -47,7 +48,7 @@ __global__ __launch_bounds__(ATT_WAVES* FG_WAVE) void paged_attention_general_ke
     const T* __restrict__ k_pages, const T* __restrict__ v_pages,
     const int* __restrict__ block_table, int bt_stride, const int* __restrict__ seq_of_token,
     const int* __restrict__ positions, int n_tokens, int n_heads, int n_kv, int hd,
-    int page_size, float scale, int window, const float* __restrict__ sinks) {
+    int page_size, float scale, int window, const float* __restrict__ sinks, const float* __restrict__ dist) {
   __shared__ float q_s[ATT_WAVES][ATT_MAX_HD];
   __shared__ float p_s[ATT_WAVES][ATT_TILE];
   const int lane = threadIdx.x % FG_WAVE, wave = threadIdx.x / FG_WAVE;
@@ -91,6 +92,7 @@ __global__ __launch_bounds__(ATT_WAVES* FG_WAVE) void paged_attention_general_ke
         for (int e = 0; e < 8; ++e) acc += qs[d + e] * kv.v[e];
       }
       s = acc * scale;
+      if (dist) s -= dist[2 * h] * log1pf(dist[2 * h + 1] * (float)(pos - key));
     }
     const float m_new = fmaxf(m, wave_max(s));
     const float p = valid ? expf(s - m_new) : 0.f;
@@ -147,7 +149,7 @@ extern "C" int fg_paged_attention_general_sink(
     const void* q, int q_stride, void* out, int out_stride, const void* k_pages,
     const void* v_pages, const int* block_table, int bt_stride, const int* seq_of_token,
     const int* positions, int n_tokens, int n_heads, int n_kv, int hd, int page_size,
-    float scale, int window, const float* sinks, int dtype, hipStream_t stream) {
+    float scale, int window, const float* sinks, const float* dist, int dtype, hipStream_t stream) {
   if (n_tokens <= 0) return FG_OK;
   if (hd <= 0 || hd % 8 || hd > ATT_MAX_HD || page_size <= 0 || page_size % 8 || n_kv <= 0 ||
       n_heads <= 0 || n_heads % n_kv)
@@ -160,12 +162,12 @@ extern "C" int fg_paged_attention_general_sink(
     paged_attention_general_kernel<float><<<grid, ATT_WAVES * FG_WAVE, 0, stream>>>(
         (const float*)q, q_stride, (float*)out, out_stride, (const float*)k_pages,
         (const float*)v_pages, block_table, bt_stride, seq_of_token, positions, n_tokens,
-        n_heads, n_kv, hd, page_size, scale, window, sinks);
+        n_heads, n_kv, hd, page_size, scale, window, sinks, dist);
   else if (dtype == FG_BF16)
     paged_attention_general_kernel<bf16_t><<<grid, ATT_WAVES * FG_WAVE, 0, stream>>>(
         (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)k_pages,
         (const bf16_t*)v_pages, block_table, bt_stride, seq_of_token, positions, n_tokens,
-        n_heads, n_kv, hd, page_size, scale, window, sinks);
+        n_heads, n_kv, hd, page_size, scale, window, sinks, dist);
   else
     return FG_ERR_ARG;
   return fg_launch_status();
@@ -178,5 +180,5 @@ extern "C" int fg_paged_attention_general(
     float scale, int window, int dtype, hipStream_t stream) {
   return fg_paged_attention_general_sink(q, q_stride, out, out_stride, k_pages, v_pages, block_table, bt_stride,
                                          seq_of_token, positions, n_tokens, n_heads, n_kv, hd, page_size, scale,
-                                         window, nullptr, dtype, stream);
+                                         window, nullptr, nullptr, dtype, stream);
 }

@@ -1,7 +1,8 @@
 // Paged causal attention on the matrix cores (bf16 in, fp32 accumulate) for
 // gfx950.  Compiled once per head size: -DFG_HD=<multiple of 16, at most 256>;
 // with -DFG_EXACT_P the softmax weights keep 16 significant bits in the product
-// with the values (for models that ask for weights of more than bfloat16).
+// with the values (for models that ask for weights of more than bfloat16); with -DFG_DIST_BIAS every score
+// loses r1_h * ln(1 + r2_h * n) for a key n tokens back (`dist`: r1, r2 per query head).
 //
 // Both kernels work on *items*: an item is a run of consecutive query tokens
 // of one sequence; its rows are (token, query head of one kv head's group),
@@ -40,6 +41,11 @@ constexpr int HD = FG_HD;
 constexpr int NKS = (HD + 31) / 32;  // 32-wide steps over the head dimension (last may be half)
 constexpr int NDB = HD / 16;         // 16-wide blocks of the head dimension
 constexpr int TILE = 64;             // keys per tile
+#ifdef FG_DIST_BIAS
+constexpr bool DIST_BIAS = true;     // this build takes the scores' distance bias, and only calls with one
+#else
+constexpr bool DIST_BIAS = false;
+#endif
 
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
@@ -108,7 +114,19 @@ struct Pager {
 struct ItemRows {
   int pos;    // position of this lane's query row, -1 for a padding row
   int first;  // first key the row sees
+#ifdef FG_DIST_BIAS
+  float r1, r2;  // the row's head's numbers
+#endif
 };
+#ifdef FG_DIST_BIAS
+#define SET_DIST(me, head)               \
+  do {                                   \
+    (me).r1 = dist[2 * (head)];          \
+    (me).r2 = dist[2 * (head) + 1];      \
+  } while (0)
+#else
+#define SET_DIST(me, head) (void)dist
+#endif
 
 // One 64-key tile for one wave, operands given by loader functors.
 //   load_k(kb, ks) -> bf16x8 : K[16*kb + lane%16][32*ks + 8*(lane/16) ..+7]
@@ -169,8 +187,13 @@ __device__ __forceinline__ void attend_tile(int k0, const ItemRows (&me)[RB], co
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         float v = s[rb][kb][i];  // unscaled: the scale is positive, so it commutes with the maximum
+        [[maybe_unused]] const int key = k0 + key_of(kb, 4 * g + i);
+#ifdef FG_DIST_BIAS
+        // scaled here, in base 2: r1 ln(x) log2(e) = r1 log2(x).  (Of a key behind the query x may be anything:
+        // the select below drops it.)
+        v = fmaf(v, scale_log2, -me[rb].r1 * __builtin_amdgcn_logf(fmaf(me[rb].r2, (float)(me[rb].pos - key), 1.f)));
+#endif
         if (!ALLVIS) {
-          const int key = k0 + key_of(kb, 4 * g + i);
           // bitwise, not short-circuit: a select, no branch
           v = ((key >= me[rb].first) & (key <= me[rb].pos)) ? v : -INFINITY;
         }
@@ -178,7 +201,11 @@ __device__ __forceinline__ void attend_tile(int k0, const ItemRows (&me)[RB], co
         mx = fmaxf(mx, v);
       }
     mx = max_over_groups(mx);
+#ifdef FG_DIST_BIAS
+    const float m_new = fmaxf(m[rb], mx);
+#else
     const float m_new = fmaxf(m[rb], mx * scale_log2);
+#endif
     const float m_use = m_new == -INFINITY ? 0.f : m_new;  // a row that has seen no key yet
     const float alpha = __builtin_amdgcn_exp2f(m[rb] - m_use);  // m = -inf: 0
     float sum = 0.f;
@@ -186,7 +213,11 @@ __device__ __forceinline__ void attend_tile(int k0, const ItemRows (&me)[RB], co
     for (int kb = 0; kb < 4; ++kb)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
+#ifdef FG_DIST_BIAS
+        const float p = __builtin_amdgcn_exp2f(s[rb][kb][i] - m_use);
+#else
         const float p = __builtin_amdgcn_exp2f(fmaf(s[rb][kb][i], scale_log2, -m_use));
+#endif
         sum += p;
         pop[rb][kb >> 1][4 * (kb & 1) + i] = (__bf16)p;
 #ifdef FG_EXACT_P
@@ -354,7 +385,7 @@ __global__ __launch_bounds__(256) void attn_split_kernel(
     const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ v_pages,
     const int* __restrict__ block_table, int bt_stride, const int* __restrict__ plan,
     float* __restrict__ part_o, float* __restrict__ part_ml, int n_heads, int n_kv, int page_size,
-    int page_shift, float scale, int window, const float* __restrict__ sinks) {
+    int page_shift, float scale, int window, const float* __restrict__ sinks, const float* __restrict__ dist) {
   __shared__ float o_s[2][16][HD + 1];
   __shared__ float ml_s[2][16][2];
   const int lane = threadIdx.x % FG_WAVE, wave = threadIdx.x / FG_WAVE;
@@ -375,6 +406,7 @@ __global__ __launch_bounds__(256) void attn_split_kernel(
   ItemRows me[1] = {{-1, 0}};
   const bool my_row = r16 < it.n_tok * G;
   const int my_tok = my_row ? r16 / G : 0, my_head = my_row ? r16 % G : 0;
+  SET_DIST(me[0], kvh * G + my_head);
   if (my_row) {
     me[0].pos = it.pos0 + my_tok;
     me[0].first = first_key(me[0].pos, window);
@@ -674,14 +706,16 @@ extern "C" int fg_attn_plan(const int* items, int n_items, int window, int max_c
 // plan: what fg_attn_plan made of the items, with the same n_items, max_chunks and window.
 // max_rows: no item has more rows (tokens x heads of a kv head's group) than this, at most 16.
 // part_o: fp32 [max_chunks * n_kv * 16 * HD], part_ml: the same rows x 2.
+// dist: fp32 [n_heads, 2], in the build with FG_DIST_BIAS (null in the others).
 // sinks: fp32 [n_heads] or null: head h's softmax has one more term exp(sinks[h]) in its denominator, which
 // brings no value.
 extern "C" int fg_attn_split_sink(const void* q, int q_stride, void* out, int out_stride, const void* k_pages,
                                   const void* v_pages, const int* block_table, int bt_stride, const int* plan,
                                   int n_items, int max_chunks, int max_rows, float* part_o, float* part_ml,
                                   int n_heads, int n_kv, int hd, int page_size, float scale, int window,
-                                  const float* sinks, hipStream_t stream) {
+                                  const float* sinks, const float* dist, hipStream_t stream) {
   if (n_items <= 0) return FG_OK;
+  if (DIST_BIAS != (dist != nullptr)) return FG_ERR_ARG;
   if (hd != HD || n_kv <= 0 || n_heads % n_kv || n_heads / n_kv > 16 || page_size < 8 || page_size % 8 ||
       !(scale > 0.f) || max_chunks < 2 * n_items || max_chunks > 65535 || n_kv > 65535 ||
       q_stride % 8 || out_stride % 4 || !plan || !part_o || !part_ml || max_rows < 1 || max_rows > 16)
@@ -690,7 +724,7 @@ extern "C" int fg_attn_split_sink(const void* q, int q_stride, void* out, int ou
   attn_split_kernel<PERM><<<dim3(n_kv, max_chunks), 256, 0, stream>>>(                                         \
       (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages,    \
       block_table, bt_stride, plan, part_o, part_ml, n_heads, n_kv, page_size,                                 \
-      page_shift_of(page_size), scale, window, sinks)
+      page_shift_of(page_size), scale, window, sinks, dist)
   if (page_size % 32 == 0) LAUNCH(true); else LAUNCH(false);
 #undef LAUNCH
   if ((long long)max_chunks * n_kv * max_rows <= COMBINE_ROWS_MAX_GROUPS)
@@ -709,7 +743,7 @@ extern "C" int fg_attn_split(const void* q, int q_stride, void* out, int out_str
                              hipStream_t stream) {
   return fg_attn_split_sink(q, q_stride, out, out_stride, k_pages, v_pages, block_table, bt_stride, plan, n_items,
                             max_chunks, max_rows, part_o, part_ml, n_heads, n_kv, hd, page_size, scale, window,
-                            nullptr, stream);
+                            nullptr, nullptr, stream);
 }
 
 // ----------------------------------------------------------- without allocation
@@ -817,7 +851,8 @@ __global__ __launch_bounds__(TILE_PAIR ? 512 : 256, TILE_PAIR ? 1 : 2) void attn
     const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, int out_stride,
     const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ v_pages,
     const int* __restrict__ block_table, int bt_stride, const int* __restrict__ items, int n_heads, int n_kv,
-    int page_size, int page_shift, float scale, int window, const float* __restrict__ sinks) {
+    int page_size, int page_shift, float scale, int window, const float* __restrict__ sinks,
+    const float* __restrict__ dist) {
   constexpr int TILE_RB = TILE_PAIR ? 2 : 1;  // row blocks a wave holds
   constexpr int TILE_THREADS = TILE_PAIR ? 512 : 256;
   constexpr int NT = TILE_THREADS;
@@ -850,6 +885,7 @@ __global__ __launch_bounds__(TILE_PAIR ? 512 : 256, TILE_PAIR ? 1 : 2) void attn
     const bool my_row = row < it.n_tok * G;
     const int my_tok = my_row ? row / G : 0, my_head = my_row ? row % G : 0;
     me[rb] = ItemRows{-1, 0};
+    SET_DIST(me[rb], kvh * G + my_head);
     if (my_row) {
       me[rb].pos = it.pos0 + my_tok;
       me[rb].first = first_key(me[rb].pos, window);
@@ -1092,13 +1128,13 @@ __global__ __launch_bounds__(TILE_PAIR ? 512 : 256, TILE_PAIR ? 1 : 2) void attn
 struct TileArgs {
   const bf16_t* q; int q_stride; bf16_t* out; int out_stride; const bf16_t* k_pages; const bf16_t* v_pages;
   const int* block_table; int bt_stride; const int* items; int n_items, n_heads, n_kv, page_size; float scale;
-  int window; const float* sinks; hipStream_t stream;
+  int window; const float* sinks; const float* dist; hipStream_t stream;
 };
 template <bool PERM, bool PAIR>
 static void launch_tile(const TileArgs& a) {
   attn_tile_kernel<PERM, PAIR><<<a.n_items * a.n_kv, PAIR ? 512 : 256, 0, a.stream>>>(
       a.q, a.q_stride, a.out, a.out_stride, a.k_pages, a.v_pages, a.block_table, a.bt_stride, a.items, a.n_heads,
-      a.n_kv, a.page_size, page_shift_of(a.page_size), a.scale, a.window, a.sinks);
+      a.n_kv, a.page_size, page_shift_of(a.page_size), a.scale, a.window, a.sinks, a.dist);
 }
 // the form with two tiles at a time exists up to head size 128 only (its LDS)
 template <bool EXISTS> struct PairForm {
@@ -1112,14 +1148,16 @@ template <> struct PairForm<false> { static void go(const TileArgs&) {} };
 extern "C" int fg_attn_tile_sink(const void* q, int q_stride, void* out, int out_stride, const void* k_pages,
                                  const void* v_pages, const int* block_table, int bt_stride, const int* items,
                                  int n_items, int item_rows, int n_heads, int n_kv, int hd, int page_size,
-                                 float scale, int window, const float* sinks, hipStream_t stream) {
+                                 float scale, int window, const float* sinks, const float* dist,
+                                 hipStream_t stream) {
   if (n_items <= 0) return FG_OK;
+  if (DIST_BIAS != (dist != nullptr)) return FG_ERR_ARG;
   if (hd != HD || !(scale > 0.f) || n_kv <= 0 || n_heads % n_kv || n_heads / n_kv > item_rows || page_size < 8 || page_size % 8 ||
       (long long)n_items * n_kv > 2147483647LL || q_stride % 8 || out_stride % 4 ||
       (item_rows != TILE_ROWS && item_rows != TILE_ROWS_SMALL))
     return FG_ERR_ARG;
   const TileArgs a{(const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages,
-                   block_table, bt_stride, items, n_items, n_heads, n_kv, page_size, scale, window, sinks, stream};
+                   block_table, bt_stride, items, n_items, n_heads, n_kv, page_size, scale, window, sinks, dist, stream};
   if (TILE_PAIR_OK && item_rows == TILE_ROWS) PairForm<TILE_PAIR_OK>::go(a);
   else if (page_size % 32 == 0) launch_tile<true, false>(a);
   else launch_tile<false, false>(a);
@@ -1131,7 +1169,7 @@ extern "C" int fg_attn_tile(const void* q, int q_stride, void* out, int out_stri
                             int n_items, int item_rows, int n_heads, int n_kv, int hd, int page_size, float scale,
                             int window, hipStream_t stream) {
   return fg_attn_tile_sink(q, q_stride, out, out_stride, k_pages, v_pages, block_table, bt_stride, items, n_items,
-                           item_rows, n_heads, n_kv, hd, page_size, scale, window, nullptr, stream);
+                           item_rows, n_heads, n_kv, hd, page_size, scale, window, nullptr, nullptr, stream);
 }
 
 // query rows (tokens x heads of a kv head's group) of one item of fg_attn_tile: of the larger form, or

@@ -1,0 +1,250 @@
+// The gated delta rule: a state S [d, e] per head in fp32, kept per request and carried from step to step.
+//
+//   S <- g_t S;   u_t = beta_t (v_t - S^T k_t);   S <- S + k_t u_t^T;   o_t = S^T q_t
+//
+//  delta_prepare  what the recurrence takes of a token, from the rows of the product: a causal convolution per
+//                 channel and SiLU on q, k and v; q and k as unit vectors per head (q times q_scale); the write
+//                 strength beta = sigmoid(b) and the decay g = exp(-exp(A_log) softplus(a + dt_bias)) per head.
+//                 One fp32 row a token: [q | k | v | beta | g].  A wave a (token, head).
+//  delta_scan     the recurrence token by token.  Column c of S needs k, q and v[c] only, so a wave owns eight value
+//                 channels of a head: lane l holds column l & 7 and the key channels rg * rpl .. (rg = l >> 3) of it in
+//                 registers.  S^T k is a sum over the lanes of a column on the chain; S^T q is not, its sums are
+//                 exchanged for a whole run of tokens at once.  Operands of the next run fly while one is computed.
+//  Every sum runs in an order fixed by the sizes: what a token gets does not depend on the batch or on the cut.
+#include "common.h"
+#include "conv_inputs.h"
+
+#define DP_WAVES 4
+#define DP_MAX_PAIRS 8  // heads of up to 1,024 elements
+
+struct DeltaPrepareArgs {
+  const void* src; int src_stride;       // [T, q | k | v ...]: q from column 0, k and v right behind
+  int n_qk, d, n_v, e;                   // query/key heads of d, value heads of e
+  ConvIn conv;                           // over the q, k and v columns
+  int b_col, a_col;                      // columns of the beta and decay logits (n_v each)
+  const float* decay_rate;               // [n_v]: exp(A_log)
+  const float* dt_bias;                  // [n_v]
+  float q_scale, unit_eps;
+  float* out; int out_stride;            // [T, 2 n_qk d + n_v e + 2 n_v]
+};
+
+// grid (T, ceil((2 n_qk + n_v + 1) / 4)); the last job of a token is its scalars, a lane a head
+template <class TS>
+__global__ __launch_bounds__(DP_WAVES* FG_WAVE) void delta_prepare_kernel(const DeltaPrepareArgs a) {
+  const int lane = threadIdx.x % FG_WAVE, t = blockIdx.x, job = blockIdx.y * DP_WAVES + threadIdx.x / FG_WAVE;
+  const int qk_jobs = 2 * a.n_qk, v_base = qk_jobs * a.d;
+  if (job > qk_jobs + a.n_v) return;  // whole waves; no block barrier below
+  const TS* src = (const TS*)a.src;
+  float* out = a.out + (size_t)t * a.out_stride;
+  if (job == qk_jobs + a.n_v) {
+    const TS* row = src + (size_t)t * a.src_stride;
+    float* so = out + v_base + a.n_v * a.e;
+    for (int h = lane; h < a.n_v; h += FG_WAVE) {
+      const float b = to_f<TS>(row[a.b_col + h]);
+      const float x = to_f<TS>(row[a.a_col + h]) + a.dt_bias[h];
+      so[h] = 1.f / (1.f + expf(-b));
+      so[a.n_v + h] = expf(-a.decay_rate[h] * (fmaxf(x, 0.f) + log1pf(expf(-fabsf(x)))));
+    }
+    return;
+  }
+  const bool is_v = job >= qk_jobs;
+  const int w = is_v ? a.e : a.d;
+  const int col = is_v ? v_base + (job - qk_jobs) * a.e : job * a.d;
+  float x[DP_MAX_PAIRS][2];
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < DP_MAX_PAIRS; ++j) {
+    const int c = 2 * (lane + FG_WAVE * j);
+    x[j][0] = x[j][1] = 0.f;
+    if (c < w) {
+      conv_pair<TS>(a.conv, src, a.src_stride, t, col + c, x[j]);
+#pragma unroll
+      for (int i = 0; i < 2; ++i) x[j][i] = x[j][i] / (1.f + expf(-x[j][i]));
+      ss += x[j][0] * x[j][0] + x[j][1] * x[j][1];
+    }
+  }
+  float mul = 1.f;
+  if (!is_v) {  // uniform
+    ss = wave_sum(ss);
+    mul = rsqrtf(ss + a.unit_eps) * (job < a.n_qk ? a.q_scale : 1.f);
+  }
+#pragma unroll
+  for (int j = 0; j < DP_MAX_PAIRS; ++j) {
+    const int c = 2 * (lane + FG_WAVE * j);
+    if (c < w) *(float2*)(out + col + c) = make_float2(x[j][0] * mul, x[j][1] * mul);
+  }
+}
+
+extern "C" int fg_delta_prepare(const DeltaPrepareArgs* args, int n_tokens, int src_dtype, hipStream_t stream) {
+  if (n_tokens <= 0) return FG_OK;
+  const DeltaPrepareArgs& a = *args;
+  const int lim = 2 * FG_WAVE * DP_MAX_PAIRS;
+  if (a.n_qk <= 0 || a.n_v <= 0 || a.d <= 0 || a.d % 2 || a.d > lim || a.e <= 0 || a.e % 2 || a.e > lim || !a.src || !a.out ||
+      !a.decay_rate || !a.dt_bias || !a.conv.w || !fg_conv_ok(a.conv) || a.conv.channels < 2 * a.n_qk * a.d + a.n_v * a.e ||
+      a.out_stride % 2 || a.out_stride < 2 * a.n_qk * a.d + a.n_v * (a.e + 2))
+    return FG_ERR_ARG;
+  const dim3 grid(n_tokens, (2 * a.n_qk + a.n_v + 1 + DP_WAVES - 1) / DP_WAVES);
+  if (grid.y > 65535) return FG_ERR_ARG;
+  if (src_dtype == FG_F32) delta_prepare_kernel<float><<<grid, DP_WAVES * FG_WAVE, 0, stream>>>(a);
+  else if (src_dtype == FG_BF16) delta_prepare_kernel<bf16_t><<<grid, DP_WAVES * FG_WAVE, 0, stream>>>(a);
+  else return FG_ERR_ARG;
+  return fg_launch_status();
+}
+
+// ------------------------------------------------------------------- scan
+struct DeltaScanArgs {
+  const float* rows; int stride;         // delta_prepare's rows
+  int n_qk, d, n_v, e;
+  float* state; long long slot_stride;   // S of slot s, head h at s * slot_stride + h * d * e, [d, e]
+  const int* slot_ids; const int* q_start;
+  float* out;                            // [T, n_v * e]
+};
+
+// The sum over the eight lanes that hold a column (lane % 8 equal), in every one of them: lanes 8 apart by a
+// rotation within a row of 16, then rows and halves exchanged in the vector unit.
+__device__ __forceinline__ float column_sum(float v) {
+  v += __uint_as_float(__builtin_amdgcn_update_dpp(0, __float_as_uint(v), 0x128 /* row_ror:8 */, 0xf, 0xf, false));
+  const auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+  v = __uint_as_float(a[0]) + __uint_as_float(a[1]);
+  const auto b = __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+  return __uint_as_float(b[0]) + __uint_as_float(b[1]);
+}
+
+#define DS_TOKENS_FOR(RPL) ((RPL) <= 16 ? 8 : 4)  // tokens staged at a time
+
+// grid (B, n_v, ceil(e / 8)), one wave.  RPL >= ceil(d / 8), a multiple of 4; NJ: staged elements a lane holds of k
+// and of q per token.
+template <int RPL>
+__global__ __launch_bounds__(FG_WAVE) void delta_scan_kernel(const DeltaScanArgs a) {
+  constexpr int RUN = DS_TOKENS_FOR(RPL);
+  constexpr int NJ = (RPL + 7) / 8;  // 64 lanes, up to 8 RPL channels
+  // [RUN][2][8 parts of RPL + 4]: k, q; key channel r of part p = r / rpl at p * (RPL + 4) + r % rpl, zeros behind rpl
+  constexpr int PS = RPL + 4, VS = 8 * PS;
+  __shared__ __attribute__((aligned(16))) float lds[RUN * 2 * VS];
+  const int lane = threadIdx.x;
+  const int b = blockIdx.x, h = blockIdx.y;
+  const int rg = lane >> 3, col = blockIdx.z * 8 + (lane & 7);
+  const bool col_ok = col < a.e;
+  const int d = a.d, e = a.e, rpl = (d + 7) / 8, r0 = rg * rpl;
+  const int hq = h / (a.n_v / a.n_qk);
+  const int t_begin = a.q_start[b], t_end = a.q_start[b + 1];
+  if (t_begin >= t_end) return;  // uniform
+  float* S_mem = a.state + (size_t)a.slot_ids[b] * a.slot_stride + (size_t)h * d * e;
+  float S[RPL];
+#pragma unroll
+  for (int i = 0; i < RPL; ++i) S[i] = (i < rpl && r0 + i < d && col_ok) ? S_mem[(size_t)(r0 + i) * e + col] : 0.f;
+  for (int i = lane; i < RUN * 2 * VS; i += FG_WAVE) lds[i] = 0.f;
+  int src[NJ], dst[NJ];
+  bool mine[NJ];
+#pragma unroll
+  for (int j = 0; j < NJ; ++j) {
+    const int r = lane + FG_WAVE * j;
+    mine[j] = r < d;
+    src[j] = hq * d + min(r, d - 1);
+    dst[j] = (r / rpl) * PS + r % rpl;
+  }
+  const int k_col = a.n_qk * d, v_col = 2 * k_col + h * e + min(col, e - 1);
+  const int b_col = 2 * k_col + a.n_v * e + h, g_col = b_col + a.n_v;
+  float pk[RUN][NJ], pq[RUN][NJ], pv[RUN], pb[RUN], pg[RUN];
+  auto fetch = [&](int t0) {
+#pragma unroll
+    for (int tt = 0; tt < RUN; ++tt) {
+      const float* row = a.rows + (size_t)min(t0 + tt, t_end - 1) * a.stride;
+#pragma unroll
+      for (int j = 0; j < NJ; ++j) {
+        pk[tt][j] = row[k_col + src[j]];
+        pq[tt][j] = row[src[j]];
+      }
+      pv[tt] = row[v_col];
+      pb[tt] = row[b_col];
+      pg[tt] = row[g_col];
+    }
+  };
+  fetch(t_begin);
+  for (int t0 = t_begin; t0 < t_end; t0 += RUN) {
+    const int n = min(RUN, t_end - t0);
+    __syncthreads();  // the run before has been read
+    float v[RUN], beta[RUN], g[RUN];
+#pragma unroll
+    for (int tt = 0; tt < RUN; ++tt) {
+      v[tt] = pv[tt];
+      beta[tt] = pb[tt];
+      g[tt] = pg[tt];
+#pragma unroll
+      for (int j = 0; j < NJ; ++j) {
+        if (mine[j]) {
+          lds[tt * 2 * VS + dst[j]] = pk[tt][j];
+          lds[tt * 2 * VS + VS + dst[j]] = pq[tt][j];
+        }
+      }
+    }
+    __syncthreads();
+    if (t0 + RUN < t_end) fetch(t0 + RUN);
+    float acc[RUN];
+#pragma unroll
+    for (int tt = 0; tt < RUN; ++tt) {
+      acc[tt] = 0.f;
+      if (tt < n) {  // uniform
+        const float4* kp = (const float4*)(lds + tt * 2 * VS + rg * PS);
+        const float4* qp = (const float4*)(lds + tt * 2 * VS + VS + rg * PS);
+        float kv[RPL], part[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int i4 = 0; i4 < RPL / 4; ++i4) {
+          const float4 k4 = kp[i4];
+          kv[4 * i4] = k4.x; kv[4 * i4 + 1] = k4.y; kv[4 * i4 + 2] = k4.z; kv[4 * i4 + 3] = k4.w;
+#pragma unroll
+          for (int u = 0; u < 4; ++u) {
+            S[4 * i4 + u] *= g[tt];
+            part[u] += S[4 * i4 + u] * kv[4 * i4 + u];
+          }
+        }
+        const float ks = column_sum((part[0] + part[1]) + (part[2] + part[3]));
+        const float uv = beta[tt] * (v[tt] - ks);
+        float op[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int i4 = 0; i4 < RPL / 4; ++i4) {
+          const float4 q4 = qp[i4];
+          const float qq[4] = {q4.x, q4.y, q4.z, q4.w};
+#pragma unroll
+          for (int u = 0; u < 4; ++u) {
+            S[4 * i4 + u] += kv[4 * i4 + u] * uv;
+            op[u] += S[4 * i4 + u] * qq[u];
+          }
+        }
+        acc[tt] = (op[0] + op[1]) + (op[2] + op[3]);
+      }
+    }
+#pragma unroll
+    for (int tt = 0; tt < RUN; ++tt) acc[tt] = column_sum(acc[tt]);
+    if (rg == 0 && col_ok) {
+#pragma unroll
+      for (int tt = 0; tt < RUN; ++tt)
+        if (tt < n) a.out[(size_t)(t0 + tt) * ((size_t)a.n_v * e) + h * e + col] = acc[tt];
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < RPL; ++i)
+    if (i < rpl && r0 + i < d && col_ok) S_mem[(size_t)(r0 + i) * e + col] = S[i];
+}
+
+static bool delta_scan_ok(const DeltaScanArgs& a, int n_seqs) {
+  return a.n_qk > 0 && a.n_v > 0 && a.n_v % a.n_qk == 0 && a.d > 0 && a.d <= 512 && a.e > 0 && a.n_v <= 65535 &&
+         n_seqs <= 65535 && (a.e + 7) / 8 <= 65535 && a.rows && a.state && a.slot_ids && a.q_start && a.out &&
+         a.stride >= 2 * a.n_qk * a.d + a.n_v * (a.e + 2);
+}
+
+extern "C" int fg_delta_scan(const DeltaScanArgs* args, int n_seqs, hipStream_t stream) {
+  if (n_seqs <= 0) return FG_OK;
+  const DeltaScanArgs& a = *args;
+  if (!delta_scan_ok(a, n_seqs)) return FG_ERR_ARG;
+  const dim3 grid(n_seqs, a.n_v, (a.e + 7) / 8);
+  const int rpl = (a.d + 7) / 8;
+  if (rpl <= 4) delta_scan_kernel<4><<<grid, FG_WAVE, 0, stream>>>(a);
+  else if (rpl <= 8) delta_scan_kernel<8><<<grid, FG_WAVE, 0, stream>>>(a);
+  else if (rpl <= 12) delta_scan_kernel<12><<<grid, FG_WAVE, 0, stream>>>(a);
+  else if (rpl <= 16) delta_scan_kernel<16><<<grid, FG_WAVE, 0, stream>>>(a);
+  else if (rpl <= 24) delta_scan_kernel<24><<<grid, FG_WAVE, 0, stream>>>(a);
+  else if (rpl <= 32) delta_scan_kernel<32><<<grid, FG_WAVE, 0, stream>>>(a);
+  else delta_scan_kernel<64><<<grid, FG_WAVE, 0, stream>>>(a);
+  return fg_launch_status();
+}

@@ -1,8 +1,8 @@
 // Per-head work around an attention or a recurrence that is no plain matrix product:
 //
 //  heads_prepare   what lies between the product that makes queries, keys and values and the
-//                  attention: a bias, an RMS norm per head (over the head's first dimensions),
-//                  the rotation of a run of dimensions, the queries to a buffer of their own (heads
+//                  attention: a causal convolution per channel, a bias, an RMS norm per head (over the
+//                  head's first dimensions) or over all of a token's query (key) columns, the rotation of a run of dimensions, the queries to a buffer of their own (heads
 //                  padded with zeros to the cache's head size) and keys and values into their cache
 //                  pages.  A value is either columns of its own or the first dimensions of its
 //                  processed key (a latent that serves as key and as value).
@@ -14,6 +14,7 @@
 // All arithmetic between a load and a store is fp32; a result is rounded once, at the store.
 #include "common.h"
 #include "kv_layout.h"
+#include "conv_inputs.h"
 
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef float f32x4 __attribute__((ext_vector_type(4)));
@@ -36,14 +37,15 @@ struct PrepareArgs {
   int norm_plain;                    // a head with norm dims and no norm weight is divided by its root mean square
   const int* positions; float q_temp_coef; int q_temp_every;  // queries times 1 + coef * ln(floor((p + 1) / every) + 1)
   const void* v_first; int v_first_stride; float v_blend;     // values become (1 - v_blend) v + v_blend v_first[t, head, :]
+  int row_norm;                      // the norms run over all n_q * q_w (n_kv * k_w) columns at once; weights [n * w]
+  ConvIn conv;  // before anything else, on the query and key columns (channel = source column)
 };
 
-// grid (T, ceil((n_q + n_kv) / HP_WAVES)); a wave a (token, head).  Lane l holds the pairs l, l + 64, ..
-template <class TS, class TA>
-__global__ __launch_bounds__(HP_WAVES* FG_WAVE) void heads_prepare_kernel(const PrepareArgs a) {
-  const int lane = threadIdx.x % FG_WAVE, wave = threadIdx.x / FG_WAVE;
-  const int t = blockIdx.x, job = blockIdx.y * HP_WAVES + wave;
-  if (job >= a.n_q + a.n_kv) return;  // whole waves; no block barrier below
+// A wave's (token, head): lane l holds the pairs l, l + 64, ..  CONV: the convolution comes first.  ROWN: the
+// norm's factor comes from the caller (row_rstd_q, row_rstd_k).
+template <class TS, class TA, bool CONV, bool ROWN>
+__device__ __forceinline__ void prepare_head(const PrepareArgs& a, int t, int job, float row_rstd_q, float row_rstd_k) {
+  const int lane = threadIdx.x % FG_WAVE;
   const bool is_q = job < a.n_q;
   const int head = is_q ? job : job - a.n_q;
   int slot = -1;
@@ -63,8 +65,12 @@ __global__ __launch_bounds__(HP_WAVES* FG_WAVE) void heads_prepare_kernel(const 
     const int d = 2 * (lane + FG_WAVE * j);
     x[j][0] = x[j][1] = 0.f;
     if (d < w) {
-      x[j][0] = to_f<TS>(row[col + d]);
-      x[j][1] = to_f<TS>(row[col + d + 1]);
+      if (CONV) {
+        conv_pair<TS>(a.conv, (const TS*)a.src, a.src_stride, t, col + d, x[j]);
+      } else {
+        x[j][0] = to_f<TS>(row[col + d]);
+        x[j][1] = to_f<TS>(row[col + d + 1]);
+      }
       if (a.bias) {
         x[j][0] += a.bias[col + d];
         x[j][1] += a.bias[col + d + 1];
@@ -75,7 +81,17 @@ __global__ __launch_bounds__(HP_WAVES* FG_WAVE) void heads_prepare_kernel(const 
   // a query's temperature grows with the logarithm of its position, in steps of `every` positions
   const bool tempered = is_q && a.positions && a.q_temp_every > 0;  // uniform
   const float temp = tempered ? 1.f + a.q_temp_coef * logf((float)((a.positions[t] + 1) / a.q_temp_every) + 1.f) : 1.f;
-  if (norm_w || (a.norm_plain && norm_dims > 0)) {  // uniform
+  if (ROWN) {
+    const float rstd = is_q ? row_rstd_q : row_rstd_k;
+#pragma unroll
+    for (int j = 0; j < HP_MAX_PAIRS; ++j) {
+      const int d = 2 * (lane + FG_WAVE * j);
+      if (d < w) {
+        x[j][0] = x[j][0] * rstd * norm_w[head * w + d];
+        x[j][1] = x[j][1] * rstd * norm_w[head * w + d + 1];
+      }
+    }
+  } else if (norm_w || (a.norm_plain && norm_dims > 0)) {  // uniform
     ss = wave_sum(ss);
     const float rstd = rsqrtf(ss / (float)norm_dims + a.eps);
 #pragma unroll
@@ -152,6 +168,49 @@ __global__ __launch_bounds__(HP_WAVES* FG_WAVE) void heads_prepare_kernel(const 
   }
 }
 
+// grid (T, ceil((n_q + n_kv) / HP_WAVES)); a wave a (token, head)
+template <class TS, class TA, bool CONV>
+__global__ __launch_bounds__(HP_WAVES* FG_WAVE) void heads_prepare_kernel(const PrepareArgs a) {
+  const int job = blockIdx.y * HP_WAVES + threadIdx.x / FG_WAVE;
+  if (job >= a.n_q + a.n_kv) return;  // whole waves; no block barrier below
+  prepare_head<TS, TA, CONV, false>(a, blockIdx.x, job, 0.f, 0.f);
+}
+
+// Norms over all of a token's query columns and all its key columns: a workgroup a token, whose waves take the
+// heads in turns once the two sums of squares are there.
+#define HP_ROW_WAVES 8
+template <class TS, class TA>
+__global__ __launch_bounds__(HP_ROW_WAVES* FG_WAVE) void heads_prepare_row_kernel(const PrepareArgs a) {
+  __shared__ float red[2][HP_ROW_WAVES];
+  const int t = blockIdx.x, wave = threadIdx.x / FG_WAVE, lane = threadIdx.x % FG_WAVE;
+  const TS* row = (const TS*)a.src + (size_t)t * a.src_stride;
+  const int nq = a.n_q * a.q_w, nk = a.n_kv * a.k_w;
+  float sq = 0.f, sk = 0.f;
+  for (int i = threadIdx.x; i < nq; i += HP_ROW_WAVES * FG_WAVE) {
+    const float v = to_f<TS>(row[a.q_col + i]) + (a.bias ? a.bias[a.q_col + i] : 0.f);
+    sq += v * v;
+  }
+  for (int i = threadIdx.x; i < nk; i += HP_ROW_WAVES * FG_WAVE) {
+    const float v = to_f<TS>(row[a.k_col + i]) + (a.bias ? a.bias[a.k_col + i] : 0.f);
+    sk += v * v;
+  }
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  if (lane == 0) {
+    red[0][wave] = sq;
+    red[1][wave] = sk;
+  }
+  __syncthreads();
+  sq = sk = 0.f;
+#pragma unroll
+  for (int i = 0; i < HP_ROW_WAVES; ++i) {
+    sq += red[0][i];
+    sk += red[1][i];
+  }
+  const float rq = nq ? rsqrtf(sq / (float)nq + a.eps) : 0.f, rk = nk ? rsqrtf(sk / (float)nk + a.eps) : 0.f;
+  for (int job = wave; job < a.n_q + a.n_kv; job += HP_ROW_WAVES) prepare_head<TS, TA, false, true>(a, t, job, rq, rk);
+}
+
 extern "C" int fg_heads_prepare(const PrepareArgs* args, int n_tokens, int src_dtype, int act_dtype,
                                 hipStream_t stream) {
   if (n_tokens <= 0) return FG_OK;
@@ -169,14 +228,21 @@ extern "C" int fg_heads_prepare(const PrepareArgs* args, int n_tokens, int src_d
   const int jobs = a.n_q + a.n_kv;
   dim3 grid(n_tokens, (jobs + HP_WAVES - 1) / HP_WAVES);
   if (grid.y > 65535) return FG_ERR_ARG;
-  if (src_dtype == FG_F32 && act_dtype == FG_F32)
-    heads_prepare_kernel<float, float><<<grid, HP_WAVES * FG_WAVE, 0, stream>>>(a);
-  else if (src_dtype == FG_F32 && act_dtype == FG_BF16)
-    heads_prepare_kernel<float, bf16_t><<<grid, HP_WAVES * FG_WAVE, 0, stream>>>(a);
-  else if (src_dtype == FG_BF16 && act_dtype == FG_BF16)
-    heads_prepare_kernel<bf16_t, bf16_t><<<grid, HP_WAVES * FG_WAVE, 0, stream>>>(a);
-  else
+  if (a.conv.w && (!fg_conv_ok(a.conv) || (a.n_q && a.q_col + a.n_q * a.q_w > a.conv.channels) ||
+                   (a.n_kv && a.k_col + a.n_kv * a.k_w > a.conv.channels)))
     return FG_ERR_ARG;
+  if (a.row_norm && (a.conv.w || (a.n_q && !a.q_norm_w) || (a.n_kv && !a.k_norm_w))) return FG_ERR_ARG;
+#define GO(TS, TA)                                                                                              \
+  do {                                                                                                          \
+    if (a.row_norm) heads_prepare_row_kernel<TS, TA><<<n_tokens, HP_ROW_WAVES * FG_WAVE, 0, stream>>>(a);       \
+    else if (a.conv.w) heads_prepare_kernel<TS, TA, true><<<grid, HP_WAVES * FG_WAVE, 0, stream>>>(a);          \
+    else heads_prepare_kernel<TS, TA, false><<<grid, HP_WAVES * FG_WAVE, 0, stream>>>(a);                       \
+  } while (0)
+  if (src_dtype == FG_F32 && act_dtype == FG_F32) GO(float, float);
+  else if (src_dtype == FG_F32 && act_dtype == FG_BF16) GO(float, bf16_t);
+  else if (src_dtype == FG_BF16 && act_dtype == FG_BF16) GO(bf16_t, bf16_t);
+  else return FG_ERR_ARG;
+#undef GO
   return fg_launch_status();
 }
 
@@ -188,11 +254,12 @@ struct HeadLinearArgs {
   const float* gate; int gate_stride;  // gate[t * gate_stride + h] or null: y *= sigmoid(gate)
   int T, H, N, K;
   int tail, y_hw;  // y[t, h, N + j] = x[t, h, K + j] for j < tail; zeros from N + tail to y_hw
+  const float* bias;  // [H, N] or null, added to the product
 };
 
 // Any dtype: grid (T, H), 256 threads; x's head goes through LDS, a thread an output element.
 #define HL_MAX_K 1024
-template <class T>
+template <class T, class TY>
 __global__ __launch_bounds__(256) void head_linear_kernel(const HeadLinearArgs a) {
   __shared__ float x_s[HL_MAX_K];
   const int t = blockIdx.x, h = blockIdx.y;
@@ -201,24 +268,26 @@ __global__ __launch_bounds__(256) void head_linear_kernel(const HeadLinearArgs a
   __syncthreads();
   float gv = 1.f;
   if (a.gate) gv = 1.f / (1.f + expf(-a.gate[(size_t)t * a.gate_stride + h]));
-  T* y = (T*)a.y + (size_t)t * a.y_stride + (size_t)h * a.y_hs;
+  TY* y = (TY*)a.y + (size_t)t * a.y_stride + (size_t)h * a.y_hs;
   const T* w = (const T*)a.w + (size_t)h * a.N * a.K;
   for (int n = threadIdx.x; n < a.y_hw; n += 256) {
     float acc = 0.f;
     if (n < a.N) {
       const T* wr = w + (size_t)n * a.K;
       for (int k = 0; k < a.K; ++k) acc += to_f<T>(wr[k]) * x_s[k];  // k ascending
+      if (a.bias) acc += a.bias[(size_t)h * a.N + n];
       acc *= gv;
     } else if (n < a.N + a.tail) {
       acc = to_f<T>(x[a.K + n - a.N]);
     }
-    y[n] = from_f<T>(acc);
+    y[n] = from_f<TY>(acc);
   }
 }
 
 // bfloat16 on the matrix cores: grid (ceil(T / 64), ceil(N / 64), H), 4 waves; a wave takes 16
 // output channels and 64 tokens (four blocks of 16), operands straight from memory.  K % 8 == 0 and
 // rows of x 16-byte aligned.  acc[mb][i] = y[token 16 mb + (lane & 15)][channel 4 (lane >> 4) + i].
+template <class TY>
 __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const HeadLinearArgs a) {
   const int lane = threadIdx.x % FG_WAVE, wave = threadIdx.x / FG_WAVE;
   const int r16 = lane & 15, g = lane >> 4;
@@ -254,11 +323,11 @@ __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const HeadLinearA
       if (t >= a.T) continue;
       float gv = 1.f;
       if (a.gate) gv = 1.f / (1.f + __expf(-a.gate[(size_t)t * a.gate_stride + h]));
-      bf16_t* y = (bf16_t*)a.y + (size_t)t * a.y_stride + (size_t)h * a.y_hs;
+      TY* y = (TY*)a.y + (size_t)t * a.y_stride + (size_t)h * a.y_hs;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int n = n0 + 4 * g + i;
-        if (n < a.N) y[n] = (bf16_t)(acc[mb][i] * gv);
+        if (n < a.N) y[n] = from_f<TY>((acc[mb][i] + (a.bias ? a.bias[(size_t)h * a.N + n] : 0.f)) * gv);
       }
     }
   }
@@ -268,12 +337,13 @@ __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const HeadLinearA
       const int t = m0 + e / extra, j = e % extra;
       if (t >= a.T) break;
       const bf16_t v = j < a.tail ? xh[(size_t)t * a.x_stride + a.K + j] : (bf16_t)0.f;
-      ((bf16_t*)a.y)[(size_t)t * a.y_stride + (size_t)h * a.y_hs + a.N + j] = v;
+      ((TY*)a.y)[(size_t)t * a.y_stride + (size_t)h * a.y_hs + a.N + j] = from_f<TY>(to_f<bf16_t>(v));
     }
   }
 }
 
-extern "C" int fg_head_linear(const HeadLinearArgs* args, int dtype, int use_mfma, hipStream_t stream) {
+// dtype: of x and w; out_dtype: of y, the same or fp32
+extern "C" int fg_head_linear(const HeadLinearArgs* args, int dtype, int out_dtype, int use_mfma, hipStream_t stream) {
   const HeadLinearArgs& a = *args;
   if (a.T <= 0) return FG_OK;
   if (a.H <= 0 || a.N <= 0 || a.K <= 0 || a.tail < 0 || a.y_hw < a.N + a.tail || a.x_hs < a.K + a.tail ||
@@ -282,24 +352,29 @@ extern "C" int fg_head_linear(const HeadLinearArgs* args, int dtype, int use_mfm
   if (use_mfma) {
     if (dtype != FG_BF16 || a.K % 8 || a.x_stride % 8 || a.x_hs % 8 || a.H > 65535 || (a.N + 63) / 64 > 65535)
       return FG_ERR_ARG;
-    head_linear_mfma_kernel<<<dim3((a.T + 63) / 64, (a.N + 63) / 64, a.H), 256, 0, stream>>>(a);
+    const dim3 grid((a.T + 63) / 64, (a.N + 63) / 64, a.H);
+    if (out_dtype == FG_BF16) head_linear_mfma_kernel<bf16_t><<<grid, 256, 0, stream>>>(a);
+    else if (out_dtype == FG_F32) head_linear_mfma_kernel<float><<<grid, 256, 0, stream>>>(a);
+    else return FG_ERR_ARG;
     return fg_launch_status();
   }
   if (a.K > HL_MAX_K || a.H > 65535) return FG_ERR_ARG;
-  if (dtype == FG_F32) head_linear_kernel<float><<<dim3(a.T, a.H), 256, 0, stream>>>(a);
-  else if (dtype == FG_BF16) head_linear_kernel<bf16_t><<<dim3(a.T, a.H), 256, 0, stream>>>(a);
+  const dim3 grid(a.T, a.H);
+  if (dtype == FG_F32 && out_dtype == FG_F32) head_linear_kernel<float, float><<<grid, 256, 0, stream>>>(a);
+  else if (dtype == FG_BF16 && out_dtype == FG_BF16) head_linear_kernel<bf16_t, bf16_t><<<grid, 256, 0, stream>>>(a);
+  else if (dtype == FG_BF16 && out_dtype == FG_F32) head_linear_kernel<bf16_t, float><<<grid, 256, 0, stream>>>(a);
   else return FG_ERR_ARG;
   return fg_launch_status();
 }
 
 // ---------------------------------------------------------------- head_norm_gate
-// out[t, h, :] = x[t, h, :] * rsqrt(mean(x[t, h, :]^2) + eps) * w * silu(g[t, h, :]); x fp32 [T, H * e],
+// out[t, h, :] = x[t, h, :] * rsqrt(mean(x[t, h, :]^2) + eps) * w * silu(g[t, h, :]) * out_scale; x fp32 [T, H * e],
 // g (act dtype) columns of a wider row.  grid (T, ceil(H / 4)); a wave a (token, head).
 #define HN_MAX 16  // elements a lane holds: heads of up to 1,024
-template <class TA>
+template <class TA, class TG>
 __global__ __launch_bounds__(HP_WAVES* FG_WAVE) void head_norm_gate_kernel(
-    const float* __restrict__ x, const float* __restrict__ w, const TA* __restrict__ gate, int gate_stride,
-    TA* __restrict__ out, int H, int e, float eps) {
+    const float* __restrict__ x, const float* __restrict__ w, const TG* __restrict__ gate, int gate_stride,
+    TA* __restrict__ out, int out_stride, int H, int e, float eps, float out_scale) {
   const int lane = threadIdx.x % FG_WAVE, wave = threadIdx.x / FG_WAVE;
   const int t = blockIdx.x, h = blockIdx.y * HP_WAVES + wave;
   if (h >= H) return;
@@ -313,33 +388,34 @@ __global__ __launch_bounds__(HP_WAVES* FG_WAVE) void head_norm_gate_kernel(
     ss += v[j] * v[j];
   }
   ss = wave_sum(ss);
-  const float rstd = rsqrtf(ss / (float)e + eps);
-  const TA* gr = gate + (size_t)t * gate_stride + (size_t)h * e;
-  TA* o = out + ((size_t)t * H + h) * e;
+  const float rstd = rsqrtf(ss / (float)e + eps) * out_scale;
+  const TG* gr = gate + (size_t)t * gate_stride + (size_t)h * e;
+  TA* o = out + (size_t)t * out_stride + (size_t)h * e;
 #pragma unroll
   for (int j = 0; j < HN_MAX; ++j) {
     const int d = lane + FG_WAVE * j;
     if (d < e) {
-      const float gv = to_f<TA>(gr[d]);
+      const float gv = to_f<TG>(gr[d]);
       o[d] = from_f<TA>(v[j] * rstd * w[d] * (gv / (1.f + expf(-gv))));
     }
   }
 }
 
 extern "C" int fg_head_norm_gate(const float* x, const float* w, const void* gate, int gate_stride, void* out,
-                                 int n_tokens, int H, int e, float eps, int act_dtype, hipStream_t stream) {
+                                 int out_stride, int n_tokens, int H, int e, float eps, float out_scale, int act_dtype, int gate_dtype,
+                                 hipStream_t stream) {
   if (n_tokens <= 0) return FG_OK;
-  if (H <= 0 || e <= 0 || e > HN_MAX * FG_WAVE || gate_stride < H * e || (H + HP_WAVES - 1) / HP_WAVES > 65535)
+  if (H <= 0 || e <= 0 || e > HN_MAX * FG_WAVE || gate_stride < H * e || out_stride < H * e || (H + HP_WAVES - 1) / HP_WAVES > 65535)
     return FG_ERR_ARG;
   dim3 grid(n_tokens, (H + HP_WAVES - 1) / HP_WAVES);
-  if (act_dtype == FG_F32)
-    head_norm_gate_kernel<float><<<grid, HP_WAVES * FG_WAVE, 0, stream>>>(x, w, (const float*)gate, gate_stride,
-                                                                         (float*)out, H, e, eps);
-  else if (act_dtype == FG_BF16)
-    head_norm_gate_kernel<bf16_t><<<grid, HP_WAVES * FG_WAVE, 0, stream>>>(x, w, (const bf16_t*)gate, gate_stride,
-                                                                          (bf16_t*)out, H, e, eps);
-  else
-    return FG_ERR_ARG;
+#define GO(TA, TG)                                                                                             \
+  head_norm_gate_kernel<TA, TG><<<grid, HP_WAVES * FG_WAVE, 0, stream>>>(x, w, (const TG*)gate, gate_stride,   \
+                                                                         (TA*)out, out_stride, H, e, eps, out_scale)
+  if (act_dtype == FG_F32 && gate_dtype == FG_F32) GO(float, float);
+  else if (act_dtype == FG_BF16 && gate_dtype == FG_BF16) GO(bf16_t, bf16_t);
+  else if (act_dtype == FG_BF16 && gate_dtype == FG_F32) GO(bf16_t, float);
+  else return FG_ERR_ARG;
+#undef GO
   return fg_launch_status();
 }
 

@@ -36,20 +36,38 @@ extern "C" int fg_embed(const void* table, int table_dtype, const int* tokens, f
   return fg_launch_status();
 }
 
+// What is added to element i of the stream where it is scaled first: a row of the activation dtype, or partial sums
+// added up in order, times `scale`.
+template <class TA>
+__device__ __forceinline__ float scaled_delta(const TA* drow, const float* prow, int n_parts, size_t part_stride, int i,
+                                              float scale) {
+  float d = drow ? to_f<TA>(drow[i]) : 0.f;
+  if (prow)
+    for (int p = 0; p < n_parts; ++p) d += prow[p * part_stride + i];
+  return d * scale;
+}
+
 // -------------------------------------------------- additions to the stream
 // h[t] = ((h[t] + delta[t]) + again[t]) + row, all fp32, in that order: what a layer left to be added
 // (rows of the activation dtype, or fp32 partial sums in order), then rows that enter the stream once
-// more (the embedding's output), then one vector for all tokens.  Each of the three may be absent.
+// more (the embedding's output), then one vector for all tokens.  Each of the three may be absent.  With `scale`
+// what a layer left is multiplied by it, element by element, first.
 template <class TA>
 __global__ __launch_bounds__(ROWS_THREADS) void stream_add_kernel(
     float* __restrict__ h, const TA* __restrict__ delta, const float* __restrict__ parts, int n_parts,
-    size_t part_stride, const float* __restrict__ again, const float* __restrict__ row, int dim) {
+    size_t part_stride, const float* __restrict__ scale, const float* __restrict__ again,
+    const float* __restrict__ row, int dim) {
   const size_t t = blockIdx.x;
   for (int i = threadIdx.x; i < dim; i += ROWS_THREADS) {
     float v = h[t * dim + i];
-    if (delta) v += to_f<TA>(delta[t * dim + i]);
-    if (parts)
-      for (int p = 0; p < n_parts; ++p) v += parts[p * part_stride + t * dim + i];
+    if (scale) {
+      v += scaled_delta<TA>(delta ? delta + t * dim : nullptr, parts ? parts + t * dim : nullptr, n_parts, part_stride, i,
+                            scale[i]);
+    } else {
+      if (delta) v += to_f<TA>(delta[t * dim + i]);
+      if (parts)
+        for (int p = 0; p < n_parts; ++p) v += parts[p * part_stride + t * dim + i];
+    }
     if (again) v += again[t * dim + i];
     if (row) v += row[i];
     h[t * dim + i] = v;
@@ -57,16 +75,16 @@ __global__ __launch_bounds__(ROWS_THREADS) void stream_add_kernel(
 }
 
 extern "C" int fg_stream_add(float* h, const void* delta, int delta_dtype, const float* parts, int n_parts,
-                             long long part_stride, const float* again, const float* row, int n_rows, int dim,
-                             hipStream_t stream) {
+                             long long part_stride, const float* scale, const float* again, const float* row,
+                             int n_rows, int dim, hipStream_t stream) {
   if (n_rows <= 0) return FG_OK;
   if (dim <= 0 || (parts && n_parts < 1)) return FG_ERR_ARG;
   if (delta_dtype == FG_F32)
     stream_add_kernel<float><<<n_rows, ROWS_THREADS, 0, stream>>>(h, (const float*)delta, parts, n_parts,
-                                                                  (size_t)part_stride, again, row, dim);
+                                                                  (size_t)part_stride, scale, again, row, dim);
   else if (delta_dtype == FG_BF16)
     stream_add_kernel<bf16_t><<<n_rows, ROWS_THREADS, 0, stream>>>(h, (const bf16_t*)delta, parts, n_parts,
-                                                                   (size_t)part_stride, again, row, dim);
+                                                                   (size_t)part_stride, scale, again, row, dim);
   else
     return FG_ERR_ARG;
   return fg_launch_status();
@@ -94,30 +112,31 @@ extern "C" int fg_add_rows(const void* a, const void* b, float* out, long long n
 
 // x[t][i] *= sigmoid(g[t][i]) (or g[t][i] itself when the sigmoid was taken where g was made), fp32
 // inside, one rounding.  Rows of x and g have strides of their own (g may be columns of a wider product).
-template <class TA>
-__global__ __launch_bounds__(ROWS_THREADS) void gate_mul_kernel(TA* __restrict__ x, int ldx, const TA* __restrict__ g,
+template <class TA, class TG>
+__global__ __launch_bounds__(ROWS_THREADS) void gate_mul_kernel(TA* __restrict__ x, int ldx, const TG* __restrict__ g,
                                                                 int ldg, int width, int sigmoid) {
   const size_t t = blockIdx.y;
   const int i = blockIdx.x * ROWS_THREADS + threadIdx.x;
   if (i >= width) return;
-  float gv = to_f<TA>(g[t * ldg + i]);
+  float gv = to_f<TG>(g[t * ldg + i]);
   if (sigmoid) gv = 1.f / (1.f + expf(-gv));
   x[t * ldx + i] = from_f<TA>(to_f<TA>(x[t * ldx + i]) * gv);
 }
 
 extern "C" int fg_gate_mul(void* x, int ldx, const void* g, int ldg, int n_rows, int width, int sigmoid, int dtype,
-                           hipStream_t stream) {
+                           int g_dtype, hipStream_t stream) {
   if (n_rows <= 0) return FG_OK;
   if (width <= 0 || ldx < width || ldg < width) return FG_ERR_ARG;
   for (int r0 = 0; r0 < n_rows; r0 += 65535) {
     const int nr = n_rows - r0 < 65535 ? n_rows - r0 : 65535;
     dim3 grid((width + ROWS_THREADS - 1) / ROWS_THREADS, nr);
-    if (dtype == FG_F32)
-      gate_mul_kernel<float><<<grid, ROWS_THREADS, 0, stream>>>((float*)x + (size_t)r0 * ldx, ldx,
-                                                                (const float*)g + (size_t)r0 * ldg, ldg, width, sigmoid);
-    else if (dtype == FG_BF16)
-      gate_mul_kernel<bf16_t><<<grid, ROWS_THREADS, 0, stream>>>((bf16_t*)x + (size_t)r0 * ldx, ldx,
-                                                                 (const bf16_t*)g + (size_t)r0 * ldg, ldg, width, sigmoid);
+#define GO(TA, TG)                                                                                              \
+  gate_mul_kernel<TA, TG><<<grid, ROWS_THREADS, 0, stream>>>((TA*)x + (size_t)r0 * ldx, ldx, (const TG*)g + (size_t)r0 * ldg, \
+                                                             ldg, width, sigmoid)
+    if (dtype == FG_F32 && g_dtype == FG_F32) GO(float, float);
+    else if (dtype == FG_BF16 && g_dtype == FG_BF16) GO(bf16_t, bf16_t);
+    else if (dtype == FG_BF16 && g_dtype == FG_F32) GO(bf16_t, float);
+#undef GO
     else
       return FG_ERR_ARG;
   }
@@ -131,12 +150,13 @@ extern "C" int fg_gate_mul(void* x, int ldx, const void* g, int ldg, int n_rows,
 // that reads it for the norm; a gathered call leaves h as it is (rows may
 // name a row twice).
 // What is added to h is either `delta` (rows of the activation dtype) or the sum, in order, of
-// `n_parts` fp32 partial results `parts[p]` (a matrix product whose k range was cut).
+// `n_parts` fp32 partial results `parts[p]` (a matrix product whose k range was cut).  With `scale` (fp32 [dim])
+// it is multiplied by that first, element by element.
 template <class TA, class TW>
 __global__ __launch_bounds__(ROWS_THREADS) void add_rmsnorm_kernel(
     float* __restrict__ h, const TA* __restrict__ delta, const float* __restrict__ parts, int n_parts,
-    size_t part_stride, const TW* __restrict__ w, TA* __restrict__ out, const int* __restrict__ rows, int dim,
-    float eps) {
+    size_t part_stride, const float* __restrict__ scale, const TW* __restrict__ w, TA* __restrict__ out,
+    const int* __restrict__ rows, int dim, float eps) {
   __shared__ float red[16];
   const int r = blockIdx.x;
   const size_t src = rows ? (size_t)rows[r] : (size_t)r;
@@ -146,9 +166,13 @@ __global__ __launch_bounds__(ROWS_THREADS) void add_rmsnorm_kernel(
   float ss = 0.f;
   for (int i = threadIdx.x; i < dim; i += ROWS_THREADS) {
     float v = hrow[i];
-    if (drow) v += to_f<TA>(drow[i]);
-    if (parts)
-      for (int p = 0; p < n_parts; ++p) v += parts[p * part_stride + src * dim + i];
+    if (scale) {
+      v += scaled_delta<TA>(drow, parts ? parts + src * dim : nullptr, n_parts, part_stride, i, scale[i]);
+    } else {
+      if (drow) v += to_f<TA>(drow[i]);
+      if (parts)
+        for (int p = 0; p < n_parts; ++p) v += parts[p * part_stride + src * dim + i];
+    }
     if (adds && !rows) hrow[i] = v;
     ss += v * v;
   }
@@ -158,7 +182,9 @@ __global__ __launch_bounds__(ROWS_THREADS) void add_rmsnorm_kernel(
   for (int i = threadIdx.x; i < dim; i += ROWS_THREADS) {
     // each thread re-reads only what it wrote itself above
     float v = hrow[i];
-    if (rows) {
+    if (rows && scale) {
+      v += scaled_delta<TA>(drow, parts ? parts + src * dim : nullptr, n_parts, part_stride, i, scale[i]);
+    } else if (rows) {
       if (drow) v += to_f<TA>(drow[i]);
       if (parts)
         for (int p = 0; p < n_parts; ++p) v += parts[p * part_stride + src * dim + i];
@@ -173,8 +199,8 @@ __global__ __launch_bounds__(ROWS_THREADS) void add_rmsnorm_kernel(
 template <class TA, class TW, int NIT>
 __global__ __launch_bounds__(ROWS_THREADS) void add_rmsnorm_vec_kernel(
     float* __restrict__ h, const TA* __restrict__ delta, const float* __restrict__ parts, int n_parts,
-    size_t part_stride, const TW* __restrict__ w, TA* __restrict__ out, const int* __restrict__ rows, int dim,
-    float eps) {
+    size_t part_stride, const float* __restrict__ scale, const TW* __restrict__ w, TA* __restrict__ out,
+    const int* __restrict__ rows, int dim, float eps) {
   __shared__ float red[16];
   const int r = blockIdx.x;
   const size_t src = rows ? (size_t)rows[r] : (size_t)r;
@@ -194,7 +220,42 @@ __global__ __launch_bounds__(ROWS_THREADS) void add_rmsnorm_vec_kernel(
   for (int it = 0; it < NIT; ++it) load8<float>(hrow + ec[it], v[it]);
 #pragma unroll
   for (int it = 0; it < NIT; ++it) load8<TW>(w + ec[it], wv[it]);
-  if (drow) {
+  if (scale && (drow || parts)) {  // uniform
+    float sv[NIT][8], d[NIT][8];
+#pragma unroll
+    for (int it = 0; it < NIT; ++it) load8<float>(scale + ec[it], sv[it]);
+    if (drow) {
+#pragma unroll
+      for (int it = 0; it < NIT; ++it) load8<TA>(drow + ec[it], d[it]);
+    } else {
+#pragma unroll
+      for (int it = 0; it < NIT; ++it)
+#pragma unroll
+        for (int i = 0; i < 8; ++i) d[it][i] = 0.f;
+    }
+    if (parts) {
+      constexpr int PB = 4;  // partial results whose loads are in flight together
+      for (int p0 = 0; p0 < n_parts; p0 += PB) {
+        float dp[NIT][PB][8];
+#pragma unroll
+        for (int it = 0; it < NIT; ++it)
+#pragma unroll
+          for (int p = 0; p < PB; ++p)
+            load8<float>(parts + (size_t)min(p0 + p, n_parts - 1) * part_stride + src * dim + ec[it], dp[it][p]);
+#pragma unroll
+        for (int it = 0; it < NIT; ++it)
+#pragma unroll
+          for (int p = 0; p < PB; ++p)
+#pragma unroll
+            for (int i = 0; i < 8; ++i) d[it][i] += p0 + p < n_parts ? dp[it][p][i] : 0.f;
+      }
+    }
+#pragma unroll
+    for (int it = 0; it < NIT; ++it)
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[it][i] += d[it][i] * sv[it][i];
+  }
+  if (drow && !scale) {
     float d[NIT][8];
 #pragma unroll
     for (int it = 0; it < NIT; ++it) load8<TA>(drow + ec[it], d[it]);
@@ -203,7 +264,7 @@ __global__ __launch_bounds__(ROWS_THREADS) void add_rmsnorm_vec_kernel(
 #pragma unroll
       for (int i = 0; i < 8; ++i) v[it][i] += d[it][i];
   }
-  if (parts) {
+  if (parts && !scale) {
     constexpr int PB = NIT <= 2 ? 8 : 4;  // partial results whose loads are in flight together
     for (int p0 = 0; p0 < n_parts; p0 += PB) {
       float dp[NIT][PB][8];
@@ -249,27 +310,27 @@ __global__ __launch_bounds__(ROWS_THREADS) void add_rmsnorm_vec_kernel(
 
 template <class TA, class TW>
 static void launch_add_rmsnorm(float* h, const void* delta, const float* parts, int n_parts, size_t part_stride,
-                               const void* w, void* out, const int* rows, int n_rows, int dim, float eps,
+                               const float* scale, const void* w, void* out, const int* rows, int n_rows, int dim, float eps,
                                hipStream_t stream) {
 #define VEC(NIT)                                                                              \
   add_rmsnorm_vec_kernel<TA, TW, NIT><<<n_rows, ROWS_THREADS, 0, stream>>>(                   \
-      h, (const TA*)delta, parts, n_parts, part_stride, (const TW*)w, (TA*)out, rows, dim, eps)
+      h, (const TA*)delta, parts, n_parts, part_stride, scale, (const TW*)w, (TA*)out, rows, dim, eps)
   if (dim % 8 == 0 && dim <= 2048) VEC(1);
   else if (dim % 8 == 0 && dim <= 4096) VEC(2);
   else if (dim % 8 == 0 && dim <= 8192) VEC(4);
   else
     add_rmsnorm_kernel<TA, TW><<<n_rows, ROWS_THREADS, 0, stream>>>(
-        h, (const TA*)delta, parts, n_parts, part_stride, (const TW*)w, (TA*)out, rows, dim, eps);
+        h, (const TA*)delta, parts, n_parts, part_stride, scale, (const TW*)w, (TA*)out, rows, dim, eps);
 #undef VEC
 }
 
 extern "C" int fg_add_rmsnorm(float* h, const void* delta, const float* parts, int n_parts,
-                              long long part_stride, const void* w, void* out, const int* rows, int n_rows,
-                              int dim, float eps, int act_dtype, int w_dtype, hipStream_t stream) {
+                              long long part_stride, const float* scale, const void* w, void* out, const int* rows,
+                              int n_rows, int dim, float eps, int act_dtype, int w_dtype, hipStream_t stream) {
   if (n_rows <= 0) return FG_OK;
   if (dim <= 0 || (parts && n_parts < 1)) return FG_ERR_ARG;
 #define LAUNCH(TA, TW) \
-  launch_add_rmsnorm<TA, TW>(h, delta, parts, n_parts, (size_t)part_stride, w, out, rows, n_rows, dim, eps, stream)
+  launch_add_rmsnorm<TA, TW>(h, delta, parts, n_parts, (size_t)part_stride, scale, w, out, rows, n_rows, dim, eps, stream)
   if (act_dtype == FG_F32 && w_dtype == FG_F32) LAUNCH(float, float);
   else if (act_dtype == FG_BF16 && w_dtype == FG_BF16) LAUNCH(bf16_t, bf16_t);
   else if (act_dtype == FG_BF16 && w_dtype == FG_F32) LAUNCH(bf16_t, float);

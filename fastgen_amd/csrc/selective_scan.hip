@@ -21,6 +21,7 @@
 // All arithmetic is fp32; the state never leaves fp32.  What a token gets depends on its sequence's earlier
 // tokens alone, in their order: not on the batch and not on how the tokens were cut into steps.
 #include "common.h"
+#include "conv_inputs.h"
 
 #define SS_THREADS 256
 #define SS_MAX_TAPS 16
@@ -30,7 +31,7 @@ __global__ __launch_bounds__(SS_THREADS) void causal_conv_kernel(
     const TS* __restrict__ x, int ldx, const float* __restrict__ taps, const float* __restrict__ bias,
     const float* __restrict__ state, int row_len, int tail_off, const int* __restrict__ slot_ids,
     const int* __restrict__ seq_of_token, const int* __restrict__ q_start, TA* __restrict__ out, int ldo, int C,
-    int K, int act) {
+    int K, int act, const float* __restrict__ in_bias) {
   const int c = blockIdx.y * SS_THREADS + threadIdx.x;
   const int t = blockIdx.x;
   if (c >= C) return;
@@ -39,9 +40,10 @@ __global__ __launch_bounds__(SS_THREADS) void causal_conv_kernel(
   const int i = t - t0;
   const float* tail = state + ((size_t)slot_ids[b] * C + c) * row_len + tail_off;
   float acc = bias ? bias[c] : 0.f;
+  const float xb = in_bias ? in_bias[c] : 0.f;  // (the tail holds inputs with it)
   for (int j = 0; j < K; ++j) {
     const int idx = i - (K - 1) + j;
-    const float v = idx >= 0 ? to_f<TS>(x[(size_t)(t0 + idx) * ldx + c]) : tail[K - 1 + idx];
+    const float v = idx >= 0 ? to_f<TS>(x[(size_t)(t0 + idx) * ldx + c]) + xb : tail[K - 1 + idx];
     acc = fmaf(v, taps[(size_t)c * K + j], acc);
   }
   if (act == 1) acc = acc / (1.f + expf(-acc));
@@ -51,7 +53,7 @@ __global__ __launch_bounds__(SS_THREADS) void causal_conv_kernel(
 extern "C" int fg_causal_conv(const void* x, int ldx, const float* taps, const float* bias, const float* state,
                               int row_len, int tail_off, const int* slot_ids, const int* seq_of_token,
                               const int* q_start, void* out, int ldo, int n_tokens, int C, int K, int act,
-                              int src_dtype, int act_dtype, hipStream_t stream) {
+                              const float* in_bias, int src_dtype, int act_dtype, hipStream_t stream) {
   if (n_tokens <= 0) return FG_OK;
   if (C <= 0 || K < 1 || K > SS_MAX_TAPS || ldx < C || ldo < C || tail_off < 0 || tail_off + K - 1 > row_len ||
       (C + SS_THREADS - 1) / SS_THREADS > 65535 || act < 0 || act > 1)
@@ -60,13 +62,47 @@ extern "C" int fg_causal_conv(const void* x, int ldx, const float* taps, const f
 #define GO(TS, TA)                                                                                             \
   causal_conv_kernel<TS, TA><<<grid, SS_THREADS, 0, stream>>>((const TS*)x, ldx, taps, bias, state, row_len,  \
                                                               tail_off, slot_ids, seq_of_token, q_start,       \
-                                                              (TA*)out, ldo, C, K, act)
+                                                              (TA*)out, ldo, C, K, act, in_bias)
   if (src_dtype == FG_F32 && act_dtype == FG_F32) GO(float, float);
   else if (src_dtype == FG_BF16 && act_dtype == FG_BF16) GO(bf16_t, bf16_t);
   else if (src_dtype == FG_F32 && act_dtype == FG_BF16) GO(float, bf16_t);
   else return FG_ERR_ARG;
 #undef GO
-#undef GO_OUT
+  return fg_launch_status();
+}
+
+// The tails of convolutions that other kernels apply (conv_inputs.h), moved on by this step's tokens: per sequence
+// and channel the last K - 1 inputs x + in_bias, old ones where the step brought fewer.  A thread a channel.
+template <class TS>
+__global__ __launch_bounds__(SS_THREADS) void conv_tail_kernel(const TS* __restrict__ x, int ldx,
+                                                               const float* __restrict__ in_bias, const ConvIn a) {
+  const int c = blockIdx.x * SS_THREADS + threadIdx.x, b = blockIdx.y;
+  if (c >= a.channels) return;
+  float* tail = a.state + (size_t)a.slot_ids[b] * a.slot_stride + (size_t)c * a.row_len + a.tail_off;
+  const int t0 = a.q_start[b], L = a.q_start[b + 1] - t0, keep = a.taps - 1;
+  const float xb = in_bias ? in_bias[c] : 0.f;
+  float nt[SS_MAX_TAPS - 1];
+#pragma unroll
+  for (int j = 0; j < SS_MAX_TAPS - 1; ++j) {
+    if (j < keep) {
+      const int src = L - keep + j;
+      nt[j] = src >= 0 ? to_f<TS>(x[(size_t)(t0 + src) * ldx + c]) + xb : tail[j + L];
+    }
+  }
+#pragma unroll
+  for (int j = 0; j < SS_MAX_TAPS - 1; ++j)
+    if (j < keep) tail[j] = nt[j];
+}
+
+extern "C" int fg_conv_tail(const void* x, int ldx, const float* in_bias, const ConvIn* args, int n_seqs, int src_dtype,
+                            hipStream_t stream) {
+  const ConvIn& a = *args;
+  if (n_seqs <= 0 || a.taps == 1) return FG_OK;
+  if (!fg_conv_ok(a) || ldx < a.channels || n_seqs > 65535) return FG_ERR_ARG;
+  const dim3 grid((a.channels + SS_THREADS - 1) / SS_THREADS, n_seqs);
+  if (src_dtype == FG_F32) conv_tail_kernel<float><<<grid, SS_THREADS, 0, stream>>>((const float*)x, ldx, in_bias, a);
+  else if (src_dtype == FG_BF16) conv_tail_kernel<bf16_t><<<grid, SS_THREADS, 0, stream>>>((const bf16_t*)x, ldx, in_bias, a);
+  else return FG_ERR_ARG;
   return fg_launch_status();
 }
 

@@ -18,7 +18,7 @@ import torch
 
 from ..config import ModelLayout, PartSpec, get_architecture, read_config_json
 from ..kernels.linear import StreamedMatrix, packing, packing_fits
-from ..kernels.ops import PostNormed, ScaledRows, post_add_rmsnorm, streams_spread
+from ..kernels.ops import PostNormed, ScaledDelta, ScaledRows, post_add_rmsnorm, stream_add, streams_spread
 from ..parts import LayerStore, PagedNeed, StateNeed, TensorSpec, build_part
 from ..parts.base import MATRIX
 from ..weights.source import RandomSource, SafetensorsSource, TensorSource, check_against_specs
@@ -190,6 +190,9 @@ class Model:
             if entry.inject is not None:
                 if isinstance(pending, PostNormed):  # a sublayer's output that is normed before it is added
                     post_add_rmsnorm(h, pending.rows, pending.weight, pending.eps, None, 0.0, None, delta_bias=pending.bias)
+                    pending = None
+                if isinstance(pending, ScaledDelta):  # ... or that is scaled per channel
+                    stream_add(h, pending.rows, None, None, delta_scale=pending.scale)
                     pending = None
                 injections[entry.inject[0]].forward(h, None if isinstance(pending, ScaledRows) else pending,
                                                     embedded, entry.inject[1])

@@ -33,7 +33,7 @@ HIPCC_FLAGS = [
     # packed fp32 instructions are kept out of the generated code
     "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
 ]
-HEADERS = ["common.h", "kv_layout.h", "attention_static.h"]
+HEADERS = ["common.h", "kv_layout.h", "attention_static.h", "conv_inputs.h"]
 
 # library name -> source file
 LIBRARIES: Dict[str, str] = {
@@ -50,6 +50,9 @@ LIBRARIES: Dict[str, str] = {
     "selective_scan": "selective_scan.hip",
     "sigmoid_attention": "sigmoid_attention.hip",
     "streams": "streams.hip",
+    "delta_rule": "delta_rule.hip",
+    "lru": "lru.hip",
+    "mixed_attention": "mixed_attention.hip",
 }
 
 # libraries compiled once per value of a macro: name -> (source, macro, values that build_all compiles,
@@ -57,6 +60,8 @@ LIBRARIES: Dict[str, str] = {
 VARIANT_LIBRARIES: Dict[str, tuple] = {
     "attention_mfma": ("attention_mfma.hip", "FG_HD", tuple(range(16, 257, 16)), ()),
     "attention_mfma_exact": ("attention_mfma.hip", "FG_HD", tuple(range(16, 257, 16)), ("-DFG_EXACT_P=1",)),
+    "attention_mfma_exact_dist": ("attention_mfma.hip", "FG_HD", tuple(range(16, 257, 16)),
+                                  ("-DFG_EXACT_P=1", "-DFG_DIST_BIAS=1")),
     "sigmoid_attention_mfma": ("sigmoid_attention_mfma.hip", "FG_HD", tuple(range(16, 257, 16)), ()),
 }
 

@@ -105,19 +105,32 @@ def embed(table: torch.Tensor, tokens: torch.Tensor, out: torch.Tensor, scale: f
     return out
 
 
+@dataclass
+class ScaledDelta:
+    """A sublayer's output on its way into the residual stream that is multiplied by a vector first: ``rows`` is
+    ``[T, dim]`` of the activation dtype or fp32 ``[S, T, dim]`` partial sums, ``scale`` fp32 ``[dim]`` (a learned scale
+    per channel, a constant of the model, their product).  A norm on the stream takes it where it takes rows."""
+
+    rows: torch.Tensor
+    scale: torch.Tensor
+
+
 def add_rmsnorm(h: torch.Tensor, delta: Optional[torch.Tensor], weight: torch.Tensor, eps: float,
-                out: torch.Tensor, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+                out: torch.Tensor, rows: Optional[torch.Tensor] = None,
+                delta_scale: Optional[torch.Tensor] = None) -> torch.Tensor:
     """``h += delta`` (fp32 residual stream), ``out = rmsnorm(h) * weight``.
 
     ``delta`` is ``[T, dim]`` of ``out``'s dtype, or fp32 ``[S, T, dim]``: partial
     sums of a matrix product whose k range was cut, added in order.  With
+    ``delta_scale`` (fp32 ``[dim]``) it is multiplied by that first, element by element.  With
     ``rows`` only those rows of ``h`` are normed, into consecutive rows of
     ``out``, and ``h`` is left unchanged.  Norm as in
     ``fastgen/kernels/rmsnorm.py:33-60``.
     """
-    _gpu(h, delta, weight, out, rows)
+    _gpu(h, delta, weight, out, rows, delta_scale)
     _need(h.dtype == torch.float32 and h.dim() == 2 and h.is_contiguous(), "h must be contiguous float32 [T, dim]")
     T, dim = h.shape
+    _f32_vec(delta_scale, dim, "delta_scale")
     n_rows = T if rows is None else rows.numel()
     if rows is not None:
         _i32(rows, "rows")
@@ -132,8 +145,8 @@ def add_rmsnorm(h: torch.Tensor, delta: Optional[torch.Tensor], weight: torch.Te
         _need(delta.shape == h.shape and delta.is_contiguous() and delta.dtype == out.dtype,
               "delta must be contiguous, shaped like h, of out's dtype")
     st = _lib.load("rows").fg_add_rmsnorm(
-        _ptr(h), _ptr(delta), _ptr(parts), n_parts, ctypes.c_longlong(part_stride), _ptr(weight), _ptr(out),
-        _ptr(rows), n_rows, dim, ctypes.c_float(eps), _code(out), _code(weight), _stream(out))
+        _ptr(h), _ptr(delta), _ptr(parts), n_parts, ctypes.c_longlong(part_stride), _ptr(delta_scale), _ptr(weight),
+        _ptr(out), _ptr(rows), n_rows, dim, ctypes.c_float(eps), _code(out), _code(weight), _stream(out))
     _check(st, "add_rmsnorm")
     return out
 
@@ -152,11 +165,12 @@ def _delta_args(h: torch.Tensor, delta: Optional[torch.Tensor], what: str):
 
 
 def stream_add(h: torch.Tensor, delta: Optional[torch.Tensor], again: Optional[torch.Tensor],
-               row: Optional[torch.Tensor]) -> torch.Tensor:
+               row: Optional[torch.Tensor], delta_scale: Optional[torch.Tensor] = None) -> torch.Tensor:
     """``h = ((h + delta) + again) + row`` in place on the fp32 stream ``h [T, dim]``, in that order:
-    ``delta`` as :func:`add_rmsnorm` takes it, ``again`` fp32 ``[T, dim]``, ``row`` fp32 ``[dim]`` for
+    ``delta`` (and ``delta_scale``) as :func:`add_rmsnorm` takes them, ``again`` fp32 ``[T, dim]``, ``row`` fp32 ``[dim]`` for
     every token.  Each may be None."""
-    _gpu(h, delta, again, row)
+    _gpu(h, delta, again, row, delta_scale)
+    _f32_vec(delta_scale, h.shape[1], "delta_scale")
     _need(h.dtype == torch.float32 and h.dim() == 2 and h.is_contiguous(), "h must be contiguous float32 [T, dim]")
     T, dim = h.shape
     if again is not None:
@@ -164,8 +178,8 @@ def stream_add(h: torch.Tensor, delta: Optional[torch.Tensor], again: Optional[t
               "again must be contiguous float32, shaped like h")
     if row is not None:
         _need(row.dtype == torch.float32 and row.shape == (dim,) and row.is_contiguous(), "row must be float32 [dim]")
-    st = _lib.load("rows").fg_stream_add(_ptr(h), *_delta_args(h, delta, "stream_add"), _ptr(again), _ptr(row), T, dim,
-                                         _stream(h))
+    st = _lib.load("rows").fg_stream_add(_ptr(h), *_delta_args(h, delta, "stream_add"), _ptr(delta_scale), _ptr(again),
+                                         _ptr(row), T, dim, _stream(h))
     _check(st, "stream_add")
     return h
 
@@ -184,13 +198,13 @@ def add_rows(a: torch.Tensor, b: torch.Tensor) -> torch.Tensor:
 
 def gate_mul(x: torch.Tensor, gate: torch.Tensor, sigmoid: bool = True) -> torch.Tensor:
     """``x *= sigmoid(gate)`` in place (``x *= gate`` with ``sigmoid=False``); ``x`` and ``gate`` are
-    ``[T, width]`` with unit column stride and row strides of their own."""
+    ``[T, width]`` with unit column stride and row strides of their own, of one dtype or ``gate`` fp32."""
     _gpu(x, gate)
     _need(x.dim() == 2 and gate.dim() == 2 and x.shape[0] == gate.shape[0] and gate.shape[1] >= x.shape[1]
-          and x.dtype == gate.dtype and x.stride(1) == 1 and gate.stride(1) == 1,
-          "x [T, width] and gate [T, >= width] must share a dtype and have unit column stride")
+          and gate.dtype in (x.dtype, torch.float32) and x.stride(1) == 1 and gate.stride(1) == 1,
+          "x [T, width] and gate [T, >= width] must have unit column stride, gate x's dtype or float32")
     st = _lib.load("rows").fg_gate_mul(_ptr(x), x.stride(0), _ptr(gate), gate.stride(0), x.shape[0], x.shape[1],
-                                       int(sigmoid), _code(x), _stream(x))
+                                       int(sigmoid), _code(x), _code(gate), _stream(x))
     _check(st, "gate_mul")
     return x
 
@@ -381,6 +395,12 @@ def rope_kv_write(qkv: torch.Tensor, positions: torch.Tensor, freqs: Optional[to
 
 
 # ------------------------------------------------------------------ attention
+def _distance_ok(distance: Optional[torch.Tensor], n_heads: int) -> None:
+    if distance is not None:
+        _need(distance.dtype == torch.float32 and distance.is_contiguous() and distance.shape == (n_heads, 2),
+              "distance must be contiguous float32 [H, 2]")
+
+
 def _sinks_ok(sinks: Optional[torch.Tensor], n_heads: int) -> None:
     if sinks is not None:
         _need(sinks.dtype == torch.float32 and sinks.is_contiguous() and sinks.shape == (n_heads,),
@@ -390,7 +410,8 @@ def _sinks_ok(sinks: Optional[torch.Tensor], n_heads: int) -> None:
 def paged_attention_general(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
                             block_table: torch.Tensor, seq_of_token: torch.Tensor, positions: torch.Tensor,
                             n_heads: int, scale: float, window: int = 0,
-                            sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                            sinks: Optional[torch.Tensor] = None,
+                            distance: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Causal attention of every token over its sequence's cached keys.
 
     ``q`` is ``[T, >= H*hd]`` (the first ``H*hd`` columns are the query heads;
@@ -399,9 +420,12 @@ def paged_attention_general(q: torch.Tensor, out: torch.Tensor, k_pages: torch.T
     denominator, which brings no value.  ``window`` > 0: a token at position ``p`` sees the keys
     ``p - window + 1 .. p``; ``window`` < 0: the keys up to ``p`` of its own block of ``-window`` positions,
     blocks counted from position 0 of the sequence (:func:`block_mask`); 0: every key up to ``p``.
+    ``distance``: fp32 ``[H, 2]``; head ``h``'s score of a key ``n`` tokens back loses
+    ``distance[h, 0] * ln(1 + distance[h, 1] * n)``.
     """
-    _gpu(q, out, k_pages, v_pages, block_table, seq_of_token, positions, sinks)
+    _gpu(q, out, k_pages, v_pages, block_table, seq_of_token, positions, sinks, distance)
     _sinks_ok(sinks, n_heads)
+    _distance_ok(distance, n_heads)
     T = q.shape[0]
     _need(k_pages.dim() == 4 and k_pages.is_contiguous(), "k_pages must be contiguous [n_pages, KV, P, hd]")
     n_pages, n_kv, page_size, hd = k_pages.shape
@@ -420,7 +444,7 @@ def paged_attention_general(q: torch.Tensor, out: torch.Tensor, k_pages: torch.T
     st = _lib.load("attention").fg_paged_attention_general_sink(
         _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(k_pages), _ptr(v_pages), _ptr(block_table),
         block_table.stride(0), _ptr(seq_of_token), _ptr(positions), T, n_heads, n_kv, hd, page_size,
-        ctypes.c_float(scale), int(window or 0), _ptr(sinks), _code(q), _stream(q))
+        ctypes.c_float(scale), int(window or 0), _ptr(sinks), _ptr(distance), _code(q), _stream(q))
     _check(st, "paged_attention_general")
     return out
 
@@ -457,16 +481,19 @@ def _split_target_blocks() -> int:
 _SPLIT_MIN_TILES = int(os.environ.get("FG_SPLIT_MIN_TILES", 4))
 
 
-def _mfma_attention(head_dim: int, exact: bool = False):
-    """The matrix-core attention library for this head size: the plain build, or the one whose softmax
-    weights keep 16 significant bits (a model that asks for it loads only that one)."""
+def _mfma_attention(head_dim: int, exact: bool = False, dist: bool = False):
+    """The matrix-core attention library for this head size: the plain build, the one whose softmax
+    weights keep 16 significant bits, or the one that does and whose scores take a distance bias (a model
+    loads only what it asks for)."""
+    if dist:
+        return _lib.load(f"attention_mfma_exact_dist@{head_dim}")
     return _lib.load(f"attention_mfma_exact@{head_dim}" if exact else f"attention_mfma@{head_dim}")
 
 
-def attention_tile_rows(head_dim: int, small: bool = False, exact: bool = False) -> int:
+def attention_tile_rows(head_dim: int, small: bool = False, exact: bool = False, dist: bool = False) -> int:
     """Query rows of one item of the tile kernel for this head size: of its larger form (128 rows up to
     head size 128), or of the form with ``small`` items (64 rows, more and lighter workgroups)."""
-    return int(_mfma_attention(head_dim, exact).fg_attn_tile_rows(int(small)))
+    return int(_mfma_attention(head_dim, exact, dist).fg_attn_tile_rows(int(small)))
 
 
 def attention_items(q_lens, q_start, n_cached, group_size: int, tile_rows: int = 64):
@@ -505,7 +532,7 @@ def _plan_ints(lib, max_chunks: int) -> int:
 
 
 def attention_plan(items: torch.Tensor, n_items: int, max_chunks: int, head_dim: int, window: int = 0,
-                   min_tiles: int = 4, exact: bool = False) -> torch.Tensor:
+                   min_tiles: int = 4, exact: bool = False, dist: bool = False) -> torch.Tensor:
     """Cuts the key ranges of ``items`` (device int32 ``[n_items, 4]``, 16-byte aligned) into chunks of
     the same number of 64-key tiles, a multiple of ``min_tiles``, on the device: a captured step cuts
     anew for the lengths of every replay.  The int32 plan that :func:`paged_attention_mfma` takes."""
@@ -513,7 +540,7 @@ def attention_plan(items: torch.Tensor, n_items: int, max_chunks: int, head_dim:
     _i32(items, "items")
     _need(items.data_ptr() % 16 == 0 and items.numel() >= 4 * n_items > 0, "items must be [n, 4], 16-byte aligned")
     _need(max_chunks >= 2 * n_items and min_tiles >= 1, "max_chunks must be at least twice the number of items")
-    lib = _mfma_attention(head_dim, exact)  # the plan is the same for every head size and build
+    lib = _mfma_attention(head_dim, exact, dist)  # the plan is the same for every head size and build
     plan = torch.empty(_plan_ints(lib, max_chunks), dtype=torch.int32, device=items.device)
     _check(lib.fg_attn_plan(_ptr(items), n_items, int(window or 0), max_chunks, min_tiles, _ptr(plan),
                             _stream(items)), "attn_plan")
@@ -538,7 +565,8 @@ def paged_attention_mfma(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tens
                          big_items: Optional[torch.Tensor], n_heads: int, scale: float, window: int = 0,
                          plan: Optional[torch.Tensor] = None, max_chunks: Optional[int] = None,
                          min_tiles: int = 4, max_rows: int = 16, tile_rows: Optional[int] = None,
-                         exact_weights: bool = False, sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                         exact_weights: bool = False, sinks: Optional[torch.Tensor] = None,
+                         distance: Optional[torch.Tensor] = None) -> torch.Tensor:
     """bf16 attention on the matrix cores.  ``small_items`` / ``big_items`` are
     device int32 ``[n, 4]`` lists from :func:`attention_items` (16-byte aligned);
     every query token of the step must be covered by exactly one item.
@@ -549,10 +577,12 @@ def paged_attention_mfma(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tens
     With items of both kinds the tile kernel runs on a second stream beside the split kernel and
     the current stream waits for it before this returns (not while a graph is captured, not with
     ``FG_ONE_STREAM=1``).  ``exact_weights``: the build of the kernels in which the softmax weights enter
-    the product with the values as two bfloat16 terms (16 significant bits).  ``sinks``: as
-    :func:`paged_attention_general`."""
-    _gpu(q, out, k_pages, v_pages, block_table, small_items, big_items, plan, sinks)
+    the product with the values as two bfloat16 terms (16 significant bits).  ``sinks`` and ``distance``: as
+    :func:`paged_attention_general` (a build of the kernels with exact weights takes the distance bias)."""
+    _gpu(q, out, k_pages, v_pages, block_table, small_items, big_items, plan, sinks, distance)
     _sinks_ok(sinks, n_heads)
+    _distance_ok(distance, n_heads)
+    dist = distance is not None
     n_pages, n_kv, page_size, hd = k_pages.shape
     _need(q.dtype == torch.bfloat16 and out.dtype == torch.bfloat16 and k_pages.dtype == torch.bfloat16
           and v_pages.dtype == torch.bfloat16, "the MFMA attention kernels take bfloat16")
@@ -567,7 +597,7 @@ def paged_attention_mfma(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tens
     _need(out.shape == (T, n_heads * hd) and out.stride(1) == 1 and out.stride(0) % 4 == 0, "out must be [T, H*hd]")
     _need(block_table.dim() == 2 and block_table.dtype == torch.int32 and block_table.stride(1) == 1,
           "block_table must be int32 [B, max_pages]")
-    lib = _mfma_attention(hd, exact_weights)
+    lib = _mfma_attention(hd, exact_weights, dist)
     G = n_heads // n_kv
     beside = None
     if (small_items is not None and small_items.numel() and big_items is not None and big_items.numel()
@@ -586,7 +616,7 @@ def paged_attention_mfma(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tens
             max_chunks = attention_chunks_for(n, n_kv)
         _need(2 * n <= max_chunks <= 65535, "the chunk list holds at least two chunks an item and at most 65535")
         if plan is None:
-            plan = attention_plan(small_items, n, max_chunks, hd, window, min_tiles, exact_weights)
+            plan = attention_plan(small_items, n, max_chunks, hd, window, min_tiles, exact_weights, dist)
         _need(plan.dtype == torch.int32 and plan.numel() == _plan_ints(lib, max_chunks),
               "the plan does not fit the items and max_chunks")
         part_o = torch.empty((max_chunks * n_kv * 16, hd), dtype=torch.float32, device=q.device)
@@ -594,11 +624,11 @@ def paged_attention_mfma(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tens
         st = lib.fg_attn_split_sink(
             _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(k_pages), _ptr(v_pages), _ptr(block_table),
             block_table.stride(0), _ptr(plan), n, max_chunks, max_rows, _ptr(part_o), _ptr(part_ml), n_heads, n_kv, hd,
-            page_size, ctypes.c_float(scale), int(window or 0), _ptr(sinks), _stream(q))
+            page_size, ctypes.c_float(scale), int(window or 0), _ptr(sinks), _ptr(distance), _stream(q))
         _check(st, "attn_split")
     if big_items is not None and big_items.numel():
-        tile_rows = attention_tile_rows(hd, False, exact_weights) if tile_rows is None else int(tile_rows)
-        _need(tile_rows in (attention_tile_rows(hd, False, exact_weights), attention_tile_rows(hd, True, exact_weights)),
+        tile_rows = attention_tile_rows(hd, False, exact_weights, dist) if tile_rows is None else int(tile_rows)
+        _need(tile_rows in (attention_tile_rows(hd, False, exact_weights, dist), attention_tile_rows(hd, True, exact_weights, dist)),
               "tile_rows is no form of the tile kernel")
         _need(G <= tile_rows, "too many query heads per kv head for the tile kernel")
         _i32(big_items, "big_items")
@@ -606,7 +636,7 @@ def paged_attention_mfma(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tens
         st = lib.fg_attn_tile_sink(
             _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(k_pages), _ptr(v_pages), _ptr(block_table),
             block_table.stride(0), _ptr(big_items), big_items.numel() // 4, tile_rows, n_heads, n_kv, hd, page_size,
-            ctypes.c_float(scale), int(window or 0), _ptr(sinks),
+            ctypes.c_float(scale), int(window or 0), _ptr(sinks), _ptr(distance),
             ctypes.c_void_p(beside.cuda_stream) if beside else _stream(q))
         _check(st, "attn_tile")
         if beside is not None:
@@ -616,7 +646,8 @@ def paged_attention_mfma(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tens
 
 def paged_attention(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
                     group, ctx, n_heads: int, scale: float, window: int = 0,
-                    exact_weights: bool = False, sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                    exact_weights: bool = False, sinks: Optional[torch.Tensor] = None,
+                    distance: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Attention for one step: picks the kernel for the step's dtype and shape.
     ``exact_weights``: see :func:`paged_attention_mfma` (the general kernel's weights are fp32 anyway).
 
@@ -630,7 +661,8 @@ def paged_attention(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v
     G = n_heads // n_kv
     if q.dtype != torch.bfloat16 or hd % 16 or hd > MFMA_MAX_HEAD_DIM or G > 16:
         return paged_attention_general(q, out, k_pages, v_pages, group.block_table, ctx.seq_of_token,
-                                       ctx.positions, n_heads, scale, window, sinks)
+                                       ctx.positions, n_heads, scale, window, sinks, distance)
+    dist = distance is not None
     items_key = ("attention_items", G, hd, n_kv)  # (how a step is cut into items depends on all three)
     plan = ctx.scratch.get(items_key)
     if plan is None:
@@ -639,13 +671,13 @@ def paged_attention(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v
             # already (and are refreshed with it when the step is a replayed graph)
             plan = (ctx.seq_records, None, ctx.n_seqs, None)
         else:
-            tile_rows = attention_tile_rows(hd, False, exact_weights)
+            tile_rows = attention_tile_rows(hd, False, exact_weights, dist)
             small, big = attention_items(ctx.q_lens, ctx.q_start_host, ctx.n_cached, G, tile_rows)
-            if 0 < len(big) * n_kv <= compute_units() // 2 and attention_tile_rows(hd, True, exact_weights) < tile_rows:
+            if 0 < len(big) * n_kv <= compute_units() // 2 and attention_tile_rows(hd, True, exact_weights, dist) < tile_rows:
                 # so few items that half the compute units would stand idle: items of half the rows, whose
                 # lighter workgroups share a unit (prompt portions of up to 512 tokens: 11.6 / 17.6 us
                 # against 14.1 / 19.5 at 256 / 512 tokens; equal at 1,024, slower beyond)
-                tile_rows = attention_tile_rows(hd, True, exact_weights)
+                tile_rows = attention_tile_rows(hd, True, exact_weights, dist)
                 small, big = attention_items(ctx.q_lens, ctx.q_start_host, ctx.n_cached, G, tile_rows)
             both = upload(np.concatenate([small, big]).reshape(-1), torch.int32, q.device)
             plan = (both[: small.size] if small.size else None, both[small.size:] if big.size else None, len(small),
@@ -660,12 +692,12 @@ def paged_attention(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v
         split_plan = ctx.scratch.get(key)
         if split_plan is None:
             split_plan = ctx.scratch[key] = attention_plan(small_d, n_small, chunks, hd, window, _SPLIT_MIN_TILES,
-                                                           exact_weights)
+                                                           exact_weights, dist)
     # rows of the largest small item: one token a sequence in a decode step (also a captured one)
     rows = G * int(ctx.q_lens.max()) if big_d is None else 16
     return paged_attention_mfma(q, out, k_pages, v_pages, group.block_table, small_d, big_d, n_heads, scale,
                                 window, split_plan, chunks, max_rows=min(16, rows), tile_rows=tile_rows,
-                                exact_weights=exact_weights, sinks=sinks)
+                                exact_weights=exact_weights, sinks=sinks, distance=distance)
 
 
 # ----------------------------------------------------------------------- gemm
@@ -1164,6 +1196,72 @@ def moe_combine(y: torch.Tensor, weight: torch.Tensor, plus: Optional[torch.Tens
     return out
 
 
+class _ConvIn(ctypes.Structure):
+    _fields_ = [("w", ctypes.c_void_p), ("taps", ctypes.c_int), ("state", ctypes.c_void_p),
+                ("slot_stride", ctypes.c_longlong), ("channels", ctypes.c_int), ("row_len", ctypes.c_int),
+                ("tail_off", ctypes.c_int), ("slot_ids", ctypes.c_void_p), ("seq_of_token", ctypes.c_void_p),
+                ("q_start", ctypes.c_void_p), ("move", ctypes.c_int)]
+
+
+CONV_MAX_TAPS = 16
+
+
+@dataclass
+class ConvInputs:
+    """A causal convolution per channel that a kernel applies where it reads its rows: ``taps`` fp32 ``[C, K]`` (the
+    last tap meets the token itself), and the state fp32 ``[n_slots, C, row_len]`` (slots and channels may have strides
+    of their own) whose rows hold the last ``K - 1`` inputs of earlier steps, oldest first, from column ``tail_off``
+    on, with the step's vectors to find them.  ``moves``: every
+    sequence of the step brings one token, and the kernel moves the tails on; else the caller does
+    (:func:`conv_tail`), behind every kernel that reads them."""
+
+    taps: torch.Tensor
+    state: torch.Tensor
+    tail_off: int
+    slot_ids: torch.Tensor
+    seq_of_token: torch.Tensor
+    q_start: torch.Tensor
+    moves: bool
+
+    def check(self, T: int, what: str) -> None:
+        C, K = self.taps.shape
+        _gpu(self.taps, self.state, self.slot_ids, self.seq_of_token, self.q_start)
+        _need(self.taps.dtype == torch.float32 and self.taps.is_contiguous() and 1 <= K <= CONV_MAX_TAPS,
+              f"{what}: taps must be contiguous float32 [C, 1..{CONV_MAX_TAPS}]")
+        _need(self.state.dtype == torch.float32 and self.state.dim() == 3 and self.state.shape[1] == C
+              and (self.state.stride(2) == 1 or self.state.shape[2] <= 1) and self.tail_off >= 0
+              and self.tail_off + K - 1 <= self.state.shape[2],
+              f"{what}: the state must be float32 [n_slots, C, >= tail_off + K - 1], rows contiguous")
+        _i32(self.seq_of_token, "seq_of_token", T)
+        _i32(self.slot_ids, "slot_ids")
+        _i32(self.q_start, "q_start")
+
+    def args(self) -> "_ConvIn":
+        C, K = self.taps.shape
+        a = _ConvIn()
+        a.w, a.taps, a.state, a.slot_stride = self.taps.data_ptr(), K, self.state.data_ptr(), self.state.stride(0)
+        a.channels, a.row_len, a.tail_off = C, self.state.stride(1), int(self.tail_off)
+        a.slot_ids, a.seq_of_token, a.q_start = self.slot_ids.data_ptr(), self.seq_of_token.data_ptr(), self.q_start.data_ptr()
+        a.move = int(bool(self.moves))
+        return a
+
+
+def conv_tail(x: torch.Tensor, conv: ConvInputs, n_seqs: int, in_bias: Optional[torch.Tensor] = None) -> None:
+    """Moves the convolutions' tails on by the step's tokens: every sequence's state row gets its last ``K - 1`` rows of
+    ``x [T, >= C]`` (plus ``in_bias`` fp32 ``[C]``), old ones where the step brought fewer."""
+    _gpu(x, in_bias)
+    C, K = conv.taps.shape
+    _rows_of_width(x, x.shape[0], C, "x")
+    _f32_vec(in_bias, C, "in_bias")
+    conv.check(x.shape[0], "conv_tail")
+    _i32(conv.slot_ids, "slot_ids", n_seqs)
+    _i32(conv.q_start, "q_start", n_seqs + 1)
+    a = conv.args()
+    st = _lib.load("selective_scan").fg_conv_tail(_ptr(x), x.stride(0), _ptr(in_bias), ctypes.byref(a), int(n_seqs), _code(x),
+                                                  _stream(x))
+    _check(st, "conv_tail")
+
+
 # ------------------------------------------------------------- per-head work
 class _PrepareArgs(ctypes.Structure):
     _fields_ = [("src", ctypes.c_void_p), ("src_stride", ctypes.c_int), ("bias", ctypes.c_void_p),
@@ -1176,7 +1274,8 @@ class _PrepareArgs(ctypes.Structure):
                 ("k_pages", ctypes.c_void_p), ("v_pages", ctypes.c_void_p), ("page_size", ctypes.c_int),
                 ("hd_c", ctypes.c_int), ("norm_plain", ctypes.c_int), ("positions", ctypes.c_void_p),
                 ("q_temp_coef", ctypes.c_float), ("q_temp_every", ctypes.c_int), ("v_first", ctypes.c_void_p),
-                ("v_first_stride", ctypes.c_int), ("v_blend", ctypes.c_float)]
+                ("v_first_stride", ctypes.c_int), ("v_blend", ctypes.c_float), ("row_norm", ctypes.c_int),
+                ("conv", _ConvIn)]
 
 
 def _f32_vec(t: Optional[torch.Tensor], n: int, name: str) -> None:
@@ -1193,7 +1292,8 @@ def heads_prepare(src: torch.Tensor, bias: Optional[torch.Tensor], eps: float,
                   rotate_q: bool = True, rotate_k: bool = True, slots: Optional[torch.Tensor] = None, k_pages: Optional[torch.Tensor] = None,
                   v_pages: Optional[torch.Tensor] = None, norm_plain: bool = False,
                   positions: Optional[torch.Tensor] = None, q_temp_coef: float = 0.0, q_temp_every: int = 0,
-                  v_first: Optional[torch.Tensor] = None, v_blend: float = 0.0) -> Optional[torch.Tensor]:
+                  v_first: Optional[torch.Tensor] = None, v_blend: float = 0.0, row_norm: bool = False,
+                  conv: Optional[ConvInputs] = None) -> Optional[torch.Tensor]:
     """What lies between a product's rows ``src [T, width]`` (fp32, or the activation dtype) and an attention.
 
     Per token and head: add ``bias`` (fp32, per column of ``src``); RMS-norm the head's first ``*_norm_dims``
@@ -1209,7 +1309,11 @@ def heads_prepare(src: torch.Tensor, bias: Optional[torch.Tensor], eps: float,
     ``norm_plain``: heads with norm dimensions but no norm weight are divided by their root mean square.
     ``positions`` with ``q_temp_every > 0``: after its norm a query at position ``p`` is multiplied by
     ``1 + q_temp_coef * ln(floor((p + 1) / q_temp_every) + 1)``.  ``v_first [T, n_kv * v_width]`` (of ``src``'s
-    dtype, unit column stride): the values become ``(1 - v_blend) v + v_blend v_first`` before they are stored."""
+    dtype, unit column stride): the values become ``(1 - v_blend) v + v_blend v_first`` before they are stored.
+
+    ``row_norm``: the norms run over all ``n_q * q_width`` query columns at once, and over all ``n_kv * k_width`` key
+    columns; ``q_norm`` and ``k_norm`` then have a weight per column.  ``conv``: the query and key columns pass a
+    causal convolution before anything else (its channel ``c`` is column ``c`` of ``src``)."""
     _gpu(src, bias, q_norm, q_out, k_norm, table, slots, k_pages, v_pages, positions, v_first)
     _need(src.dim() == 2 and src.stride(1) == 1, "src must be [T, width] with unit column stride")
     T, width = src.shape
@@ -1226,7 +1330,7 @@ def heads_prepare(src: torch.Tensor, bias: Optional[torch.Tensor], eps: float,
         _need(q_col >= 0 and q_col + n_q * q_width <= width, "the query heads lie outside src")
         _need(q_width % 2 == 0 and q_out_width % 2 == 0 and q_out_width <= 1024, "head widths must be even, at most 1024")
         _need(0 <= q_norm_dims <= q_width and q_norm_dims % 2 == 0, "q_norm_dims must be even and at most q_width")
-        _f32_vec(q_norm, q_norm_dims, "q_norm")
+        _f32_vec(q_norm, n_q * q_width if row_norm else q_norm_dims, "q_norm")
         _need(q_norm is None or q_norm_dims > 0, "a norm needs dimensions to run over")
         act = q_out.dtype
         a.q_col, a.q_w, a.q_norm_dims, a.q_norm_w = q_col, q_width, q_norm_dims, q_norm.data_ptr() if q_norm is not None else None
@@ -1247,7 +1351,7 @@ def heads_prepare(src: torch.Tensor, bias: Optional[torch.Tensor], eps: float,
         _need(v_col < 0 and v_width <= k_width or v_col >= 0 and v_col + n_kv * v_width <= width,
               "the values lie outside src (or, taken from the keys, are wider than they)")
         _need(0 <= k_norm_dims <= k_width and k_norm_dims % 2 == 0, "k_norm_dims must be even and at most k_width")
-        _f32_vec(k_norm, k_norm_dims, "k_norm")
+        _f32_vec(k_norm, n_kv * k_width if row_norm else k_norm_dims, "k_norm")
         _need(k_norm is None or k_norm_dims > 0, "a norm needs dimensions to run over")
         a.k_col, a.k_w, a.k_norm_dims, a.k_norm_w = k_col, k_width, k_norm_dims, k_norm.data_ptr() if k_norm is not None else None
         a.v_col, a.v_w = (v_col if v_col >= 0 else -1), v_width
@@ -1270,6 +1374,16 @@ def heads_prepare(src: torch.Tensor, bias: Optional[torch.Tensor], eps: float,
         _need(v_first.dtype == src.dtype and v_first.dim() == 2 and v_first.stride(1) == 1 and v_first.shape[0] == T
               and v_first.shape[1] >= n_kv * v_width, "v_first must be [T, >= n_kv * v_width] of src's dtype")
         a.v_first, a.v_first_stride, a.v_blend = v_first.data_ptr(), v_first.stride(0), float(v_blend)
+    if row_norm:
+        _need(conv is None and (not n_q or q_norm is not None) and (not n_kv or k_norm is not None),
+              "a norm over the whole projection needs weights and does not go with a convolution")
+        a.row_norm = 1
+    if conv is not None:
+        conv.check(T, "heads_prepare")
+        C, K = conv.taps.shape
+        _need((not n_q or q_col + n_q * q_width <= C) and (not n_kv or k_col + n_kv * k_width <= C),
+              "the convolution must cover the query and key columns")
+        a.conv = conv.args()
     st = _lib.load("heads").fg_heads_prepare(ctypes.byref(a), T, _code(src), _DTYPE_CODE[act], _stream(src))
     _check(st, "heads_prepare")
     return q_out
@@ -1279,16 +1393,16 @@ class _HeadLinearArgs(ctypes.Structure):
     _fields_ = [("x", ctypes.c_void_p), ("x_stride", ctypes.c_int), ("x_hs", ctypes.c_int), ("w", ctypes.c_void_p),
                 ("y", ctypes.c_void_p), ("y_stride", ctypes.c_int), ("y_hs", ctypes.c_int), ("gate", ctypes.c_void_p),
                 ("gate_stride", ctypes.c_int), ("T", ctypes.c_int), ("H", ctypes.c_int), ("N", ctypes.c_int),
-                ("K", ctypes.c_int), ("tail", ctypes.c_int), ("y_hw", ctypes.c_int)]
+                ("K", ctypes.c_int), ("tail", ctypes.c_int), ("y_hw", ctypes.c_int), ("bias", ctypes.c_void_p)]
 
 
 def head_linear(x: torch.Tensor, x_head_stride: int, w: torch.Tensor, out: torch.Tensor, out_head_stride: int,
-                tail: int = 0, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                tail: int = 0, gate: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
     """A product per head: ``out[t, h * out_head_stride + n] = sum_k w[h, n, k] * x[t, h * x_head_stride + k]``
-    for ``w [H, N, K]``; with fp32 ``gate [T, >= H]`` (unit column stride) the result is multiplied by
+    (plus fp32 ``bias [H, N]``) for ``w [H, N, K]``, in ``x``'s dtype or fp32; with fp32 ``gate [T, >= H]`` (unit column stride) the result is multiplied by
     ``sigmoid(gate[t, h])``.  The ``tail`` columns of ``x``'s head behind ``K`` are copied behind the ``N``
     results, and what is left of the ``out_head_stride`` columns is set to zero."""
-    _gpu(x, w, out, gate)
+    _gpu(x, w, out, gate, bias)
     _need(w.dim() == 3 and w.is_contiguous(), "w must be contiguous [H, N, K]")
     H, N, K = w.shape
     T = x.shape[0]
@@ -1296,8 +1410,11 @@ def head_linear(x: torch.Tensor, x_head_stride: int, w: torch.Tensor, out: torch
           "x must be [T, >= H * x_head_stride] with heads at least K + tail wide")
     _need(out.dim() == 2 and out.stride(1) == 1 and out.shape[0] == T and out_head_stride >= N + tail
           and out.shape[1] >= H * out_head_stride, "out must be [T, >= H * out_head_stride] with heads at least N + tail wide")
-    _need(x.dtype == w.dtype == out.dtype, "x, w and out must share a dtype")
+    _need(x.dtype == w.dtype and out.dtype in (x.dtype, torch.float32), "x and w must share a dtype, out's too or float32")
     a = _HeadLinearArgs()
+    _f32_vec(bias, H * N, "bias")
+    if bias is not None:
+        a.bias = bias.data_ptr()
     a.x, a.x_stride, a.x_hs, a.w = x.data_ptr(), x.stride(0), x_head_stride, w.data_ptr()
     a.y, a.y_stride, a.y_hs = out.data_ptr(), out.stride(0), out_head_stride
     if gate is not None:
@@ -1308,14 +1425,14 @@ def head_linear(x: torch.Tensor, x_head_stride: int, w: torch.Tensor, out: torch
     mfma = (x.dtype == torch.bfloat16 and K % 8 == 0 and x.stride(0) % 8 == 0 and x_head_stride % 8 == 0
             and x.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0)
     _need(mfma or K <= 1024, "heads of more than 1024 inputs need bfloat16 rows aligned to 16 bytes")
-    st = _lib.load("heads").fg_head_linear(ctypes.byref(a), _code(x), int(mfma), _stream(x))
+    st = _lib.load("heads").fg_head_linear(ctypes.byref(a), _code(x), _code(out), int(mfma), _stream(x))
     _check(st, "head_linear")
     return out
 
 
 def head_norm_gate(x: torch.Tensor, weight: torch.Tensor, eps: float, gate: torch.Tensor, n_heads: int,
-                   out: torch.Tensor) -> torch.Tensor:
-    """``out[t, h, :] = rmsnorm(x[t, h, :]) * weight * silu(gate[t, h, :])`` for fp32 ``x [T, H*e]``, fp32
+                   out: torch.Tensor, out_scale: float = 1.0) -> torch.Tensor:
+    """``out[t, h, :] = rmsnorm(x[t, h, :]) * weight * silu(gate[t, h, :]) * out_scale`` for fp32 ``x [T, H*e]``, fp32
     ``weight [e]`` shared by the heads, ``gate [T, >= H*e]`` (unit column stride) and ``out [T, H*e]`` of the
     activation dtype."""
     _gpu(x, weight, gate, out)
@@ -1323,11 +1440,12 @@ def head_norm_gate(x: torch.Tensor, weight: torch.Tensor, eps: float, gate: torc
     T, e = x.shape[0], x.shape[1] // n_heads
     _f32_vec(weight, e, "weight")
     _need(e <= 1024, "heads of at most 1024 elements")
-    _need(out.shape == x.shape and out.is_contiguous(), "out must be contiguous [T, H*e]")
+    _need(out.shape == x.shape and out.stride(1) == 1, "out must be [T, H*e] with unit column stride")
     _need(gate.dim() == 2 and gate.stride(1) == 1 and gate.shape[0] == T and gate.shape[1] >= n_heads * e
-          and gate.dtype == out.dtype, "gate must be [T, >= H*e] of out's dtype")
-    st = _lib.load("heads").fg_head_norm_gate(_ptr(x), _ptr(weight), _ptr(gate), gate.stride(0), _ptr(out), T, n_heads,
-                                              e, ctypes.c_float(eps), _code(out), _stream(out))
+          and gate.dtype in (out.dtype, torch.float32), "gate must be [T, >= H*e] of out's dtype or float32")
+    st = _lib.load("heads").fg_head_norm_gate(_ptr(x), _ptr(weight), _ptr(gate), gate.stride(0), _ptr(out), out.stride(0),
+                                              T, n_heads, e, ctypes.c_float(eps), ctypes.c_float(out_scale), _code(out),
+                                              _code(gate), _stream(out))
     _check(st, "head_norm_gate")
     return out
 
@@ -1577,15 +1695,17 @@ def _rows_of_width(t: torch.Tensor, T: int, width: int, name: str) -> None:
 
 def causal_conv(x: torch.Tensor, taps: torch.Tensor, bias: Optional[torch.Tensor], state: torch.Tensor, tail_off: int,
                 slot_ids: torch.Tensor, seq_of_token: torch.Tensor, q_start: torch.Tensor, out: torch.Tensor,
-                activation: Optional[str] = None) -> torch.Tensor:
+                activation: Optional[str] = None, in_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
     """A short causal convolution per channel over each sequence's tokens: ``out[t, c] = act(bias[c] + sum_j
-    taps[c, j] x[t - (K - 1) + j, c])``, the last tap on the token itself.  ``x [T, >= C]``; ``taps`` fp32
+    taps[c, j] (x[t - (K - 1) + j, c] + in_bias[c]))``, the last tap on the token itself.  ``x [T, >= C]``; ``taps`` fp32
     ``[C, K]``; tokens before this step's first are the last ``K - 1`` inputs of earlier steps, which
     ``state`` fp32 ``[n_slots, C, row_len]`` holds from column ``tail_off`` on at row ``slot_ids[seq]`` (zeros for
-    a new request).  The state is read only (:func:`selective_scan` moves it on).  ``activation``: None or ``silu``."""
-    _gpu(x, taps, bias, state, slot_ids, seq_of_token, q_start, out)
+    a new request; with ``in_bias`` already in them).  The state is read only (:func:`selective_scan` and
+    :func:`lru_scan` move it on).  ``activation``: None or ``silu``."""
+    _gpu(x, taps, bias, state, slot_ids, seq_of_token, q_start, out, in_bias)
     C, K = taps.shape
     T = x.shape[0]
+    _f32_vec(in_bias, C, "in_bias")
     _need(taps.dtype == torch.float32 and taps.is_contiguous(), "taps must be contiguous float32 [C, K]")
     _f32_vec(bias, C, "bias")
     _rows_of_width(x, T, C, "x")
@@ -1599,7 +1719,7 @@ def causal_conv(x: torch.Tensor, taps: torch.Tensor, bias: Optional[torch.Tensor
     st = _lib.load("selective_scan").fg_causal_conv(
         _ptr(x), x.stride(0), _ptr(taps), _ptr(bias), _ptr(state), state.shape[2], int(tail_off), _ptr(slot_ids),
         _ptr(seq_of_token), _ptr(q_start), _ptr(out), out.stride(0), T, C, K, 1 if activation == "silu" else 0,
-        _code(x), _code(out), _stream(out))
+        _ptr(in_bias), _code(x), _code(out), _stream(out))
     _check(st, "causal_conv")
     return out
 
@@ -1872,4 +1992,218 @@ def sigmoid_attention(q: torch.Tensor, head_dim: int, out: torch.Tensor, v_head_
             a.partial, a.n_chunks = partial.data_ptr(), n_chunks
     st = _lib.load("sigmoid_attention").fg_sigmoid_attention(ctypes.byref(a), _code(q), _stream(q))
     _check(st, "sigmoid_attention")
+    return out
+
+
+# ------------------------------------------- softmax attention with mixed heads
+class _MixedAttentionArgs(ctypes.Structure):
+    _fields_ = [("q", ctypes.c_void_p), ("q_stride", ctypes.c_int), ("q_hs", ctypes.c_int), ("k_pages", ctypes.c_void_p),
+                ("v_pages", ctypes.c_void_p), ("block_table", ctypes.c_void_p), ("bt_stride", ctypes.c_int),
+                ("seq_of_token", ctypes.c_void_p), ("positions", ctypes.c_void_p), ("n_tokens", ctypes.c_int),
+                ("n_heads", ctypes.c_int), ("n_kv", ctypes.c_int), ("d", ctypes.c_int), ("e", ctypes.c_int),
+                ("hd_c", ctypes.c_int), ("page_size", ctypes.c_int), ("scale", ctypes.c_float), ("softcap", ctypes.c_float),
+                ("window", ctypes.c_int), ("talk", ctypes.c_void_p), ("out_scale", ctypes.c_float), ("out", ctypes.c_void_p),
+                ("out_stride", ctypes.c_int)]
+
+
+def mixed_attention(q: torch.Tensor, head_dim: int, out: torch.Tensor, v_head_dim: int, k_pages: torch.Tensor,
+                    v_pages: torch.Tensor, block_table: torch.Tensor, seq_of_token: torch.Tensor, positions: torch.Tensor,
+                    n_heads: int, scale: float, talk: torch.Tensor, softcap: float = 0.0, window: int = 0,
+                    out_scale: float = 1.0) -> torch.Tensor:
+    """Causal softmax attention over the paged cache whose heads' weights are mixed after the softmax.
+
+    For the query at flat row ``t`` (position ``p`` of sequence ``seq_of_token[t]``) and every key it sees (``window`` as
+    :func:`paged_attention_general` takes it): ``s_h = q_h . k_j * scale``, through ``softcap * tanh(s_h / softcap)`` if
+    that is positive; ``p_h`` the softmax over the keys; ``w_h = sum_g talk[h, g] p_g`` (fp32 ``[H, H]``);
+    ``out[t, h] = sum_j w_h(j) v_j * out_scale`` with the values of head ``h``'s own key/value head.  ``q [T, >= H *
+    head_dim]`` and ``out [T, >= H * v_head_dim]`` have the cache's dtype; keys and values are the first ``head_dim`` and
+    ``v_head_dim`` elements of heads in ``k_pages [n_pages, G, P, hd]`` and ``v_pages [n_pages, G, hd, P]``, keys padded
+    with zeros to a multiple of 8.  All of it in fp32, one rounding."""
+    T, H, G, hd, P, a = _mixed_operands(_MixedAttentionArgs(), q, head_dim, out, v_head_dim, k_pages, v_pages, block_table,
+                                        positions, n_heads, scale, talk, softcap, window, out_scale)
+    _gpu(seq_of_token)
+    _i32(seq_of_token, "seq_of_token", T)
+    a.seq_of_token, a.hd_c = seq_of_token.data_ptr(), hd
+    _check(_lib.load("mixed_attention").fg_mixed_attention(ctypes.byref(a), _code(q), _stream(q)), "mixed_attention")
+    return out
+
+
+def _mixed_operands(a, q, head_dim, out, v_head_dim, k_pages, v_pages, block_table, positions, n_heads, scale, talk, softcap,
+                    window, out_scale):
+    """Checks what the kernels of attention with mixed heads have in common and fills it into ``a``."""
+    _gpu(q, out, k_pages, v_pages, block_table, positions, talk)
+    T, H, d, e = q.shape[0], int(n_heads), int(head_dim), int(v_head_dim)
+    _need(k_pages.dim() == 4 and k_pages.is_contiguous(), "k_pages must be contiguous [n_pages, G, P, hd]")
+    n_pages, G, P, hd = k_pages.shape
+    _need(v_pages.is_contiguous() and v_pages.shape == (n_pages, G, hd, P) and v_pages.dtype == k_pages.dtype,
+          "v_pages must be contiguous [n_pages, G, hd, P] of k_pages' dtype")
+    _need(H > 0 and H % G == 0 and 0 < d <= hd and 0 < e <= hd and hd % 8 == 0 and P % 8 == 0,
+          "heads must be a multiple of the cache's heads, head sizes at most the cache's")
+    _need(q.dtype == k_pages.dtype and out.dtype == k_pages.dtype, "q and out must have the cache's dtype")
+    _rows_of_width(q, T, H * d, "q")
+    _rows_of_width(out, T, H * e, "out")
+    _need(block_table.dim() == 2 and block_table.dtype == torch.int32 and block_table.stride(1) == 1, "block_table must be int32 [B, pages]")
+    _i32(positions, "positions", T)
+    _need(talk.dtype == torch.float32 and talk.is_contiguous() and talk.shape == (H, H), "talk must be contiguous float32 [H, H]")
+    _need(softcap >= 0, "softcap must not be negative")
+    a.q, a.q_stride, a.q_hs = q.data_ptr(), q.stride(0), d
+    a.k_pages, a.v_pages, a.block_table, a.bt_stride = k_pages.data_ptr(), v_pages.data_ptr(), block_table.data_ptr(), block_table.stride(0)
+    a.positions, a.n_tokens, a.n_heads, a.n_kv, a.d, a.e, a.page_size = positions.data_ptr(), T, H, G, d, e, P
+    a.scale, a.softcap, a.window, a.talk, a.out_scale = float(scale), float(softcap), int(window or 0), talk.data_ptr(), float(out_scale)
+    a.out, a.out_stride = out.data_ptr(), out.stride(0)
+    return T, H, G, hd, P, a
+
+
+# ------------------------------------------------------------ gated delta rule
+class _DeltaPrepareArgs(ctypes.Structure):
+    _fields_ = [("src", ctypes.c_void_p), ("src_stride", ctypes.c_int), ("n_qk", ctypes.c_int), ("d", ctypes.c_int),
+                ("n_v", ctypes.c_int), ("e", ctypes.c_int), ("conv", _ConvIn), ("b_col", ctypes.c_int), ("a_col", ctypes.c_int),
+                ("decay_rate", ctypes.c_void_p), ("dt_bias", ctypes.c_void_p), ("q_scale", ctypes.c_float),
+                ("unit_eps", ctypes.c_float), ("out", ctypes.c_void_p), ("out_stride", ctypes.c_int)]
+
+
+class _DeltaScanArgs(ctypes.Structure):
+    _fields_ = [("rows", ctypes.c_void_p), ("stride", ctypes.c_int), ("n_qk", ctypes.c_int), ("d", ctypes.c_int),
+                ("n_v", ctypes.c_int), ("e", ctypes.c_int), ("state", ctypes.c_void_p), ("slot_stride", ctypes.c_longlong),
+                ("slot_ids", ctypes.c_void_p), ("q_start", ctypes.c_void_p), ("out", ctypes.c_void_p)]
+
+
+def delta_prepare(src: torch.Tensor, n_qk: int, head_dim: int, n_v: int, v_head_dim: int, conv: ConvInputs, b_col: int,
+                  a_col: int, decay_rate: torch.Tensor, dt_bias: torch.Tensor, q_scale: float, unit_eps: float,
+                  out: torch.Tensor) -> torch.Tensor:
+    """What the gated delta rule takes of a token: ``out`` fp32 ``[T, q | k | v | beta | g]`` from the rows ``src [T, q | k |
+    v | ...]`` of a product (``n_qk`` query and key heads of ``head_dim``, ``n_v`` value heads of ``v_head_dim``).  q, k and v
+    pass ``conv`` and SiLU; every q and k head becomes ``x / sqrt(sum(x^2) + unit_eps)``, q times ``q_scale``;
+    ``beta = sigmoid(src[b_col + h])``; ``g = exp(-decay_rate[h] softplus(src[a_col + h] + dt_bias[h]))``."""
+    _gpu(src, decay_rate, dt_bias, out)
+    T, C = src.shape[0], 2 * n_qk * head_dim + n_v * v_head_dim
+    _need(min(n_qk, n_v, head_dim, v_head_dim) > 0 and n_v % n_qk == 0 and head_dim % 2 == 0 and v_head_dim % 2 == 0
+          and max(head_dim, v_head_dim) <= 1024, "heads must be even, at most 1024 wide, value heads a multiple of the others")
+    conv.check(T, "delta_prepare")
+    _need(conv.taps.shape[0] == C, "the convolution must have a channel for every column of q, k and v")
+    _rows_of_width(src, T, max(C, b_col + n_v, a_col + n_v), "src")
+    _need(min(b_col, a_col) >= 0, "the scalars' columns must lie inside src")
+    _f32_vec(decay_rate, n_v, "decay_rate")
+    _f32_vec(dt_bias, n_v, "dt_bias")
+    _need(out.dtype == torch.float32 and out.dim() == 2 and out.stride(1) == 1 and out.shape[0] == T
+          and out.shape[1] >= C + 2 * n_v and out.stride(0) % 2 == 0 and out.data_ptr() % 8 == 0,
+          "out must be float32 [T, >= q | k | v | beta | g], rows 8-byte aligned")
+    a = _DeltaPrepareArgs()
+    a.src, a.src_stride, a.n_qk, a.d, a.n_v, a.e = src.data_ptr(), src.stride(0), n_qk, head_dim, n_v, v_head_dim
+    a.conv, a.b_col, a.a_col = conv.args(), b_col, a_col
+    a.decay_rate, a.dt_bias, a.q_scale, a.unit_eps = decay_rate.data_ptr(), dt_bias.data_ptr(), float(q_scale), float(unit_eps)
+    a.out, a.out_stride = out.data_ptr(), out.stride(0)
+    _check(_lib.load("delta_rule").fg_delta_prepare(ctypes.byref(a), T, _code(src), _stream(src)), "delta_prepare")
+    return out
+
+
+def delta_scan(rows: torch.Tensor, n_qk: int, head_dim: int, n_v: int, v_head_dim: int, state: torch.Tensor,
+               slot_ids: torch.Tensor, q_start: torch.Tensor, n_seqs: int, out: torch.Tensor, q_start_host=None) -> torch.Tensor:
+    """The gated delta rule for every sequence of the step, in fp32: per value head ``h`` (query/key head ``h // (n_v /
+    n_qk)``) ``S <- g S``; ``u = beta (v - S^T k)``; ``S <- S + k u^T``; ``out[t, h] = S^T q``.
+
+    ``rows`` are :func:`delta_prepare`'s; ``state`` fp32 ``[n_slots, n_v, head_dim, v_head_dim]`` (slots may have a stride of
+    their own) is read at ``slot_ids[b]`` and left as the sequence's last token leaves it; ``out`` fp32 ``[T, n_v *
+    v_head_dim]``."""
+    _gpu(rows, state, slot_ids, q_start, out)
+    T, d, e = rows.shape[0], int(head_dim), int(v_head_dim)
+    _need(rows.dtype == torch.float32, "rows must be float32")
+    _rows_of_width(rows, T, 2 * n_qk * d + n_v * (e + 2), "rows")
+    _need(n_v % n_qk == 0 and d <= 512, "value heads a multiple of the others, at most 512 key channels")
+    _need(state.dtype == torch.float32 and state.dim() == 4 and tuple(state.shape[1:]) == (n_v, d, e)
+          and state.stride(3) == 1 and state.stride(2) == e and state.stride(1) == d * e, "state must be float32 [n_slots, n_v, d, e]")
+    _need(out.dtype == torch.float32 and out.is_contiguous() and out.shape == (T, n_v * e), "out must be contiguous float32 [T, n_v * e]")
+    _i32(slot_ids, "slot_ids", n_seqs)
+    _i32(q_start, "q_start", n_seqs + 1)
+    a = _DeltaScanArgs()
+    a.rows, a.stride, a.n_qk, a.d, a.n_v, a.e = rows.data_ptr(), rows.stride(0), n_qk, d, n_v, e
+    a.state, a.slot_stride, a.slot_ids, a.q_start = state.data_ptr(), state.stride(0), slot_ids.data_ptr(), q_start.data_ptr()
+    a.out = out.data_ptr()
+    _check(_lib.load("delta_rule").fg_delta_scan(ctypes.byref(a), int(n_seqs), _stream(rows)), "delta_scan")
+    return out
+
+
+# ------------------------------------------------- real-gated linear recurrence
+class _LruArgs(ctypes.Structure):
+    _fields_ = [("u", ctypes.c_void_p), ("ldu", ctypes.c_int), ("gates", ctypes.c_void_p), ("ldg", ctypes.c_int),
+                ("block", ctypes.c_int), ("decay", ctypes.c_void_p), ("y", ctypes.c_void_p), ("ldy", ctypes.c_int),
+                ("y_bias", ctypes.c_void_p), ("out_scale", ctypes.c_float), ("x_raw", ctypes.c_void_p), ("ldx", ctypes.c_int),
+                ("x_bias", ctypes.c_void_p), ("taps", ctypes.c_int), ("state", ctypes.c_void_p), ("row_len", ctypes.c_int),
+                ("slot_ids", ctypes.c_void_p), ("q_start", ctypes.c_void_p), ("out", ctypes.c_void_p), ("ldo", ctypes.c_int),
+                ("C", ctypes.c_int), ("chunk_log", ctypes.c_void_p), ("chunk_state", ctypes.c_void_p), ("pass_", ctypes.c_int)]
+
+
+LRU_CHUNK = 32  # tokens of a chunk where long runs of tokens are scanned chunk by chunk, side by side
+LRU_CHUNKED_FROM = 96  # the shortest run of tokens of one sequence for which a step is scanned so
+
+
+def _chunk_plan(q_start_host, n_seqs: int, chunk: int, device):
+    """The chunks of every sequence's tokens: (their number, device int32 first tokens ``[n + 1]``, first chunk of each
+    sequence ``[n_seqs + 1]``, ``0 .. n - 1``)."""
+    starts, seq_chunk = [], [0]
+    for b in range(n_seqs):
+        starts.extend(range(int(q_start_host[b]), int(q_start_host[b + 1]), chunk))
+        seq_chunk.append(len(starts))
+    n = len(starts)
+    _need(n <= 65535 and n_seqs <= 65535, "too many chunks or sequences in one step")
+    plan = upload(np.asarray(starts + [int(q_start_host[n_seqs])] + seq_chunk + list(range(n)), dtype=np.int32),
+                  torch.int32, device)
+    return n, plan[: n + 1], plan[n + 1 : n + n_seqs + 2], plan[n + n_seqs + 2 :]
+
+
+def lru_scan(u: torch.Tensor, gates: torch.Tensor, block: int, decay: torch.Tensor, y: torch.Tensor,
+             y_bias: Optional[torch.Tensor], out_scale: float, x_raw: Optional[torch.Tensor], x_bias: Optional[torch.Tensor],
+             taps: int, state: torch.Tensor, slot_ids: torch.Tensor, q_start: torch.Tensor, n_seqs: int, out: torch.Tensor,
+             q_start_host=None) -> torch.Tensor:
+    """A real-gated linear recurrence per channel, in fp32: with ``r, i`` the sigmoids of ``gates`` and ``log a = -r decay[c]``,
+    ``S <- a S + sqrt(1 - a^2) i u``; ``out = S * gelu_tanh(y + y_bias) * out_scale``.
+
+    ``u [T, >= C]`` and ``out`` have the activation dtype; ``gates`` fp32 ``[T, >= 2 C]``: per block of ``block`` channels
+    its logits of ``r``, then its logits of ``i``; ``decay`` fp32 ``[C]``, positive; ``y`` fp32 ``[T, >= C]``; ``state`` fp32
+    ``[n_slots, C, row_len]`` holds ``S`` in its first column and, behind it, the last ``taps - 1`` rows of ``x_raw + x_bias``
+    (fp32, the input of the convolution that made ``u``); both move on by the step's tokens.
+
+    ``q_start_host``: ``q_start`` on the host.  With it, a step in which a sequence brings ``LRU_CHUNKED_FROM`` tokens or
+    more is scanned in chunks of ``LRU_CHUNK`` tokens side by side; the result differs from the token-by-token scan's by
+    rounding (a chunk's decay is the exponential of a sum, not a product)."""
+    _gpu(u, gates, decay, y, y_bias, x_raw, x_bias, state, slot_ids, q_start, out)
+    C, T = decay.numel(), u.shape[0]
+    _f32_vec(decay, C, "decay")
+    _f32_vec(y_bias, C, "y_bias")
+    _f32_vec(x_bias, C, "x_bias")
+    _rows_of_width(u, T, C, "u")
+    _rows_of_width(out, T, C, "out")
+    _rows_of_width(gates, T, 2 * C, "gates")
+    _rows_of_width(y, T, C, "y")
+    _need(block > 0 and C % block == 0, "the channels must be a multiple of a block's")
+    _need(u.dtype == out.dtype and gates.dtype == torch.float32 and y.dtype == torch.float32, "u and out share a dtype; gates and y are float32")
+    a = _LruArgs()
+    _need(1 <= taps <= CONV_MAX_TAPS and (taps == 1 or x_raw is not None), "the convolution's input is needed to move its tail on")
+    if taps > 1:
+        _rows_of_width(x_raw, T, C, "x_raw")
+        _need(x_raw.dtype == torch.float32, "x_raw must be float32")
+        a.x_raw, a.ldx = x_raw.data_ptr(), x_raw.stride(0)
+    _need(state.dtype == torch.float32 and state.dim() == 3 and state.is_contiguous() and state.shape[1] == C
+          and state.shape[2] >= taps, "state must be contiguous float32 [n_slots, C, >= taps]")
+    _i32(slot_ids, "slot_ids", n_seqs)
+    _i32(q_start, "q_start", n_seqs + 1)
+    a.u, a.ldu, a.gates, a.ldg, a.block, a.decay = u.data_ptr(), u.stride(0), gates.data_ptr(), gates.stride(0), int(block), decay.data_ptr()
+    a.y, a.ldy, a.y_bias = y.data_ptr(), y.stride(0), (y_bias.data_ptr() if y_bias is not None else None)
+    a.out_scale, a.x_bias, a.taps = float(out_scale), (x_bias.data_ptr() if x_bias is not None else None), int(taps)
+    a.state, a.row_len, a.slot_ids, a.q_start = state.data_ptr(), state.shape[2], slot_ids.data_ptr(), q_start.data_ptr()
+    a.out, a.ldo, a.C = out.data_ptr(), out.stride(0), C
+    lib = _lib.load("lru")
+    lens = np.diff(np.asarray(q_start_host[: n_seqs + 1])) if q_start_host is not None else None
+    if lens is None or not len(lens) or int(lens.max()) < LRU_CHUNKED_FROM or torch.cuda.is_current_stream_capturing():
+        _check(lib.fg_lru_scan(ctypes.byref(a), int(n_seqs), _code(out), _stream(out)), "lru_scan")
+        return out
+    n_chunks, chunk_start, seq_chunk, _ = _chunk_plan(q_start_host, n_seqs, LRU_CHUNK, u.device)
+    sums = torch.empty((2, n_chunks, C), dtype=torch.float32, device=u.device)
+    a.chunk_log, a.chunk_state = sums[0].data_ptr(), sums[1].data_ptr()
+    a.q_start, a.pass_ = chunk_start.data_ptr(), 1
+    _check(lib.fg_lru_scan(ctypes.byref(a), n_chunks, _code(out), _stream(out)), "lru_scan (chunks' sums)")
+    a.q_start = q_start.data_ptr()
+    _check(lib.fg_lru_chunk_states(ctypes.byref(a), _ptr(seq_chunk), int(n_seqs), _stream(out)), "lru_chunk_states")
+    a.q_start, a.pass_ = chunk_start.data_ptr(), 2
+    _check(lib.fg_lru_scan(ctypes.byref(a), n_chunks, _code(out), _stream(out)), "lru_scan (chunks' outputs)")
     return out

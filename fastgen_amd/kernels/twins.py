@@ -27,17 +27,21 @@ def embed(table: torch.Tensor, tokens: torch.Tensor, out: torch.Tensor, scale: f
     return out
 
 
-def _added(delta: Optional[torch.Tensor]):
-    """What a ``delta`` argument adds, in order: rows ``[T, dim]``, or fp32 partial sums ``[S, T, dim]``."""
+def _added(delta: Optional[torch.Tensor], scale: Optional[torch.Tensor] = None):
+    """What a ``delta`` argument adds, in order: rows ``[T, dim]``, or fp32 partial sums ``[S, T, dim]``; with ``scale
+    [dim]`` one term, their sum times it."""
     if delta is None:
         return []
+    if scale is not None:
+        return [(delta.float().sum(0) if delta.dim() == 3 else delta.float()) * scale.float()]
     return [delta[s] for s in range(delta.shape[0])] if delta.dim() == 3 else [delta.float()]
 
 
 def stream_add(h: torch.Tensor, delta: Optional[torch.Tensor], again: Optional[torch.Tensor],
-               row: Optional[torch.Tensor]) -> torch.Tensor:
-    """``h = ((h + delta) + again) + row`` in place, fp32, in that order; each term may be None."""
-    for d in _added(delta):
+               row: Optional[torch.Tensor], delta_scale: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``h = ((h + delta) + again) + row`` in place, fp32, in that order; each term may be None; ``delta`` is multiplied
+    by ``delta_scale`` first, if there is one."""
+    for d in _added(delta, delta_scale):
         h += d
     if again is not None:
         h += again

@@ -18,8 +18,9 @@ from .base import (
     registered_parts,
     unregister_part,
 )
-from . import (attention, block, differential_attention, embedding, feed_forward, injection, latent_attention,  # noqa: F401
-               linear_attention, moe, norm, position, selective_scan, sigmoid_attention)  # register the built-in parts
+from . import (attention, block, delta_rule, differential_attention, embedding, feed_forward, injection,  # noqa: F401
+               latent_attention, linear_attention, linear_recurrence, mixed_attention, moe, norm, position, rows_mixer,
+               selective_scan, sigmoid_attention)  # register the built-in parts
 
 __all__ = [
     "MATRIX", "TABLE_INT", "VECTOR", "FeedForward", "Injection", "LayerStore", "Mixer", "Norm", "PagedNeed", "Part",

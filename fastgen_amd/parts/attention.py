@@ -14,7 +14,9 @@ more than bfloat16's digits), ``bias`` (q, k and v have biases, added in fp32
 where the product's fp32 result is read), ``qk_norm`` (an RMS norm per head on
 q and on k, one weight for all heads, before any rotation), ``sink`` (a learned
 number per head whose exponential is one more term of the softmax's
-denominator), ``v_head_dim`` (values of another width than keys: the cache
+denominator; ``"one"``: that term is 1 for every head), ``conv_taps`` (q and k pass a short causal convolution per
+channel behind their projections; the last ``taps - 1`` projected rows are per-request state), ``distance_bias`` (two
+numbers per head; a key ``n`` tokens back loses ``r1 ln(1 + r2 n)`` of its score), ``v_head_dim`` (values of another width than keys: the cache
 holds both padded with zeros to one width), ``has_kv`` = False (a layer that
 reads another layer's keys and values has only its queries), ``cache_window``
 (how long the cache keeps a key, where later layers read this layer's cache
@@ -29,7 +31,7 @@ import torch
 
 from ..kernels import ops
 from ..kernels.linear import StreamedMatrix, linear, skinny_ok, streamed
-from .base import LayerStore, Mixer, PagedNeed, TensorSpec, build_part, place, register_part, MATRIX, VECTOR
+from .base import LayerStore, Mixer, PagedNeed, StateNeed, TensorSpec, build_part, place, register_part, MATRIX, VECTOR
 
 
 class Attention(Mixer):
@@ -58,20 +60,32 @@ class Attention(Mixer):
         self.qk_norm = bool(o.get("qk_norm", False))
         self.qk_norm_eps = float(o.get("qk_norm_eps", 1e-6))
         self.sink = bool(o.get("sink", False))
+        self.sink_is_one = o.get("sink") == "one"
+        self.conv_taps = int(o.get("conv_taps", 0))
+        self.distance_bias = bool(o.get("distance_bias", False))
+        if not 0 <= self.conv_taps <= ops.CONV_MAX_TAPS:
+            raise ValueError(f"{self.prefix}: {self.conv_taps} taps are not supported (at most {ops.CONV_MAX_TAPS})")
+        if self.distance_bias and not self.exact_weights:
+            raise ValueError(f"{self.prefix}: the kernels with a distance bias are built with exact weights")
         self.has_kv = bool(o.get("has_kv", True))
         self.v_head_dim = int(o.get("v_head_dim") or self.head_dim)
         self.cache_window: Optional[int] = o.get("cache_window", self.window) or None
         # the width of a head in the cache: keys and values of different widths are padded with zeros to one
         # width, a multiple of 16 (what the matrix-core kernels take)
         # the general form: what the product gives goes through a kernel of its own on its way to the attention
-        self.prepared = self.bias or self.qk_norm or not self.has_kv or self.v_head_dim != self.head_dim
+        self.prepared = (self.bias or self.qk_norm or not self.has_kv or self.v_head_dim != self.head_dim
+                         or self.conv_taps > 0)
         self.cache_dim = -(-max(self.head_dim, self.v_head_dim) // 16) * 16 if self.prepared else self.head_dim
-        if self.prepared and (self.value_from_key or self.output_gate):
-            raise ValueError(f"{self.prefix}: value_from_key and output_gate do not go with bias, qk_norm, v_head_dim or has_kv")
+        plain_keys = not (self.bias or self.qk_norm) and o["position"].kind == "none" and self.v_head_dim == self.head_dim
+        if self.prepared and self.value_from_key and not (plain_keys and self.has_kv):
+            raise ValueError(f"{self.prefix}: value_from_key does not go with bias, qk_norm, v_head_dim, has_kv or, behind a"
+                             " convolution, with a rotation")
+        if self.conv_taps and not self.has_kv:
+            raise ValueError(f"{self.prefix}: a convolution on the keys needs keys")
         if self.v_head_dim % 2 or self.cache_dim > 512:
             raise ValueError(f"{self.prefix}: value size {self.v_head_dim} is not supported (even, at most 512)")
         self.position = build_part("position", o["position"])
-        self.b_qkv = self.q_norm_w = self.k_norm_w = self.sinks = None
+        self.b_qkv = self.q_norm_w = self.k_norm_w = self.sinks = self.conv_w = self.distance = None
         self.wqkv: Optional[StreamedMatrix] = None
         self.wo: Optional[StreamedMatrix] = None
         self.freqs: Optional[torch.Tensor] = None
@@ -85,7 +99,7 @@ class Attention(Mixer):
             if not self.value_from_key:
                 specs.append(TensorSpec(self._name("v_proj.weight"), (vw, self.dim)))
         if self.output_gate:
-            specs.append(TensorSpec(self._name("gate_proj.weight"), (q, self.dim)))
+            specs.append(TensorSpec(self._name("gate_proj.weight"), (self.n_heads * self.v_head_dim, self.dim)))
         if self.bias:
             specs.append(TensorSpec(self._name("q_proj.bias"), (q,), VECTOR))
             if self.has_kv:
@@ -95,8 +109,13 @@ class Attention(Mixer):
             specs.append(TensorSpec(self._name("q_norm.weight"), (self.head_dim,), VECTOR, ("one_plus_normal", 0.01)))
             if self.has_kv:
                 specs.append(TensorSpec(self._name("k_norm.weight"), (self.head_dim,), VECTOR, ("one_plus_normal", 0.01)))
-        if self.sink:
+        if self.sink and not self.sink_is_one:
             specs.append(TensorSpec(self._name("sinks"), (self.n_heads,), VECTOR, ("normal", 1.0)))
+        if self.conv_taps:
+            specs += [TensorSpec(self._name("q_conv.weight"), (q, self.conv_taps), VECTOR, ("normal", 0.5)),
+                      TensorSpec(self._name("k_conv.weight"), (kv, self.conv_taps), VECTOR, ("normal", 0.5))]
+        if self.distance_bias:
+            specs += [TensorSpec(self._name(f"distance.{n}"), (self.n_heads,), VECTOR, ("one_plus_normal", 0.1)) for n in ("r1", "r2")]
         return specs + [TensorSpec(self._name("o_proj.weight"), (self.dim, self.n_heads * self.v_head_dim))]
 
     def load(self, tensors: Mapping[str, torch.Tensor], dtype: torch.dtype, device: Any) -> None:
@@ -109,15 +128,10 @@ class Attention(Mixer):
             if not self.value_from_key:
                 mats.append(tensors[self._name("v_proj.weight")])
         if self.output_gate:
-            mats.append(tensors[self._name("gate_proj.weight")])
+            mats.append(self._padded_heads(tensors[self._name("gate_proj.weight")], 0))
         self.wqkv = streamed(place(torch.cat(mats, dim=0), MATRIX, dtype, device))
-        wo = tensors[self._name("o_proj.weight")]
-        if self.cache_dim != self.v_head_dim:
-            # the attention's output rows hold heads of the cache's width: zero columns meet the padding
-            wide = wo.new_zeros(self.dim, self.n_heads, self.cache_dim)
-            wide[:, :, : self.v_head_dim] = wo.view(self.dim, self.n_heads, self.v_head_dim)
-            wo = wide.view(self.dim, self.n_heads * self.cache_dim)
-        self.wo = streamed(place(wo, MATRIX, dtype, device))
+        # the attention's output rows hold heads of the cache's width: zero columns meet the padding
+        self.wo = streamed(place(self._padded_heads(tensors[self._name("o_proj.weight")], 1), MATRIX, dtype, device))
         self.freqs = self.position.frequencies_on(device)
         if self.bias:
             names = ["q_proj.bias"] + (["k_proj.bias", "v_proj.bias"] if self.has_kv else [])
@@ -128,7 +142,29 @@ class Attention(Mixer):
             self.q_norm_w = f32("q_norm.weight")
             self.k_norm_w = f32("k_norm.weight") if self.has_kv else None
         if self.sink:
-            self.sinks = f32("sinks")
+            self.sinks = torch.zeros(self.n_heads, device=device) if self.sink_is_one else f32("sinks")
+        if self.conv_taps:
+            if self.position.rotary_dim and getattr(self.position, "pairing", "") == "half":
+                raise ValueError(f"{self.prefix}: convolutions with rows rearranged for the rotation are not supported")
+            self.conv_w = torch.cat([f32("q_conv.weight"), f32("k_conv.weight")]).contiguous()
+        if self.distance_bias:
+            self.distance = torch.stack([f32("distance.r1"), f32("distance.r2")], dim=1).contiguous()
+
+    def _padded_heads(self, w: torch.Tensor, axis: int) -> torch.Tensor:
+        """The rows (columns) of heads of ``v_head_dim`` spread to heads of the cache's width, zeros between."""
+        if self.cache_dim == self.v_head_dim:
+            return w
+        w = w if axis == 0 else w.t()
+        wide = w.new_zeros(self.n_heads, self.cache_dim, w.shape[1])
+        wide[:, : self.v_head_dim] = w.reshape(self.n_heads, self.v_head_dim, -1)
+        wide = wide.reshape(self.n_heads * self.cache_dim, -1)
+        return wide if axis == 0 else wide.t().contiguous()
+
+    def state_need(self) -> Optional[StateNeed]:
+        if not self.conv_taps:
+            return None
+        # (one column where there is one tap: never empty)
+        return StateNeed(((self.n_heads + self.n_kv_heads) * self.head_dim, max(1, self.conv_taps - 1)), torch.float32)
 
     def paged_need(self) -> PagedNeed:
         return PagedNeed(self.n_kv_heads, self.cache_dim, self.cache_window)
@@ -177,7 +213,7 @@ class Attention(Mixer):
             gate_done = False
         out = torch.empty((rows.shape[0], q_width), dtype=rows.dtype, device=rows.device)
         ops.paged_attention(qkv, out, store.k_pages, store.v_pages, group, ctx, self.n_heads, self.scale,
-                            self.window or 0, exact_weights=self.exact_weights, sinks=self.sinks)
+                            self.window or 0, exact_weights=self.exact_weights, sinks=self.sinks, distance=self.distance)
         if gate is not None:
             ops.gate_mul(out, gate, sigmoid=not gate_done)
         return linear(out, self.wo, partials_ok=True, residual=then)
@@ -192,7 +228,7 @@ class Attention(Mixer):
         return table
 
     def _forward_prepared(self, x, ctx: Any, store: LayerStore, then=None):
-        """The general form: the product's fp32 rows go through ``heads_prepare`` (bias, the norms per
+        """The general form: the product's fp32 rows go through ``heads_prepare`` (convolution, bias, the norms per
         head, rotation, padding to the cache's head width, cache write), then attention and output
         projection."""
         if isinstance(x, ops.ScaledRows):
@@ -203,17 +239,28 @@ class Attention(Mixer):
         rows = linear(x, self.wqkv, out_dtype=torch.float32)
         q = torch.empty((x.shape[0], self.n_heads * hc), dtype=x.dtype, device=x.device)
         writes = store.owns and self.has_kv
+        v_col = -1 if self.value_from_key else q_width + kv_width  # (the value is the key as it is stored)
+        gate_col = q_width + (kv_width if self.has_kv else 0) + (
+            self.n_kv_heads * self.v_head_dim if self.has_kv and not self.value_from_key else 0)
+        conv = None
+        if self.conv_taps:
+            moves = ctx.graph_capacity > 0 or ctx.max_q_len == 1
+            conv = ops.ConvInputs(self.conv_w, store.state, 0, ctx.slot_ids, ctx.seq_of_token, ctx.q_start, moves)
         ops.heads_prepare(
             rows, self.b_qkv, self.qk_norm_eps, n_q=self.n_heads, q_col=0, q_width=d, q_norm=self.q_norm_w,
             q_norm_dims=d if self.qk_norm else 0, q_out=q, q_out_width=hc,
             n_kv=self.n_kv_heads if writes else 0, k_col=q_width, k_width=d, k_norm=self.k_norm_w,
-            k_norm_dims=d if self.qk_norm else 0, v_col=q_width + kv_width, v_width=self.v_head_dim,
+            k_norm_dims=d if self.qk_norm else 0, v_col=v_col, v_width=self.v_head_dim,
             table=self._rope_table(ctx), rot_start=0, rotary_dim=self.position.rotary_dim,
             slots=group.slots if writes else None, k_pages=store.k_pages if writes else None,
-            v_pages=store.v_pages if writes else None)
+            v_pages=store.v_pages if writes else None, conv=conv)
+        if conv is not None and not conv.moves:
+            ops.conv_tail(rows, conv, ctx.n_seqs)
         out = torch.empty_like(q)
         ops.paged_attention(q, out, store.k_pages, store.v_pages, group, ctx, self.n_heads, self.scale,
-                            self.window or 0, exact_weights=self.exact_weights, sinks=self.sinks)
+                            self.window or 0, exact_weights=self.exact_weights, sinks=self.sinks, distance=self.distance)
+        if self.output_gate:
+            ops.gate_mul(out, rows[:, gate_col:])
         return linear(out, self.wo, partials_ok=True)
 
 

@@ -58,6 +58,49 @@ class PreNormBlock:
 register_part("arrangement", "pre_norm", lambda spec, *parts: PreNormBlock(*parts))
 
 
+class ScaledPreNormBlock(Part):
+    """``h += mult * ls1 (.) mixer(norm(h)); h += mult * ls2 (.) ffn(norm(h))``: a pre-norm layer whose sublayers' outputs are
+    multiplied per channel by a learned vector (``ls1 [dim]``, ``ls2 [dim]``) and by a constant before they are added.
+    The products' rows go on as :class:`~fastgen_amd.kernels.ops.ScaledDelta`: the norm that follows scales them, adds
+    them and norms the stream in one kernel, in fp32.  A layer without a feed-forward has the first half only.
+    Options: ``dim``, ``mult``, ``scaled`` (False: there are no vectors); the spec's prefix is the layer's."""
+
+    folds_norms = False
+
+    def __init__(self, spec, mixer: Mixer, ffn: Optional[FeedForward], mixer_norm: Norm, ffn_norm: Optional[Norm]) -> None:
+        super().__init__(spec)
+        self.dim = int(spec.options["dim"])
+        self.mult = float(spec.options.get("mult", 1.0))
+        self.scaled = bool(spec.options.get("scaled", True))
+        if ffn is not None and ffn_norm is None:
+            raise ValueError("a feed-forward needs its norm")
+        self.mixer, self.ffn, self.mixer_norm, self.ffn_norm = mixer, ffn, mixer_norm, ffn_norm
+        _no_output_bias(ffn, "pre-norm")
+        self.scales: dict = {}
+
+    def _sublayers(self):
+        return ("ls1", "ls2") if self.ffn is not None else ("ls1",)
+
+    def tensor_specs(self):
+        return [TensorSpec(self._name(n), (self.dim,), VECTOR, ("one_plus_normal", 0.1)) for n in self._sublayers()] if self.scaled else []
+
+    def load(self, tensors, dtype, device) -> None:
+        for n in self._sublayers():
+            ls = tensors[self._name(n)].to(device=device, dtype=torch.float32) if self.scaled else torch.ones(self.dim, device=device)
+            self.scales[n] = (self.mult * ls).contiguous()
+
+    def forward(self, h: torch.Tensor, pending, ctx: Any, store: LayerStore):
+        x = self.mixer_norm.forward(h, pending, ctx.act_dtype)
+        mixed = ops.ScaledDelta(self.mixer.forward(x, ctx, store), self.scales["ls1"])
+        if self.ffn is None:
+            return mixed
+        x = self.ffn_norm.forward(h, mixed, ctx.act_dtype)
+        return ops.ScaledDelta(self.ffn.forward(x), self.scales["ls2"])
+
+
+register_part("arrangement", "pre_norm_scaled", ScaledPreNormBlock)
+
+
 class ParallelBlock:
     """``x = norm(h); h += mixer(x) + ffn(x)``: one norm, both sublayers read its output, and their
     sum (taken first, in fp32) goes to the residual stream.  A layer without a feed-forward adds its
