@@ -62,6 +62,7 @@ VARIANT_LIBRARIES: Dict[str, tuple] = {
     "attention_mfma_exact": ("attention_mfma.hip", "FG_HD", tuple(range(16, 257, 16)), ("-DFG_EXACT_P=1",)),
     "attention_mfma_exact_dist": ("attention_mfma.hip", "FG_HD", tuple(range(16, 257, 16)),
                                   ("-DFG_EXACT_P=1", "-DFG_DIST_BIAS=1")),
+    "mixed_attention_mfma": ("mixed_attention_mfma.hip", "FG_HD", tuple(range(16, 257, 16)), ()),
     "sigmoid_attention_mfma": ("sigmoid_attention_mfma.hip", "FG_HD", tuple(range(16, 257, 16)), ()),
 }
 

@@ -2028,6 +2028,91 @@ def mixed_attention(q: torch.Tensor, head_dim: int, out: torch.Tensor, v_head_di
     return out
 
 
+class _MixedTileArgs(ctypes.Structure):
+    _fields_ = [("q", ctypes.c_void_p), ("q_stride", ctypes.c_int), ("q_hs", ctypes.c_int), ("k_pages", ctypes.c_void_p),
+                ("v_pages", ctypes.c_void_p), ("block_table", ctypes.c_void_p), ("bt_stride", ctypes.c_int),
+                ("items", ctypes.c_void_p), ("n_items", ctypes.c_int), ("n_tokens", ctypes.c_int), ("n_heads", ctypes.c_int),
+                ("n_kv", ctypes.c_int), ("d", ctypes.c_int), ("e", ctypes.c_int), ("page_size", ctypes.c_int),
+                ("scale", ctypes.c_float), ("softcap", ctypes.c_float), ("window", ctypes.c_int), ("talk", ctypes.c_void_p),
+                ("talk_low", ctypes.c_int), ("out_scale", ctypes.c_float), ("out", ctypes.c_void_p), ("out_stride", ctypes.c_int),
+                ("stats", ctypes.c_void_p), ("partial", ctypes.c_void_p), ("n_chunks", ctypes.c_int), ("chunk_keys", ctypes.c_int),
+                ("part_ml", ctypes.c_void_p)]
+
+
+MIXED_TILE_TOKENS = 16  # query tokens of an item of the matrix-core kernel
+MIXED_TILE_HEADS = 16  # the most heads it mixes
+_MIXED_TILE = 32  # keys of a tile
+_MIXED_CHUNK = 256  # keys of a chunk of a prompt portion's item, at least
+_MIXED_DECODE_CHUNK = 128  # keys of a chunk of a decoded token, at least (a tile for each of four waves)
+
+
+def mixed_attention_mfma_ok(dtype: torch.dtype, n_heads: int, cache_dim: int, page_size: int) -> bool:
+    """Whether :func:`mixed_attention_mfma` takes these sizes."""
+    return (dtype == torch.bfloat16 and n_heads <= MIXED_TILE_HEADS and cache_dim % 16 == 0 and cache_dim <= MFMA_MAX_HEAD_DIM
+            and page_size % 32 == 0)
+
+
+def mixed_attention_items(q_lens, q_start, n_cached):
+    """The step's sequences as items for :func:`mixed_attention_mfma`: two int32 arrays ``[n, 4]`` of (sequence, first flat
+    token, tokens, position of the first token): sequences that bring one token, and the others' tokens cut into runs
+    of up to 16, those with the most keys first."""
+    single = [(b, int(q_start[b]), 1, int(n_cached[b])) for b, n in enumerate(q_lens) if int(n) == 1]
+    items = [(b, int(q_start[b]) + i, min(MIXED_TILE_TOKENS, int(n) - i), int(n_cached[b]) + i)
+             for b, n in enumerate(q_lens) if int(n) > 1 for i in range(0, int(n), MIXED_TILE_TOKENS)]
+    items.sort(key=lambda it: -(it[3] + it[2]))
+    as_arr = lambda x: np.asarray(x, dtype=np.int32).reshape(-1, 4)
+    return as_arr(single), as_arr(items)
+
+
+def mixed_attention_mfma(q: torch.Tensor, head_dim: int, out: torch.Tensor, v_head_dim: int, k_pages: torch.Tensor,
+                         v_pages: torch.Tensor, block_table: torch.Tensor, single: Optional[torch.Tensor],
+                         items: Optional[torch.Tensor], max_keys: int, n_heads: int, scale: float, talk: torch.Tensor,
+                         softcap: float = 0.0, window: int = 0, out_scale: float = 1.0, talk_low: bool = True) -> torch.Tensor:
+    """:func:`mixed_attention` in bfloat16 on the matrix cores: at most 16 heads, pages of a multiple of 32 keys, cache
+    heads of a multiple of 16 up to 256.  ``single`` / ``items`` (device int32 ``[n, 4]``, 16-byte aligned, from
+    :func:`mixed_attention_items`): the tokens that are decoded alone and the runs of prompt portions; every token of the
+    step is covered once.  ``max_keys``: no sequence has more keys than this.  ``talk_low``: False promises that ``talk``
+    holds bfloat16 numbers.  The weights keep 16 significant bits; the result differs from the general kernel's by
+    rounding."""
+    T, H, G, hd, P, a = _mixed_operands(_MixedTileArgs(), q, head_dim, out, v_head_dim, k_pages, v_pages, block_table, None,
+                                        n_heads, scale, talk, softcap, window, out_scale)
+    _need(mixed_attention_mfma_ok(q.dtype, H, hd, P), "bfloat16, at most 16 heads, pages of a multiple of 32 keys, head sizes of"
+          " a multiple of 16 up to 256")
+    _gpu(single, items)
+    lib = _lib.load(f"mixed_attention_mfma@{hd}")
+    a.talk_low = int(bool(talk_low))
+    dev, window = q.device, int(window or 0)
+
+    def aim(which: torch.Tensor, tokens: int) -> int:
+        """Point the arguments at these items; the most keys one of them sees, counted from its first tile."""
+        _i32(which, "items")
+        _need(which.dim() == 2 and which.shape[1] == 4 and which.data_ptr() % 16 == 0, "items must be [n, 4], 16-byte aligned")
+        a.items, a.n_items = which.data_ptr(), which.shape[0]
+        span = max(int(max_keys), 1)
+        return min(span, window + tokens - 1 + _MIXED_TILE - 1) if window > 0 else span
+
+    def chunks(span: int, at_least: int, groups: int, most: int) -> int:
+        """Chunks of at least ``at_least`` keys that give ``groups`` workgroups over all items; their number."""
+        n = max(1, min(-(-span // at_least), -(-groups // a.n_items), most))
+        a.chunk_keys = -(-(-(-span // n)) // at_least) * at_least if n > 1 else -(-span // _MIXED_TILE) * _MIXED_TILE
+        a.n_chunks = -(-span // a.chunk_keys)
+        return a.n_chunks
+
+    if single is not None and single.shape[0]:
+        n = chunks(aim(single, 1), _MIXED_DECODE_CHUNK, compute_units(), int(lib.fg_mixed_attention_max_chunks()))
+        partial = torch.empty((n, a.n_items, G, 16, hd), dtype=torch.float32, device=dev)
+        part_ml = torch.empty((n, a.n_items, 16, 2), dtype=torch.float32, device=dev)
+        a.partial, a.part_ml = partial.data_ptr(), part_ml.data_ptr()
+        _check(lib.fg_mixed_attention_decode(ctypes.byref(a), _stream(q)), "mixed_attention (decoded tokens)")
+    if items is not None and items.shape[0]:
+        n = chunks(aim(items, MIXED_TILE_TOKENS), _MIXED_CHUNK, 2 * compute_units(), 65535)
+        stats = torch.empty((T, H, 2), dtype=torch.float32, device=dev)
+        partial = torch.empty((n, T, H * int(v_head_dim)), dtype=torch.float32, device=dev) if n > 1 else None
+        a.stats, a.partial, a.part_ml = stats.data_ptr(), (partial.data_ptr() if n > 1 else None), None
+        _check(lib.fg_mixed_attention_tiles(ctypes.byref(a), _stream(q)), "mixed_attention (prompt portions)")
+    return out
+
+
 def _mixed_operands(a, q, head_dim, out, v_head_dim, k_pages, v_pages, block_table, positions, n_heads, scale, talk, softcap,
                     window, out_scale):
     """Checks what the kernels of attention with mixed heads have in common and fills it into ``a``."""
@@ -2043,12 +2128,14 @@ def _mixed_operands(a, q, head_dim, out, v_head_dim, k_pages, v_pages, block_tab
     _rows_of_width(q, T, H * d, "q")
     _rows_of_width(out, T, H * e, "out")
     _need(block_table.dim() == 2 and block_table.dtype == torch.int32 and block_table.stride(1) == 1, "block_table must be int32 [B, pages]")
-    _i32(positions, "positions", T)
     _need(talk.dtype == torch.float32 and talk.is_contiguous() and talk.shape == (H, H), "talk must be contiguous float32 [H, H]")
+    if positions is not None:
+        _i32(positions, "positions", T)
+        a.positions = positions.data_ptr()
     _need(softcap >= 0, "softcap must not be negative")
     a.q, a.q_stride, a.q_hs = q.data_ptr(), q.stride(0), d
     a.k_pages, a.v_pages, a.block_table, a.bt_stride = k_pages.data_ptr(), v_pages.data_ptr(), block_table.data_ptr(), block_table.stride(0)
-    a.positions, a.n_tokens, a.n_heads, a.n_kv, a.d, a.e, a.page_size = positions.data_ptr(), T, H, G, d, e, P
+    a.n_tokens, a.n_heads, a.n_kv, a.d, a.e, a.page_size = T, H, G, d, e, P
     a.scale, a.softcap, a.window, a.talk, a.out_scale = float(scale), float(softcap), int(window or 0), talk.data_ptr(), float(out_scale)
     a.out, a.out_stride = out.data_ptr(), out.stride(0)
     return T, H, G, hd, P, a

@@ -14,6 +14,7 @@ from __future__ import annotations
 
 from typing import Any, List, Mapping, Optional
 
+import numpy as np
 import torch
 
 from ..kernels import ops
@@ -46,7 +47,8 @@ class MixedAttention(RowsMixer):
         self.position = build_part("position", o["position"])
         self.in_width = self.n_heads * self.head_dim + self.n_kv_heads * (self.head_dim + self.v_head_dim)
         self.out_width = self.n_heads * self.v_head_dim
-        self.freqs = self.q_norm_w = self.k_norm_w = self.talk = self.talk_mfma = None
+        self.freqs = self.q_norm_w = self.k_norm_w = self.talk = None
+        self.talk_low = True
 
     def tensor_specs(self) -> List[TensorSpec]:
         H, G, d, e = self.n_heads, self.n_kv_heads, self.head_dim, self.v_head_dim
@@ -72,6 +74,7 @@ class MixedAttention(RowsMixer):
         self.q_norm_w = f32(arranged("q_norm.weight", self.n_heads))
         self.k_norm_w = f32(arranged("k_norm.weight", self.n_kv_heads))
         self.talk = f32(tensors[self._name("head_mix")])
+        self.talk_low = not bool(torch.equal(self.talk, self.talk.to(torch.bfloat16).float()))
         self.freqs = self.position.frequencies_on(device)
 
     def paged_need(self) -> PagedNeed:
@@ -95,8 +98,30 @@ class MixedAttention(RowsMixer):
             n_kv=G, k_col=H * d, k_width=d, k_norm=self.k_norm_w, k_norm_dims=d, v_col=(H + G) * d, v_width=e,
             table=self._rope_table(ctx), rot_start=0, rotary_dim=self.position.rotary_dim,
             slots=group.slots, k_pages=store.k_pages, v_pages=store.v_pages, row_norm=True)
-        ops.mixed_attention(q, d, out, e, store.k_pages, store.v_pages, group.block_table, ctx.seq_of_token, ctx.positions, H,
-                            self.scale, self.talk, self.softcap, self.window or 0, out_scale)
+        if not ops.mixed_attention_mfma_ok(out.dtype, H, self.cache_dim, store.k_pages.shape[2]):
+            ops.mixed_attention(q, d, out, e, store.k_pages, store.v_pages, group.block_table, ctx.seq_of_token, ctx.positions,
+                                H, self.scale, self.talk, self.softcap, self.window or 0, out_scale)
+            return
+        single, portions = self._items(ctx, out.device)
+        ops.mixed_attention_mfma(q, d, out, e, store.k_pages, store.v_pages, group.block_table, single, portions,
+                                 ctx.graph_capacity or ctx.max_kv_len, H, self.scale, self.talk, self.softcap,
+                                 self.window or 0, out_scale, self.talk_low)
+
+    @staticmethod
+    def _items(ctx: Any, device: Any):
+        """The step's items for the matrix-core kernels, shared by the layers."""
+        plan = ctx.scratch.get("mixed_attention_items")
+        if plan is None:
+            if ctx.seq_records is not None and ctx.max_q_len == 1:
+                # every sequence is one token: its records are in the step's buffer already (and are refreshed with it
+                # when the step is a replayed graph)
+                plan = (ctx.seq_records, None)
+            else:
+                single, portions = ops.mixed_attention_items(ctx.q_lens, ctx.q_start_host, ctx.n_cached)
+                both = ops.upload(np.concatenate([single, portions]), torch.int32, device)
+                plan = (both[: len(single)] if len(single) else None, both[len(single) :] if len(portions) else None)
+            ctx.scratch["mixed_attention_items"] = plan
+        return plan
 
 
 register_part("mixer", "mixed_attention", MixedAttention)
