@@ -4,13 +4,15 @@
 //
 //  delta_prepare  what the recurrence takes of a token, from the rows of the product: a causal convolution per
 //                 channel and SiLU on q, k and v; q and k as unit vectors per head (q times q_scale); the write
-//                 strength beta = sigmoid(b) and the decay g = exp(-exp(A_log) softplus(a + dt_bias)) per head.
-//                 One fp32 row a token: [q | k | v | beta | g].  A wave a (token, head).
+//                 strength beta = sigmoid(b) and the decay's logarithm log g = -exp(A_log) softplus(a + dt_bias) per
+//                 head.  One fp32 row a token: [q | k | v | beta | log g].  A wave a (token, head).
 //  delta_scan     the recurrence token by token.  Column c of S needs k, q and v[c] only, so a wave owns eight value
 //                 channels of a head: lane l holds column l & 7 and the key channels rg * rpl .. (rg = l >> 3) of it in
 //                 registers.  S^T k is a sum over the lanes of a column on the chain; S^T q is not, its sums are
 //                 exchanged for a whole run of tokens at once.  Operands of the next run fly while one is computed.
-//  Every sum runs in an order fixed by the sizes: what a token gets does not depend on the batch or on the cut.
+//                 Every sum runs in an order fixed by the sizes: the result does not depend on the batch or the cut.
+//  delta_chunk_*  long prompts, 64 tokens at a time as matrix products (the WY form of the products of the tokens'
+//                 rank-one changes), see below: the same within rounding.
 #include "common.h"
 #include "conv_inputs.h"
 
@@ -43,7 +45,7 @@ __global__ __launch_bounds__(DP_WAVES* FG_WAVE) void delta_prepare_kernel(const 
       const float b = to_f<TS>(row[a.b_col + h]);
       const float x = to_f<TS>(row[a.a_col + h]) + a.dt_bias[h];
       so[h] = 1.f / (1.f + expf(-b));
-      so[a.n_v + h] = expf(-a.decay_rate[h] * (fmaxf(x, 0.f) + log1pf(expf(-fabsf(x)))));
+      so[a.n_v + h] = -a.decay_rate[h] * (fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))));
     }
     return;
   }
@@ -157,7 +159,7 @@ __global__ __launch_bounds__(FG_WAVE) void delta_scan_kernel(const DeltaScanArgs
       }
       pv[tt] = row[v_col];
       pb[tt] = row[b_col];
-      pg[tt] = row[g_col];
+      pg[tt] = row[g_col];  // (its logarithm)
     }
   };
   fetch(t_begin);
@@ -169,7 +171,7 @@ __global__ __launch_bounds__(FG_WAVE) void delta_scan_kernel(const DeltaScanArgs
     for (int tt = 0; tt < RUN; ++tt) {
       v[tt] = pv[tt];
       beta[tt] = pb[tt];
-      g[tt] = pg[tt];
+      g[tt] = expf(pg[tt]);
 #pragma unroll
       for (int j = 0; j < NJ; ++j) {
         if (mine[j]) {
@@ -246,5 +248,289 @@ extern "C" int fg_delta_scan(const DeltaScanArgs* args, int n_seqs, hipStream_t 
   else if (rpl <= 24) delta_scan_kernel<24><<<grid, FG_WAVE, 0, stream>>>(a);
   else if (rpl <= 32) delta_scan_kernel<32><<<grid, FG_WAVE, 0, stream>>>(a);
   else delta_scan_kernel<64><<<grid, FG_WAVE, 0, stream>>>(a);
+  return fg_launch_status();
+}
+
+// ------------------------------------------------------------------ chunks
+// Within a chunk let L_t = the sum of log g up to token t, and S0 the state it starts from.  The writes u_t obey
+//   (I + A) U = diag(beta) V - diag(beta exp(L)) K S0,   A[t, s] = beta_t exp(L_t - L_s) k_t . k_s  (s < t),
+// the outputs and the state behind the chunk of n tokens are
+//   O = diag(exp(L)) Q S0 + M U,   M[t, s] = exp(L_t - L_s) q_t . k_s  (s <= t),
+//   S = exp(L_n) S0 + K^T diag(exp(L_n - L)) U.
+// delta_chunk_prepare makes T = (I + A)^-1 and M for every chunk and head side by side; delta_chunk_scan walks a
+// sequence's chunks in order, a workgroup 16 value channels of a head.  All products are fp32
+// (v_mfma_f32_16x16x4_f32); an operand's k index runs as 16 j + 4 (lane / 16) + i over the four products i of a block
+// j, so that a lane reads its operands as float4 and a result (rows 4 (lane / 16) + i) is the next product's second
+// operand as it is.  Tokens beyond a chunk's last have beta = 0 and change nothing.
+#define DC 64  // tokens of a chunk
+#define DC_LD (DC + 4)
+
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+
+struct DeltaChunks {
+  const int* chunk_start;  // [n_chunks + 1] first flat tokens
+  const int* seq_chunk;    // [n_seqs + 1] first chunk of each sequence
+  float* T; float* M;      // [n_chunks, n_v, 64, 64]; blocks of 16 x 16 above the diagonal are not written
+  float* L;                // [n_chunks, n_v, 64]
+};
+
+__device__ __forceinline__ f32x4 mfma4(const float4& x, const float4& y, f32x4 acc) {
+  acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x.x, y.x, acc, 0, 0, 0);
+  acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x.y, y.y, acc, 0, 0, 0);
+  acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x.z, y.z, acc, 0, 0, 0);
+  return __builtin_amdgcn_mfma_f32_16x16x4f32(x.w, y.w, acc, 0, 0, 0);
+}
+
+// grid (n_chunks, n_v), 4 waves; NDM >= d / 16
+template <int NDM>
+__global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(const DeltaScanArgs a, const DeltaChunks ch) {
+  __shared__ __attribute__((aligned(16))) float A_s[DC][DC_LD], T_s[DC][DC_LD];
+  __shared__ float L_s[DC], beta_s[DC];
+  const int lane = threadIdx.x % FG_WAVE, wave = threadIdx.x / FG_WAVE, g = lane >> 4, r16 = lane & 15;
+  const int c = blockIdx.x, h = blockIdx.y, hq = h / (a.n_v / a.n_qk), nd = a.d / 16;
+  const int t0 = ch.chunk_start[c], n = ch.chunk_start[c + 1] - t0;
+  const int k_col = a.n_qk * a.d, b_col = 2 * k_col + a.n_v * a.e + h;
+  const size_t at = (size_t)c * a.n_v + h;
+  if (wave == 0) {
+    const float* row = a.rows + (size_t)(t0 + min(lane, n - 1)) * a.stride;
+    float L = lane < n ? row[b_col + a.n_v] : 0.f;
+#pragma unroll
+    for (int m = 1; m < DC; m <<= 1) {
+      const float o = __shfl_up(L, m, FG_WAVE);
+      if (lane >= m) L += o;
+    }
+    L_s[lane] = L;
+    beta_s[lane] = lane < n ? row[b_col] : 0.f;
+    ch.L[at * DC + lane] = L;
+  }
+  __syncthreads();
+  float4 kf[NDM], qf[NDM];
+  {
+    const float* row = a.rows + (size_t)(t0 + min(16 * wave + r16, n - 1)) * a.stride + hq * a.d + 4 * g;
+#pragma unroll
+    for (int j = 0; j < NDM; ++j) {
+      if (j < nd) {  // uniform
+        qf[j] = *(const float4*)(row + 16 * j);
+        kf[j] = *(const float4*)(row + k_col + 16 * j);
+      }
+    }
+  }
+  for (int b = 0; b <= wave; ++b) {
+    const float* row = a.rows + (size_t)(t0 + min(16 * b + r16, n - 1)) * a.stride + k_col + hq * a.d + 4 * g;
+    f32x4 kk = {0.f, 0.f, 0.f, 0.f}, qk = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < NDM; ++j) {
+      if (j < nd) {
+        const float4 o = *(const float4*)(row + 16 * j);
+        kk = mfma4(kf[j], o, kk);
+        qk = mfma4(qf[j], o, qk);
+      }
+    }
+    const int s = 16 * b + r16;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int t = 16 * wave + 4 * g + i;
+      const float dec = expf(L_s[t] - L_s[s]);  // (not used above the diagonal)
+      A_s[t][s] = s < t ? beta_s[t] * dec * kk[i] : 0.f;
+      ch.M[at * DC * DC + t * DC + s] = s <= t ? dec * qk[i] : 0.f;
+    }
+  }
+  __syncthreads();
+  {  // the inverse of the diagonal block of this wave: a lane a column
+    float x[16];
+#pragma unroll
+    for (int t = 0; t < 16; ++t) {
+      float v = t == r16 ? 1.f : 0.f;
+#pragma unroll
+      for (int s = 0; s < t; ++s) v -= A_s[16 * wave + t][16 * wave + s] * x[s];
+      x[t] = v;
+    }
+    if (g == 0) {
+#pragma unroll
+      for (int t = 0; t < 16; ++t) T_s[16 * wave + t][16 * wave + r16] = x[t];
+    }
+  }
+  __syncthreads();
+  for (int i = wave + 1; i < 4; ++i) {  // block column `wave`, downwards: T_ij = -T_ii sum_k A_ik T_kj
+    f32x4 y = {0.f, 0.f, 0.f, 0.f};
+    for (int k = wave; k < i; ++k) {
+      const float4 av = *(const float4*)&A_s[16 * i + r16][16 * k + 4 * g];
+      const float4 tv = make_float4(T_s[16 * k + 4 * g][16 * wave + r16], T_s[16 * k + 4 * g + 1][16 * wave + r16],
+                                    T_s[16 * k + 4 * g + 2][16 * wave + r16], T_s[16 * k + 4 * g + 3][16 * wave + r16]);
+      y = mfma4(av, tv, y);
+    }
+    const float4 tii = *(const float4*)&T_s[16 * i + r16][16 * i + 4 * g];
+    const f32x4 res = mfma4(tii, make_float4(-y[0], -y[1], -y[2], -y[3]), f32x4{0.f, 0.f, 0.f, 0.f});
+#pragma unroll
+    for (int r = 0; r < 4; ++r) T_s[16 * i + 4 * g + r][16 * wave + r16] = res[r];
+  }
+  __syncthreads();
+  for (int e = threadIdx.x; e < DC * DC / 4; e += 256) {
+    const int t = e / (DC / 4), s = 4 * (e % (DC / 4));
+    if (s / 16 <= t / 16) *(float4*)(ch.T + at * DC * DC + t * DC + s) = *(const float4*)&T_s[t][s];
+  }
+}
+
+// grid (n_seqs, n_v, ceil(e / 16)), 4 waves: wave w takes tokens 16 w .. of a chunk, and the key channels of the
+// blocks w, w + 4, .. of the state.
+template <int NDM>
+__global__ __launch_bounds__(256) void delta_chunk_scan_kernel(const DeltaScanArgs a, const DeltaChunks ch) {
+  constexpr int NT = (NDM + 3) / 4;
+  __shared__ __attribute__((aligned(16))) float S_s[16][16 * NDM + 4];             // the state, by value channel
+  __shared__ __attribute__((aligned(16))) float X_s[16][DC_LD], U_s[16][DC_LD], D_s[16][DC_LD];
+  const int lane = threadIdx.x % FG_WAVE, wave = threadIdx.x / FG_WAVE, g = lane >> 4, r16 = lane & 15;
+  const int b = blockIdx.x, h = blockIdx.y, col = blockIdx.z * 16 + r16;
+  const bool col_ok = col < a.e;
+  const int d = a.d, e = a.e, nd = d / 16, hq = h / (a.n_v / a.n_qk);
+  const int k_col = a.n_qk * d, v_col = 2 * k_col + h * e + min(col, e - 1), b_col = 2 * k_col + a.n_v * e + h;
+  float* S_mem = a.state + (size_t)a.slot_ids[b] * a.slot_stride + (size_t)h * d * e;
+  f32x4 S[NT];
+#pragma unroll
+  for (int m = 0; m < NT; ++m) {
+    const int ti = wave + 4 * m;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) S[m][i] = ti < nd && col_ok ? S_mem[(size_t)(16 * ti + 4 * g + i) * e + col] : 0.f;
+    if (ti < nd) *(f32x4*)&S_s[r16][16 * ti + 4 * g] = S[m];
+  }
+  const int c_end = ch.seq_chunk[b + 1];
+  float4 kf[NDM], qf[NDM];
+  auto ask_rows = [&](int c) {  // this wave's 16 tokens of chunk c as first operands
+    const int t0 = ch.chunk_start[c], n = ch.chunk_start[c + 1] - t0;
+    const float* row = a.rows + (size_t)(t0 + min(16 * wave + r16, n - 1)) * a.stride + hq * d + 4 * g;
+#pragma unroll
+    for (int j = 0; j < NDM; ++j) {
+      if (j < nd) {  // uniform
+        qf[j] = *(const float4*)(row + 16 * j);
+        kf[j] = *(const float4*)(row + k_col + 16 * j);
+      }
+    }
+  };
+  int c = ch.seq_chunk[b];
+  if (c < c_end) ask_rows(c);
+  for (; c < c_end; ++c) {
+    const int t0 = ch.chunk_start[c], n = ch.chunk_start[c + 1] - t0;
+    const size_t at = (size_t)c * a.n_v + h;
+    // what the later phases need, asked for now
+    float4 tf[4], mf[4];
+    const float* t_row = ch.T + at * DC * DC + (size_t)(16 * wave + r16) * DC + 4 * g;
+    const float* m_row = ch.M + at * DC * DC + (size_t)(16 * wave + r16) * DC + 4 * g;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      if (j <= wave) {  // uniform in the wave
+        tf[j] = *(const float4*)(t_row + 16 * j);
+        mf[j] = *(const float4*)(m_row + 16 * j);
+      }
+    }
+    float beta[4], eL[4], eD[4], v[4];
+    const float L_end = ch.L[at * DC + DC - 1];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int t = 16 * wave + 4 * g + i;
+      const float L = ch.L[at * DC + t];
+      const float* row = a.rows + (size_t)(t0 + min(t, n - 1)) * a.stride;
+      beta[i] = t < n ? row[b_col] : 0.f;
+      v[i] = row[v_col];
+      eL[i] = expf(L);
+      eD[i] = expf(L_end - L);
+    }
+    __syncthreads();  // S_s is complete
+    // ---- 1. X = beta (V - exp(L) K S), and exp(L) Q S
+    f32x4 ks = {0.f, 0.f, 0.f, 0.f}, o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < NDM; ++j) {
+      if (j < nd) {
+        const float4 sv = *(const float4*)&S_s[r16][16 * j + 4 * g];
+        ks = mfma4(kf[j], sv, ks);
+        o = mfma4(qf[j], sv, o);
+      }
+    }
+    if (c + 1 < c_end) ask_rows(c + 1);
+    // the chunk's keys as first operands of K^T U: channel 16 ti + r16, token 16 j + 4 g + i
+    float kt[NT][4][4];
+#pragma unroll
+    for (int m = 0; m < NT; ++m) {
+      if (wave + 4 * m < nd) {
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            kt[m][j][i] = a.rows[(size_t)(t0 + min(16 * j + 4 * g + i, n - 1)) * a.stride + k_col + hq * d +
+                                 16 * (wave + 4 * m) + r16];
+      }
+    }
+    f32x4 x;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      x[i] = beta[i] * (v[i] - eL[i] * ks[i]);
+      o[i] *= eL[i];
+    }
+    *(f32x4*)&X_s[r16][16 * wave + 4 * g] = x;
+    __syncthreads();
+    // ---- 2. U = T X
+    f32x4 u = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (j <= wave) u = mfma4(tf[j], *(const float4*)&X_s[r16][16 * j + 4 * g], u);
+    *(f32x4*)&U_s[r16][16 * wave + 4 * g] = u;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) u[i] *= eD[i];
+    *(f32x4*)&D_s[r16][16 * wave + 4 * g] = u;
+    __syncthreads();
+    // ---- 3. O = exp(L) Q S + M U
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (j <= wave) o = mfma4(mf[j], *(const float4*)&U_s[r16][16 * j + 4 * g], o);
+    if (col_ok) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int t = 16 * wave + 4 * g + i;
+        if (t < n) a.out[(size_t)(t0 + t) * ((size_t)a.n_v * e) + h * e + col] = o[i];
+      }
+    }
+    // ---- 4. S = exp(L_n) S + K^T diag(exp(L_n - L)) U
+    const float all = expf(L_end);
+#pragma unroll
+    for (int m = 0; m < NT; ++m) {
+      const int ti = wave + 4 * m;
+      if (ti < nd) {
+        S[m] *= all;
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          S[m] = mfma4(make_float4(kt[m][j][0], kt[m][j][1], kt[m][j][2], kt[m][j][3]), *(const float4*)&D_s[r16][16 * j + 4 * g], S[m]);
+        *(f32x4*)&S_s[r16][16 * ti + 4 * g] = S[m];  // (everybody has read the old state: two barriers ago)
+      }
+    }
+  }
+#pragma unroll
+  for (int m = 0; m < NT; ++m) {
+    const int ti = wave + 4 * m;
+    if (ti < nd && col_ok) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) S_mem[(size_t)(16 * ti + 4 * g + i) * e + col] = S[m][i];
+    }
+  }
+}
+
+extern "C" int fg_delta_chunk_tokens() { return DC; }
+
+// d a multiple of 16 up to 256, rows 16-byte aligned
+extern "C" int fg_delta_chunk_scan(const DeltaScanArgs* args, const DeltaChunks* chunks, int n_chunks, int n_seqs,
+                                   hipStream_t stream) {
+  if (n_seqs <= 0 || n_chunks <= 0) return FG_OK;
+  const DeltaScanArgs& a = *args;
+  const DeltaChunks& ch = *chunks;
+  if (!delta_scan_ok(a, n_seqs) || a.d % 16 || a.d > 256 || a.stride % 4 || ((uintptr_t)a.rows & 15) || n_chunks > 2147483647 / 64 ||
+      !ch.chunk_start || !ch.seq_chunk || !ch.T || !ch.M || !ch.L)
+    return FG_ERR_ARG;
+  const dim3 pgrid(n_chunks, a.n_v), sgrid(n_seqs, a.n_v, (a.e + 15) / 16);
+#define GO(NDM)                                                               \
+  do {                                                                        \
+    delta_chunk_prepare_kernel<NDM><<<pgrid, 256, 0, stream>>>(a, ch);        \
+    delta_chunk_scan_kernel<NDM><<<sgrid, 256, 0, stream>>>(a, ch);           \
+  } while (0)
+  if (a.d <= 64) GO(4);
+  else if (a.d <= 128) GO(8);
+  else GO(16);
+#undef GO
   return fg_launch_status();
 }

@@ -2155,13 +2155,21 @@ class _DeltaScanArgs(ctypes.Structure):
                 ("slot_ids", ctypes.c_void_p), ("q_start", ctypes.c_void_p), ("out", ctypes.c_void_p)]
 
 
+class _DeltaChunks(ctypes.Structure):
+    _fields_ = [("chunk_start", ctypes.c_void_p), ("seq_chunk", ctypes.c_void_p), ("T", ctypes.c_void_p), ("M", ctypes.c_void_p),
+                ("L", ctypes.c_void_p)]
+
+
+DELTA_CHUNKED_FROM = 64  # the shortest run of tokens of one sequence for which a step is taken chunk by chunk
+
+
 def delta_prepare(src: torch.Tensor, n_qk: int, head_dim: int, n_v: int, v_head_dim: int, conv: ConvInputs, b_col: int,
                   a_col: int, decay_rate: torch.Tensor, dt_bias: torch.Tensor, q_scale: float, unit_eps: float,
                   out: torch.Tensor) -> torch.Tensor:
-    """What the gated delta rule takes of a token: ``out`` fp32 ``[T, q | k | v | beta | g]`` from the rows ``src [T, q | k |
+    """What the gated delta rule takes of a token: ``out`` fp32 ``[T, q | k | v | beta | log g]`` from the rows ``src [T, q | k |
     v | ...]`` of a product (``n_qk`` query and key heads of ``head_dim``, ``n_v`` value heads of ``v_head_dim``).  q, k and v
     pass ``conv`` and SiLU; every q and k head becomes ``x / sqrt(sum(x^2) + unit_eps)``, q times ``q_scale``;
-    ``beta = sigmoid(src[b_col + h])``; ``g = exp(-decay_rate[h] softplus(src[a_col + h] + dt_bias[h]))``."""
+    ``beta = sigmoid(src[b_col + h])``; ``log g = -decay_rate[h] softplus(src[a_col + h] + dt_bias[h])``."""
     _gpu(src, decay_rate, dt_bias, out)
     T, C = src.shape[0], 2 * n_qk * head_dim + n_v * v_head_dim
     _need(min(n_qk, n_v, head_dim, v_head_dim) > 0 and n_v % n_qk == 0 and head_dim % 2 == 0 and v_head_dim % 2 == 0
@@ -2174,7 +2182,7 @@ def delta_prepare(src: torch.Tensor, n_qk: int, head_dim: int, n_v: int, v_head_
     _f32_vec(dt_bias, n_v, "dt_bias")
     _need(out.dtype == torch.float32 and out.dim() == 2 and out.stride(1) == 1 and out.shape[0] == T
           and out.shape[1] >= C + 2 * n_v and out.stride(0) % 2 == 0 and out.data_ptr() % 8 == 0,
-          "out must be float32 [T, >= q | k | v | beta | g], rows 8-byte aligned")
+          "out must be float32 [T, >= q | k | v | beta | log g], rows 8-byte aligned")
     a = _DeltaPrepareArgs()
     a.src, a.src_stride, a.n_qk, a.d, a.n_v, a.e = src.data_ptr(), src.stride(0), n_qk, head_dim, n_v, v_head_dim
     a.conv, a.b_col, a.a_col = conv.args(), b_col, a_col
@@ -2191,7 +2199,11 @@ def delta_scan(rows: torch.Tensor, n_qk: int, head_dim: int, n_v: int, v_head_di
 
     ``rows`` are :func:`delta_prepare`'s; ``state`` fp32 ``[n_slots, n_v, head_dim, v_head_dim]`` (slots may have a stride of
     their own) is read at ``slot_ids[b]`` and left as the sequence's last token leaves it; ``out`` fp32 ``[T, n_v *
-    v_head_dim]``."""
+    v_head_dim]``.
+
+    ``q_start_host``: ``q_start`` on the host.  With it, a step in which a sequence brings ``DELTA_CHUNKED_FROM`` tokens or
+    more takes chunks of tokens at a time as matrix products (fp32) where the sizes allow; the result differs from the
+    token-by-token scan's by rounding."""
     _gpu(rows, state, slot_ids, q_start, out)
     T, d, e = rows.shape[0], int(head_dim), int(v_head_dim)
     _need(rows.dtype == torch.float32, "rows must be float32")
@@ -2206,7 +2218,20 @@ def delta_scan(rows: torch.Tensor, n_qk: int, head_dim: int, n_v: int, v_head_di
     a.rows, a.stride, a.n_qk, a.d, a.n_v, a.e = rows.data_ptr(), rows.stride(0), n_qk, d, n_v, e
     a.state, a.slot_stride, a.slot_ids, a.q_start = state.data_ptr(), state.stride(0), slot_ids.data_ptr(), q_start.data_ptr()
     a.out = out.data_ptr()
-    _check(_lib.load("delta_rule").fg_delta_scan(ctypes.byref(a), int(n_seqs), _stream(rows)), "delta_scan")
+    lib = _lib.load("delta_rule")
+    lens = np.diff(np.asarray(q_start_host[: n_seqs + 1])) if q_start_host is not None else None
+    if (lens is None or not len(lens) or int(lens.max()) < DELTA_CHUNKED_FROM or d % 16 or d > 256 or rows.stride(0) % 4
+            or rows.data_ptr() % 16 or torch.cuda.is_current_stream_capturing()):
+        _check(lib.fg_delta_scan(ctypes.byref(a), int(n_seqs), _stream(rows)), "delta_scan")
+        return out
+    size = int(lib.fg_delta_chunk_tokens())
+    n_chunks, chunk_start, seq_chunk, _ = _chunk_plan(q_start_host, n_seqs, size, rows.device)
+    room = torch.empty((n_chunks, n_v, 2 * size + 1, size), dtype=torch.float32, device=rows.device)
+    flat, per = room.view(-1), n_chunks * n_v * size * size
+    ch = _DeltaChunks()
+    ch.chunk_start, ch.seq_chunk = chunk_start.data_ptr(), seq_chunk.data_ptr()
+    ch.T, ch.M, ch.L = flat.data_ptr(), flat[per:].data_ptr(), flat[2 * per :].data_ptr()
+    _check(lib.fg_delta_chunk_scan(ctypes.byref(a), ctypes.byref(ch), n_chunks, int(n_seqs), _stream(rows)), "delta_scan (chunks)")
     return out
 
 

@@ -63,15 +63,13 @@ def gate_mul(x: torch.Tensor, gate: torch.Tensor, sigmoid: bool = True) -> torch
 
 
 def add_rmsnorm(h: torch.Tensor, delta: Optional[torch.Tensor], weight: torch.Tensor, eps: float,
-                out: torch.Tensor, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """``h += delta`` (a ``[T, dim]`` tensor, or fp32 ``[S, T, dim]`` partial sums added in order), then
-    ``out = h * rsqrt(mean(h^2) + eps) * weight``; with ``rows`` only those rows, and ``h`` stays as it was."""
+                out: torch.Tensor, rows: Optional[torch.Tensor] = None,
+                delta_scale: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``h += delta`` (a ``[T, dim]`` tensor, or fp32 ``[S, T, dim]`` partial sums added in order; their sum times
+    ``delta_scale [dim]`` if there is one), then ``out = h * rsqrt(mean(h^2) + eps) * weight``; with ``rows`` only those rows, and ``h`` stays as it was."""
     total = h.clone()
-    if delta is not None and delta.dim() == 3:
-        for s in range(delta.shape[0]):
-            total += delta[s]
-    elif delta is not None:
-        total += delta.float()
+    for d in _added(delta, delta_scale):
+        total += d
     if rows is None:
         h.copy_(total)
     else:
@@ -226,12 +224,14 @@ def _gather_kv(pages: torch.Tensor, unpack, table_row: torch.Tensor, n: int) -> 
 def paged_attention_general(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
                             block_table: torch.Tensor, seq_of_token: torch.Tensor, positions: torch.Tensor,
                             n_heads: int, scale: float, window: int = 0,
-                            sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                            sinks: Optional[torch.Tensor] = None,
+                            distance: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Token ``t`` of sequence ``b`` at position ``p`` attends keys ``0..p`` (``p-window+1..p`` with a window; with a
     negative one the keys up to ``p`` of its block of ``-window`` positions, blocks counted from 0)
     of its sequence, read through ``block_table[b]``; query head ``h`` reads kv head ``h // (H / KV)``;
     softmax of ``scale * q.k`` in fp32 (``fastgen/forward.py:176-258``).  With ``sinks`` head ``h``'s softmax runs
-    over one more score, ``sinks[h]`` as it is, whose weight meets no value."""
+    over one more score, ``sinks[h]`` as it is, whose weight meets no value.  With ``distance [H, 2]`` a key ``n`` tokens
+    back loses ``distance[h, 0] ln(1 + distance[h, 1] n)`` of its score."""
     n_kv, P, hd = k_pages.shape[1], k_pages.shape[2], k_pages.shape[3]
     G = n_heads // n_kv
     for t in range(q.shape[0]):
@@ -242,6 +242,9 @@ def paged_attention_general(q: torch.Tensor, out: torch.Tensor, k_pages: torch.T
         qt = q[t, : n_heads * hd].float().view(n_heads, hd)
         for h in range(n_heads):
             s = (k[lo:, h // G] @ qt[h]) * scale
+            if distance is not None:
+                n = (p - torch.arange(lo, p + 1)).to(distance.device)
+                s = s - distance[h, 0].float() * torch.log1p(distance[h, 1].float() * n.float())
             if sinks is not None:
                 s = torch.cat([s, sinks[h].float().reshape(1)])
             w = torch.softmax(s, 0)[: p + 1 - lo]
@@ -254,7 +257,8 @@ def paged_attention_mfma(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tens
                          big_items: Optional[torch.Tensor], n_heads: int, scale: float, window: int = 0,
                          plan=None, max_chunks=None, min_tiles: int = 4, max_rows: int = 16,
                          tile_rows=None, exact_weights: bool = False,
-                         sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                         sinks: Optional[torch.Tensor] = None,
+                         distance: Optional[torch.Tensor] = None) -> torch.Tensor:
     """The same attention for tokens listed as items (sequence, first flat token, tokens, position of the
     first token).  How the kernels cut the work (``plan`` and what follows it) does not change the result;
     ``exact_weights`` only says how many digits of the softmax weights the kernel keeps (here: all)."""
@@ -267,16 +271,17 @@ def paged_attention_mfma(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tens
             seq_of_token[first : first + n] = b
             positions[first : first + n] = torch.arange(pos, pos + n, dtype=torch.int32)
     return paged_attention_general(q, out, k_pages, v_pages, block_table, seq_of_token, positions, n_heads, scale,
-                                   window, sinks)
+                                   window, sinks, distance)
 
 
 def paged_attention(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
                     group, ctx, n_heads: int, scale: float, window: int = 0,
-                    exact_weights: bool = False, sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                    exact_weights: bool = False, sinks: Optional[torch.Tensor] = None,
+                    distance: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Attention of one step: the block table from the layer's cache group, sequences and positions of the
     tokens from the step's context."""
     return paged_attention_general(q, out, k_pages, v_pages, group.block_table, ctx.seq_of_token, ctx.positions,
-                                   n_heads, scale, window, sinks)
+                                   n_heads, scale, window, sinks, distance)
 
 
 def gemm_nt(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = None,
@@ -512,17 +517,26 @@ def heads_prepare(src: torch.Tensor, bias: Optional[torch.Tensor], eps: float,
                   rotate_q: bool = True, rotate_k: bool = True, slots: Optional[torch.Tensor] = None,
                   k_pages: Optional[torch.Tensor] = None, v_pages: Optional[torch.Tensor] = None, norm_plain: bool = False,
                   positions: Optional[torch.Tensor] = None, q_temp_coef: float = 0.0, q_temp_every: int = 0,
-                  v_first: Optional[torch.Tensor] = None, v_blend: float = 0.0) -> Optional[torch.Tensor]:
-    """Bias, a norm over the first dimensions of each head (``norm_plain``: also without a weight), the query's
+                  v_first: Optional[torch.Tensor] = None, v_blend: float = 0.0, row_norm: bool = False,
+                  conv=None) -> Optional[torch.Tensor]:
+    """A causal convolution on the columns that ``conv`` covers (whose tails move on if ``conv.moves``), bias, a norm over the first dimensions of each head (``norm_plain``: also without a weight; ``row_norm``: over all
+    query columns and over all key columns instead), the query's
     temperature ``1 + q_temp_coef * ln(floor((p + 1) / q_temp_every) + 1)``, the rotation of a run of pairs; queries to
     ``q_out`` and keys and values (blended with ``v_first``: ``(1 - v_blend) v + v_blend v_first``) to their pages,
     every head padded with zeros to its destination's width."""
     T = src.shape[0]
-    x = src.float() + (bias.float()[None, : src.shape[1]] if bias is not None else 0.0)
+    x = src.float()
+    if conv is not None:
+        x = torch.cat([_convolved(src, conv), x[:, conv.taps.shape[0] :]], dim=1)
+        if conv.moves:
+            conv_tail(src, conv, int(conv.q_start.numel()) - 1)
+    x = x + (bias.float()[None, : src.shape[1]] if bias is not None else 0.0)
 
     def heads(col, n, width, norm_w, norm_dims, turn, is_q=False):
         y = x[:, col : col + n * width].reshape(T, n, width).clone()
-        if norm_w is not None or (norm_plain and norm_dims > 0):
+        if row_norm:
+            y = y * torch.rsqrt((y * y).mean((1, 2), keepdim=True) + eps) * norm_w.float().view(n, width)
+        elif norm_w is not None or (norm_plain and norm_dims > 0):
             part = y[..., :norm_dims]
             part = part * torch.rsqrt((part * part).mean(-1, keepdim=True) + eps)
             y[..., :norm_dims] = part * norm_w.float()[:norm_dims] if norm_w is not None else part
@@ -552,14 +566,16 @@ def heads_prepare(src: torch.Tensor, bias: Optional[torch.Tensor], eps: float,
 
 
 def head_linear(x: torch.Tensor, x_head_stride: int, w: torch.Tensor, out: torch.Tensor, out_head_stride: int,
-                tail: int = 0, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """``out[t, h, :N] = w[h] @ x[t, h, :K]`` (times ``sigmoid(gate[t, h])``), then ``tail`` columns of ``x`` copied
+                tail: int = 0, gate: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``out[t, h, :N] = w[h] @ x[t, h, :K] + bias[h]`` (times ``sigmoid(gate[t, h])``), then ``tail`` columns of ``x`` copied
     through, then zeros up to ``out_head_stride``."""
     H, N, K = w.shape
     T = x.shape[0]
     for h in range(H):
         xh = x[:, h * x_head_stride : h * x_head_stride + K + tail].float()
         y = xh[:, :K] @ w[h].float().T
+        if bias is not None:
+            y = y + bias[h].float()
         if gate is not None:
             y = y * torch.sigmoid(gate[:, h].float())[:, None]
         full = torch.zeros(T, out_head_stride, device=x.device)
@@ -570,13 +586,13 @@ def head_linear(x: torch.Tensor, x_head_stride: int, w: torch.Tensor, out: torch
 
 
 def head_norm_gate(x: torch.Tensor, weight: torch.Tensor, eps: float, gate: torch.Tensor, n_heads: int,
-                   out: torch.Tensor) -> torch.Tensor:
-    """RMS norm of every head of fp32 ``x [T, H*e]`` with one weight ``[e]``, times ``silu(gate)``."""
+                   out: torch.Tensor, out_scale: float = 1.0) -> torch.Tensor:
+    """RMS norm of every head of fp32 ``x [T, H*e]`` with one weight ``[e]``, times ``silu(gate)`` and ``out_scale``."""
     T, e = x.shape[0], x.shape[1] // n_heads
     y = x.view(T, n_heads, e)
     y = y * torch.rsqrt((y * y).mean(-1, keepdim=True) + eps) * weight.float()
     g = gate[:, : n_heads * e].float().reshape(T, n_heads, e)
-    out.copy_((y * g * torch.sigmoid(g)).reshape(T, -1).to(out.dtype))
+    out.copy_((y * g * torch.sigmoid(g) * out_scale).reshape(T, -1).to(out.dtype))
     return out
 
 
@@ -620,15 +636,16 @@ def gated_mul(gate_up: torch.Tensor, bias: Optional[torch.Tensor], activation: s
 # ------------------------------------------------- selective state-space recurrence
 def causal_conv(x: torch.Tensor, taps: torch.Tensor, bias: Optional[torch.Tensor], state: torch.Tensor, tail_off: int,
                 slot_ids: torch.Tensor, seq_of_token: torch.Tensor, q_start: torch.Tensor, out: torch.Tensor,
-                activation: Optional[str] = None) -> torch.Tensor:
-    """Per sequence: the last ``K - 1`` inputs that the state holds, then this step's, convolved per channel."""
+                activation: Optional[str] = None, in_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Per sequence: the last ``K - 1`` inputs that the state holds, then this step's (plus ``in_bias``), convolved per
+    channel."""
     C, K = taps.shape
     for b in range(q_start.numel() - 1):
         t0, t1 = int(q_start[b]), int(q_start[b + 1])
         if t1 <= t0:
             continue
         tail = state[int(slot_ids[b]), :, tail_off : tail_off + K - 1].T  # [K - 1, C], oldest first
-        seq = torch.cat([tail.float(), x[t0:t1, :C].float()])
+        seq = torch.cat([tail.float(), x[t0:t1, :C].float() + (in_bias.float() if in_bias is not None else 0.0)])
         y = sum(seq[j : j + t1 - t0] * taps[:, j].float() for j in range(K))
         if bias is not None:
             y = y + bias.float()
@@ -636,6 +653,23 @@ def causal_conv(x: torch.Tensor, taps: torch.Tensor, bias: Optional[torch.Tensor
             y = y * torch.sigmoid(y)
         out[t0:t1, :C] = y.to(out.dtype)
     return out
+
+
+def _convolved(x: torch.Tensor, conv) -> torch.Tensor:
+    """fp32 ``[T, C]``: the first ``C`` columns of ``x`` behind ``conv`` (:class:`~fastgen_amd.kernels.ops.ConvInputs`)."""
+    out = torch.empty((x.shape[0], conv.taps.shape[0]), dtype=torch.float32, device=x.device)
+    return causal_conv(x, conv.taps, None, conv.state, conv.tail_off, conv.slot_ids, conv.seq_of_token, conv.q_start, out)
+
+
+def conv_tail(x: torch.Tensor, conv, n_seqs: int, in_bias: Optional[torch.Tensor] = None) -> None:
+    """Every sequence's state row gets its last ``K - 1`` inputs, old ones where the step brought fewer."""
+    C, K = conv.taps.shape
+    for b in range(n_seqs):
+        t0, t1 = int(conv.q_start[b]), int(conv.q_start[b + 1])
+        tail = conv.state[int(conv.slot_ids[b]), :, conv.tail_off : conv.tail_off + K - 1]
+        new = x[t0:t1, :C].float() + (in_bias.float() if in_bias is not None else 0.0)
+        if K > 1:
+            tail.copy_(torch.cat([tail.T, new])[-(K - 1) :].T.clone())
 
 
 def selective_scan(u: torch.Tensor, dt: torch.Tensor, dt_bias: Optional[torch.Tensor], A: torch.Tensor, bc: torch.Tensor,
@@ -738,3 +772,105 @@ def streams_step(x: torch.Tensor, update, in_weights: Optional[torch.Tensor], no
         n = u if norm_weight is None else u / torch.sqrt((u * u).mean(-1, keepdim=True) + eps) * norm_weight.float()
         out.copy_(n.to(out.dtype))
     return out if out is not None else u_out
+
+
+# ------------------------------------------------------- softmax attention with mixed heads
+def mixed_attention(q: torch.Tensor, head_dim: int, out: torch.Tensor, v_head_dim: int, k_pages: torch.Tensor,
+                    v_pages: torch.Tensor, block_table: torch.Tensor, seq_of_token: torch.Tensor, positions: torch.Tensor,
+                    n_heads: int, scale: float, talk: torch.Tensor, softcap: float = 0.0, window: int = 0,
+                    out_scale: float = 1.0) -> torch.Tensor:
+    """Scores over the keys a token sees, soft-capped, softmaxed per head, the heads' weights mixed by ``talk``, then the
+    values of each head's own key/value head."""
+    H, d, e = n_heads, head_dim, v_head_dim
+    rep = H // k_pages.shape[1]
+    for t in range(q.shape[0]):
+        b, p = int(seq_of_token[t]), int(positions[t])
+        first = max(0, p - window + 1) if window > 0 else p - p % -window if window < 0 else 0
+        k = _gather_kv(k_pages, unpack_k, block_table[b], p + 1)[first:, :, :d]
+        v = _gather_kv(v_pages, unpack_v, block_table[b], p + 1)[first:, :, :e]
+        s = torch.einsum("hd,jhd->hj", q[t, : H * d].float().view(H, d), k.repeat_interleave(rep, dim=1)) * scale
+        if softcap > 0:
+            s = softcap * torch.tanh(s / softcap)
+        w = talk.float() @ torch.softmax(s, dim=-1)
+        o = torch.einsum("hj,jhe->he", w, v.repeat_interleave(rep, dim=1)) * out_scale
+        out[t, : H * e] = o.reshape(-1).to(out.dtype)
+    return out
+
+
+def mixed_attention_mfma(q: torch.Tensor, head_dim: int, out: torch.Tensor, v_head_dim: int, k_pages: torch.Tensor,
+                         v_pages: torch.Tensor, block_table: torch.Tensor, single: Optional[torch.Tensor],
+                         items: Optional[torch.Tensor], max_keys: int, n_heads: int, scale: float, talk: torch.Tensor,
+                         softcap: float = 0.0, window: int = 0, out_scale: float = 1.0, talk_low: bool = True) -> torch.Tensor:
+    """The same for the tokens that the items name."""
+    for which in (single, items):
+        for seq, tok0, n, pos0 in (which.tolist() if which is not None else ()):
+            rows = slice(tok0, tok0 + n)
+            mixed_attention(q[rows], head_dim, out[rows], v_head_dim, k_pages, v_pages, block_table,
+                            torch.full((n,), seq, dtype=torch.int32), torch.arange(pos0, pos0 + n, dtype=torch.int32), n_heads,
+                            scale, talk, softcap, window, out_scale)
+    return out
+
+
+# ------------------------------------------------------------ gated delta rule
+def delta_prepare(src: torch.Tensor, n_qk: int, head_dim: int, n_v: int, v_head_dim: int, conv, b_col: int, a_col: int,
+                  decay_rate: torch.Tensor, dt_bias: torch.Tensor, q_scale: float, unit_eps: float,
+                  out: torch.Tensor) -> torch.Tensor:
+    """``[q | k | v | beta | log g]`` a token: q, k, v behind the convolution and SiLU, q and k as unit vectors per head."""
+    T, n = src.shape[0], n_qk * head_dim
+    y = _convolved(src, conv)
+    if conv.moves:
+        conv_tail(src, conv, int(conv.q_start.numel()) - 1)
+    y = y * torch.sigmoid(y)
+    for i, mul in ((0, q_scale), (1, 1.0)):
+        x = y[:, i * n : (i + 1) * n].view(T, n_qk, head_dim)
+        y[:, i * n : (i + 1) * n] = (x * torch.rsqrt((x * x).sum(-1, keepdim=True) + unit_eps) * mul).reshape(T, n)
+    C = y.shape[1]
+    out[:, :C] = y
+    out[:, C : C + n_v] = torch.sigmoid(src[:, b_col : b_col + n_v].float())
+    out[:, C + n_v : C + 2 * n_v] = -decay_rate * torch.nn.functional.softplus(src[:, a_col : a_col + n_v].float() + dt_bias)
+    return out
+
+
+def delta_scan(rows: torch.Tensor, n_qk: int, head_dim: int, n_v: int, v_head_dim: int, state: torch.Tensor,
+               slot_ids: torch.Tensor, q_start: torch.Tensor, n_seqs: int, out: torch.Tensor, q_start_host=None) -> torch.Tensor:
+    """Per sequence and value head, token by token: ``S <- g S``, ``u = beta (v - S^T k)``, ``S <- S + k u^T``, ``o = S^T q``."""
+    d, e, n = head_dim, v_head_dim, n_qk * head_dim
+    rep = n_v // n_qk
+    for b in range(n_seqs):
+        S = state[int(slot_ids[b])]
+        for t in range(int(q_start[b]), int(q_start[b + 1])):
+            r = rows[t]
+            q = r[:n].view(n_qk, d).repeat_interleave(rep, 0)
+            k = r[n : 2 * n].view(n_qk, d).repeat_interleave(rep, 0)
+            v = r[2 * n : 2 * n + n_v * e].view(n_v, e)
+            beta, log_g = r[2 * n + n_v * e :][:n_v], r[2 * n + n_v * (e + 1) :][:n_v]
+            S.mul_(torch.exp(log_g)[:, None, None])
+            u = beta[:, None] * (v - torch.einsum("hde,hd->he", S, k))
+            S.add_(k[:, :, None] * u[:, None, :])
+            out[t] = torch.einsum("hde,hd->he", S, q).reshape(-1)
+    return out
+
+
+# ------------------------------------------------- real-gated linear recurrence
+def lru_scan(u: torch.Tensor, gates: torch.Tensor, block: int, decay: torch.Tensor, y: torch.Tensor,
+             y_bias: Optional[torch.Tensor], out_scale: float, x_raw: Optional[torch.Tensor], x_bias: Optional[torch.Tensor],
+             taps: int, state: torch.Tensor, slot_ids: torch.Tensor, q_start: torch.Tensor, n_seqs: int, out: torch.Tensor,
+             q_start_host=None) -> torch.Tensor:
+    """``S <- a S + sqrt(1 - a^2) i u``, ``log a = -r decay``, ``out = S gelu(y + y_bias) out_scale``; the state's rows hold ``S``
+    and behind it the convolution's last ``taps - 1`` inputs."""
+    C = decay.numel()
+    g = gates[:, : 2 * C].float().view(-1, C // block, 2, block)
+    r, i = torch.sigmoid(g[:, :, 0].reshape(-1, C)), torch.sigmoid(g[:, :, 1].reshape(-1, C))
+    log_a = -r * decay.float()
+    drive = torch.sqrt(-torch.expm1(2 * log_a)) * i * u[:, :C].float()
+    mul = _gelu_tanh(y[:, :C].float() + (y_bias.float() if y_bias is not None else 0.0)) * out_scale
+    for b in range(n_seqs):
+        row = state[int(slot_ids[b])]
+        t0, t1 = int(q_start[b]), int(q_start[b + 1])
+        for t in range(t0, t1):
+            row[:, 0] = torch.exp(log_a[t]) * row[:, 0] + drive[t]
+            out[t, :C] = (row[:, 0] * mul[t]).to(out.dtype)
+        if taps > 1:
+            new = x_raw[t0:t1, :C].float() + (x_bias.float() if x_bias is not None else 0.0)
+            row[:, 1:taps] = torch.cat([row[:, 1:taps].T, new])[-(taps - 1) :].T.clone()
+    return out

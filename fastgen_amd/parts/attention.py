@@ -48,11 +48,6 @@ class Attention(Mixer):
         self.window: Optional[int] = o.get("window") or None
         if self.n_heads % self.n_kv_heads:
             raise ValueError(f"n_heads={self.n_heads} is not a multiple of n_kv_heads={self.n_kv_heads}")
-        if self.head_dim % 8 or self.head_dim > 512:
-            raise ValueError(
-                f"{self.prefix}: head size {self.head_dim} is not supported: the cache and the attention"
-                " kernels work in chunks of 8 head dimensions, up to 512"
-            )
         self.value_from_key = bool(o.get("value_from_key", False))
         self.output_gate = bool(o.get("output_gate", False))
         self.exact_weights = bool(o.get("exact_weights", False))
@@ -76,6 +71,11 @@ class Attention(Mixer):
         self.prepared = (self.bias or self.qk_norm or not self.has_kv or self.v_head_dim != self.head_dim
                          or self.conv_taps > 0)
         self.cache_dim = -(-max(self.head_dim, self.v_head_dim) // 16) * 16 if self.prepared else self.head_dim
+        if self.head_dim % (2 if self.prepared else 8) or self.head_dim > 512:
+            raise ValueError(
+                f"{self.prefix}: head size {self.head_dim} is not supported: the cache and the attention"
+                " kernels work in chunks of 8 head dimensions (padded heads: of 2), up to 512"
+            )
         plain_keys = not (self.bias or self.qk_norm) and o["position"].kind == "none" and self.v_head_dim == self.head_dim
         if self.prepared and self.value_from_key and not (plain_keys and self.has_kv):
             raise ValueError(f"{self.prefix}: value_from_key does not go with bias, qk_norm, v_head_dim, has_kv or, behind a"

@@ -91,7 +91,8 @@ class GatedDeltaRule(RowsMixer):
         tails = store.state[:, self._matrix :].view(slots, C, -1)
         moves = ctx.graph_capacity > 0 or ctx.max_q_len == 1
         conv = ops.ConvInputs(self.conv_w, tails, 0, ctx.slot_ids, ctx.seq_of_token, ctx.q_start, moves)
-        ready = torch.empty((T, C + 2 * H), dtype=torch.float32, device=rows.device)
+        # (rows of a multiple of 4: the chunked scan reads them as vectors)
+        ready = torch.empty((T, -(-(C + 2 * H) // 4) * 4), dtype=torch.float32, device=rows.device)
         ops.delta_prepare(rows, G, d, H, e, conv, C + H * e, C + H * e + H, self.decay_rate, self.dt_bias, d ** -0.5,
                           self.unit_eps, ready)
         if not moves:

@@ -341,3 +341,56 @@ def plain_weights(config: Mapping, seed: int, stored: torch.dtype = torch.bfloat
             mat(f"l{i}.mlp.up", mlp["ff"], D, 2 * D ** -0.5)
             mat(f"l{i}.mlp.down", D, mlp["ff"])
     return {k: v.to(stored).float() for k, v in w.items()}
+
+
+# ---------------------------------------------------------------- configurations
+def _parallel(heads, kv, dim, vdim, rot, window, softcap, width, blocks, conv, scales, base=900.0):
+    left = {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": vdim, "scale": dim ** -0.5}
+    if rot:
+        left["rot"] = {"base": base, "dims": rot}
+    if window:
+        left["mask"] = {"size": window}
+    if softcap:
+        left["softcap"] = softcap
+    return {"left": left, "right": {"width": width, "blocks": blocks, "conv": conv}, "left_scale": scales[0],
+            "right_scale": scales[1]}
+
+
+def _attention(heads, kv, dim, window, conv):
+    m = {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "conv": conv}
+    if window:
+        m["mask"] = {"size": window}
+    return m
+
+
+def _delta(heads, kv, dim, vdim, conv):
+    return {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": vdim, "conv": conv}
+
+
+def _model(width, vocab, layers, embed=3.0, mult=0.7, eps=1e-5):
+    return {"architecture": "Ropelix", "width": width, "vocab": vocab, "embedding": {"scale": embed}, "residual_mult": mult,
+            "norm": {"eps": eps}, "layers": [
+                {"type": t, "mixer": m, "mlp": None if f is None else {"kind": "dense", "ff": f[0], "limit": f[1]}}
+                for t, m, f in layers]}
+
+
+# every mixer, one of each kind without a feed-forward
+TRIO = _model(64, 96, [
+    ("parallel", _parallel(4, 2, 16, 24, 8, 20, 8.0, 48, 3, 4, (0.8, 0.4)), (56, 1.5)),
+    ("delta", _delta(4, 2, 16, 24, 3), (40, 0.9)),
+    ("attention", _attention(4, 2, 16, 23, 2), (56, 1.5)),
+    ("delta", _delta(3, 3, 32, 16, 2), None)])
+# heads that are no power of two, a head size that is no multiple of 16 (or of 8), one key head a query head, values
+# narrower than keys, every dimension rotated, no window, no cap, one block, one tap, widths that are no multiple of 8
+ODD = _model(72, 50, [
+    ("attention", _attention(3, 3, 20, None, 1), (44, 0.6)),
+    ("parallel", _parallel(3, 3, 12, 6, 12, None, None, 36, 1, 1, (1.0, -0.5)), None),
+    ("delta", _delta(6, 2, 10, 14, 1), (20, 2.0))], embed=1.0, mult=1.0, eps=1e-6)
+# twenty heads (more than the matrix-core kernels mix or group) and twelve (one group), windows of one page
+WIDE = _model(64, 80, [
+    ("parallel", _parallel(20, 4, 8, 8, 4, 16, 3.0, 64, 4, 5, (0.5, 1.5)), (48, 1.0)),
+    ("attention", _attention(20, 1, 8, 16, 4), (48, 1.0)),
+    ("parallel", _parallel(12, 1, 16, 16, 6, 64, 12.0, 16, 2, 2, (1.3, 0.7)), (48, 1.0))])
+ONLY_MIXED = _model(48, 64, [("parallel", _parallel(4, 2, 16, 16, 8, 32, None, 16, 2, 2, (1.0, 0.3)), None)], mult=1.0)
+ONLY_CONV = _model(48, 64, [("attention", _attention(4, 1, 16, 32, 3), None)], mult=1.0)
+ONLY_DELTA = _model(48, 64, [("delta", _delta(4, 2, 16, 16, 4), None)], mult=1.0)
