@@ -319,13 +319,23 @@ def cases(tmp_path_factory):
 
 
 def _against(got, runs, dtype, what):
-    """float32: against the float64 run, three times what the plain float32 run is off; bfloat16: against the float32
-    run, twice what the plain bfloat16 run is off.  (The yardstick is the worst over the step's requests: a request
-    of one token has little rounding of its own.)"""
-    want, low = (runs[torch.float64], runs[torch.float32]) if dtype == torch.float32 else (runs[torch.float32], runs[torch.bfloat16])
-    level = max(float((low[r].double() - want[r].double()).abs().max()) for r in want)
-    noise = {r: want[r].double() + level for r in want}
-    assert_close(got, {r: w.double() if dtype == torch.float32 else w for r, w in want.items()}, dtype, noise, what)
+    """float32: against the float64 run, three times what the plain float32 run is off at its worst.  bfloat16: the
+    root mean square over all logits of all requests at most 1.3 times the plain bfloat16 run's, and no position off by
+    more than four times that run's worst (single positions may stand on an edge where rounding counts for more)."""
+    if dtype == torch.float32:
+        want, low = runs[torch.float64], runs[torch.float32]
+        level = max(float((low[r].double() - want[r]).abs().max()) for r in want)
+        assert_close(got, want, dtype, {r: want[r] + level for r in want}, what)
+        return
+    want, low = runs[torch.float64], runs[torch.bfloat16]
+    for r in want:
+        assert got[r].shape == want[r].shape and torch.isfinite(got[r]).all(), f"{what} {r}"
+    flat = lambda runs_: torch.cat([(runs_[r].double() - want[r]).flatten() for r in want])
+    g, l = flat(got), flat(low)
+    scale = max(float(want[r].abs().max()) for r in want)
+    rms = lambda e: float(e.pow(2).mean().sqrt())
+    assert rms(g) <= 1.3 * rms(l) + 1e-4 * scale, f"{what}: root mean square {rms(g):.3e}, the plain run's {rms(l):.3e}"
+    assert float(g.abs().max()) <= 4 * float(l.abs().max()) + 1e-3 * scale, f"{what}: worst {float(g.abs().max()):.3e} against {float(l.abs().max()):.3e}"
 
 
 def _all_traces(lengths):
@@ -466,14 +476,18 @@ def test_keys_at_the_edges_of_windows_and_pages(tmp_path):
 
 @pytest.mark.parametrize("kind", ["delta", "lru", "sink"])
 def test_a_state_that_remembers_and_a_sink_that_counts(tmp_path, kind):
-    """Recurrences that hardly forget: changing the first 40 of 600 tokens changes the last logits, whole, in portions,
+    """Recurrences that hardly forget: changing the first 40 tokens of hundreds changes the last logits, whole, in portions,
     decoded alone, through slots that another request held.  The one in the softmax's denominator takes a visible share."""
     config = copy.deepcopy({"delta": ONLY_DELTA, "lru": ONLY_MIXED, "sink": ONLY_CONV}[kind])
+    n = {"delta": 200, "lru": 600, "sink": 120}[kind]
+    if kind == "delta":  # (keys of 64: a later write leaves most of an earlier one standing)
+        config["layers"][0]["mixer"].update(dim=64)
+    elif kind == "sink":
+        config["layers"][0]["mixer"].update(mask={"size": 5}, scale=0.05)
+        config["embedding"]["scale"] = 0.5  # (the stream is mostly what the layer added)
     w = plain_weights(config, 9)
-    n = 600 if kind != "sink" else 120
     if kind == "delta":
         w["l0.mix.A_log"].fill_(-9.0)
-        w["l0.mix.b"] *= 0.3
     elif kind == "lru":
         w["l0.mix.right.lam"].fill_(-9.0)
         config["layers"][0]["mixer"].update(left_scale=0.1, right_scale=2.0)
@@ -483,7 +497,6 @@ def test_a_state_that_remembers_and_a_sink_that_counts(tmp_path, kind):
     want = runs[torch.float32]["s"]
     scale = float(want.abs().max())
     if kind == "sink":
-        w2, x = dict(w), 0.0
         no_sink = plain_without_sink(w, config, toks["s"])
         assert float(((no_sink - want).abs().amax(-1) > 0.02 * scale).float().mean()) > 0.3, "the sink does not count"
     else:
