@@ -9,6 +9,7 @@
     python bench.py --workload gisodra      # the Gisodra design beside the dense Llama at equal sizes
     python bench.py --workload zudisun      # the Zudisun design beside Gisodra and the dense Llama at equal sizes
     python bench.py --workload sodotar      # the Sodotar design beside Gisodra and the dense Llama at equal sizes
+    python bench.py --workload ropelix      # the Ropelix design beside Gisodra and the dense Llama at equal sizes
 
 The model has the layer sizes of Llama 3.1 8B (32 layers, hidden 4096, 32
 heads, 8 kv heads, head size 128, feed-forward 14336, vocabulary 128256,
@@ -863,6 +864,227 @@ def sodotar_workload(prefill_tokens: int = 2048, batch: int = 8, context: int = 
     return 0
 
 
+# Ropelix at sizes that resemble a real model's layers: eight layers in the order delta rule, parallel (attention with
+# mixed heads beside a linear recurrence), convolved attention, delta rule, twice.  Beside it: Gisodra (the framework's
+# closest model: windowed attention and recurrent layers side by side) and the dense Llama, both of the same width,
+# heads, head size, feed-forward width and number of layers.
+ROPELIX_SIZES = {
+    "w1024": dict(width=1024, heads=16, kv_heads=4, dim=64, ff=2816, window=1024, delta_heads=8, delta_kv=4, delta_dim=64,
+                  delta_vdim=128, rec_width=1024, blocks=16, conv=4, vocab=32000),
+    "w2048": dict(width=2048, heads=16, kv_heads=4, dim=128, ff=5632, window=4096, delta_heads=16, delta_kv=8, delta_dim=128,
+                  delta_vdim=128, rec_width=2048, blocks=16, conv=4, vocab=32000),
+}
+
+
+def _ropelix_configs(z: dict):
+    mlp = dict(kind="dense", ff=z["ff"], limit=7.0)
+    attn = dict(heads=z["heads"], kv_heads=z["kv_heads"], dim=z["dim"], vdim=z["dim"], scale=z["dim"] ** -0.5,
+                mask=dict(size=z["window"]))
+    delta = dict(type="delta", mlp=mlp, mixer=dict(heads=z["delta_heads"], kv_heads=z["delta_kv"], dim=z["delta_dim"],
+                                                   vdim=z["delta_vdim"], conv=z["conv"]))
+    parallel = dict(type="parallel", mlp=mlp, mixer=dict(
+        left=dict(attn, softcap=30.0, rot=dict(base=500000.0, dims=z["dim"] // 2)), left_scale=0.7, right_scale=0.7,
+        right=dict(width=z["rec_width"], blocks=z["blocks"], conv=z["conv"])))
+    conv = dict(type="attention", mlp=mlp, mixer=dict(attn, conv=z["conv"]))
+    layers = [delta, parallel, conv, delta] * 2
+    new = dict(architecture="Ropelix", width=z["width"], vocab=z["vocab"], embedding=dict(scale=8.0), residual_mult=0.5,
+               norm=dict(eps=1e-6), layers=layers)
+    hybrid, dense = _gisodra_configs(GISODRA_SIZES["w1024" if z["width"] == 1024 else "w2048"])
+    return new, hybrid, dense
+
+
+def _ropelix_kernels(z: dict, rows: int, context: int) -> dict:
+    """The design's own kernels at ``rows`` tokens (one prompt of ``rows`` tokens, or ``rows`` sequences of one token at
+    ``context`` cached ones), each beside the like kernel of the framework's other models on operands of the same
+    size: microseconds, and the shares of the memory roofline (the bytes the kernel has to move), of the matrix
+    cores' (its bf16 products' flops) and of the fp32 vector units' (the flops that are fp32 by design)."""
+    import numpy as np
+    import torch
+
+    from fastgen_amd.kernels import ops
+    from fastgen_amd.parts.position import distance_table
+
+    D, H, G, d, P, K = z["width"], z["heads"], z["kv_heads"], z["dim"], PAGE, z["conv"]
+    g = torch.Generator(device="cuda").manual_seed(rows)
+    rnd = lambda *shape: (torch.randn(*shape, generator=g, device="cuda") * 0.05).to(torch.bfloat16)
+    f32 = lambda *shape: torch.randn(*shape, generator=g, device="cuda")
+    i32 = lambda values: torch.tensor(values, dtype=torch.int32, device="cuda")
+    decode = rows <= 16
+    n_seqs = rows if decode else 1
+    out = {}
+
+    def put(name, fn, nbytes, flops=0, vector_flops=0):
+        t = _time(fn)
+        out[name] = {"us": round(t * 1e6, 1), "hbm_frac": round(nbytes / t / PEAK_HBM, 4),
+                     "mfma_frac": round(flops / t / PEAK_FLOPS["bf16"], 4),
+                     "fp32_vector_frac": round(vector_flops / t / PEAK_FLOPS["fp32"], 4)}
+
+    # ---- the step: `rows` tokens of one sequence, or one of each of `rows` sequences
+    q_lens, q_start_host, n_cached = (([1] * rows, list(range(rows + 1)), [context] * rows) if decode else ([rows], [0, rows], [0]))
+    q_start, slot_ids = i32(q_start_host), torch.arange(n_seqs, dtype=torch.int32, device="cuda")
+    host = np.array(q_start_host)
+    seq_of_token = i32(list(range(rows)) if decode else [0] * rows)
+    positions = i32([context] * rows if decode else list(range(rows)))
+    keys = context + 1 if decode else rows
+    pages_seq = -(-keys // P)
+    bt = torch.arange(n_seqs * pages_seq, dtype=torch.int32, device="cuda").view(n_seqs, pages_seq)
+    slots = (torch.arange(rows, dtype=torch.int32, device="cuda") * pages_seq * P + context if decode
+             else torch.arange(rows, dtype=torch.int32, device="cuda")).contiguous()
+    kp, vp = rnd(n_seqs * pages_seq, G, P, d), rnd(n_seqs * pages_seq, G, d, P)
+    pairs = n_seqs * keys if decode else rows * (rows + 1) // 2  # (the windows are as long as the sequences, or longer)
+    kv_bytes = (n_seqs * keys * 2 * G * d + 2 * rows * H * d) * 2
+    # ---- attention with mixed heads; beside sigmoid attention (which mixes the scores) and the plain softmax attention
+    q, o = rnd(rows, H * d), torch.empty(rows, H * d, dtype=torch.bfloat16, device="cuda")
+    talk = (torch.eye(H, device="cuda") + 0.1 * f32(H, H)).to(torch.bfloat16).float()
+    single, runs = ops.mixed_attention_items(q_lens, q_start_host, n_cached)
+    up = lambda items: ops.upload(items, torch.int32, "cuda") if len(items) else None
+    single_d, runs_d = up(single), up(runs)
+    put("mixed_attention", lambda: ops.mixed_attention_mfma(q, d, o, d, kp, vp, bt, single_d, runs_d, keys, H, d ** -0.5, talk, 30.0,
+                                                            z["window"], 0.7, False), kv_bytes, 4 * pairs * H * d, pairs * (2 * H * H + 8 * H))
+    put("mixed_attention, general kernel (what float32 runs)", lambda: ops.mixed_attention(
+        q, d, o, d, kp, vp, bt, seq_of_token, positions, H, d ** -0.5, talk, 30.0, z["window"], 0.7), kv_bytes, 0,
+        pairs * (4 * H * d + 2 * H * H + 8 * H))
+    rel, pb = distance_table(f32(32, H), 2048.0).contiguous(), f32(H) - 3.0
+    s_items = ops.upload(np.array(single) if decode else ops.sigmoid_attention_items(q_lens, q_start_host, n_cached), torch.int32, "cuda")
+    s_mixed = ops.sigmoid_attention_mixed(d ** -0.5, H, rel, talk, pb, "cuda")
+    put("sigmoid_attention (zudisun)", lambda: ops.sigmoid_attention(q, d, o, d, kp, vp, bt, seq_of_token, positions, H, d ** -0.5, rel,
+                                                                     talk, pb, None, split_for=keys, items=s_items, mixed=s_mixed),
+        kv_bytes, 4 * pairs * H * d, pairs * (2 * H * H + 8 * H))
+    # ---- attention with a distance bias; beside the same without
+    dist, sinks = torch.rand(H, 2, generator=g, device="cuda"), torch.zeros(H, device="cuda")
+    for name, bias in (("attention (distance bias, sink)", dist), ("attention (gisodra: sink)", None)):
+        small, big = ops.attention_items(np.array(q_lens), host, np.array(n_cached), H // G, ops.attention_tile_rows(d, False, True, bias is not None))
+        sm, bg = up(small), up(big)
+        plan = (ops.attention_plan(sm, len(small), ops.attention_chunks_for(len(small), G), d, z["window"], 4, True, bias is not None)
+                if sm is not None else None)
+        put(name, lambda: ops.paged_attention_mfma(q, o, kp, vp, bt, sm, bg, H, d ** -0.5, z["window"], plan, exact_weights=True, sinks=sinks,
+                                                   distance=bias), kv_bytes, 4 * pairs * H * d)
+    # ---- between a product and an attention
+    src = f32(rows, (H + 2 * G) * d)
+    table = ops.rope_table(positions, f32(d // 4).abs())
+    qn, kn, hn = f32(H * d), f32(G * d), f32(d)
+    conv = ops.ConvInputs(f32((H + G) * d, K), torch.zeros(n_seqs + 1, (H + G) * d, K - 1, device="cuda"), 0, slot_ids, seq_of_token,
+                          q_start, decode)
+    heads = dict(n_q=H, q_col=0, q_width=d, q_out=q, q_out_width=d, n_kv=G, k_col=H * d, k_width=d, v_width=d, slots=slots,
+                 k_pages=kp, v_pages=vp)
+    moved = src.numel() * 4 + rows * (H + 2 * G) * d * 2
+    put("heads_prepare (norms over whole projections, rotation)", lambda: ops.heads_prepare(
+        src, None, 1e-6, q_norm=qn, q_norm_dims=d, k_norm=kn, k_norm_dims=d, v_col=(H + G) * d, table=table, rotary_dim=d // 2,
+        row_norm=True, **heads), moved)
+    put("heads_prepare (convolution)", lambda: ops.heads_prepare(src, None, 1e-6, v_col=-1, conv=conv, **heads),
+        rows * (H + G) * d * 4 + rows * (H + 2 * G) * d * 2)
+    put("heads_prepare (gisodra: norms per head)", lambda: ops.heads_prepare(
+        src, None, 1e-6, q_norm=hn, q_norm_dims=d, k_norm=hn, k_norm_dims=d, v_col=(H + G) * d, **heads), moved)
+    if not decode:
+        put("conv_tail", lambda: ops.conv_tail(src, conv, n_seqs), n_seqs * (H + G) * d * K * 4)
+    gate32, gate16 = f32(rows, H * d), rnd(rows, H * d)
+    put("gate_mul (fp32 gate)", lambda: ops.gate_mul(o, gate32), rows * H * d * 8)
+    put("gate_mul (buderax: bf16 gate)", lambda: ops.gate_mul(o, gate16), rows * H * d * 6)
+    # ---- the delta rule; beside gisodra's recurrence with a state of equal size
+    Hd, Gd, dd, e = z["delta_heads"], z["delta_kv"], z["delta_dim"], z["delta_vdim"]
+    C = 2 * Gd * dd + Hd * e
+    raw = f32(rows, C + Hd * e + 2 * Hd)
+    total = Hd * dd * e + C * (K - 1)
+    state = torch.zeros(n_seqs + 1, total, device="cuda")
+    dconv = ops.ConvInputs(f32(C, K), state[:, Hd * dd * e :].view(n_seqs + 1, C, K - 1), 0, slot_ids, seq_of_token, q_start, decode)
+    ready = torch.empty(rows, -(-(C + 2 * Hd) // 4) * 4, device="cuda")
+    rate, dtb = f32(Hd).abs(), f32(Hd)
+    put("delta_prepare", lambda: ops.delta_prepare(raw, Gd, dd, Hd, e, dconv, C + Hd * e, C + Hd * e + Hd, rate, dtb, dd ** -0.5, 1e-6, ready),
+        rows * (C + 2 * Hd) * 8)
+    o32 = torch.empty(rows, Hd * e, device="cuda")
+    S = state[:, : Hd * dd * e].view(n_seqs + 1, Hd, dd, e)
+    scan = lambda h: ops.delta_scan(ready, Gd, dd, Hd, e, S, slot_ids, q_start, n_seqs, o32, h)
+    scan_bytes = 2 * n_seqs * Hd * dd * e * 4 + rows * (C + 2 * Hd + Hd * e) * 4
+    put("delta_scan", lambda: scan(host), scan_bytes, 0, 7 * rows * Hd * dd * e)
+    gw = 2 * Hd * dd + 2 * Hd * e
+    rows16, zz, zb = rnd(rows, gw), f32(rows, Hd * dd), f32(Hd * dd)
+    gstate = torch.zeros(n_seqs + 1, Hd, dd, e, device="cuda")
+    gscan = lambda h: ops.decay_scan(rows16, 0, Hd * dd, 2 * Hd * dd, zz, zb, 16.0, dd ** -0.5, gstate, slot_ids, q_start, n_seqs, o32,
+                                     q_start_host=h)
+    g_bytes = 2 * n_seqs * Hd * dd * e * 4 + rows * (2 * Hd * dd + Hd * e) * 2 + rows * (Hd * dd + Hd * e) * 4
+    put("decay_scan (gisodra)", lambda: gscan(host), g_bytes, 0, 5 * rows * Hd * dd * e)
+    if not decode:
+        put("delta_scan, token by token", lambda: scan(None), scan_bytes, 0, 7 * rows * Hd * dd * e)
+        put("decay_scan (gisodra), token by token", lambda: gscan(None), g_bytes, 0, 5 * rows * Hd * dd * e)
+    o16, nw = torch.empty(rows, Hd * e, dtype=torch.bfloat16, device="cuda"), f32(e)
+    put("head_norm_gate (fp32 gate)", lambda: ops.head_norm_gate(o32, nw, 1e-6, raw[:, C:], Hd, o16), rows * Hd * e * 10)
+    put("head_norm_gate (gisodra: bf16 gate)", lambda: ops.head_norm_gate(o32, nw, 1e-6, rows16[:, : Hd * e], Hd, o16), rows * Hd * e * 8)
+    # ---- the linear recurrence; beside the selective scan with as many channels (16 states each) and a product per head
+    W, n = z["rec_width"], z["rec_width"] // z["blocks"]
+    yx, taps, cb, lam = f32(rows, 2 * W), f32(W, K), f32(W), f32(W).abs() + 0.01
+    rstate = torch.zeros(n_seqs + 1, W, K, device="cuda")
+    u, gates = torch.empty(rows, W, dtype=torch.bfloat16, device="cuda"), torch.empty(rows, 2 * W, device="cuda")
+    put("causal_conv (fp32 rows, input bias)", lambda: ops.causal_conv(yx[:, W:], taps, cb, rstate, 1, slot_ids, seq_of_token, q_start, u,
+                                                                       in_bias=cb), rows * W * 6)
+    xz = rnd(rows, 2 * W)
+    put("causal_conv (zudisun)", lambda: ops.causal_conv(xz, taps, cb, rstate, 1, slot_ids, seq_of_token, q_start, u, activation="silu"),
+        rows * W * 4)
+    wg, gb = rnd(z["blocks"], 2 * n, n), f32(z["blocks"], 2 * n)
+    put("head_linear (gates, fp32 out)", lambda: ops.head_linear(u, n, wg, gates, 2 * n, bias=gb), rows * W * (2 + 8) + wg.numel() * 2,
+        2 * rows * W * 2 * n)
+    y16 = torch.empty(rows, 2 * W, dtype=torch.bfloat16, device="cuda")
+    put("head_linear (gisodra: bf16 out)", lambda: ops.head_linear(u, n, wg, y16, 2 * n), rows * W * (2 + 4) + wg.numel() * 2,
+        2 * rows * W * 2 * n)
+    r16 = torch.empty(rows, W, dtype=torch.bfloat16, device="cuda")
+    put("lru_scan", lambda: ops.lru_scan(u, gates, n, lam, yx, cb, 0.7, yx[:, W:], cb, K, rstate, slot_ids, q_start, n_seqs, r16, host),
+        rows * W * (2 + 8 + 4 + 2) + 2 * n_seqs * W * K * 4, 0, 40 * rows * W)
+    A, narrow, sstate = -f32(W, 16).abs() - 0.1, rnd(rows, 96), torch.zeros(n_seqs + 1, W, 16 + K - 1, device="cuda")
+    put("selective_scan (zudisun, 16 states a channel)", lambda: ops.selective_scan(
+        u, yx[:, :W], cb, A, narrow, 64, 80, cb, xz[:, W:], xz, K, sstate, slot_ids, q_start, n_seqs, r16, q_start_host=host),
+        rows * W * (2 + 4 + 2 + 2) + 2 * n_seqs * W * (16 + K - 1) * 4, 0, 6 * rows * W * 16)
+    # ---- the stream and the feed-forward's activation
+    h, delta, w, ls = f32(rows, D), rnd(rows, D), f32(D), f32(D)
+    normed = torch.empty(rows, D, dtype=torch.bfloat16, device="cuda")
+    put("add_rmsnorm (scaled per channel)", lambda: ops.add_rmsnorm(h, delta, w, 1e-6, normed, None, ls), rows * D * 12)
+    put("add_rmsnorm (llama)", lambda: ops.add_rmsnorm(h, delta, w, 1e-6, normed), rows * D * 12)
+    F = z["ff"]
+    gu, gu16 = f32(rows, 2 * F), rnd(rows, 2 * F)
+    put("gated_mul (limited, fp32 rows)", lambda: ops.gated_mul(gu, None, "limited", torch.bfloat16, None, 7.0, 1.702), rows * F * 10)
+    put("silu_mul (llama, bf16 rows)", lambda: ops.silu_mul(gu16), rows * F * 6)
+    return out
+
+
+def ropelix_workload(prefill_tokens: int = 2048, batch: int = 8, context: int = 1024, steps: int = 32, warmup: int = 8) -> int:
+    """Prefill and decode throughput of Ropelix models with random bfloat16 weights beside Gisodra and dense Llama models of
+    equal sizes, and the design's own kernels beside the other models' like ones.  One JSON line."""
+    import torch
+
+    from fastgen_amd.engine import Engine
+
+    results = {}
+    for name, z in ROPELIX_SIZES.items():
+        new, hybrid, dense = _ropelix_configs(z)
+        row = {"layers": len(new["layers"])}
+        for label, cfg in (("ropelix", new), ("gisodra", hybrid), ("llama", dense)):
+            engine = Engine.from_config(cfg, seed=5, dtype=torch.bfloat16, page_size=PAGE,
+                                        max_tokens=max(batch * (context + 256), prefill_tokens + PAGE), max_batch=batch,
+                                        max_step_tokens=prefill_tokens)
+            g = torch.Generator().manual_seed(0)
+            prompt = lambda n: torch.randint(0, z["vocab"], (n,), generator=g).tolist()
+            pre = min(engine.time_prefill(prompt(prefill_tokens), repeats=5))
+            dt = engine.time_decode([prompt(context) for _ in range(batch)], steps=steps, warmup=warmup)
+            row[label] = {"prefill_tok_s": round(prefill_tokens / pre, 1), "prefill_ms": round(pre * 1e3, 3),
+                          "decode_tok_s": round(batch * steps / dt, 1), "decode_ms_per_step": round(dt / steps * 1e3, 4),
+                          "weights_gb": round(engine.model.weight_bytes() / 1e9, 3)}
+            print(f"[bench] {name} {label}: {row[label]}", file=sys.stderr, flush=True)
+            del engine
+            torch.cuda.empty_cache()
+        row["kernels_prefill"] = _ropelix_kernels(z, prefill_tokens, context)
+        row["kernels_decode"] = _ropelix_kernels(z, batch, context)
+        print(f"[bench] {name} kernels: {row['kernels_prefill']} {row['kernels_decode']}", file=sys.stderr, flush=True)
+        results[name] = row
+    first = results[next(iter(results))]
+    print(json.dumps({
+        "metric": "Ropelix beside Gisodra and the dense Llama at equal sizes: prefill and decode tok/s", "unit": "tokens/s",
+        "value": first["ropelix"]["decode_tok_s"], "n_gpus": 1, "steps": steps, "warmup": warmup, "higher_is_better": True,
+        "dtype": "bf16", "data": "synthetic",
+        "config": {"prefill_tokens": prefill_tokens, "decode_batch": batch, "decode_context": context, "page_size": PAGE,
+                   "sizes": ROPELIX_SIZES},
+        "results": results,
+    }), flush=True)
+    return 0
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -880,9 +1102,10 @@ def main() -> int:
                          " 2,048); more are fed untimed, in portions")
     ap.add_argument("--dtype", choices=["bf16", "fp32"], default="bf16")
     ap.add_argument("--no-points", action="store_true", help="skip decode at batch 1 and 64")
-    ap.add_argument("--workload", choices=["decode", "serve", "readme", "buderax", "gisodra", "zudisun", "sodotar"], default="decode",
+    ap.add_argument("--workload", choices=["decode", "serve", "readme", "buderax", "gisodra", "zudisun", "sodotar", "ropelix"],
+                    default="decode",
                     help="decode (default): the step benchmark; serve: continuous batching of 256 requests; "
-                         "readme: the load of the reference's README; buderax, gisodra, zudisun, sodotar: that design beside the "
+                         "readme: the load of the reference's README; buderax, gisodra, zudisun, sodotar, ropelix: that design beside the "
                          "dense Llama at equal sizes")
     ap.add_argument("--step-budget", type=int, default=2048, help="tokens a step of the serve workload")
     ap.add_argument("--show-choices", action="store_true",
@@ -899,6 +1122,8 @@ def main() -> int:
         return gisodra_workload(prefill_tokens=a.prefill_tokens, batch=a.batch, steps=min(a.steps, 32), warmup=a.warmup)
     if a.workload == "sodotar":
         return sodotar_workload(prefill_tokens=a.prefill_tokens, batch=a.batch, steps=min(a.steps, 32), warmup=a.warmup)
+    if a.workload == "ropelix":
+        return ropelix_workload(prefill_tokens=a.prefill_tokens, batch=a.batch, steps=min(a.steps, 32), warmup=a.warmup)
     if a.workload == "zudisun":
         return zudisun_workload(prefill_tokens=a.prefill_tokens, batch=a.batch, steps=min(a.steps, 32), warmup=a.warmup)
     if a.workload == "buderax":

@@ -31,7 +31,7 @@ struct DeltaPrepareArgs {
 };
 
 // grid (T, ceil((2 n_qk + n_v + 1) / 4)); the last job of a token is its scalars, a lane a head
-template <class TS>
+template <class TS, int NP>
 __global__ __launch_bounds__(DP_WAVES* FG_WAVE) void delta_prepare_kernel(const DeltaPrepareArgs a) {
   const int lane = threadIdx.x % FG_WAVE, t = blockIdx.x, job = blockIdx.y * DP_WAVES + threadIdx.x / FG_WAVE;
   const int qk_jobs = 2 * a.n_qk, v_base = qk_jobs * a.d;
@@ -52,10 +52,10 @@ __global__ __launch_bounds__(DP_WAVES* FG_WAVE) void delta_prepare_kernel(const 
   const bool is_v = job >= qk_jobs;
   const int w = is_v ? a.e : a.d;
   const int col = is_v ? v_base + (job - qk_jobs) * a.e : job * a.d;
-  float x[DP_MAX_PAIRS][2];
+  float x[NP][2];
   float ss = 0.f;
 #pragma unroll
-  for (int j = 0; j < DP_MAX_PAIRS; ++j) {
+  for (int j = 0; j < NP; ++j) {
     const int c = 2 * (lane + FG_WAVE * j);
     x[j][0] = x[j][1] = 0.f;
     if (c < w) {
@@ -71,7 +71,7 @@ __global__ __launch_bounds__(DP_WAVES* FG_WAVE) void delta_prepare_kernel(const 
     mul = rsqrtf(ss + a.unit_eps) * (job < a.n_qk ? a.q_scale : 1.f);
   }
 #pragma unroll
-  for (int j = 0; j < DP_MAX_PAIRS; ++j) {
+  for (int j = 0; j < NP; ++j) {
     const int c = 2 * (lane + FG_WAVE * j);
     if (c < w) *(float2*)(out + col + c) = make_float2(x[j][0] * mul, x[j][1] * mul);
   }
@@ -87,9 +87,17 @@ extern "C" int fg_delta_prepare(const DeltaPrepareArgs* args, int n_tokens, int 
     return FG_ERR_ARG;
   const dim3 grid(n_tokens, (2 * a.n_qk + a.n_v + 1 + DP_WAVES - 1) / DP_WAVES);
   if (grid.y > 65535) return FG_ERR_ARG;
-  if (src_dtype == FG_F32) delta_prepare_kernel<float><<<grid, DP_WAVES * FG_WAVE, 0, stream>>>(a);
-  else if (src_dtype == FG_BF16) delta_prepare_kernel<bf16_t><<<grid, DP_WAVES * FG_WAVE, 0, stream>>>(a);
+  const int widest = a.d > a.e ? a.d : a.e;
+#define GO(TS)                                                                                                 \
+  do {                                                                                                         \
+    if (widest <= 2 * FG_WAVE) delta_prepare_kernel<TS, 1><<<grid, DP_WAVES * FG_WAVE, 0, stream>>>(a);        \
+    else if (widest <= 4 * FG_WAVE) delta_prepare_kernel<TS, 2><<<grid, DP_WAVES * FG_WAVE, 0, stream>>>(a);   \
+    else delta_prepare_kernel<TS, DP_MAX_PAIRS><<<grid, DP_WAVES * FG_WAVE, 0, stream>>>(a);                   \
+  } while (0)
+  if (src_dtype == FG_F32) GO(float);
+  else if (src_dtype == FG_BF16) GO(bf16_t);
   else return FG_ERR_ARG;
+#undef GO
   return fg_launch_status();
 }
 

@@ -42,8 +42,8 @@ struct PrepareArgs {
 };
 
 // A wave's (token, head): lane l holds the pairs l, l + 64, ..  CONV: the convolution comes first.  ROWN: the
-// norm's factor comes from the caller (row_rstd_q, row_rstd_k).
-template <class TS, class TA, bool CONV, bool ROWN>
+// norm's factor comes from the caller (row_rstd_q, row_rstd_k).  NP: pairs a lane holds, for heads of up to 128 NP.
+template <class TS, class TA, int NP, bool CONV, bool ROWN>
 __device__ __forceinline__ void prepare_head(const PrepareArgs& a, int t, int job, float row_rstd_q, float row_rstd_k) {
   const int lane = threadIdx.x % FG_WAVE;
   const bool is_q = job < a.n_q;
@@ -58,10 +58,10 @@ __device__ __forceinline__ void prepare_head(const PrepareArgs& a, int t, int jo
   const int norm_dims = is_q ? a.q_norm_dims : a.k_norm_dims;
   const float* norm_w = is_q ? a.q_norm_w : a.k_norm_w;
   const TS* row = (const TS*)a.src + (size_t)t * a.src_stride;
-  float x[HP_MAX_PAIRS][2];
+  float x[NP][2];
   float ss = 0.f;
 #pragma unroll
-  for (int j = 0; j < HP_MAX_PAIRS; ++j) {
+  for (int j = 0; j < NP; ++j) {
     const int d = 2 * (lane + FG_WAVE * j);
     x[j][0] = x[j][1] = 0.f;
     if (d < w) {
@@ -84,7 +84,7 @@ __device__ __forceinline__ void prepare_head(const PrepareArgs& a, int t, int jo
   if (ROWN) {
     const float rstd = is_q ? row_rstd_q : row_rstd_k;
 #pragma unroll
-    for (int j = 0; j < HP_MAX_PAIRS; ++j) {
+    for (int j = 0; j < NP; ++j) {
       const int d = 2 * (lane + FG_WAVE * j);
       if (d < w) {
         x[j][0] = x[j][0] * rstd * norm_w[head * w + d];
@@ -95,7 +95,7 @@ __device__ __forceinline__ void prepare_head(const PrepareArgs& a, int t, int jo
     ss = wave_sum(ss);
     const float rstd = rsqrtf(ss / (float)norm_dims + a.eps);
 #pragma unroll
-    for (int j = 0; j < HP_MAX_PAIRS; ++j) {
+    for (int j = 0; j < NP; ++j) {
       const int d = 2 * (lane + FG_WAVE * j);
       if (d < norm_dims) {
         x[j][0] = x[j][0] * rstd * (norm_w ? norm_w[d] : 1.f);
@@ -105,14 +105,14 @@ __device__ __forceinline__ void prepare_head(const PrepareArgs& a, int t, int jo
   }
   if (tempered) {
 #pragma unroll
-    for (int j = 0; j < HP_MAX_PAIRS; ++j) {
+    for (int j = 0; j < NP; ++j) {
       x[j][0] *= temp;
       x[j][1] *= temp;
     }
   }
   if (a.table && (is_q ? a.rot_q : a.rot_k)) {  // uniform
 #pragma unroll
-    for (int j = 0; j < HP_MAX_PAIRS; ++j) {
+    for (int j = 0; j < NP; ++j) {
       const int d = 2 * (lane + FG_WAVE * j);
       if (d >= a.rot_start && d < a.rot_start + a.rotary_dim && d < w) {
         const float2 cs = *(const float2*)(a.table + ((size_t)t * (a.rotary_dim / 2) + (d - a.rot_start) / 2) * 2);
@@ -125,7 +125,7 @@ __device__ __forceinline__ void prepare_head(const PrepareArgs& a, int t, int jo
   if (is_q) {
     TA* o = (TA*)a.q_out + (size_t)t * a.q_out_stride + (size_t)head * a.q_out_hw;
 #pragma unroll
-    for (int j = 0; j < HP_MAX_PAIRS; ++j) {
+    for (int j = 0; j < NP; ++j) {
       const int d = 2 * (lane + FG_WAVE * j);
       if (d < a.q_out_hw) {  // (x is zero from w on)
         o[d] = from_f<TA>(x[j][0]);
@@ -140,7 +140,7 @@ __device__ __forceinline__ void prepare_head(const PrepareArgs& a, int t, int jo
   TA* kp = (TA*)a.k_pages + ((size_t)page * a.n_kv + head) * head_elems;
   TA* vp = (TA*)a.v_pages + ((size_t)page * a.n_kv + head) * head_elems;
 #pragma unroll
-  for (int j = 0; j < HP_MAX_PAIRS; ++j) {
+  for (int j = 0; j < NP; ++j) {
     const int d = 2 * (lane + FG_WAVE * j);
     if (d < a.hd_c) {
       TA* dst = kp + lay.k_off(off, d);  // d is even: d + 1 lies in the same chunk of 8
@@ -169,17 +169,17 @@ __device__ __forceinline__ void prepare_head(const PrepareArgs& a, int t, int jo
 }
 
 // grid (T, ceil((n_q + n_kv) / HP_WAVES)); a wave a (token, head)
-template <class TS, class TA, bool CONV>
+template <class TS, class TA, int NP, bool CONV>
 __global__ __launch_bounds__(HP_WAVES* FG_WAVE) void heads_prepare_kernel(const PrepareArgs a) {
   const int job = blockIdx.y * HP_WAVES + threadIdx.x / FG_WAVE;
   if (job >= a.n_q + a.n_kv) return;  // whole waves; no block barrier below
-  prepare_head<TS, TA, CONV, false>(a, blockIdx.x, job, 0.f, 0.f);
+  prepare_head<TS, TA, NP, CONV, false>(a, blockIdx.x, job, 0.f, 0.f);
 }
 
 // Norms over all of a token's query columns and all its key columns: a workgroup a token, whose waves take the
 // heads in turns once the two sums of squares are there.
 #define HP_ROW_WAVES 8
-template <class TS, class TA>
+template <class TS, class TA, int NP>
 __global__ __launch_bounds__(HP_ROW_WAVES* FG_WAVE) void heads_prepare_row_kernel(const PrepareArgs a) {
   __shared__ float red[2][HP_ROW_WAVES];
   const int t = blockIdx.x, wave = threadIdx.x / FG_WAVE, lane = threadIdx.x % FG_WAVE;
@@ -208,7 +208,7 @@ __global__ __launch_bounds__(HP_ROW_WAVES* FG_WAVE) void heads_prepare_row_kerne
     sk += red[1][i];
   }
   const float rq = nq ? rsqrtf(sq / (float)nq + a.eps) : 0.f, rk = nk ? rsqrtf(sk / (float)nk + a.eps) : 0.f;
-  for (int job = wave; job < a.n_q + a.n_kv; job += HP_ROW_WAVES) prepare_head<TS, TA, false, true>(a, t, job, rq, rk);
+  for (int job = wave; job < a.n_q + a.n_kv; job += HP_ROW_WAVES) prepare_head<TS, TA, NP, false, true>(a, t, job, rq, rk);
 }
 
 extern "C" int fg_heads_prepare(const PrepareArgs* args, int n_tokens, int src_dtype, int act_dtype,
@@ -232,17 +232,26 @@ extern "C" int fg_heads_prepare(const PrepareArgs* args, int n_tokens, int src_d
                    (a.n_kv && a.k_col + a.n_kv * a.k_w > a.conv.channels)))
     return FG_ERR_ARG;
   if (a.row_norm && (a.conv.w || (a.n_q && !a.q_norm_w) || (a.n_kv && !a.k_norm_w))) return FG_ERR_ARG;
-#define GO(TS, TA)                                                                                              \
-  do {                                                                                                          \
-    if (a.row_norm) heads_prepare_row_kernel<TS, TA><<<n_tokens, HP_ROW_WAVES * FG_WAVE, 0, stream>>>(a);       \
-    else if (a.conv.w) heads_prepare_kernel<TS, TA, true><<<grid, HP_WAVES * FG_WAVE, 0, stream>>>(a);          \
-    else heads_prepare_kernel<TS, TA, false><<<grid, HP_WAVES * FG_WAVE, 0, stream>>>(a);                       \
+  int widest = a.n_q ? (a.q_w > a.q_out_hw ? a.q_w : a.q_out_hw) : 0;
+  if (a.n_kv && a.hd_c > widest) widest = a.hd_c;
+#define GO1(TS, TA, NP)                                                                                           \
+  do {                                                                                                            \
+    if (a.row_norm) heads_prepare_row_kernel<TS, TA, NP><<<n_tokens, HP_ROW_WAVES * FG_WAVE, 0, stream>>>(a);     \
+    else if (a.conv.w) heads_prepare_kernel<TS, TA, NP, true><<<grid, HP_WAVES * FG_WAVE, 0, stream>>>(a);        \
+    else heads_prepare_kernel<TS, TA, NP, false><<<grid, HP_WAVES * FG_WAVE, 0, stream>>>(a);                     \
+  } while (0)
+#define GO(TS, TA)                                                  \
+  do {                                                              \
+    if (widest <= 2 * FG_WAVE) GO1(TS, TA, 1);                      \
+    else if (widest <= 4 * FG_WAVE) GO1(TS, TA, 2);                 \
+    else GO1(TS, TA, HP_MAX_PAIRS);                                 \
   } while (0)
   if (src_dtype == FG_F32 && act_dtype == FG_F32) GO(float, float);
   else if (src_dtype == FG_F32 && act_dtype == FG_BF16) GO(float, bf16_t);
   else if (src_dtype == FG_BF16 && act_dtype == FG_BF16) GO(bf16_t, bf16_t);
   else return FG_ERR_ARG;
 #undef GO
+#undef GO1
   return fg_launch_status();
 }
 

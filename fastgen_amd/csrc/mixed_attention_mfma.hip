@@ -467,8 +467,8 @@ __global__ __launch_bounds__(MT_THREADS) void mixed_tile_combine_kernel(const Mi
 // grid (n_items, n_chunks, ceil(n_kv / CB)); an item is one token
 __global__ __launch_bounds__(MT_THREADS) void mixed_decode_kernel(const MixedTileArgs a) {
   extern __shared__ __attribute__((aligned(16))) char lds[];
-  bf16x8* q_s = (bf16x8*)lds;                                   // [n_kv][NKS][64 lanes]: the queries of each group
-  float* o_s = (float*)(lds + (size_t)a.n_kv * NKS * FG_WAVE * 16);  // [2][CB][NDB][64 lanes][4]
+  bf16x8* q_s = (bf16x8*)lds;  // [n_kv][NKS][64 lanes]: the queries of each group
+  float* o_s = (float*)lds;  // in their place once the waves have ended their keys: [2][CB][NDB][64 lanes][4]
   __shared__ float ml_s[2][HP][2];
   const int tid = threadIdx.x, lane = tid % FG_WAVE, wave = tid / FG_WAVE;
   const int g = lane >> 4, row = lane & 15;
@@ -603,6 +603,7 @@ __global__ __launch_bounds__(MT_THREADS) void mixed_decode_kernel(const MixedTil
         o[c][db] = fs * o[c][db] + fo * other;
       }
   };
+  __syncthreads();  // (the queries are no longer read)
   if (wave >= 2) put(wave - 2);
   __syncthreads();
   if (wave < 2) take(wave);
@@ -720,8 +721,8 @@ extern "C" int fg_mixed_attention_decode(const MixedTileArgs* args, hipStream_t 
   const MixedTileArgs& a = *args;
   if (a.n_items <= 0) return FG_OK;
   if (!mixed_ok(a) || !a.partial || !a.part_ml || a.n_chunks > MD_MAX_CHUNKS) return FG_ERR_ARG;
-  const size_t lds = (size_t)a.n_kv * NKS * FG_WAVE * 16 + (size_t)2 * CB * NDB * FG_WAVE * 16;
-  if (lds > 160 * 1024 - 1024) return FG_ERR_ARG;
+  const int q_units = a.n_kv * NKS, o_units = 2 * CB * NDB;  // at most 128 and 64: n_kv <= 16, HD <= 256
+  const size_t lds = (size_t)(q_units > o_units ? q_units : o_units) * FG_WAVE * 16;
   if (hipFuncSetAttribute((const void*)mixed_decode_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
     return FG_ERR_LAUNCH;
   mixed_decode_kernel<<<dim3(a.n_items, a.n_chunks, (a.n_kv + CB - 1) / CB), MT_THREADS, lds, stream>>>(a);

@@ -142,7 +142,7 @@ def _random_pages(n, G, d, e, P, dtype, seed):
 
 MIXED = [(4, 2, 16, 24, 150, 64, 20, 8.0), (6, 3, 96, 64, 230, 64, 0, 0.0), (16, 4, 128, 128, 333, 64, 100, 30.0),
          (12, 12, 32, 16, 130, 32, 33, 0.0), (15, 5, 24, 40, 200, 32, 64, 5.0), (16, 1, 32, 32, 700, 64, 0, 10.0),
-         (1, 1, 16, 16, 70, 32, 1, 0.0), (10, 2, 160, 176, 140, 64, 50, 4.0), (20, 4, 8, 8, 90, 16, 16, 3.0), (3, 3, 12, 6, 75, 8, 0, 0.0)]
+         (1, 1, 16, 16, 70, 32, 1, 0.0), (10, 2, 160, 176, 140, 64, 50, 4.0), (16, 16, 256, 208, 90, 64, 40, 8.0), (20, 4, 8, 8, 90, 16, 16, 3.0), (3, 3, 12, 6, 75, 8, 0, 0.0)]
 
 
 @pytest.mark.parametrize("H,G,d,e,n,P,window,cap", MIXED)
