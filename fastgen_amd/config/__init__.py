@@ -13,6 +13,7 @@ from . import gisodra as _gisodra  # registers Gisodra
 from . import zudisun as _zudisun  # registers Zudisun
 from . import sodotar as _sodotar  # registers Sodotar
 from . import ropelix as _ropelix  # registers Ropelix
+from . import poselorn as _poselorn  # registers Poselorn
 
 __all__ = [
     "Architecture",

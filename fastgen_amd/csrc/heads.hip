@@ -8,7 +8,8 @@
 //                  processed key (a latent that serves as key and as value).
 //  head_linear     y[t, h, :] = W_h x[t, h, :] with a matrix per head, an optional sigmoid gate per
 //                  (token, head), and a run of x's columns behind the product's copied through.
-//  head_norm_gate  RMS norm per head of fp32 rows times silu(gate).
+//  head_norm_gate  RMS norm per head of fp32 rows times silu(gate) or sigmoid(gate); row_norm_gate: one norm over all
+//                  of a row's heads.
 //  head_diff_norm  the difference of two attention maps' outputs per head, divided by its root mean square.
 //
 // All arithmetic between a load and a store is fp32; a result is rounded once, at the store.
@@ -378,12 +379,12 @@ extern "C" int fg_head_linear(const HeadLinearArgs* args, int dtype, int out_dty
 
 // ---------------------------------------------------------------- head_norm_gate
 // out[t, h, :] = x[t, h, :] * rsqrt(mean(x[t, h, :]^2) + eps) * w * silu(g[t, h, :]) * out_scale; x fp32 [T, H * e],
-// g (act dtype) columns of a wider row.  grid (T, ceil(H / 4)); a wave a (token, head).
+// g (act dtype) columns of a wider row.  `sigmoid`: the gate's sigmoid in its silu's place.  grid (T, ceil(H / 4)); a wave a (token, head).
 #define HN_MAX 16  // elements a lane holds: heads of up to 1,024
 template <class TA, class TG>
 __global__ __launch_bounds__(HP_WAVES* FG_WAVE) void head_norm_gate_kernel(
     const float* __restrict__ x, const float* __restrict__ w, const TG* __restrict__ gate, int gate_stride,
-    TA* __restrict__ out, int out_stride, int H, int e, float eps, float out_scale) {
+    TA* __restrict__ out, int out_stride, int H, int e, float eps, float out_scale, int sigmoid) {
   const int lane = threadIdx.x % FG_WAVE, wave = threadIdx.x / FG_WAVE;
   const int t = blockIdx.x, h = blockIdx.y * HP_WAVES + wave;
   if (h >= H) return;
@@ -405,25 +406,78 @@ __global__ __launch_bounds__(HP_WAVES* FG_WAVE) void head_norm_gate_kernel(
     const int d = lane + FG_WAVE * j;
     if (d < e) {
       const float gv = to_f<TG>(gr[d]);
-      o[d] = from_f<TA>(v[j] * rstd * w[d] * (gv / (1.f + expf(-gv))));
+      o[d] = from_f<TA>(v[j] * rstd * w[d] * ((sigmoid ? 1.f : gv) / (1.f + expf(-gv))));
     }
   }
 }
 
 extern "C" int fg_head_norm_gate(const float* x, const float* w, const void* gate, int gate_stride, void* out,
-                                 int out_stride, int n_tokens, int H, int e, float eps, float out_scale, int act_dtype, int gate_dtype,
-                                 hipStream_t stream) {
+                                 int out_stride, int n_tokens, int H, int e, float eps, float out_scale, int sigmoid, int act_dtype,
+                                 int gate_dtype, hipStream_t stream) {
   if (n_tokens <= 0) return FG_OK;
   if (H <= 0 || e <= 0 || e > HN_MAX * FG_WAVE || gate_stride < H * e || out_stride < H * e || (H + HP_WAVES - 1) / HP_WAVES > 65535)
     return FG_ERR_ARG;
   dim3 grid(n_tokens, (H + HP_WAVES - 1) / HP_WAVES);
 #define GO(TA, TG)                                                                                             \
   head_norm_gate_kernel<TA, TG><<<grid, HP_WAVES * FG_WAVE, 0, stream>>>(x, w, (const TG*)gate, gate_stride,   \
-                                                                         (TA*)out, out_stride, H, e, eps, out_scale)
+                                                                         (TA*)out, out_stride, H, e, eps, out_scale, sigmoid)
   if (act_dtype == FG_F32 && gate_dtype == FG_F32) GO(float, float);
   else if (act_dtype == FG_BF16 && gate_dtype == FG_BF16) GO(bf16_t, bf16_t);
   else if (act_dtype == FG_BF16 && gate_dtype == FG_F32) GO(bf16_t, float);
   else return FG_ERR_ARG;
+#undef GO
+  return fg_launch_status();
+}
+
+// ---------------------------------------------------------------- row_norm_gate
+// out[t, :] = x[t, :] * rsqrt(mean(x[t, :]^2) + eps) * w * sigmoid(g[t, :]) * out_scale over W columns; x fp32 [T, W], g
+// (fp32) columns of a wider row.  A workgroup a row, which it keeps in registers: NIT elements a thread.
+#define RN_THREADS 256
+#define RN_MAX 64
+template <class TA, int NIT>
+__global__ __launch_bounds__(RN_THREADS) void row_norm_gate_kernel(
+    const float* __restrict__ x, const float* __restrict__ w, const float* __restrict__ gate, int gate_stride,
+    TA* __restrict__ out, int out_stride, int W, float eps, float out_scale) {
+  __shared__ float red[16];
+  const size_t t = blockIdx.x;
+  const float* xr = x + t * W;
+  const float* gr = gate + t * gate_stride;
+  float v[NIT], gv[NIT], wv[NIT], ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < NIT; ++j) {  // (never conditional: beyond the row its last element, which counts for nothing)
+    const int c = min((int)threadIdx.x + RN_THREADS * j, W - 1);
+    v[j] = xr[c];
+    gv[j] = gr[c];
+    wv[j] = w[c];
+  }
+#pragma unroll
+  for (int j = 0; j < NIT; ++j)
+    if ((int)threadIdx.x + RN_THREADS * j < W) ss += v[j] * v[j];
+  ss = block_sum(ss, red);
+  const float rstd = rsqrtf(ss / (float)W + eps) * out_scale;
+#pragma unroll
+  for (int j = 0; j < NIT; ++j) {
+    const int c = threadIdx.x + RN_THREADS * j;
+    if (c < W) out[t * out_stride + c] = from_f<TA>(v[j] * rstd * wv[j] / (1.f + expf(-gv[j])));
+  }
+}
+
+extern "C" int fg_row_norm_gate(const float* x, const float* w, const float* gate, int gate_stride, void* out, int out_stride,
+                                int n_tokens, int W, float eps, float out_scale, int act_dtype, hipStream_t stream) {
+  if (n_tokens <= 0) return FG_OK;
+  if (W <= 0 || W > RN_MAX * RN_THREADS || gate_stride < W || out_stride < W) return FG_ERR_ARG;
+#define GO(TA, NIT) row_norm_gate_kernel<TA, NIT><<<n_tokens, RN_THREADS, 0, stream>>>(x, w, gate, gate_stride, (TA*)out, out_stride, W, eps, out_scale)
+#define LAUNCH(TA)                                  \
+  do {                                              \
+    if (W <= 2 * RN_THREADS) GO(TA, 2);             \
+    else if (W <= 8 * RN_THREADS) GO(TA, 8);        \
+    else if (W <= 16 * RN_THREADS) GO(TA, 16);      \
+    else GO(TA, RN_MAX);                            \
+  } while (0)
+  if (act_dtype == FG_F32) LAUNCH(float);
+  else if (act_dtype == FG_BF16) LAUNCH(bf16_t);
+  else return FG_ERR_ARG;
+#undef LAUNCH
 #undef GO
   return fg_launch_status();
 }

@@ -7,6 +7,9 @@
 //  down     per tile: y[pair] = act W_down^T in fp32, one row per pair
 //  combine  out[t] = plus[t] + sum_j weight[t][j] * y[t * top + j], in fp32, j ascending
 //
+// Experts from a number on may be identities: the router scores them like the others, but the sort makes no tiles of
+// their pairs and combine takes the token's own row of x for their output.
+//
 // A tile's rows do not depend on one another: every output element is one dot product over k in an
 // order fixed by k alone, so a token's result is the same whatever else the step holds and wherever
 // the sort puts it.  The bf16 kernels run on the matrix cores (v_mfma_f32_16x16x32_bf16, the expert's
@@ -32,7 +35,8 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 // neighbouring experts (a group's rank: the sum of its two largest choice scores; the experts of the other
 // groups cannot be chosen); the weights are the chosen experts' scores without the correction, divided by
 // their sum (+ 1e-20) and multiplied by `weight_scale`.  A third way (`sigmoid_scores` = 2): the scores are the
-// softmax of the logits over all experts; choice, groups and weights as with sigmoid scores.
+// softmax of the logits over all experts; choice, groups and weights as with sigmoid scores.  `group_max`: a group
+// ranks by its largest choice score alone.  `raw_weights`: the chosen scores are not divided by their sum.
 //
 // `n_extra`: the router matrix has that many rows more than there are experts; their logits (no bias) take no
 // part in the choice and are stored as they are in `extra [n_tokens, n_extra]` (a gate of a shared expert, say).
@@ -43,6 +47,7 @@ struct RouteMode {
   float weight_scale;
   int n_extra;
   float* extra;
+  int group_max, raw_weights;
 };
 template <class T, int WAVES, int EPW>
 __global__ __launch_bounds__(64 * WAVES) void moe_route_kernel(
@@ -114,7 +119,7 @@ __global__ __launch_bounds__(64 * WAVES) void moe_route_kernel(
             const float v = z[g * per + i];
             if (v > a) { b = a; a = v; } else if (v > b) { b = v; }
           }
-          rank[g] = per > 1 ? a + b : a;
+          rank[g] = per > 1 && !mode.group_max ? a + b : a;
         }
       }
       __syncthreads();
@@ -156,7 +161,7 @@ __global__ __launch_bounds__(64 * WAVES) void moe_route_kernel(
   if (threadIdx.x == 0 && mode.sigmoid_scores) {
     float sum = 0.f;
     for (int j = 0; j < top; ++j) sum += chosen[j];
-    for (int j = 0; j < top; ++j) weight[t * top + j] = chosen[j] / (sum + 1e-20f) * mode.weight_scale;
+    for (int j = 0; j < top; ++j) weight[t * top + j] = (mode.raw_weights ? chosen[j] : chosen[j] / (sum + 1e-20f)) * mode.weight_scale;
   } else if (threadIdx.x == 0) {
     const float m = chosen[0];  // the largest
     float sum = 0.f;
@@ -168,14 +173,14 @@ __global__ __launch_bounds__(64 * WAVES) void moe_route_kernel(
 extern "C" int fg_moe_route_mode(const void* x, int ldx, int dtype, const float* wr, const float* bias, int n_tokens,
                                  int dim, int n_experts, int top, int* choice, float* weight, int sigmoid_scores,
                                  const float* correction, int n_groups, int keep_groups, float weight_scale,
-                                 int n_extra, float* extra, hipStream_t stream) {
+                                 int n_extra, float* extra, int group_max, int raw_weights, hipStream_t stream) {
   if (n_tokens <= 0) return FG_OK;
   if (sigmoid_scores < 0 || sigmoid_scores > 2 || n_extra < 0 || (n_extra > 0 && !extra)) return FG_ERR_ARG;
   if (dim <= 0 || ldx < dim || n_experts <= 0 || top < 1 || top > n_experts) return FG_ERR_ARG;
   if (n_groups < 1 || n_experts % n_groups || keep_groups < 1 || keep_groups > n_groups ||
       top > keep_groups * (n_experts / n_groups) || (!sigmoid_scores && (correction || n_groups > 1)))
     return FG_ERR_ARG;
-  const RouteMode mode = {sigmoid_scores, correction, n_groups, keep_groups, weight_scale, n_extra, extra};
+  const RouteMode mode = {sigmoid_scores, correction, n_groups, keep_groups, weight_scale, n_extra, extra, group_max, raw_weights};
   const size_t lds = (size_t)(2 * n_experts + n_extra + top + n_groups) * sizeof(float);
   if (lds > 60000) return FG_ERR_ARG;
 #define GO(T, WAVES, EPW)                                                                                        \
@@ -196,16 +201,17 @@ extern "C" int fg_moe_route_mode(const void* x, int ldx, int dtype, const float*
 extern "C" int fg_moe_route(const void* x, int ldx, int dtype, const float* wr, const float* bias, int n_tokens, int dim,
                             int n_experts, int top, int* choice, float* weight, hipStream_t stream) {
   return fg_moe_route_mode(x, ldx, dtype, wr, bias, n_tokens, dim, n_experts, top, choice, weight, 0, nullptr, 1, 1, 1.f,
-                           0, nullptr, stream);
+                           0, nullptr, 0, 0, stream);
 }
 
 // -------------------------------------------------------------------- sort
 // One workgroup.  sorted[pos] = pair (token * top + j) for the pairs in the order of their experts;
-// tiles[i] = (expert, first pos, rows, 0) for i < max_tiles, rows = 0 for tiles that do not exist.
+// tiles[i] = (expert, first pos, rows, 0) for i < max_tiles, rows = 0 for tiles that do not exist.  Experts from
+// n_tiled on have no tiles.
 // LDS: 3 * n_experts ints (count, first pos, first tile).
 #define SORT_THREADS 1024
 __global__ __launch_bounds__(SORT_THREADS) void moe_sort_kernel(
-    const int* __restrict__ choice, int n_pairs, int n_experts, int tile_rows, int max_tiles,
+    const int* __restrict__ choice, int n_pairs, int n_experts, int n_tiled, int tile_rows, int max_tiles,
     int* __restrict__ sorted, int* __restrict__ tiles) {
   extern __shared__ int sm[];
   int* count = sm;
@@ -221,7 +227,7 @@ __global__ __launch_bounds__(SORT_THREADS) void moe_sort_kernel(
     for (int base = 0; base < n_experts; base += FG_WAVE) {
       const int e = base + lane;
       const int c = e < n_experts ? count[e] : 0;
-      const int nt = (c + tile_rows - 1) / tile_rows;
+      const int nt = e < n_tiled ? (c + tile_rows - 1) / tile_rows : 0;
       int sc = c, st = nt;
 #pragma unroll
       for (int d = 1; d < FG_WAVE; d <<= 1) {
@@ -241,7 +247,7 @@ __global__ __launch_bounds__(SORT_THREADS) void moe_sort_kernel(
   __syncthreads();
   for (int e = threadIdx.x; e < n_experts; e += SORT_THREADS) {
     const int c = count[e], f = first[e];
-    for (int i = 0, r = 0; r < c; ++i, r += tile_rows) {
+    for (int i = 0, r = 0; r < c && e < n_tiled; ++i, r += tile_rows) {
       const int at = first_tile[e] + i;
       if (at < max_tiles) *(int4*)(tiles + 4 * (size_t)at) = make_int4(e, f + r, min(tile_rows, c - r), 0);
     }
@@ -254,12 +260,12 @@ __global__ __launch_bounds__(SORT_THREADS) void moe_sort_kernel(
   }
 }
 
-extern "C" int fg_moe_sort(const int* choice, int n_pairs, int n_experts, int tile_rows, int max_tiles, int* sorted,
-                           int* tiles, hipStream_t stream) {
+extern "C" int fg_moe_sort(const int* choice, int n_pairs, int n_experts, int n_tiled, int tile_rows, int max_tiles,
+                           int* sorted, int* tiles, hipStream_t stream) {
   if (n_pairs <= 0) return FG_OK;
-  if (n_experts <= 0 || tile_rows <= 0 || max_tiles <= 0 || (size_t)3 * n_experts * sizeof(int) > 60000) return FG_ERR_ARG;
-  moe_sort_kernel<<<1, SORT_THREADS, (size_t)3 * n_experts * sizeof(int), stream>>>(choice, n_pairs, n_experts, tile_rows,
-                                                                                    max_tiles, sorted, tiles);
+  if (n_experts <= 0 || n_tiled < 0 || n_tiled > n_experts || tile_rows <= 0 || max_tiles <= 0 || (size_t)3 * n_experts * sizeof(int) > 60000) return FG_ERR_ARG;
+  moe_sort_kernel<<<1, SORT_THREADS, (size_t)3 * n_experts * sizeof(int), stream>>>(choice, n_pairs, n_experts, n_tiled,
+                                                                                    tile_rows, max_tiles, sorted, tiles);
   return fg_launch_status();
 }
 
@@ -670,16 +676,26 @@ extern "C" int fg_moe_down(const void* act, int lda, const void* wd, int ldw, co
 // out[t] = plus[t] + sum_j weight[t][j] * y[t * top + j]: the weighted sum first, j ascending, all fp32.
 // plus: rows of the activation dtype, or (n_plus > 0) fp32 partial sums plus[p * plus_stride + t * ldp + d],
 // whose sum, in order, is what is added.  plus_gate (fp32, one number a token at plus_gate[t * gate_stride]): the
-// rows of plus are multiplied by its sigmoid before they are added.
-template <class TP>
+// rows of plus are multiplied by its sigmoid before they are added.  choice [n_tokens, top] (or null): the output of an
+// expert from n_tiled on is the token's row of x.
+struct CombineIdentity {
+  const int* choice; int n_tiled;
+  const void* x; int ldx;
+};
+template <class TP, class TX>
 __global__ __launch_bounds__(256) void moe_combine_kernel(
     const float* __restrict__ y, const float* __restrict__ weight, const TP* __restrict__ plus, int ldp, int n_plus,
-    size_t plus_stride, int top, int dim, float* __restrict__ out, const float* __restrict__ plus_gate, int gate_stride) {
+    size_t plus_stride, int top, int dim, float* __restrict__ out, const float* __restrict__ plus_gate, int gate_stride,
+    const CombineIdentity id) {
   const int t = blockIdx.x;
   const float pg = plus_gate ? 1.f / (1.f + expf(-plus_gate[(size_t)t * gate_stride])) : 1.f;
   for (int d = threadIdx.x; d < dim; d += 256) {
     float s = 0.f;
-    for (int j = 0; j < top; ++j) s = fmaf(weight[(size_t)t * top + j], y[((size_t)t * top + j) * dim + d], s);
+    for (int j = 0; j < top; ++j) {
+      const size_t p = (size_t)t * top + j;
+      const float o = id.choice && id.choice[p] >= id.n_tiled ? to_f<TX>(((const TX*)id.x)[(size_t)t * id.ldx + d]) : y[p * dim + d];
+      s = fmaf(weight[p], o, s);
+    }
     if (plus) {
       float m = to_f<TP>(plus[(size_t)t * ldp + d]);
       for (int p = 1; p < n_plus; ++p) m += to_f<TP>(plus[p * plus_stride + (size_t)t * ldp + d]);
@@ -689,21 +705,38 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(
   }
 }
 
-extern "C" int fg_moe_combine_gated(const float* y, const float* weight, const void* plus, int ldp, int plus_dtype,
-                                    int n_plus, long long plus_stride, int n_tokens, int top, int dim, float* out,
-                                    const float* plus_gate, int gate_stride, hipStream_t stream) {
+extern "C" int fg_moe_combine_identity(const float* y, const float* weight, const void* plus, int ldp, int plus_dtype,
+                                       int n_plus, long long plus_stride, int n_tokens, int top, int dim, float* out,
+                                       const float* plus_gate, int gate_stride, const int* choice, int n_tiled, const void* x,
+                                       int ldx, int x_dtype, hipStream_t stream) {
   if (n_tokens <= 0) return FG_OK;
   if (plus_gate && (!plus || gate_stride < 1)) return FG_ERR_ARG;
   if (top <= 0 || dim <= 0 || (plus && (ldp < dim || n_plus < 1)) || (n_plus > 1 && plus_dtype != FG_F32)) return FG_ERR_ARG;
-  if (plus_dtype == FG_F32)
-    moe_combine_kernel<float><<<n_tokens, 256, 0, stream>>>(y, weight, (const float*)plus, ldp, n_plus, (size_t)plus_stride,
-                                                            top, dim, out, plus_gate, gate_stride);
-  else if (plus_dtype == FG_BF16)
-    moe_combine_kernel<bf16_t><<<n_tokens, 256, 0, stream>>>(y, weight, (const bf16_t*)plus, ldp, n_plus,
-                                                             (size_t)plus_stride, top, dim, out, plus_gate, gate_stride);
+  if (choice && (!x || ldx < dim || n_tiled < 0)) return FG_ERR_ARG;
+  const CombineIdentity id = {choice, n_tiled, x, ldx};
+  if (x_dtype != FG_F32 && x_dtype != FG_BF16) return FG_ERR_ARG;
+  if (plus_dtype == FG_F32 && x_dtype == FG_F32)
+    moe_combine_kernel<float, float><<<n_tokens, 256, 0, stream>>>(y, weight, (const float*)plus, ldp, n_plus, (size_t)plus_stride,
+                                                                   top, dim, out, plus_gate, gate_stride, id);
+  else if (plus_dtype == FG_F32)
+    moe_combine_kernel<float, bf16_t><<<n_tokens, 256, 0, stream>>>(y, weight, (const float*)plus, ldp, n_plus, (size_t)plus_stride,
+                                                                    top, dim, out, plus_gate, gate_stride, id);
+  else if (plus_dtype == FG_BF16 && x_dtype == FG_BF16)
+    moe_combine_kernel<bf16_t, bf16_t><<<n_tokens, 256, 0, stream>>>(y, weight, (const bf16_t*)plus, ldp, n_plus,
+                                                                     (size_t)plus_stride, top, dim, out, plus_gate, gate_stride, id);
+  else if (plus_dtype == FG_BF16 && !choice)
+    moe_combine_kernel<bf16_t, float><<<n_tokens, 256, 0, stream>>>(y, weight, (const bf16_t*)plus, ldp, n_plus,
+                                                                    (size_t)plus_stride, top, dim, out, plus_gate, gate_stride, id);
   else
     return FG_ERR_ARG;
   return fg_launch_status();
+}
+
+extern "C" int fg_moe_combine_gated(const float* y, const float* weight, const void* plus, int ldp, int plus_dtype,
+                                    int n_plus, long long plus_stride, int n_tokens, int top, int dim, float* out,
+                                    const float* plus_gate, int gate_stride, hipStream_t stream) {
+  return fg_moe_combine_identity(y, weight, plus, ldp, plus_dtype, n_plus, plus_stride, n_tokens, top, dim, out, plus_gate,
+                                 gate_stride, nullptr, 0, nullptr, 0, FG_F32, stream);
 }
 
 extern "C" int fg_moe_combine(const float* y, const float* weight, const void* plus, int ldp, int plus_dtype, int n_plus,

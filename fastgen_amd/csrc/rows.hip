@@ -656,6 +656,55 @@ extern "C" int fg_gated_mul(const void* gu, const float* bias, void* out, int n_
   return fg_gated_mul_act(gu, bias, out, n_rows, hidden, act, 0.f, 1.f, src_dtype, act_dtype, stream);
 }
 
+// ------------------------------------------- act(x + b), any source dtype
+// The activation of a feed-forward without a gate: square of ReLU (0), ReLU (1), SiLU (2) or the tanh form of GELU (3) of
+// rows (fp32, or the activation dtype) plus a bias per column (fp32, or none).  hidden % 8 == 0.
+template <class TS, class TA>
+__global__ __launch_bounds__(ROWS_THREADS) void bias_act_kernel(const TS* __restrict__ x, const float* __restrict__ bias,
+                                                                TA* __restrict__ out, int hidden, int act) {
+  const int e = (blockIdx.x * ROWS_THREADS + threadIdx.x) * 8;
+  if (e >= hidden) return;
+  float v[8], r[8];
+  load8<TS>(x + (size_t)blockIdx.y * hidden + e, v);
+  if (bias) {
+    float b[8];
+    load8<float>(bias + e, b);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] += b[i];
+  }
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const float z = v[i];
+    if (act <= 1) {
+      const float p = fmaxf(z, 0.f);
+      r[i] = act == 0 ? p * p : p;
+    } else if (act == 2) {
+      r[i] = z / (1.f + expf(-z));
+    } else {
+      r[i] = 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+    }
+  }
+  store8<TA>(out + (size_t)blockIdx.y * hidden + e, r);
+}
+
+extern "C" int fg_bias_act(const void* x, const float* bias, void* out, int n_rows, int hidden, int act, int src_dtype,
+                           int act_dtype, hipStream_t stream) {
+  if (n_rows <= 0) return FG_OK;
+  if (hidden <= 0 || hidden % 8 || act < 0 || act > 3) return FG_ERR_ARG;
+  for (int r0 = 0; r0 < n_rows; r0 += 65535) {
+    const int nr = n_rows - r0 < 65535 ? n_rows - r0 : 65535;
+    const dim3 grid((hidden + ROWS_THREADS * 8 - 1) / (ROWS_THREADS * 8), nr);
+    const size_t o = (size_t)r0 * hidden;
+#define GO(TS, TA) bias_act_kernel<TS, TA><<<grid, ROWS_THREADS, 0, stream>>>((const TS*)x + o, bias, (TA*)out + o, hidden, act)
+    if (src_dtype == FG_F32 && act_dtype == FG_F32) GO(float, float);
+    else if (src_dtype == FG_F32 && act_dtype == FG_BF16) GO(float, bf16_t);
+    else if (src_dtype == FG_BF16 && act_dtype == FG_BF16) GO(bf16_t, bf16_t);
+    else return FG_ERR_ARG;
+#undef GO
+  }
+  return fg_launch_status();
+}
+
 // ------------------------------------------------------------- soft cap
 // x = cap * tanh(x / cap) in place on fp32 (logits).
 __global__ __launch_bounds__(ROWS_THREADS) void softcap_kernel(float* __restrict__ x, size_t n, float cap) {

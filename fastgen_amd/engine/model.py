@@ -18,7 +18,8 @@ import torch
 
 from ..config import ModelLayout, PartSpec, get_architecture, read_config_json
 from ..kernels.linear import StreamedMatrix, packing, packing_fits
-from ..kernels.ops import PostNormed, ScaledDelta, ScaledRows, post_add_rmsnorm, stream_add, streams_spread
+from ..kernels.ops import (PostNormed, ScaledDelta, ScaledRows, StreamTerms, post_add_rmsnorm, stream_add, stream_terms,
+                           streams_spread)
 from ..parts import LayerStore, PagedNeed, StateNeed, TensorSpec, build_part
 from ..parts.base import MATRIX
 from ..weights.source import RandomSource, SafetensorsSource, TensorSource, check_against_specs
@@ -193,6 +194,9 @@ class Model:
                     pending = None
                 if isinstance(pending, ScaledDelta):  # ... or that is scaled per channel
                     stream_add(h, pending.rows, None, None, delta_scale=pending.scale)
+                    pending = None
+                if isinstance(pending, StreamTerms) and not injections[entry.inject[0]].takes_terms:
+                    stream_terms(h, pending)
                     pending = None
                 injections[entry.inject[0]].forward(h, None if isinstance(pending, ScaledRows) else pending,
                                                     embedded, entry.inject[1])

@@ -53,6 +53,9 @@ LIBRARIES: Dict[str, str] = {
     "delta_rule": "delta_rule.hip",
     "lru": "lru.hip",
     "mixed_attention": "mixed_attention.hip",
+    "stream_terms": "stream_terms.hip",
+    "low_rank": "low_rank.hip",
+    "lightning": "lightning.hip",
 }
 
 # libraries compiled once per value of a macro: name -> (source, macro, values that build_all compiles,

@@ -11,7 +11,7 @@ from __future__ import annotations
 import ctypes
 from dataclasses import dataclass
 import os
-from typing import Dict, Optional, Tuple
+from typing import Dict, List, Optional, Sequence, Tuple
 
 import numpy as np
 
@@ -316,6 +316,107 @@ def post_add_rmsnorm(h: torch.Tensor, delta: Optional[torch.Tensor], post_weight
         _code(w_any) if w_any is not None else F32, _ptr(delta_bias), _stream(h))
     _check(st, "post_add_rmsnorm")
     return out
+
+
+# ------------------------------------------------ several terms at once
+@dataclass
+class StreamTerm:
+    """A sublayer's output on its way into the residual stream: ``scale (.) n(rows + bias)``.  ``rows`` is ``[T, dim]`` of the
+    activation dtype or fp32 ``[S, T, dim]`` partial sums; ``bias`` and ``scale`` are fp32 ``[dim]`` or None; with ``norm_eps``
+    ``n`` divides by the root mean square over the row (eps inside the root), else it does nothing."""
+
+    rows: torch.Tensor
+    scale: Optional[torch.Tensor] = None
+    bias: Optional[torch.Tensor] = None
+    norm_eps: Optional[float] = None
+
+
+@dataclass
+class StreamTerms:
+    """What the sublayers of a layer leave to be added, all at once (:func:`stream_terms`).  A norm on the stream takes it
+    where it takes rows to be added."""
+
+    terms: List[StreamTerm]
+
+    @classmethod
+    def of(cls, delta) -> "StreamTerms":
+        """Any form of what a layer leaves to be added, as terms."""
+        if delta is None:
+            return cls([])
+        if isinstance(delta, StreamTerms):
+            return delta
+        if isinstance(delta, ScaledDelta):
+            return cls([StreamTerm(delta.rows, delta.scale)])
+        if isinstance(delta, PostNormed):
+            return cls([StreamTerm(delta.rows, delta.weight.float(), delta.bias, delta.eps)])
+        if isinstance(delta, torch.Tensor):
+            return cls([StreamTerm(delta)])
+        raise KernelArgumentError(f"{type(delta).__name__} is nothing that can be added to the one plain stream")
+
+
+STREAM_TERMS_MAX = 3
+
+
+class _StreamTerm(ctypes.Structure):
+    _fields_ = [("rows", ctypes.c_void_p), ("parts", ctypes.c_void_p), ("n_parts", ctypes.c_int), ("part_stride", ctypes.c_longlong),
+                ("bias", ctypes.c_void_p), ("scale", ctypes.c_void_p), ("normed", ctypes.c_int), ("eps", ctypes.c_float)]
+
+
+class _StreamTermsArgs(ctypes.Structure):
+    _fields_ = [("h", ctypes.c_void_p), ("term", _StreamTerm * STREAM_TERMS_MAX), ("n_terms", ctypes.c_int), ("again", ctypes.c_void_p),
+                ("w", ctypes.c_void_p * 2), ("out", ctypes.c_void_p * 2), ("rows", ctypes.c_void_p), ("dim", ctypes.c_int),
+                ("eps", ctypes.c_float)]
+
+
+def stream_terms(h: torch.Tensor, delta: StreamTerms, again: Optional[torch.Tensor] = None,
+                 norms: Sequence[Tuple[torch.Tensor, torch.Tensor]] = (), eps: float = 0.0,
+                 rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``h += sum of the terms`` (in order), ``h += again`` (fp32 ``[T, dim]``) on the fp32 stream ``h [T, dim]``, and for each
+    ``(weight [dim], out)`` of ``norms`` (at most two) ``out = h / rms(h) * weight``: one kernel, all in fp32.  With ``rows``
+    only those rows are computed, into consecutive rows of the outs, and ``h`` is left as it was."""
+    tensors = [h, again, rows] + [t for n in norms for t in n]
+    for t in delta.terms:
+        tensors += [t.rows, t.scale, t.bias]
+    _gpu(*tensors)
+    _need(h.dtype == torch.float32 and h.dim() == 2 and h.is_contiguous(), "h must be contiguous float32 [T, dim]")
+    T, dim = h.shape
+    _need(dim <= 16384 and len(delta.terms) <= STREAM_TERMS_MAX and len(norms) <= 2, "at most 16384 columns, three terms, two norms")
+    n_rows = T if rows is None else rows.numel()
+    if rows is not None:
+        _i32(rows, "rows")
+        _need(len(norms) > 0, "a gathered call needs an out")
+    a = _StreamTermsArgs()
+    a.h, a.dim, a.eps, a.n_terms = h.data_ptr(), dim, float(eps), len(delta.terms)
+    act = norms[0][1].dtype if norms else None
+    for c, t in zip(a.term, delta.terms):
+        if t.rows.dim() == 3:
+            _need(t.rows.dtype == torch.float32 and t.rows.shape[1:] == h.shape and t.rows.stride(2) == 1 and t.rows.stride(1) == dim
+                  and (t.rows.shape[0] == 1 or t.rows.stride(0) % 4 == 0 or dim % 8), "partial sums must be float32 [S, T, dim] with contiguous rows")
+            c.parts, c.n_parts, c.part_stride = t.rows.data_ptr(), t.rows.shape[0], t.rows.stride(0)
+        elif t.rows.dtype == torch.float32 and act not in (None, torch.float32):
+            _need(t.rows.shape == h.shape and t.rows.is_contiguous(), "a term must be contiguous and shaped like h")
+            c.parts, c.n_parts, c.part_stride = t.rows.data_ptr(), 1, 0
+        else:
+            act = act or t.rows.dtype
+            _need(t.rows.shape == h.shape and t.rows.is_contiguous() and t.rows.dtype == act,
+                  "a term must be contiguous, shaped like h, of the outs' dtype or float32")
+            c.rows = t.rows.data_ptr()
+        _f32_vec(t.bias, dim, "a term's bias")
+        _f32_vec(t.scale, dim, "a term's scale")
+        c.bias, c.scale = (x.data_ptr() if x is not None else None for x in (t.bias, t.scale))
+        c.normed, c.eps = int(t.norm_eps is not None), float(t.norm_eps or 0.0)
+    if again is not None:
+        _need(again.dtype == torch.float32 and again.shape == h.shape and again.is_contiguous(), "again must be contiguous float32, shaped like h")
+        a.again = again.data_ptr()
+    w_code = F32
+    for k, (w, out) in enumerate(norms):
+        _need(w.shape == (dim,) and w.is_contiguous() and w.dtype == norms[0][0].dtype, "the norms' weights must be [dim] of one dtype")
+        _need(out.is_contiguous() and out.shape == (n_rows, dim) and out.dtype == act, "the outs must be contiguous [rows, dim] of one dtype")
+        a.w[k], a.out[k], w_code = w.data_ptr(), out.data_ptr(), _code(w)
+    a.rows = rows.data_ptr() if rows is not None else None
+    _check(_lib.load("stream_terms").fg_stream_terms(ctypes.byref(a), n_rows, _DTYPE_CODE[act or torch.float32], w_code, _stream(h)),
+           "stream_terms")
+    return h
 
 
 def softcap(x: torch.Tensor, cap: float) -> torch.Tensor:
@@ -1052,7 +1153,8 @@ MOE_TILE_ROWS = (16, 32, 64, 128, 256)  # rows of one expert that a tile of the 
 
 def moe_route(x: torch.Tensor, router: torch.Tensor, bias: Optional[torch.Tensor], top: int,
               sigmoid_scores: bool = False, correction: Optional[torch.Tensor] = None, n_groups: int = 1,
-              keep_groups: int = 1, weight_scale: float = 1.0, softmax_scores: bool = False, n_extra: int = 0):
+              keep_groups: int = 1, weight_scale: float = 1.0, softmax_scores: bool = False, n_extra: int = 0,
+              group_max: bool = False, raw_weights: bool = False):
     """Per row of ``x [T, dim]``: fp32 logits ``x router^T + bias`` (``router`` fp32 ``[E, dim]``), the
     ``top`` largest (ties: the lower expert), and the softmax over those.  Returns int32 ``[T, top]``
     experts and fp32 ``[T, top]`` weights, the largest logit first.
@@ -1062,7 +1164,8 @@ def moe_route(x: torch.Tensor, router: torch.Tensor, bias: Optional[torch.Tensor
     groups of neighbours (a group ranks by the sum of its two largest choice scores; ties: the lower group);
     the weights are the chosen experts' scores, without the correction, divided by their sum (+ 1e-20)
     and multiplied by ``weight_scale``.  ``softmax_scores``: the same with the softmax of the logits over all
-    experts as the scores.
+    experts as the scores.  ``group_max``: a group ranks by its largest choice score alone; ``raw_weights``: the chosen
+    experts' scores are not divided by their sum.
 
     ``n_extra``: ``router`` has that many rows behind the experts'; their logits (without bias) take no part in
     the choice and are returned as a third result, fp32 ``[T, n_extra]`` (the gate of a shared expert, say)."""
@@ -1080,6 +1183,7 @@ def moe_route(x: torch.Tensor, router: torch.Tensor, bias: Optional[torch.Tensor
     weight = torch.empty((T, top), dtype=torch.float32, device=x.device)
     _f32_vec(correction, E, "correction")
     scored = sigmoid_scores or softmax_scores
+    _need(scored or not (group_max or raw_weights), "group_max and raw_weights go with sigmoid or softmax scores")
     _need(scored or (correction is None and n_groups == 1), "correction and groups go with sigmoid or softmax scores")
     extra = torch.empty((T, n_extra), dtype=torch.float32, device=x.device) if n_extra else None
     _need(n_groups >= 1 and E % n_groups == 0 and 1 <= keep_groups <= n_groups and top <= keep_groups * (E // n_groups),
@@ -1087,7 +1191,8 @@ def moe_route(x: torch.Tensor, router: torch.Tensor, bias: Optional[torch.Tensor
     st = _lib.load("moe").fg_moe_route_mode(_ptr(x), x.stride(0), _code(x), _ptr(router), _ptr(bias), T, dim, E, top,
                                             _ptr(choice), _ptr(weight), 2 if softmax_scores else int(bool(sigmoid_scores)),
                                             _ptr(correction), int(n_groups), int(keep_groups),
-                                            ctypes.c_float(weight_scale), int(n_extra), _ptr(extra), _stream(x))
+                                            ctypes.c_float(weight_scale), int(n_extra), _ptr(extra), int(bool(group_max)),
+                                            int(bool(raw_weights)), _stream(x))
     _check(st, "moe_route")
     return (choice, weight, extra) if n_extra else (choice, weight)
 
@@ -1097,18 +1202,20 @@ def moe_max_tiles(n_pairs: int, n_experts: int, tile_rows: int) -> int:
     return min(n_pairs, n_pairs // tile_rows + n_experts)
 
 
-def moe_sort(choice: torch.Tensor, n_experts: int, tile_rows: int):
+def moe_sort(choice: torch.Tensor, n_experts: int, tile_rows: int, n_identity: int = 0):
     """The (row, choice) pairs of ``choice [T, top]`` in the order of their experts, cut into tiles of
     at most ``tile_rows`` rows of one expert, on the device.  Returns int32 ``sorted [T * top]`` (pair
     ``t * top + j`` at each sorted place) and int32 ``tiles [max_tiles, 4]``: (expert, first sorted
-    place, rows, 0), rows = 0 for tiles that this step does not have."""
+    place, rows, 0), rows = 0 for tiles that this step does not have.  The last ``n_identity`` experts have no tiles: their
+    output is their input (:func:`moe_combine`)."""
     _gpu(choice)
     _i32(choice, "choice")
+    _need(0 <= n_identity <= n_experts, "n_identity of the experts")
     n_pairs = choice.numel()
-    max_tiles = moe_max_tiles(n_pairs, n_experts, tile_rows)
+    max_tiles = moe_max_tiles(n_pairs, n_experts - n_identity, tile_rows)
     sorted_ = torch.empty((n_pairs,), dtype=torch.int32, device=choice.device)
     tiles = torch.empty((max_tiles, 4), dtype=torch.int32, device=choice.device)
-    st = _lib.load("moe").fg_moe_sort(_ptr(choice), n_pairs, n_experts, tile_rows, max_tiles, _ptr(sorted_), _ptr(tiles),
+    st = _lib.load("moe").fg_moe_sort(_ptr(choice), n_pairs, n_experts, n_experts - n_identity, tile_rows, max_tiles, _ptr(sorted_), _ptr(tiles),
                                       _stream(choice))
     _check(st, "moe_sort")
     return sorted_, tiles
@@ -1167,12 +1274,14 @@ def moe_down(act: torch.Tensor, w_down: torch.Tensor, sorted_: torch.Tensor, til
 
 
 def moe_combine(y: torch.Tensor, weight: torch.Tensor, plus: Optional[torch.Tensor] = None,
-                plus_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                plus_gate: Optional[torch.Tensor] = None, choice: Optional[torch.Tensor] = None, n_tiled: int = 0,
+                x: Optional[torch.Tensor] = None) -> torch.Tensor:
     """fp32 ``[1, T, dim]``: ``plus[t] + sum_j weight[t, j] * y[t * top + j]``, the weighted sum first, ``j``
     ascending.  ``plus``: ``[T, dim]`` rows of any supported dtype, fp32 ``[S, T, dim]`` partial sums (a
     product whose k range was cut; summed in order), or None.  ``plus_gate``: fp32 ``[T]`` (any stride): the rows
-    of ``plus`` are multiplied by ``sigmoid(plus_gate[t])`` before they are added."""
-    _gpu(y, weight, plus, plus_gate)
+    of ``plus`` are multiplied by ``sigmoid(plus_gate[t])`` before they are added.  With ``choice [T, top]`` the output of
+    an expert from ``n_tiled`` on is the token's row of ``x [T, dim]``, whatever ``y`` holds there."""
+    _gpu(y, weight, plus, plus_gate, choice, x)
     if plus_gate is not None:
         _need(plus is not None and plus_gate.dtype == torch.float32 and plus_gate.dim() == 1
               and plus_gate.shape[0] == weight.shape[0] and plus_gate.stride(0) >= 1, "plus_gate must be float32 [T], with plus")
@@ -1188,10 +1297,16 @@ def moe_combine(y: torch.Tensor, weight: torch.Tensor, plus: Optional[torch.Tens
     elif plus is not None:
         _need(plus.shape == (T, dim) and plus.stride(1) == 1, "plus must be [T, dim]")
         ldp, n_plus = plus.stride(0), 1
+    if choice is not None:
+        _i32(choice, "choice", T * top)
+        _need(x is not None and x.dim() == 2 and x.shape == (T, dim) and x.stride(1) == 1, "x must be [T, dim] with unit column stride")
+        if plus is not None and plus.dtype == torch.bfloat16:
+            _need(x.dtype == torch.bfloat16, "bfloat16 rows are added to outputs of a bfloat16 x")
     out = torch.empty((1, T, dim), dtype=torch.float32, device=y.device)
-    st = _lib.load("moe").fg_moe_combine_gated(_ptr(y), _ptr(weight), _ptr(plus), ldp, _code(plus) if plus is not None else F32,
+    st = _lib.load("moe").fg_moe_combine_identity(_ptr(y), _ptr(weight), _ptr(plus), ldp, _code(plus) if plus is not None else F32,
                                                n_plus, ctypes.c_longlong(stride), T, top, dim, _ptr(out), _ptr(plus_gate),
-                                               plus_gate.stride(0) if plus_gate is not None else 0, _stream(y))
+                                               plus_gate.stride(0) if plus_gate is not None else 0, _ptr(choice), int(n_tiled), _ptr(x),
+                                               x.stride(0) if x is not None else 0, _code(x) if x is not None else F32, _stream(y))
     _check(st, "moe_combine")
     return out
 
@@ -1431,8 +1546,9 @@ def head_linear(x: torch.Tensor, x_head_stride: int, w: torch.Tensor, out: torch
 
 
 def head_norm_gate(x: torch.Tensor, weight: torch.Tensor, eps: float, gate: torch.Tensor, n_heads: int,
-                   out: torch.Tensor, out_scale: float = 1.0) -> torch.Tensor:
-    """``out[t, h, :] = rmsnorm(x[t, h, :]) * weight * silu(gate[t, h, :]) * out_scale`` for fp32 ``x [T, H*e]``, fp32
+                   out: torch.Tensor, out_scale: float = 1.0, sigmoid: bool = False) -> torch.Tensor:
+    """``out[t, h, :] = rmsnorm(x[t, h, :]) * weight * silu(gate[t, h, :]) * out_scale`` (``sigmoid``: the gate's sigmoid in
+    its silu's place) for fp32 ``x [T, H*e]``, fp32
     ``weight [e]`` shared by the heads, ``gate [T, >= H*e]`` (unit column stride) and ``out [T, H*e]`` of the
     activation dtype."""
     _gpu(x, weight, gate, out)
@@ -1444,9 +1560,26 @@ def head_norm_gate(x: torch.Tensor, weight: torch.Tensor, eps: float, gate: torc
     _need(gate.dim() == 2 and gate.stride(1) == 1 and gate.shape[0] == T and gate.shape[1] >= n_heads * e
           and gate.dtype in (out.dtype, torch.float32), "gate must be [T, >= H*e] of out's dtype or float32")
     st = _lib.load("heads").fg_head_norm_gate(_ptr(x), _ptr(weight), _ptr(gate), gate.stride(0), _ptr(out), out.stride(0),
-                                              T, n_heads, e, ctypes.c_float(eps), ctypes.c_float(out_scale), _code(out),
+                                              T, n_heads, e, ctypes.c_float(eps), ctypes.c_float(out_scale), int(bool(sigmoid)), _code(out),
                                               _code(gate), _stream(out))
     _check(st, "head_norm_gate")
+    return out
+
+
+def row_norm_gate(x: torch.Tensor, weight: torch.Tensor, eps: float, gate: torch.Tensor, out: torch.Tensor,
+                  out_scale: float = 1.0) -> torch.Tensor:
+    """``out[t, :W] = rmsnorm(x[t, :]) * weight * sigmoid(gate[t, :W]) * out_scale`` for fp32 ``x [T, W]``, fp32 ``weight [W]``
+    and fp32 ``gate [T, >= W]``; ``out [T, >= W]`` has the activation dtype."""
+    _gpu(x, weight, gate, out)
+    _need(x.dtype == torch.float32 and x.dim() == 2 and x.is_contiguous(), "x must be contiguous float32 [T, W]")
+    T, W = x.shape
+    _f32_vec(weight, W, "weight")
+    _rows_of_width(gate, T, W, "gate")
+    _rows_of_width(out, T, W, "out")
+    _need(gate.dtype == torch.float32 and W <= 16384, "gate must be float32, rows of at most 16384")
+    st = _lib.load("heads").fg_row_norm_gate(_ptr(x), _ptr(weight), _ptr(gate), gate.stride(0), _ptr(out), out.stride(0), T, W,
+                                             ctypes.c_float(eps), ctypes.c_float(out_scale), _code(out), _stream(out))
+    _check(st, "row_norm_gate")
     return out
 
 
@@ -1669,6 +1802,24 @@ def gated_mul(gate_up: torch.Tensor, bias: Optional[torch.Tensor], activation: s
                                             ctypes.c_float(limit), ctypes.c_float(alpha), _code(gate_up), _code(out),
                                             _stream(out))
     _check(st, "gated_mul")
+    return out
+
+
+_PLAIN_ACT_CODE = {"relu2": 0, "relu": 1, "silu": 2, "gelu_tanh": 3}
+
+
+def bias_act(x: torch.Tensor, bias: Optional[torch.Tensor], activation: str, out_dtype: torch.dtype) -> torch.Tensor:
+    """``act(x + bias)`` for contiguous ``x [T, hidden]`` (fp32, or ``out_dtype``; ``hidden`` a multiple of 8) and fp32 ``bias
+    [hidden]`` or None; ``activation`` one of ``relu2`` (the square of ReLU), ``relu``, ``silu``, ``gelu_tanh``."""
+    _gpu(x, bias)
+    _need(activation in _PLAIN_ACT_CODE, f"activation {activation!r} is not supported ({sorted(_PLAIN_ACT_CODE)})")
+    _need(x.dim() == 2 and x.is_contiguous() and x.shape[1] % 8 == 0, "x must be contiguous [T, hidden], hidden a multiple of 8")
+    _need(x.dtype == torch.float32 or x.dtype == out_dtype, "x must be float32 or of the result's dtype")
+    _f32_vec(bias, x.shape[1], "bias")
+    out = torch.empty(x.shape, dtype=out_dtype, device=x.device)
+    st = _lib.load("rows").fg_bias_act(_ptr(x), _ptr(bias), _ptr(out), x.shape[0], x.shape[1], _PLAIN_ACT_CODE[activation], _code(x),
+                                       _code(out), _stream(out))
+    _check(st, "bias_act")
     return out
 
 
@@ -2152,48 +2303,55 @@ class _DeltaPrepareArgs(ctypes.Structure):
 class _DeltaScanArgs(ctypes.Structure):
     _fields_ = [("rows", ctypes.c_void_p), ("stride", ctypes.c_int), ("n_qk", ctypes.c_int), ("d", ctypes.c_int),
                 ("n_v", ctypes.c_int), ("e", ctypes.c_int), ("state", ctypes.c_void_p), ("slot_stride", ctypes.c_longlong),
-                ("slot_ids", ctypes.c_void_p), ("q_start", ctypes.c_void_p), ("out", ctypes.c_void_p)]
+                ("slot_ids", ctypes.c_void_p), ("q_start", ctypes.c_void_p), ("out", ctypes.c_void_p), ("g_col", ctypes.c_int),
+                ("per_channel", ctypes.c_int)]
 
 
 class _DeltaChunks(ctypes.Structure):
     _fields_ = [("chunk_start", ctypes.c_void_p), ("seq_chunk", ctypes.c_void_p), ("T", ctypes.c_void_p), ("M", ctypes.c_void_p),
-                ("L", ctypes.c_void_p)]
+                ("L", ctypes.c_void_p), ("Qd", ctypes.c_void_p), ("Kd", ctypes.c_void_p), ("Ke", ctypes.c_void_p)]
 
 
 DELTA_CHUNKED_FROM = 64  # the shortest run of tokens of one sequence for which a step is taken chunk by chunk
 
 
 def delta_prepare(src: torch.Tensor, n_qk: int, head_dim: int, n_v: int, v_head_dim: int, conv: ConvInputs, b_col: int,
-                  a_col: int, decay_rate: torch.Tensor, dt_bias: torch.Tensor, q_scale: float, unit_eps: float,
+                  a_col: int, decay_rate: Optional[torch.Tensor], dt_bias: Optional[torch.Tensor], q_scale: float, unit_eps: float,
                   out: torch.Tensor) -> torch.Tensor:
     """What the gated delta rule takes of a token: ``out`` fp32 ``[T, q | k | v | beta | log g]`` from the rows ``src [T, q | k |
     v | ...]`` of a product (``n_qk`` query and key heads of ``head_dim``, ``n_v`` value heads of ``v_head_dim``).  q, k and v
     pass ``conv`` and SiLU; every q and k head becomes ``x / sqrt(sum(x^2) + unit_eps)``, q times ``q_scale``;
-    ``beta = sigmoid(src[b_col + h])``; ``log g = -decay_rate[h] softplus(src[a_col + h] + dt_bias[h])``."""
+    ``beta = sigmoid(src[b_col + h])``; ``log g = -decay_rate[h] softplus(src[a_col + h] + dt_bias[h])``.  With ``a_col < 0``
+    nothing is written behind ``beta``: the decays are made elsewhere."""
     _gpu(src, decay_rate, dt_bias, out)
+    decays = a_col >= 0
+    _need(not decays or (decay_rate is not None and dt_bias is not None), "decays need decay_rate and dt_bias")
     T, C = src.shape[0], 2 * n_qk * head_dim + n_v * v_head_dim
     _need(min(n_qk, n_v, head_dim, v_head_dim) > 0 and n_v % n_qk == 0 and head_dim % 2 == 0 and v_head_dim % 2 == 0
           and max(head_dim, v_head_dim) <= 1024, "heads must be even, at most 1024 wide, value heads a multiple of the others")
     conv.check(T, "delta_prepare")
     _need(conv.taps.shape[0] == C, "the convolution must have a channel for every column of q, k and v")
     _rows_of_width(src, T, max(C, b_col + n_v, a_col + n_v), "src")
-    _need(min(b_col, a_col) >= 0, "the scalars' columns must lie inside src")
+    _need(b_col >= 0, "the scalars' columns must lie inside src")
     _f32_vec(decay_rate, n_v, "decay_rate")
     _f32_vec(dt_bias, n_v, "dt_bias")
     _need(out.dtype == torch.float32 and out.dim() == 2 and out.stride(1) == 1 and out.shape[0] == T
-          and out.shape[1] >= C + 2 * n_v and out.stride(0) % 2 == 0 and out.data_ptr() % 8 == 0,
+          and out.shape[1] >= C + (2 if decays else 1) * n_v and out.stride(0) % 2 == 0 and out.data_ptr() % 8 == 0,
           "out must be float32 [T, >= q | k | v | beta | log g], rows 8-byte aligned")
     a = _DeltaPrepareArgs()
     a.src, a.src_stride, a.n_qk, a.d, a.n_v, a.e = src.data_ptr(), src.stride(0), n_qk, head_dim, n_v, v_head_dim
-    a.conv, a.b_col, a.a_col = conv.args(), b_col, a_col
-    a.decay_rate, a.dt_bias, a.q_scale, a.unit_eps = decay_rate.data_ptr(), dt_bias.data_ptr(), float(q_scale), float(unit_eps)
+    a.conv, a.b_col, a.a_col = conv.args(), b_col, a_col if decays else -1
+    if decays:
+        a.decay_rate, a.dt_bias = decay_rate.data_ptr(), dt_bias.data_ptr()
+    a.q_scale, a.unit_eps = float(q_scale), float(unit_eps)
     a.out, a.out_stride = out.data_ptr(), out.stride(0)
     _check(_lib.load("delta_rule").fg_delta_prepare(ctypes.byref(a), T, _code(src), _stream(src)), "delta_prepare")
     return out
 
 
 def delta_scan(rows: torch.Tensor, n_qk: int, head_dim: int, n_v: int, v_head_dim: int, state: torch.Tensor,
-               slot_ids: torch.Tensor, q_start: torch.Tensor, n_seqs: int, out: torch.Tensor, q_start_host=None) -> torch.Tensor:
+               slot_ids: torch.Tensor, q_start: torch.Tensor, n_seqs: int, out: torch.Tensor, q_start_host=None,
+               channel_decay_col: Optional[int] = None) -> torch.Tensor:
     """The gated delta rule for every sequence of the step, in fp32: per value head ``h`` (query/key head ``h // (n_v /
     n_qk)``) ``S <- g S``; ``u = beta (v - S^T k)``; ``S <- S + k u^T``; ``out[t, h] = S^T q``.
 
@@ -2201,13 +2359,19 @@ def delta_scan(rows: torch.Tensor, n_qk: int, head_dim: int, n_v: int, v_head_di
     their own) is read at ``slot_ids[b]`` and left as the sequence's last token leaves it; ``out`` fp32 ``[T, n_v *
     v_head_dim]``.
 
+    ``channel_decay_col``: the decays are per key channel (row ``c`` of ``S`` fades by ``g[c]``); ``n_v * head_dim`` logarithms
+    stand in ``rows`` from that column on, behind ``beta``.
+
     ``q_start_host``: ``q_start`` on the host.  With it, a step in which a sequence brings ``DELTA_CHUNKED_FROM`` tokens or
     more takes chunks of tokens at a time as matrix products (fp32) where the sizes allow; the result differs from the
     token-by-token scan's by rounding."""
     _gpu(rows, state, slot_ids, q_start, out)
     T, d, e = rows.shape[0], int(head_dim), int(v_head_dim)
     _need(rows.dtype == torch.float32, "rows must be float32")
-    _rows_of_width(rows, T, 2 * n_qk * d + n_v * (e + 2), "rows")
+    channel = channel_decay_col is not None
+    g_col = int(channel_decay_col) if channel else 2 * n_qk * d + n_v * (e + 1)
+    _need(g_col >= 2 * n_qk * d + n_v * (e + 1), "the decays stand behind beta")
+    _rows_of_width(rows, T, g_col + n_v * (d if channel else 1), "rows")
     _need(n_v % n_qk == 0 and d <= 512, "value heads a multiple of the others, at most 512 key channels")
     _need(state.dtype == torch.float32 and state.dim() == 4 and tuple(state.shape[1:]) == (n_v, d, e)
           and state.stride(3) == 1 and state.stride(2) == e and state.stride(1) == d * e, "state must be float32 [n_slots, n_v, d, e]")
@@ -2217,7 +2381,7 @@ def delta_scan(rows: torch.Tensor, n_qk: int, head_dim: int, n_v: int, v_head_di
     a = _DeltaScanArgs()
     a.rows, a.stride, a.n_qk, a.d, a.n_v, a.e = rows.data_ptr(), rows.stride(0), n_qk, d, n_v, e
     a.state, a.slot_stride, a.slot_ids, a.q_start = state.data_ptr(), state.stride(0), slot_ids.data_ptr(), q_start.data_ptr()
-    a.out = out.data_ptr()
+    a.out, a.g_col, a.per_channel = out.data_ptr(), g_col, int(channel)
     lib = _lib.load("delta_rule")
     lens = np.diff(np.asarray(q_start_host[: n_seqs + 1])) if q_start_host is not None else None
     if (lens is None or not len(lens) or int(lens.max()) < DELTA_CHUNKED_FROM or d % 16 or d > 256 or rows.stride(0) % 4
@@ -2231,7 +2395,121 @@ def delta_scan(rows: torch.Tensor, n_qk: int, head_dim: int, n_v: int, v_head_di
     ch = _DeltaChunks()
     ch.chunk_start, ch.seq_chunk = chunk_start.data_ptr(), seq_chunk.data_ptr()
     ch.T, ch.M, ch.L = flat.data_ptr(), flat[per:].data_ptr(), flat[2 * per :].data_ptr()
+    if channel:  # the chunks' rows with their decays multiplied in, and what is left of a state behind a chunk
+        folded = torch.empty((3, n_chunks, n_v, size, d), dtype=torch.float32, device=rows.device)
+        left = torch.empty((n_chunks, n_v, d), dtype=torch.float32, device=rows.device)
+        ch.Qd, ch.Kd, ch.Ke = (folded[i].data_ptr() for i in range(3))
+        ch.L = left.data_ptr()
     _check(lib.fg_delta_chunk_scan(ctypes.byref(a), ctypes.byref(ch), n_chunks, int(n_seqs), _stream(rows)), "delta_scan (chunks)")
+    return out
+
+
+# ------------------------------------------------ projections through a narrow middle
+@dataclass
+class LowRankJob:
+    """``out[t, n] = act(sum_k w[n, k] src[t, col + k] + bias[n])``: ``w [N, K]`` of the activation dtype, ``out`` fp32 ``[T, >=
+    N]``, ``bias`` fp32 ``[N]`` or None.  With ``rate`` (fp32 ``[ceil(N / per)]``) ``act(y) = -rate[n // per] softplus(y)``: the
+    logarithm of a decay; without, ``act(y) = y``."""
+
+    col: int
+    w: torch.Tensor
+    out: torch.Tensor
+    bias: Optional[torch.Tensor] = None
+    rate: Optional[torch.Tensor] = None
+    per: int = 1
+
+
+class _LowRankJob(ctypes.Structure):
+    _fields_ = [("col", ctypes.c_int), ("K", ctypes.c_int), ("w", ctypes.c_void_p), ("N", ctypes.c_int), ("out", ctypes.c_void_p),
+                ("out_stride", ctypes.c_int), ("bias", ctypes.c_void_p), ("kind", ctypes.c_int), ("rate", ctypes.c_void_p),
+                ("per", ctypes.c_int)]
+
+
+class _LowRankArgs(ctypes.Structure):
+    _fields_ = [("src", ctypes.c_void_p), ("src_stride", ctypes.c_int), ("job", _LowRankJob * 2), ("n_jobs", ctypes.c_int),
+                ("T", ctypes.c_int)]
+
+
+def low_rank(src: torch.Tensor, jobs: Sequence[LowRankJob]) -> None:
+    """The second halves of up to two projections through a narrow middle, whose first halves are columns of the fp32 rows
+    ``src [T, width]``, in one launch.  bfloat16 matrices with middles of multiples of 8 up to 256, aligned, meet the
+    middles rounded to bfloat16 on the matrix cores; everything else the fp32 kernel."""
+    _need(1 <= len(jobs) <= 2, "one or two products")
+    _need(src.dtype == torch.float32 and src.dim() == 2 and src.stride(1) == 1, "src must be float32 [T, width] with unit column stride")
+    T = src.shape[0]
+    a = _LowRankArgs()
+    a.src, a.src_stride, a.n_jobs, a.T = src.data_ptr(), src.stride(0), len(jobs), T
+    mfma = src.stride(0) % 8 == 0 and src.data_ptr() % 16 == 0
+    for c, j in zip(a.job, jobs):
+        _gpu(src, j.w, j.out, j.bias, j.rate)
+        _need(j.w.dim() == 2 and j.w.is_contiguous() and j.w.dtype == jobs[0].w.dtype, "w must be contiguous [N, K], of one dtype")
+        N, K = j.w.shape
+        _need(0 <= j.col and j.col + K <= src.shape[1] and K <= 4096, "the middle lies outside src, or is wider than 4096")
+        _rows_of_width(j.out, T, N, "out")
+        _need(j.out.dtype == torch.float32, "out must be float32")
+        _f32_vec(j.bias, N, "bias")
+        _need(j.per >= 1, "outputs share a rate in runs of at least one")
+        _f32_vec(j.rate, -(-N // j.per), "rate")
+        c.col, c.K, c.w, c.N, c.out, c.out_stride = j.col, K, j.w.data_ptr(), N, j.out.data_ptr(), j.out.stride(0)
+        c.bias, c.rate = (x.data_ptr() if x is not None else None for x in (j.bias, j.rate))
+        c.kind, c.per = int(j.rate is not None), int(j.per)
+        mfma = mfma and j.w.dtype == torch.bfloat16 and K % 8 == 0 and K <= 256 and j.col % 8 == 0 and j.w.data_ptr() % 16 == 0
+    _check(_lib.load("low_rank").fg_low_rank(ctypes.byref(a), _code(jobs[0].w), int(mfma), _stream(src)), "low_rank")
+
+
+# ------------------------------------------------ linear attention with a constant decay
+class _LightningArgs(ctypes.Structure):
+    _fields_ = [("rows", ctypes.c_void_p), ("stride", ctypes.c_int), ("q_col", ctypes.c_int), ("k_col", ctypes.c_int),
+                ("v_col", ctypes.c_int), ("H", ctypes.c_int), ("d", ctypes.c_int), ("e", ctypes.c_int), ("log_decay", ctypes.c_void_p),
+                ("state", ctypes.c_void_p), ("slot_stride", ctypes.c_longlong), ("slot_ids", ctypes.c_void_p),
+                ("q_start", ctypes.c_void_p), ("out", ctypes.c_void_p)]
+
+
+class _LightningChunks(ctypes.Structure):
+    _fields_ = [("chunk_start", ctypes.c_void_p), ("seq_chunk", ctypes.c_void_p), ("states", ctypes.c_void_p)]
+
+
+LIGHTNING_CHUNKED_FROM = 64  # the shortest run of tokens of one sequence for which a step is taken chunk by chunk
+
+
+def lightning_scan(rows: torch.Tensor, q_col: int, k_col: int, v_col: int, log_decay: torch.Tensor, state: torch.Tensor,
+                   slot_ids: torch.Tensor, q_start: torch.Tensor, n_seqs: int, out: torch.Tensor, q_start_host=None) -> torch.Tensor:
+    """Linear attention whose state fades by a constant per head, for every sequence of the step, in fp32:
+    ``S <- exp(log_decay[h]) S + k v^T``, ``out[t, h] = S^T q`` with ``q``, ``k``, ``v`` the silu of ``rows``' columns (``H`` heads
+    of ``d`` from ``q_col`` and ``k_col``, of ``e`` from ``v_col``).
+
+    ``rows`` fp32 ``[T, width]``; ``state`` fp32 ``[n_slots, H, d, e]`` (slots may have a stride of their own) is read at
+    ``slot_ids[b]`` and left as the sequence's last token leaves it; ``out`` fp32 ``[T, H * e]``.
+
+    ``q_start_host``: ``q_start`` on the host.  With it, a step in which a sequence brings ``LIGHTNING_CHUNKED_FROM`` tokens or
+    more takes chunks of tokens side by side as matrix products (fp32) where the sizes allow; the result differs from the
+    token-by-token scan's by rounding."""
+    _gpu(rows, log_decay, state, slot_ids, q_start, out)
+    _need(state.dtype == torch.float32 and state.dim() == 4, "state must be float32 [n_slots, H, d, e]")
+    T, (_, H, d, e) = rows.shape[0], state.shape
+    _need(state.stride(3) == 1 and state.stride(2) == e and state.stride(1) == d * e and d <= 512,
+          "a slot's state must be contiguous, with at most 512 key channels")
+    _need(rows.dtype == torch.float32 and min(q_col, k_col, v_col) >= 0, "rows must be float32")
+    _rows_of_width(rows, T, max(q_col + H * d, k_col + H * d, v_col + H * e), "rows")
+    _f32_vec(log_decay, H, "log_decay")
+    _need(out.dtype == torch.float32 and out.is_contiguous() and out.shape == (T, H * e), "out must be contiguous float32 [T, H * e]")
+    _i32(slot_ids, "slot_ids", n_seqs)
+    _i32(q_start, "q_start", n_seqs + 1)
+    a = _LightningArgs()
+    a.rows, a.stride, a.q_col, a.k_col, a.v_col = rows.data_ptr(), rows.stride(0), int(q_col), int(k_col), int(v_col)
+    a.H, a.d, a.e, a.log_decay, a.state, a.slot_stride = H, d, e, log_decay.data_ptr(), state.data_ptr(), state.stride(0)
+    a.slot_ids, a.q_start, a.out = slot_ids.data_ptr(), q_start.data_ptr(), out.data_ptr()
+    lib = _lib.load("lightning")
+    lens = np.diff(np.asarray(q_start_host[: n_seqs + 1])) if q_start_host is not None else None
+    if (lens is None or not len(lens) or int(lens.max()) < LIGHTNING_CHUNKED_FROM or d % 16 or d > 256 or rows.stride(0) % 4
+            or rows.data_ptr() % 16 or q_col % 4 or k_col % 4 or torch.cuda.is_current_stream_capturing()):
+        _check(lib.fg_lightning_scan(ctypes.byref(a), int(n_seqs), _stream(rows)), "lightning_scan")
+        return out
+    n_chunks, chunk_start, seq_chunk, _ = _chunk_plan(q_start_host, n_seqs, int(lib.fg_lightning_chunk_tokens()), rows.device)
+    states = torch.empty((n_chunks, H, d, e), dtype=torch.float32, device=rows.device)
+    ch = _LightningChunks()
+    ch.chunk_start, ch.seq_chunk, ch.states = chunk_start.data_ptr(), seq_chunk.data_ptr(), states.data_ptr()
+    _check(lib.fg_lightning_chunk_scan(ctypes.byref(a), ctypes.byref(ch), n_chunks, int(n_seqs), _stream(rows)), "lightning_scan (chunks)")
     return out
 
 

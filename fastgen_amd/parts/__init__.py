@@ -19,7 +19,7 @@ from .base import (
     unregister_part,
 )
 from . import (attention, block, delta_rule, differential_attention, embedding, feed_forward, injection,  # noqa: F401
-               latent_attention, linear_attention, linear_recurrence, mixed_attention, moe, norm, position, rows_mixer,
+               latent_attention, lightning, linear_attention, linear_recurrence, mixed_attention, moe, norm, position, rows_mixer,
                selective_scan, sigmoid_attention)  # register the built-in parts
 
 __all__ = [

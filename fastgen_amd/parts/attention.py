@@ -21,6 +21,9 @@ holds both padded with zeros to one width), ``has_kv`` = False (a layer that
 reads another layer's keys and values has only its queries), ``cache_window``
 (how long the cache keeps a key, where later layers read this layer's cache
 through longer windows than its own).
+
+In its general form (``prepared``: any of ``bias``, ``qk_norm``, ``conv_taps``, ``v_head_dim``, or the option itself) it is a
+:class:`~fastgen_amd.parts.rows_mixer.RowsMixer`, which can run beside another one on the same input.
 """
 
 from __future__ import annotations
@@ -31,10 +34,11 @@ import torch
 
 from ..kernels import ops
 from ..kernels.linear import StreamedMatrix, linear, skinny_ok, streamed
-from .base import LayerStore, Mixer, PagedNeed, StateNeed, TensorSpec, build_part, place, register_part, MATRIX, VECTOR
+from .base import LayerStore, PagedNeed, StateNeed, TensorSpec, build_part, place, register_part, MATRIX, VECTOR
+from .rows_mixer import RowsMixer
 
 
-class Attention(Mixer):
+class Attention(RowsMixer):
     folds_norms = True  # takes ScaledRows and the ``then`` request (see parts.block)
 
     def __init__(self, spec) -> None:
@@ -69,7 +73,7 @@ class Attention(Mixer):
         # width, a multiple of 16 (what the matrix-core kernels take)
         # the general form: what the product gives goes through a kernel of its own on its way to the attention
         self.prepared = (self.bias or self.qk_norm or not self.has_kv or self.v_head_dim != self.head_dim
-                         or self.conv_taps > 0)
+                         or self.conv_taps > 0 or bool(o.get("prepared", False)))
         self.cache_dim = -(-max(self.head_dim, self.v_head_dim) // 16) * 16 if self.prepared else self.head_dim
         if self.head_dim % (2 if self.prepared else 8) or self.head_dim > 512:
             raise ValueError(
@@ -85,6 +89,14 @@ class Attention(Mixer):
         if self.v_head_dim % 2 or self.cache_dim > 512:
             raise ValueError(f"{self.prefix}: value size {self.v_head_dim} is not supported (even, at most 512)")
         self.position = build_part("position", o["position"])
+        q_width, kv_width, v_width = (n * w for n, w in ((self.n_heads, self.head_dim), (self.n_kv_heads, self.head_dim),
+                                                         (self.n_kv_heads, self.v_head_dim)))
+        # columns of the product: q, k, v (or none: the values are the k columns), gate
+        self.k_col = q_width
+        self.v_col = q_width + kv_width if not self.value_from_key else q_width
+        self.gate_col = q_width + (0 if not self.has_kv else kv_width if self.value_from_key else kv_width + v_width)
+        self.out_width = self.n_heads * self.cache_dim
+        self.in_width = self.gate_col + (self.out_width if self.output_gate else 0)
         self.b_qkv = self.q_norm_w = self.k_norm_w = self.sinks = self.conv_w = self.distance = None
         self.wqkv: Optional[StreamedMatrix] = None
         self.wo: Optional[StreamedMatrix] = None
@@ -119,9 +131,13 @@ class Attention(Mixer):
         return specs + [TensorSpec(self._name("o_proj.weight"), (self.dim, self.n_heads * self.v_head_dim))]
 
     def load(self, tensors: Mapping[str, torch.Tensor], dtype: torch.dtype, device: Any) -> None:
+        self.wqkv = streamed(place(self.in_matrix(tensors), MATRIX, dtype, device))
+        self.wo = streamed(place(self.out_matrix(tensors), MATRIX, dtype, device))
+        self.load_rest(tensors, dtype, device)
+
+    def in_matrix(self, tensors: Mapping[str, torch.Tensor]) -> torch.Tensor:
         # one matrix for everything that reads the mixer's input: q, k, then v (if it has a projection
         # of its own), then the output gate
-        f32 = lambda name: tensors[self._name(name)].to(device=device, dtype=torch.float32).contiguous()
         mats = [self.position.arrange_rows(tensors[self._name("q_proj.weight")], self.n_heads)]
         if self.has_kv:
             mats.append(self.position.arrange_rows(tensors[self._name("k_proj.weight")], self.n_kv_heads))
@@ -129,18 +145,28 @@ class Attention(Mixer):
                 mats.append(tensors[self._name("v_proj.weight")])
         if self.output_gate:
             mats.append(self._padded_heads(tensors[self._name("gate_proj.weight")], 0))
-        self.wqkv = streamed(place(torch.cat(mats, dim=0), MATRIX, dtype, device))
+        return torch.cat(mats, dim=0)
+
+    def out_matrix(self, tensors: Mapping[str, torch.Tensor]) -> torch.Tensor:
         # the attention's output rows hold heads of the cache's width: zero columns meet the padding
-        self.wo = streamed(place(self._padded_heads(tensors[self._name("o_proj.weight")], 1), MATRIX, dtype, device))
+        return self._padded_heads(tensors[self._name("o_proj.weight")], 1)
+
+    def _arranged(self, v: torch.Tensor, n_heads: int) -> torch.Tensor:
+        """Numbers per row of a q or k projection (or per dimension of a head, one head) in the order of the rows as they
+        are stored for the rotation."""
+        return self.position.arrange_rows(v[:, None], n_heads)[:, 0].contiguous()
+
+    def load_rest(self, tensors: Mapping[str, torch.Tensor], dtype: torch.dtype, device: Any) -> None:
+        f32 = lambda name: tensors[self._name(name)].to(device=device, dtype=torch.float32).contiguous()
         self.freqs = self.position.frequencies_on(device)
         if self.bias:
-            names = ["q_proj.bias"] + (["k_proj.bias", "v_proj.bias"] if self.has_kv else [])
-            if self.position.rotary_dim and getattr(self.position, "pairing", "") == "half":
-                raise ValueError(f"{self.prefix}: biases with rows rearranged for the rotation are not supported")
-            self.b_qkv = torch.cat([f32(n) for n in names])
+            biases = [self._arranged(f32("q_proj.bias"), self.n_heads)]
+            if self.has_kv:
+                biases += [self._arranged(f32("k_proj.bias"), self.n_kv_heads), f32("v_proj.bias")]
+            self.b_qkv = torch.cat(biases)
         if self.qk_norm:
-            self.q_norm_w = f32("q_norm.weight")
-            self.k_norm_w = f32("k_norm.weight") if self.has_kv else None
+            self.q_norm_w = self._arranged(f32("q_norm.weight"), 1)
+            self.k_norm_w = self._arranged(f32("k_norm.weight"), 1) if self.has_kv else None
         if self.sink:
             self.sinks = torch.zeros(self.n_heads, device=device) if self.sink_is_one else f32("sinks")
         if self.conv_taps:
@@ -176,19 +202,8 @@ class Attention(Mixer):
         if self.prepared:
             return self._forward_prepared(x, ctx, store, then)
         group = ctx.groups[store.group]
-        q_width = self.n_heads * self.head_dim
-        kv_width = self.n_kv_heads * self.head_dim
-        # columns of the product: q, k, v (or none: the values are the k columns), gate
-        v_col = q_width if self.value_from_key else q_width + kv_width
-        gate_col = v_col + kv_width
-        table = None
-        if self.freqs is not None:
-            # sin and cos of the step's positions: computed by the first layer, shared by all layers
-            # that rotate with the same frequencies
-            key = ("rope_table", self.freqs.data_ptr())
-            table = ctx.scratch.get(key)
-            if table is None:
-                table = ctx.scratch[key] = ops.rope_table(ctx.positions, self.freqs)
+        q_width, v_col, gate_col = self.k_col, self.v_col, self.gate_col
+        table = self._rope_table(ctx)
         rows = x.rows if isinstance(x, ops.ScaledRows) else x
         fused = store.owns and self.head_dim % 16 == 0 and skinny_ok(rows, self.wqkv)
         if not fused and rows is not x:
@@ -221,6 +236,8 @@ class Attention(Mixer):
     def _rope_table(self, ctx: Any):
         if self.freqs is None:
             return None
+        # sin and cos of the step's positions: computed by the first layer, shared by all layers
+        # that rotate with the same frequencies
         key = ("rope_table", self.freqs.data_ptr())
         table = ctx.scratch.get(key)
         if table is None:
@@ -228,20 +245,24 @@ class Attention(Mixer):
         return table
 
     def _forward_prepared(self, x, ctx: Any, store: LayerStore, then=None):
-        """The general form: the product's fp32 rows go through ``heads_prepare`` (convolution, bias, the norms per
-        head, rotation, padding to the cache's head width, cache write), then attention and output
-        projection."""
+        """The general form: the product's fp32 rows, :meth:`mix`, output projection."""
         if isinstance(x, ops.ScaledRows):
             x = x.materialize()
+        rows = linear(x, self.wqkv, out_dtype=torch.float32)
+        out = torch.empty((x.shape[0], self.out_width), dtype=x.dtype, device=x.device)
+        self.mix(rows, ctx, store, out)
+        return linear(out, self.wo, partials_ok=True)
+
+    def mix(self, rows: torch.Tensor, ctx: Any, store: LayerStore, out: torch.Tensor, out_scale: float = 1.0) -> None:
+        """The rows go through ``heads_prepare`` (convolution, bias, the norms per head, rotation, padding to the cache's head
+        width, cache write), then attention, then the output gate."""
+        if not self.prepared or out_scale != 1.0:
+            raise ValueError(f"{self.prefix}: beside another mixer an attention is of the general form, and its result is not scaled")
         group = ctx.groups[store.group]
         d, hc = self.head_dim, self.cache_dim
-        q_width, kv_width = self.n_heads * d, self.n_kv_heads * d
-        rows = linear(x, self.wqkv, out_dtype=torch.float32)
-        q = torch.empty((x.shape[0], self.n_heads * hc), dtype=x.dtype, device=x.device)
+        q = torch.empty((out.shape[0], self.out_width), dtype=out.dtype, device=out.device)
         writes = store.owns and self.has_kv
-        v_col = -1 if self.value_from_key else q_width + kv_width  # (the value is the key as it is stored)
-        gate_col = q_width + (kv_width if self.has_kv else 0) + (
-            self.n_kv_heads * self.v_head_dim if self.has_kv and not self.value_from_key else 0)
+        v_col = -1 if self.value_from_key else self.v_col  # (the value is the key as it is stored)
         conv = None
         if self.conv_taps:
             moves = ctx.graph_capacity > 0 or ctx.max_q_len == 1
@@ -249,19 +270,18 @@ class Attention(Mixer):
         ops.heads_prepare(
             rows, self.b_qkv, self.qk_norm_eps, n_q=self.n_heads, q_col=0, q_width=d, q_norm=self.q_norm_w,
             q_norm_dims=d if self.qk_norm else 0, q_out=q, q_out_width=hc,
-            n_kv=self.n_kv_heads if writes else 0, k_col=q_width, k_width=d, k_norm=self.k_norm_w,
+            n_kv=self.n_kv_heads if writes else 0, k_col=self.k_col, k_width=d, k_norm=self.k_norm_w,
             k_norm_dims=d if self.qk_norm else 0, v_col=v_col, v_width=self.v_head_dim,
             table=self._rope_table(ctx), rot_start=0, rotary_dim=self.position.rotary_dim,
             slots=group.slots if writes else None, k_pages=store.k_pages if writes else None,
             v_pages=store.v_pages if writes else None, conv=conv)
         if conv is not None and not conv.moves:
             ops.conv_tail(rows, conv, ctx.n_seqs)
-        out = torch.empty_like(q)
+        out = out[:, : self.out_width]
         ops.paged_attention(q, out, store.k_pages, store.v_pages, group, ctx, self.n_heads, self.scale,
                             self.window or 0, exact_weights=self.exact_weights, sinks=self.sinks, distance=self.distance)
         if self.output_gate:
-            ops.gate_mul(out, rows[:, gate_col:])
-        return linear(out, self.wo, partials_ok=True)
+            ops.gate_mul(out, rows[:, self.gate_col :])
 
 
 register_part("mixer", "attention", Attention)

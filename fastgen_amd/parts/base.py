@@ -169,6 +169,7 @@ class Injection(Part):
     of the entry's ``inject`` (which pass of a loop this is)."""
 
     needs_embedding = False
+    takes_terms = False  # whether ``pending`` may be ``ops.StreamTerms``
 
     def forward(self, h: torch.Tensor, pending: Optional[torch.Tensor], embedded: Optional[torch.Tensor],
                 index: int) -> None:

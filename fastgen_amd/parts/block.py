@@ -12,10 +12,13 @@ from ..kernels.ops import ScaledRows
 from .base import VECTOR, FeedForward, LayerStore, Mixer, Norm, Part, TensorSpec, register_part
 
 
-def _no_output_bias(ffn, arrangement: str) -> None:
-    """Only an arrangement that norms a feed-forward's output adds a bias of its last projection."""
-    if ffn is not None and getattr(ffn, "bias", False):
+def _plain_outputs(mixer, ffn, arrangement: str, bias_ok: bool = False) -> None:
+    """Only an arrangement that norms a feed-forward's output, or adds its sublayers' outputs as terms, adds a bias of the
+    last projection; only the latter takes a mixer whose output is a sum of normed rows (``returns_terms``)."""
+    if not bias_ok and ffn is not None and getattr(ffn, "bias", False):
         raise ValueError(f"a {arrangement} layer does not take a feed-forward with biases")
+    if getattr(mixer, "returns_terms", False):
+        raise ValueError(f"a {arrangement} layer does not take a mixer whose output is a sum of normed rows")
 
 
 class PreNormBlock:
@@ -37,7 +40,7 @@ class PreNormBlock:
 
     def __init__(self, mixer: Mixer, ffn: FeedForward, mixer_norm: Norm, ffn_norm: Norm) -> None:
         self.mixer, self.ffn, self.mixer_norm, self.ffn_norm = mixer, ffn, mixer_norm, ffn_norm
-        _no_output_bias(ffn, "pre-norm")
+        _plain_outputs(mixer, ffn, "pre-norm")
 
     @staticmethod
     def _run(part, x, then, *args):
@@ -75,7 +78,7 @@ class ScaledPreNormBlock(Part):
         if ffn is not None and ffn_norm is None:
             raise ValueError("a feed-forward needs its norm")
         self.mixer, self.ffn, self.mixer_norm, self.ffn_norm = mixer, ffn, mixer_norm, ffn_norm
-        _no_output_bias(ffn, "pre-norm")
+        _plain_outputs(mixer, ffn, "pre-norm")
         self.scales: dict = {}
 
     def _sublayers(self):
@@ -117,7 +120,7 @@ class ParallelBlock:
         if ffn_norm is not None:
             raise ValueError("a parallel layer has one norm: its feed-forward reads the mixer's")
         self.mixer, self.ffn, self.mixer_norm = mixer, ffn, mixer_norm
-        _no_output_bias(ffn, "parallel")
+        _plain_outputs(mixer, ffn, "parallel")
 
     def forward(self, h: torch.Tensor, pending, ctx: Any, store: LayerStore):
         x = self.mixer_norm.forward(h, pending, ctx.act_dtype)
@@ -153,7 +156,7 @@ class SandwichBlock:
             raise ValueError("a sandwich layer needs the norms post_mixer and, with a feed-forward, ffn_norm and post_ffn")
         self.mixer, self.ffn, self.mixer_norm, self.ffn_norm = mixer, ffn, mixer_norm, ffn_norm
         self.post_mixer, self.post_ffn = extra["post_mixer"], extra.get("post_ffn")
-        _no_output_bias(ffn, "sandwich")
+        _plain_outputs(mixer, ffn, "sandwich")
 
     @staticmethod
     def _behind(rows, norm) -> ops.PostNormed:
@@ -184,6 +187,7 @@ class NormBehindBlock:
     def __init__(self, mixer: Mixer, ffn: Optional[FeedForward], mixer_norm: Norm, ffn_norm: Optional[Norm]) -> None:
         if ffn is not None and ffn_norm is None:
             raise ValueError("a feed-forward whose output is normed needs its norm")
+        _plain_outputs(mixer, ffn, "norm-behind", bias_ok=True)
         self.mixer, self.ffn, self.mixer_norm, self.ffn_norm = mixer, ffn, mixer_norm, ffn_norm
 
     @staticmethod
@@ -235,7 +239,7 @@ class HyperConnectionBlock(Part):
         if ffn is not None and ffn_norm is None:
             raise ValueError("a feed-forward needs its norm")
         self.mixer, self.ffn, self.mixer_norm, self.ffn_norm = mixer, ffn, mixer_norm, ffn_norm
-        _no_output_bias(ffn, "hyper-connection")
+        _plain_outputs(mixer, ffn, "hyper-connection")
         self.weights: dict = {}
 
     def _sublayers(self):
@@ -274,3 +278,52 @@ class HyperConnectionBlock(Part):
 
 
 register_part("arrangement", "hyper_connections", HyperConnectionBlock)
+
+
+class ParallelScaledBlock(Part):
+    """``h += mult * (ls1 (.) mixer(n1(h)) + ls2 (.) ffn(n2(h)))``: both sublayers read the same stream, each through a norm
+    of its own, and their outputs, multiplied per channel by a learned vector (``ls1 [dim]``, ``ls2 [dim]``) and by a
+    constant, are added at once.  The outputs go on as :class:`~fastgen_amd.kernels.ops.StreamTerms`; one kernel adds them
+    (with a bias of the feed-forward's last projection, and the norms of a mixer whose output is a sum of normed rows)
+    and makes both norms of the layer that follows, which share one root mean square.  A layer without a feed-forward adds
+    its mixer's output alone.  Options: ``dim``, ``mult``, ``scaled`` (False: there are no vectors); the spec's prefix is the
+    layer's."""
+
+    folds_norms = False
+
+    def __init__(self, spec, mixer: Mixer, ffn: Optional[FeedForward], mixer_norm: Norm, ffn_norm: Optional[Norm]) -> None:
+        super().__init__(spec)
+        self.dim = int(spec.options["dim"])
+        self.mult = float(spec.options.get("mult", 1.0))
+        self.scaled = bool(spec.options.get("scaled", True))
+        if ffn is not None and (ffn_norm is None or ffn_norm.eps != mixer_norm.eps):
+            raise ValueError("a feed-forward needs its norm, with the eps of the mixer's")
+        self.mixer, self.ffn, self.mixer_norm, self.ffn_norm = mixer, ffn, mixer_norm, ffn_norm
+        self.scales: dict = {}
+
+    def _sublayers(self):
+        return ("ls1", "ls2") if self.ffn is not None else ("ls1",)
+
+    def tensor_specs(self):
+        return [TensorSpec(self._name(n), (self.dim,), VECTOR, ("one_plus_normal", 0.1)) for n in self._sublayers()] if self.scaled else []
+
+    def load(self, tensors, dtype, device) -> None:
+        for n in self._sublayers():
+            ls = tensors[self._name(n)].to(device=device, dtype=torch.float32) if self.scaled else torch.ones(self.dim, device=device)
+            self.scales[n] = (self.mult * ls).contiguous()
+        if getattr(self.mixer, "returns_terms", False):
+            self.mixer.fold_scale(self.scales["ls1"])
+
+    def forward(self, h: torch.Tensor, pending, ctx: Any, store: LayerStore):
+        norms = [n for n in (self.mixer_norm, self.ffn_norm) if n is not None]
+        outs = [torch.empty(h.shape, dtype=ctx.act_dtype, device=h.device) for _ in norms]
+        ops.stream_terms(h, ops.StreamTerms.of(pending), None, [(n.weight, o) for n, o in zip(norms, outs)], self.mixer_norm.eps)
+        mixed = self.mixer.forward(outs[0], ctx, store)
+        terms = mixed.terms if isinstance(mixed, ops.StreamTerms) else [ops.StreamTerm(mixed, self.scales["ls1"])]
+        if self.ffn is not None:
+            fed = self.ffn.forward(outs[1])
+            terms = terms + [ops.StreamTerm(fed, self.scales["ls2"], getattr(self.ffn, "output_bias", None))]
+        return ops.StreamTerms(terms)
+
+
+register_part("arrangement", "parallel_scaled", ParallelScaledBlock)

@@ -9,7 +9,10 @@ product is stored.  The option ``activation`` puts the tanh form of GELU
 every projection has a bias: the gate's and the up projection's are added in
 fp32 where the activation is applied to the product's fp32 result; the down
 projection's (``output_bias``) is left to the kernel that adds the result to the
-residual stream."""
+residual stream.
+
+Without a gate (``mlp``): ``down(act(up(x)))`` with the square of ReLU (``"relu2"``), ReLU, SiLU or the tanh form of
+GELU, biases as above."""
 
 from __future__ import annotations
 
@@ -91,3 +94,46 @@ class SwiGLU(FeedForward):
 
 
 register_part("feed_forward", "swiglu", SwiGLU)
+
+
+class MLP(FeedForward):
+    """``down(act(up(x) + b)) + b'`` (see the module).  Options: ``dim``, ``hidden_dim``, ``activation``, ``bias``."""
+
+    def __init__(self, spec) -> None:
+        super().__init__(spec)
+        o = spec.options
+        self.dim, self.hidden_dim = int(o["dim"]), int(o["hidden_dim"])
+        self.activation = o.get("activation", "relu2")
+        if self.activation not in ("relu2", "relu", "silu", "gelu_tanh"):
+            raise ValueError(f"{self.prefix}: activation {self.activation!r} is not supported ('relu2', 'relu', 'silu', 'gelu_tanh')")
+        self.bias = bool(o.get("bias", False))
+        self.up_bias: Optional[torch.Tensor] = None
+        self.output_bias: Optional[torch.Tensor] = None
+        self.w_up: Optional[StreamedMatrix] = None
+        self.w_down: Optional[StreamedMatrix] = None
+
+    def tensor_specs(self) -> List[TensorSpec]:
+        specs = [TensorSpec(self._name("up_proj.weight"), (self.hidden_dim, self.dim)),
+                 TensorSpec(self._name("down_proj.weight"), (self.dim, self.hidden_dim))]
+        if self.bias:
+            specs += [TensorSpec(self._name("up_proj.bias"), (self.hidden_dim,), VECTOR, ("normal", 0.1)),
+                      TensorSpec(self._name("down_proj.bias"), (self.dim,), VECTOR, ("normal", 0.1))]
+        return specs
+
+    def load(self, tensors: Mapping[str, torch.Tensor], dtype: torch.dtype, device: Any) -> None:
+        up, down = tensors[self._name("up_proj.weight")], tensors[self._name("down_proj.weight")]
+        pad = -self.hidden_dim % 8
+        if pad:  # the kernels work on groups of 8 channels: what is added meets zero columns of the down projection
+            up, down = torch.cat([up, up.new_zeros(pad, self.dim)]), torch.cat([down, down.new_zeros(self.dim, pad)], dim=1)
+        self.w_up, self.w_down = streamed(place(up, MATRIX, dtype, device)), streamed(place(down, MATRIX, dtype, device))
+        if self.bias:
+            b = tensors[self._name("up_proj.bias")].to(torch.float32)
+            self.up_bias = torch.cat([b, b.new_zeros(pad)]).to(device=device).contiguous()
+            self.output_bias = tensors[self._name("down_proj.bias")].to(device=device, dtype=torch.float32).contiguous()
+
+    def forward(self, x):
+        act = ops.bias_act(linear(x, self.w_up, out_dtype=torch.float32), self.up_bias, self.activation, x.dtype)
+        return linear(act, self.w_down, partials_ok=True)
+
+
+register_part("feed_forward", "mlp", MLP)

@@ -20,7 +20,10 @@ expert is ``W_down (g * sigmoid(alpha g) * (u + 1))`` of ``g = min(W_gate x, lim
 ``u = clamp(W_up x, -limit, limit)``; ``shared_activation`` / ``shared_limit`` say the same
 of the shared expert.  ``shared_gate``: the shared expert's output is multiplied by
 ``sigmoid(w . x)`` for one more row ``w`` (``shared_gate.weight [1, dim]``), whose logit the
-router's kernel computes in fp32 beside the experts'.
+router's kernel computes in fp32 beside the experts'.  ``group_rank`` = ``"max"``: a group ranks by its largest choice
+score, not by the sum of its two largest.  ``renormalize`` = False: the chosen experts' scores are the weights as they
+are.  ``identity``: that many more experts, behind the others in the router's matrix, whose output is their input; they
+have no tensors, take part in scores, groups and choice like the others, and cost the combine a row.
 """
 
 from __future__ import annotations
@@ -44,8 +47,13 @@ class MoE(FeedForward):
         self.hidden_dim = int(o["hidden_dim"])
         self.n_experts = int(o["n_experts"])
         self.top = int(o["top"])
-        if not 1 <= self.top <= self.n_experts:
-            raise ValueError(f"{self.prefix}: top={self.top} must be between 1 and n_experts={self.n_experts}")
+        self.identity = int(o.get("identity", 0))
+        self.n_scored = self.n_experts + self.identity  # the router's outputs
+        if self.n_experts < 1 or self.identity < 0 or not 1 <= self.top <= self.n_scored:
+            raise ValueError(f"{self.prefix}: top={self.top} must be between 1 and the {self.n_scored} experts")
+        self.group_rank, self.renormalize = o.get("group_rank", "top2"), bool(o.get("renormalize", True))
+        if self.group_rank not in ("top2", "max"):
+            raise ValueError(f"{self.prefix}: group_rank {self.group_rank!r} is not supported ('top2', 'max')")
         self.router_bias = bool(o.get("router_bias", True))
         self.scoring = o.get("scoring", "softmax")
         if self.scoring not in ("softmax", "sigmoid", "softmax_all"):
@@ -58,12 +66,13 @@ class MoE(FeedForward):
         self.has_correction = bool(o.get("correction", False))
         self.n_groups, self.keep_groups = int(o.get("n_groups", 1)), int(o.get("keep_groups", o.get("n_groups", 1)))
         self.weight_scale = float(o.get("weight_scale", 1.0))
-        if self.scoring == "softmax" and (self.has_correction or self.n_groups != 1 or self.weight_scale != 1.0):
-            raise ValueError(f"{self.prefix}: correction, groups and weight_scale go with sigmoid or softmax_all scoring")
-        if (self.n_groups < 1 or self.n_experts % self.n_groups or not 1 <= self.keep_groups <= self.n_groups
-                or self.top > self.keep_groups * (self.n_experts // self.n_groups)):
+        if self.scoring == "softmax" and (self.has_correction or self.n_groups != 1 or self.weight_scale != 1.0
+                                          or not self.renormalize):
+            raise ValueError(f"{self.prefix}: correction, groups, weight_scale and raw weights go with sigmoid or softmax_all scoring")
+        if (self.n_groups < 1 or self.n_scored % self.n_groups or not 1 <= self.keep_groups <= self.n_groups
+                or self.top > self.keep_groups * (self.n_scored // self.n_groups)):
             raise ValueError(f"{self.prefix}: {self.n_groups} groups of which {self.keep_groups} stay do not fit"
-                             f" {self.n_experts} experts and top={self.top}")
+                             f" {self.n_scored} experts and top={self.top}")
         self.correction: Optional[torch.Tensor] = None
         self.shared: Optional[FeedForward] = None
         self.shared_gate = bool(o.get("shared_gate", False))
@@ -86,11 +95,11 @@ class MoE(FeedForward):
         return self._name(f"{names.get('expert', 'experts.{}').format(e)}.{names.get(which, which)}")
 
     def tensor_specs(self) -> List[TensorSpec]:
-        specs = [TensorSpec(self._name("router.weight"), (self.n_experts, self.dim), MATRIX, ("normal", 0.3))]
+        specs = [TensorSpec(self._name("router.weight"), (self.n_scored, self.dim), MATRIX, ("normal", 0.3))]
         if self.router_bias:
-            specs.append(TensorSpec(self._name("router.bias"), (self.n_experts,), VECTOR, ("normal", 0.3)))
+            specs.append(TensorSpec(self._name("router.bias"), (self.n_scored,), VECTOR, ("normal", 0.3)))
         if self.has_correction:
-            specs.append(TensorSpec(self._name("correction"), (self.n_experts,), VECTOR, ("normal", 0.1)))
+            specs.append(TensorSpec(self._name("correction"), (self.n_scored,), VECTOR, ("normal", 0.1)))
         if self.shared is not None:
             specs += self.shared.tensor_specs()
         if self.shared_gate:
@@ -134,7 +143,7 @@ class MoE(FeedForward):
         matrix-core kernels only)."""
         if self.w_gate.dtype != torch.bfloat16 or self.dim % 8:
             return 16
-        per_expert = n_rows * self.top / self.n_experts
+        per_expert = n_rows * self.top / self.n_scored
         lds_ok = min(self.dim, self.w_down.shape[2]) >= 32  # the tiles through LDS load k in steps of 32
         # a tile is computed whole whatever it holds, and every expert's last tile is half empty on average:
         # the largest tiles only where an expert has several of them
@@ -154,12 +163,14 @@ class MoE(FeedForward):
             plus = both if plus is None else torch.cat([t if t.dim() == 3 else t.float()[None] for t in (plus, both)])
         routed = ops.moe_route(x, self.router, self.bias, self.top, self.scoring == "sigmoid", self.correction,
                                self.n_groups, self.keep_groups, self.weight_scale,
-                               softmax_scores=self.scoring == "softmax_all", n_extra=int(self.shared_gate))
+                               softmax_scores=self.scoring == "softmax_all", n_extra=int(self.shared_gate),
+                               group_max=self.group_rank == "max", raw_weights=not self.renormalize)
         choice, weight = routed[0], routed[1]
-        sorted_, tiles = ops.moe_sort(choice, self.n_experts, tile_rows)
+        sorted_, tiles = ops.moe_sort(choice, self.n_scored, tile_rows, self.identity)
         act = ops.moe_gate_up(x, self.w_gate, self.w_up, sorted_, tiles, self.top, tile_rows, self.limit, self.alpha)
         y = ops.moe_down(act, self.w_down, sorted_, tiles, tile_rows)
-        return ops.moe_combine(y, weight, plus, routed[2][:, 0] if self.shared_gate else None)
+        own = dict(choice=choice, n_tiled=self.n_experts, x=x) if self.identity else {}
+        return ops.moe_combine(y, weight, plus, routed[2][:, 0] if self.shared_gate else None, **own)
 
 
 register_part("feed_forward", "moe", MoE)

@@ -38,7 +38,8 @@ class RMSNorm(Norm):
     def forward(self, h, delta, dtype, rows=None):
         """``delta`` may be :class:`~fastgen_amd.kernels.ops.PostNormed`: a sublayer's output that is normed
         itself before it is added (the norm behind a sublayer); one kernel does that norm, the addition and
-        this norm.  :class:`~fastgen_amd.kernels.ops.ScaledDelta`: rows times a vector.  ``h`` may be several residual streams ``[S, T, dim]`` (``delta``: the
+        this norm.  :class:`~fastgen_amd.kernels.ops.ScaledDelta`: rows times a vector;
+        :class:`~fastgen_amd.kernels.ops.StreamTerms`: several sublayers' outputs.  ``h`` may be several residual streams ``[S, T, dim]`` (``delta``: the
         :class:`~fastgen_amd.kernels.ops.StreamUpdate` still to be applied, or None): their sum is normed."""
         n = h.shape[-2] if rows is None else rows.numel()
         out = torch.empty((n, self.dim), dtype=dtype, device=h.device)
@@ -47,6 +48,9 @@ class RMSNorm(Norm):
         if isinstance(delta, ops.PostNormed):
             return ops.post_add_rmsnorm(h, delta.rows, delta.weight, delta.eps, self.weight, self.eps, out, rows,
                                         delta_bias=delta.bias)
+        if isinstance(delta, ops.StreamTerms):
+            ops.stream_terms(h, delta, None, [(self.weight, out)], self.eps, rows)
+            return out
         if isinstance(delta, ops.ScaledDelta):
             return ops.add_rmsnorm(h, delta.rows, self.weight, self.eps, out, rows, delta_scale=delta.scale)
         return ops.add_rmsnorm(h, delta, self.weight, self.eps, out, rows)

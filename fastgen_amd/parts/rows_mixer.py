@@ -5,8 +5,12 @@ what happens between (:meth:`RowsMixer.mix`).  Alone it is a mixer like the othe
 them on one input as one product in (both matrices stacked) and one product out (their results side by side, the two
 constant factors applied where each result is rounded): ``left_scale * left(x) + right_scale * right(x)``.
 
+With ``out_norms`` the two results have an output product each, and the mixer's output is ``left_scale * n(left(x)) (.) w_l +
+right_scale * n(right(x)) (.) w_r`` with ``n`` the division by the root mean square over the model's width (``eps``): it is
+returned as terms (:class:`~fastgen_amd.kernels.ops.StreamTerms`), which the kernel that adds them to the stream norms.
+
 ``ParallelMixers`` options: ``dim``, ``left``, ``right`` (:class:`~fastgen_amd.config.PartSpec` of mixers of this form, with
-tensor names of their own), ``left_scale``, ``right_scale``.  At most one of the two keeps pages, at most one a state.
+tensor names of their own), ``left_scale``, ``right_scale``, ``out_norms``, ``eps``.  At most one of the two keeps pages, at most one a state.
 """
 
 from __future__ import annotations
@@ -15,8 +19,9 @@ from typing import Any, List, Mapping, Optional
 
 import torch
 
+from ..kernels import ops
 from ..kernels.linear import StreamedMatrix, linear, streamed
-from .base import MATRIX, LayerStore, Mixer, PagedNeed, StateNeed, TensorSpec, build_part, place, register_part
+from .base import MATRIX, VECTOR, LayerStore, Mixer, PagedNeed, StateNeed, TensorSpec, build_part, place, register_part
 
 
 def _padded(n: int) -> int:
@@ -92,19 +97,36 @@ class ParallelMixers(Mixer):
         self.capturable = all(s.capturable for s in self.sides)
         self.w_in: Optional[StreamedMatrix] = None
         self.wo: Optional[StreamedMatrix] = None
+        self.returns_terms = bool(o.get("out_norms", False))
+        self.eps = float(o.get("eps", 0.0))
+        self.right_col = _padded(self.left.in_width)  # (the right side's columns begin where its kernels can read them as vectors)
+        self.wo_right: Optional[StreamedMatrix] = None
+        self.out_scales: List[torch.Tensor] = []
 
     @property
     def sides(self):
         return (self.left, self.right)
 
     def tensor_specs(self) -> List[TensorSpec]:
-        return self.left.tensor_specs() + self.right.tensor_specs()
+        norms = [TensorSpec(self._name(f"{n}_norm.weight"), (self.dim,), VECTOR, ("one_plus_normal", 0.1)) for n in ("left", "right")]
+        return self.left.tensor_specs() + self.right.tensor_specs() + (norms if self.returns_terms else [])
 
     def load(self, tensors: Mapping[str, torch.Tensor], dtype: torch.dtype, device: Any) -> None:
-        self.w_in = load_in(torch.cat([s.in_matrix(tensors) for s in self.sides]), dtype, device)
-        self.wo = load_out(torch.cat([s.out_matrix(tensors) for s in self.sides], dim=1), dtype, device)
+        mats = [s.in_matrix(tensors) for s in self.sides]
+        gap = mats[0].new_zeros(self.right_col - self.left.in_width, self.dim)
+        self.w_in = load_in(torch.cat([mats[0], gap, mats[1]]), dtype, device)
         for s in self.sides:
             s.load_rest(tensors, dtype, device)
+        if not self.returns_terms:
+            self.wo = load_out(torch.cat([s.out_matrix(tensors) for s in self.sides], dim=1), dtype, device)
+            return
+        self.wo, self.wo_right = (load_out(s.out_matrix(tensors), dtype, device) for s in self.sides)
+        self.out_scales = [(c * tensors[self._name(f"{n}_norm.weight")].to(device=device, dtype=torch.float32)).contiguous()
+                           for n, c in zip(("left", "right"), self.scales)]
+
+    def fold_scale(self, scale: torch.Tensor) -> None:
+        """A vector that multiplies this mixer's terms is folded into their own (once, behind ``load``)."""
+        self.out_scales = [(s * scale).contiguous() for s in self.out_scales]
 
     def paged_need(self) -> Optional[PagedNeed]:
         return self.left.paged_need() or self.right.paged_need()
@@ -114,9 +136,17 @@ class ParallelMixers(Mixer):
 
     def forward(self, x: torch.Tensor, ctx: Any, store: LayerStore) -> torch.Tensor:
         rows = linear(x, self.w_in, out_dtype=torch.float32)
+        if self.returns_terms:
+            terms = []
+            for s, own, w, scale in ((self.left, rows[:, : self.left.in_width], self.wo, self.out_scales[0]),
+                                     (self.right, rows[:, self.right_col :], self.wo_right, self.out_scales[1])):
+                out = result_rows(x.shape[0], s.out_width, x.dtype, x.device)
+                s.mix(own, ctx, store, out)
+                terms.append(ops.StreamTerm(linear(out, w, partials_ok=True), scale, None, self.eps))
+            return ops.StreamTerms(terms)
         out = result_rows(x.shape[0], self.left.out_width + self.right.out_width, x.dtype, x.device)
-        self.left.mix(rows, ctx, store, out, self.scales[0])
-        self.right.mix(rows[:, self.left.in_width :], ctx, store, out[:, self.left.out_width :], self.scales[1])
+        self.left.mix(rows[:, : self.left.in_width], ctx, store, out, self.scales[0])
+        self.right.mix(rows[:, self.right_col :], ctx, store, out[:, self.left.out_width :], self.scales[1])
         return linear(out, self.wo, partials_ok=True)
 
 
