@@ -385,13 +385,15 @@ def gemm_skinny_qkv(x, wqkv, table: Optional[torch.Tensor], slots: torch.Tensor,
 # ------------------------------------------------------------- routed experts
 def moe_route(x: torch.Tensor, router: torch.Tensor, bias: Optional[torch.Tensor], top: int,
               sigmoid_scores: bool = False, correction: Optional[torch.Tensor] = None, n_groups: int = 1,
-              keep_groups: int = 1, weight_scale: float = 1.0, softmax_scores: bool = False, n_extra: int = 0):
+              keep_groups: int = 1, weight_scale: float = 1.0, softmax_scores: bool = False, n_extra: int = 0,
+              group_max: bool = False, raw_weights: bool = False):
     """The ``top`` experts with the largest fp32 logits ``x router^T + bias`` (largest first; of equal
     logits the lower expert) and the softmax over those logits alone.  With ``sigmoid_scores``: scores
     ``sigmoid(logit)``; chosen by score plus ``correction`` inside the ``keep_groups`` groups (of ``n_groups``) whose two
     largest choice scores sum highest; weights: the chosen scores over their sum (+ 1e-20), times ``weight_scale``.
     ``softmax_scores``: the same with scores ``softmax(logits)`` over all experts.  The last ``n_extra`` rows of
-    ``router`` are no experts: their logits come back as a third result."""
+    ``router`` are no experts: their logits come back as a third result.  ``group_max``: a group ranks by its largest choice
+    score; ``raw_weights``: the weights are the chosen scores as they are (times ``weight_scale``)."""
     z = x.float() @ router.T
     E = router.shape[0] - n_extra
     z, extra = z[:, :E] + (bias if bias is not None else 0.0), z[:, E:]
@@ -404,29 +406,29 @@ def moe_route(x: torch.Tensor, router: torch.Tensor, bias: Optional[torch.Tensor
     T, E = choice.shape
     if n_groups > 1 and keep_groups < n_groups:
         per = E // n_groups
-        rank = torch.sort(choice.view(T, n_groups, per), dim=-1, descending=True).values[..., : min(2, per)].sum(-1)
+        rank = torch.sort(choice.view(T, n_groups, per), dim=-1, descending=True).values[..., : min(1 if group_max else 2, per)].sum(-1)
         order = torch.sort(rank, dim=-1, descending=True, stable=True).indices
         lost = torch.zeros(T, n_groups, dtype=torch.bool, device=x.device).scatter_(1, order[:, keep_groups:], True)
         choice = choice.masked_fill(lost[:, :, None].expand(T, n_groups, per).reshape(T, E), float("-inf"))
     idx = torch.sort(choice, dim=-1, descending=True, stable=True).indices[:, :top]
     w = score.gather(1, idx)
-    return (idx.to(torch.int32), w / (w.sum(-1, keepdim=True) + 1e-20) * weight_scale, *more)
+    return (idx.to(torch.int32), (w if raw_weights else w / (w.sum(-1, keepdim=True) + 1e-20)) * weight_scale, *more)
 
 
 def moe_max_tiles(n_pairs: int, n_experts: int, tile_rows: int) -> int:
     return min(n_pairs, n_pairs // tile_rows + n_experts)
 
 
-def moe_sort(choice: torch.Tensor, n_experts: int, tile_rows: int):
+def moe_sort(choice: torch.Tensor, n_experts: int, tile_rows: int, n_identity: int = 0):
     """The pairs (row, choice) in the order of their experts (within an expert in any order; here:
     ascending) and the tiles (expert, first sorted place, rows, 0) of at most ``tile_rows`` rows;
-    tiles that do not exist have zero rows."""
+    tiles that do not exist have zero rows.  The last ``n_identity`` experts have no tiles."""
     flat = choice.reshape(-1).long()
     order = torch.sort(flat, stable=True).indices
-    tiles = torch.zeros((moe_max_tiles(flat.numel(), n_experts, tile_rows), 4), dtype=torch.int32, device=choice.device)
+    tiles = torch.zeros((moe_max_tiles(flat.numel(), n_experts - n_identity, tile_rows), 4), dtype=torch.int32, device=choice.device)
     at, first = 0, 0
     for e, c in enumerate(torch.bincount(flat, minlength=n_experts).tolist()):
-        for r in range(0, c, tile_rows):
+        for r in range(0, c if e < n_experts - n_identity else 0, tile_rows):
             tiles[at] = torch.tensor([e, first + r, min(tile_rows, c - r), 0], dtype=torch.int32)
             at += 1
         first += c
@@ -466,9 +468,13 @@ def moe_down(act: torch.Tensor, w_down: torch.Tensor, sorted_: torch.Tensor, til
 
 
 def moe_combine(y: torch.Tensor, weight: torch.Tensor, plus: Optional[torch.Tensor] = None,
-                plus_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """fp32 ``[1, T, dim]``: ``plus[t] (* sigmoid(plus_gate[t])) + sum_j weight[t, j] * y[t * top + j]``."""
+                plus_gate: Optional[torch.Tensor] = None, choice: Optional[torch.Tensor] = None, n_tiled: int = 0,
+                x: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """fp32 ``[1, T, dim]``: ``plus[t] (* sigmoid(plus_gate[t])) + sum_j weight[t, j] * y[t * top + j]``; where ``choice[t, j]``
+    is ``n_tiled`` or more, ``x[t]`` stands for ``y``'s row."""
     T, top = weight.shape
+    if choice is not None:
+        y = torch.where((choice.reshape(-1) >= n_tiled)[:, None], x.float().repeat_interleave(top, 0), y)
     out = (weight[:, :, None] * y.view(T, top, -1)).sum(1)
     if plus is not None:
         p = plus.sum(0) if plus.dim() == 3 else plus.float()
@@ -586,13 +592,80 @@ def head_linear(x: torch.Tensor, x_head_stride: int, w: torch.Tensor, out: torch
 
 
 def head_norm_gate(x: torch.Tensor, weight: torch.Tensor, eps: float, gate: torch.Tensor, n_heads: int,
-                   out: torch.Tensor, out_scale: float = 1.0) -> torch.Tensor:
-    """RMS norm of every head of fp32 ``x [T, H*e]`` with one weight ``[e]``, times ``silu(gate)`` and ``out_scale``."""
+                   out: torch.Tensor, out_scale: float = 1.0, sigmoid: bool = False) -> torch.Tensor:
+    """RMS norm of every head of fp32 ``x [T, H*e]`` with one weight ``[e]``, times ``silu(gate)`` (or ``sigmoid(gate)``) and
+    ``out_scale``."""
     T, e = x.shape[0], x.shape[1] // n_heads
     y = x.view(T, n_heads, e)
     y = y * torch.rsqrt((y * y).mean(-1, keepdim=True) + eps) * weight.float()
     g = gate[:, : n_heads * e].float().reshape(T, n_heads, e)
-    out.copy_((y * g * torch.sigmoid(g) * out_scale).reshape(T, -1).to(out.dtype))
+    out.copy_((y * (1.0 if sigmoid else g) * torch.sigmoid(g) * out_scale).reshape(T, -1).to(out.dtype))
+    return out
+
+
+def row_norm_gate(x: torch.Tensor, weight: torch.Tensor, eps: float, gate: torch.Tensor, out: torch.Tensor,
+                  out_scale: float = 1.0) -> torch.Tensor:
+    """RMS norm of every row of fp32 ``x [T, W]`` with a weight ``[W]``, times ``sigmoid(gate)`` and ``out_scale``."""
+    W = x.shape[1]
+    y = x * torch.rsqrt((x * x).mean(-1, keepdim=True) + eps) * weight.float() * torch.sigmoid(gate[:, :W].float()) * out_scale
+    out[:, :W] = y.to(out.dtype)
+    return out
+
+
+def bias_act(x: torch.Tensor, bias: Optional[torch.Tensor], activation: str, out_dtype: torch.dtype) -> torch.Tensor:
+    """``act(x + bias)``: the square of ReLU, ReLU, SiLU or the tanh form of GELU."""
+    z = x.float() + (bias.float() if bias is not None else 0.0)
+    y = {"relu2": lambda: torch.relu(z) ** 2, "relu": lambda: torch.relu(z), "silu": lambda: z * torch.sigmoid(z),
+         "gelu_tanh": lambda: _gelu_tanh(z)}[activation]()
+    return y.to(out_dtype)
+
+
+def stream_terms(h: torch.Tensor, delta, again: Optional[torch.Tensor] = None, norms=(), eps: float = 0.0,
+                 rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``h += sum_j scale_j (.) n_j(rows_j + bias_j)``, ``h += again``, then the norms of ``h``; gathered: ``h`` stays."""
+    v = h.clone()
+    for t in delta.terms:
+        x = t.rows.sum(0) if t.rows.dim() == 3 else t.rows.float()
+        if t.bias is not None:
+            x = x + t.bias
+        if t.norm_eps is not None:
+            x = x * torch.rsqrt((x * x).mean(-1, keepdim=True) + t.norm_eps)
+        v = v + (x if t.scale is None else x * t.scale)
+    if again is not None:
+        v = v + again
+    if rows is None:
+        h.copy_(v)
+    else:
+        v = v[rows.long()]
+    for w, out in norms:
+        out.copy_((v * torch.rsqrt((v * v).mean(-1, keepdim=True) + eps) * w.float()).to(out.dtype))
+    return h
+
+
+def low_rank(src: torch.Tensor, jobs) -> None:
+    """``out = W2 z + b`` for columns ``z`` of ``src`` in ``W2``'s dtype; with a rate ``-rate softplus(.)``."""
+    for j in jobs:
+        N, K = j.w.shape
+        y = src[:, j.col : j.col + K].to(j.w.dtype).float() @ j.w.float().T
+        if j.bias is not None:
+            y = y + j.bias
+        if j.rate is not None:
+            y = -j.rate.repeat_interleave(j.per)[:N] * torch.nn.functional.softplus(y)
+        j.out[:, :N] = y
+
+
+def lightning_scan(rows: torch.Tensor, q_col: int, k_col: int, v_col: int, log_decay: torch.Tensor, state: torch.Tensor,
+                   slot_ids: torch.Tensor, q_start: torch.Tensor, n_seqs: int, out: torch.Tensor, q_start_host=None) -> torch.Tensor:
+    """Per sequence and head, token by token: ``S <- exp(log_decay) S + k v^T``, ``o = S^T q``, silu on q, k and v."""
+    _, H, d, e = state.shape
+    a = torch.exp(log_decay.to(state.dtype))[:, None, None]
+    y = rows * torch.sigmoid(rows)
+    for b in range(n_seqs):
+        S = state[int(slot_ids[b])]
+        for t in range(int(q_start[b]), int(q_start[b + 1])):
+            q, k, v = (y[t, c : c + H * w].view(H, w) for c, w in ((q_col, d), (k_col, d), (v_col, e)))
+            S.mul_(a).add_(k[:, :, None] * v[:, None, :])
+            out[t] = torch.einsum("hde,hd->he", S, q).reshape(-1)
     return out
 
 
@@ -813,7 +886,7 @@ def mixed_attention_mfma(q: torch.Tensor, head_dim: int, out: torch.Tensor, v_he
 
 # ------------------------------------------------------------ gated delta rule
 def delta_prepare(src: torch.Tensor, n_qk: int, head_dim: int, n_v: int, v_head_dim: int, conv, b_col: int, a_col: int,
-                  decay_rate: torch.Tensor, dt_bias: torch.Tensor, q_scale: float, unit_eps: float,
+                  decay_rate: Optional[torch.Tensor], dt_bias: Optional[torch.Tensor], q_scale: float, unit_eps: float,
                   out: torch.Tensor) -> torch.Tensor:
     """``[q | k | v | beta | log g]`` a token: q, k, v behind the convolution and SiLU, q and k as unit vectors per head."""
     T, n = src.shape[0], n_qk * head_dim
@@ -827,13 +900,15 @@ def delta_prepare(src: torch.Tensor, n_qk: int, head_dim: int, n_v: int, v_head_
     C = y.shape[1]
     out[:, :C] = y
     out[:, C : C + n_v] = torch.sigmoid(src[:, b_col : b_col + n_v].float())
-    out[:, C + n_v : C + 2 * n_v] = -decay_rate * torch.nn.functional.softplus(src[:, a_col : a_col + n_v].float() + dt_bias)
+    if a_col >= 0:
+        out[:, C + n_v : C + 2 * n_v] = -decay_rate * torch.nn.functional.softplus(src[:, a_col : a_col + n_v].float() + dt_bias)
     return out
 
 
 def delta_scan(rows: torch.Tensor, n_qk: int, head_dim: int, n_v: int, v_head_dim: int, state: torch.Tensor,
-               slot_ids: torch.Tensor, q_start: torch.Tensor, n_seqs: int, out: torch.Tensor, q_start_host=None) -> torch.Tensor:
-    """Per sequence and value head, token by token: ``S <- g S``, ``u = beta (v - S^T k)``, ``S <- S + k u^T``, ``o = S^T q``."""
+               slot_ids: torch.Tensor, q_start: torch.Tensor, n_seqs: int, out: torch.Tensor, q_start_host=None,
+               channel_decay_col: Optional[int] = None) -> torch.Tensor:
+    """Per sequence and value head, token by token: ``S <- g S`` (a number, or one per key channel), ``u = beta (v - S^T k)``, ``S <- S + k u^T``, ``o = S^T q``."""
     d, e, n = head_dim, v_head_dim, n_qk * head_dim
     rep = n_v // n_qk
     for b in range(n_seqs):
@@ -843,8 +918,10 @@ def delta_scan(rows: torch.Tensor, n_qk: int, head_dim: int, n_v: int, v_head_di
             q = r[:n].view(n_qk, d).repeat_interleave(rep, 0)
             k = r[n : 2 * n].view(n_qk, d).repeat_interleave(rep, 0)
             v = r[2 * n : 2 * n + n_v * e].view(n_v, e)
-            beta, log_g = r[2 * n + n_v * e :][:n_v], r[2 * n + n_v * (e + 1) :][:n_v]
-            S.mul_(torch.exp(log_g)[:, None, None])
+            beta, log_g = r[2 * n + n_v * e :][:n_v], r[2 * n + n_v * (e + 1) :][:n_v, None]
+            if channel_decay_col is not None:
+                log_g = r[channel_decay_col:][: n_v * d].view(n_v, d)
+            S.mul_(torch.exp(log_g)[:, :, None])
             u = beta[:, None] * (v - torch.einsum("hde,hd->he", S, k))
             S.add_(k[:, :, None] * u[:, None, :])
             out[t] = torch.einsum("hde,hd->he", S, q).reshape(-1)

@@ -247,10 +247,11 @@ def plain_greedy(weights: Mapping[str, torch.Tensor], config: Mapping, prompt: L
 
 
 # --------------------------------------------------------------------- weights
-def plain_weights(config: Mapping, seed: int, stored: torch.dtype = torch.bfloat16, a_rank: int = 6, g_rank: int = 10
-                  ) -> Dict[str, torch.Tensor]:
+def plain_weights(config: Mapping, seed: int, stored: torch.dtype = torch.bfloat16, a_rank: int = 6, g_rank: int = 10,
+                  decisive: bool = False) -> Dict[str, torch.Tensor]:
     """Random tensors of a configuration, by the names of the checkpoint, with the values that ``stored`` can hold
-    (as float32).  ``a_rank`` / ``g_rank``: the narrow middles, which only the tensors' shapes give."""
+    (as float32).  ``a_rank`` / ``g_rank``: the narrow middles, which only the tensors' shapes give.
+    ``decisive``: corrections so far apart that they alone decide which experts are chosen, whatever the rounding."""
     g = torch.Generator().manual_seed(seed)
     D, V = config["width"], config["vocab"]
     w: Dict[str, torch.Tensor] = {}
@@ -312,6 +313,8 @@ def plain_weights(config: Mapping, seed: int, stored: torch.dtype = torch.bfloat
             n = r["experts"] + r.get("identity", 0)
             mat(f"{p}.router", n, D)
             vec(f"{p}.correction", n, mean=-0.05, std=0.1)
+            if decisive:
+                w[f"{p}.correction"] = 2.0 * (torch.randperm(n, generator=g) - n // 2)
             for e in range(r["experts"]):
                 mat(f"{p}.e{e}.gate", ff, D)
                 mat(f"{p}.e{e}.up", ff, D)

@@ -27,7 +27,8 @@ KERNEL_OPS = ["embed", "add_rmsnorm", "rmsnorm", "silu_mul", "rope_table", "rope
               "moe_sort", "moe_gate_up", "moe_down", "moe_combine", "gelu_mul", "post_add_rmsnorm", "softcap",
               "heads_prepare", "head_linear", "head_norm_gate", "decay_scan", "gated_mul", "causal_conv", "selective_scan",
               "sigmoid_attention", "scale_logits", "head_diff_norm", "streams_spread", "streams_step", "conv_tail",
-              "mixed_attention", "mixed_attention_mfma", "delta_prepare", "delta_scan", "lru_scan"]
+              "mixed_attention", "mixed_attention_mfma", "delta_prepare", "delta_scan", "lru_scan", "stream_terms", "row_norm_gate",
+              "bias_act", "low_rank", "lightning_scan"]
 
 
 @pytest.mark.parametrize("name", KERNEL_OPS + ["interleave_gate_up"])
