@@ -97,11 +97,12 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_kernel(
   // wave issues LPW loads a stage to the end, so the count it waits for stays the same)
   auto issue = [&](int s) {
     const int k = k_begin + 32 * min(s, n_stages - 1);
-    const int koff = k + 8 * g < k_end ? k : k_begin;  // a chunk beyond the k range: any readable one, zeroed at use
+    // a chunk beyond the k range: the range's first one of the row (a packed W has zeros there), zeroed at use
+    const int koff = k + 8 * g < k_end ? k : k_begin - 8 * g;
     bf16_t* slot = ring + (size_t)(s % NST) * NB * BLOCK;
 #pragma unroll
     for (int j = 0; j < LPW; ++j)
-      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src[j] + (size_t)koff * step[j]),
+      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src[j] + (ptrdiff_t)(step[j] == 1 ? koff : k * 16)),
                                        (__attribute__((address_space(3))) void*)(slot + (wave + NW * j) * BLOCK), 16, 0, 0);
   };
 

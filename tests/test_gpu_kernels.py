@@ -413,6 +413,31 @@ def test_gemm_tiled_and_k_splits(ops, tile_rows, M, N, K, S):
                        ops.gemm_tiled(x.to(DEV), w.to(DEV), k_splits=S, tile_rows=tile_rows))
 
 
+@pytest.mark.parametrize("K", [8, 16, 24, 40, 72])
+def test_products_of_few_columns_do_not_look_behind_their_operands(ops, K):
+    """k ranges shorter than a step of the kernels: what lies behind x and W in memory (NaN here) must not count."""
+    N = 40
+    torch.manual_seed(K)
+
+    def with_nan_behind(t):
+        room = torch.full((t.numel() + 4096,), float("nan"), dtype=t.dtype, device=DEV)
+        room[: t.numel()] = t.reshape(-1).to(DEV)
+        return room[: t.numel()].view(t.shape)
+
+    for M in (1, 7, 16, 40, 64, 100, 130, 300):
+        x, w = torch.randn(M, K).bfloat16(), (torch.randn(N, K) * K**-0.5).bfloat16()
+        want = x.double() @ w.double().T
+        xd, wd = with_nan_behind(x), with_nan_behind(w)
+        for weight in (wd, ops.pack_weight(wd)):
+            runs = [ops.gemm_tiled(xd, weight, torch.float32, tile_rows=r) for r in (128, 256)]
+            if M <= 128:
+                runs.append(ops.gemm_skinny(xd, weight, torch.float32, wide=True))
+            if M <= 64:
+                runs.append(ops.gemm_skinny(xd, weight, torch.float32, wide=False))
+            for got in runs:
+                assert (got.cpu().double() - want).abs().max() <= 1e-4 * want.abs().max() + 1e-6
+
+
 @pytest.mark.parametrize("M,F,K", [(129, 328, 240), (256, 14336, 4096), (70, 8, 64)])
 def test_gemm_tiled_gate_up_epilogue(ops, M, F, K):
     torch.manual_seed(F)
