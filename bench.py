@@ -10,6 +10,7 @@
     python bench.py --workload zudisun      # the Zudisun design beside Gisodra and the dense Llama at equal sizes
     python bench.py --workload sodotar      # the Sodotar design beside Gisodra and the dense Llama at equal sizes
     python bench.py --workload ropelix      # the Ropelix design beside Gisodra and the dense Llama at equal sizes
+    python bench.py --workload poselorn     # the Poselorn design beside Ropelix and the dense Llama at equal sizes
 
 The model has the layer sizes of Llama 3.1 8B (32 layers, hidden 4096, 32
 heads, 8 kv heads, head size 128, feed-forward 14336, vocabulary 128256,
@@ -1085,6 +1086,211 @@ def ropelix_workload(prefill_tokens: int = 2048, batch: int = 8, context: int = 
     return 0
 
 
+# Poselorn at the sizes of the Ropelix workload: eight layers in the order delta rule with a decay per channel (dense
+# feed-forward), parallel (windowed attention beside linear attention; experts), parallel, delta rule (experts), twice, each
+# run once.  Beside it Ropelix (the framework's closest model: the delta rule and attention beside a recurrence) and the
+# dense Llama, of the same width, heads, head size and number of layers; the experts that a token uses are together as wide
+# as half the dense feed-forward.
+POSELORN_SIZES = {
+    "w1024": dict(ROPELIX_SIZES["w1024"], rank=64, lin_heads=8, lin_dim=64, lin_vdim=128, experts=28, identity=4, groups=4, keep=2,
+                  top=4, expert_ff=352),
+    "w2048": dict(ROPELIX_SIZES["w2048"], rank=128, lin_heads=16, lin_dim=128, lin_vdim=128, experts=28, identity=4, groups=4, keep=2,
+                  top=4, expert_ff=704),
+}
+
+
+def _poselorn_configs(z: dict):
+    dense = dict(kind="dense", ff=z["ff"])
+    moe = dict(kind="moe", expert=dict(ff=z["expert_ff"]), router=dict(
+        experts=z["experts"], identity=z["identity"], top=z["top"], groups=dict(count=z["groups"], keep=z["keep"])))
+    delta = dict(type="channel_delta", mixer=dict(heads=z["delta_heads"], kv_heads=z["delta_kv"], dim=z["delta_dim"], vdim=z["delta_vdim"],
+                                                  conv=z["conv"], decay_rank=z["rank"], gate_rank=z["rank"]))
+    decay = [1.0 - 2.0 ** -(1 + i % 10) for i in range(z["lin_heads"])]
+    parallel = dict(type="parallel", mlp=moe, mixer=dict(
+        left=dict(heads=z["heads"], kv_heads=z["kv_heads"], dim=z["dim"], vdim=z["dim"], scale=z["dim"] ** -0.5,
+                  mask=dict(size=z["window"]), rot=dict(base=500000.0, dims=z["dim"])),
+        right=dict(heads=z["lin_heads"], dim=z["lin_dim"], vdim=z["lin_vdim"], decay=decay)))
+    layers = [dict(delta, mlp=dense), parallel, parallel, dict(delta, mlp=moe)] * 2
+    new = dict(architecture="Poselorn", width=z["width"], vocab=z["vocab"], embedding=dict(scale=8.0), residual_mult=0.5,
+               norm=dict(eps=1e-6), layers=layers)
+    near, _, llama = _ropelix_configs(z)
+    return new, near, llama
+
+
+def _poselorn_kernels(z: dict, rows: int, context: int) -> dict:
+    """The design's own kernels at ``rows`` tokens (one prompt of ``rows`` tokens, or ``rows`` sequences of one token at
+    ``context`` cached ones), each beside the like kernel of the framework's other models on operands of the same
+    size: microseconds, and the shares of the memory roofline (the bytes the kernel has to move), of the matrix
+    cores' (its bf16 products' flops) and of the fp32 units' (the flops that are fp32 by design; the fp32 matrix products
+    have the same peak)."""
+    import numpy as np
+    import torch
+
+    from fastgen_amd.kernels import ops
+
+    D, H, G, d, P, K = z["width"], z["heads"], z["kv_heads"], z["dim"], PAGE, z["conv"]
+    g = torch.Generator(device="cuda").manual_seed(rows)
+    rnd = lambda *shape: (torch.randn(*shape, generator=g, device="cuda") * 0.05).to(torch.bfloat16)
+    f32 = lambda *shape: torch.randn(*shape, generator=g, device="cuda")
+    i32 = lambda values: torch.tensor(values, dtype=torch.int32, device="cuda")
+    decode = rows <= 16
+    n_seqs = rows if decode else 1
+    out = {}
+
+    def put(name, fn, nbytes, flops=0, vector_flops=0):
+        t = _time(fn)
+        out[name] = {"us": round(t * 1e6, 1), "hbm_frac": round(nbytes / t / PEAK_HBM, 4),
+                     "mfma_frac": round(flops / t / PEAK_FLOPS["bf16"], 4),
+                     "fp32_frac": round(vector_flops / t / PEAK_FLOPS["fp32"], 4)}
+
+    # ---- the step: `rows` tokens of one sequence, or one of each of `rows` sequences
+    q_lens, q_start_host, n_cached = (([1] * rows, list(range(rows + 1)), [context] * rows) if decode else ([rows], [0, rows], [0]))
+    q_start, slot_ids = i32(q_start_host), torch.arange(n_seqs, dtype=torch.int32, device="cuda")
+    host = np.array(q_start_host)
+    seq_of_token = i32(list(range(rows)) if decode else [0] * rows)
+    positions = i32([context] * rows if decode else list(range(rows)))
+    keys = context + 1 if decode else rows
+    pages_seq = -(-keys // P)
+    bt = torch.arange(n_seqs * pages_seq, dtype=torch.int32, device="cuda").view(n_seqs, pages_seq)
+    slots = (torch.arange(rows, dtype=torch.int32, device="cuda") * pages_seq * P + context if decode
+             else torch.arange(rows, dtype=torch.int32, device="cuda")).contiguous()
+    kp, vp = rnd(n_seqs * pages_seq, G, P, d), rnd(n_seqs * pages_seq, G, d, P)
+    w = min(z["window"], keys)
+    pairs = n_seqs * w if decode else w * (w + 1) // 2 + (rows - w) * w
+    kv_bytes = (n_seqs * w * 2 * G * d + 2 * rows * H * d) * 2
+    # ---- attention in a window, beside the same with a sink
+    q, o = rnd(rows, H * d), torch.empty(rows, H * d, dtype=torch.bfloat16, device="cuda")
+    up = lambda items: ops.upload(items, torch.int32, "cuda") if len(items) else None
+    small, big = ops.attention_items(np.array(q_lens), host, np.array(n_cached), H // G, ops.attention_tile_rows(d, False, True))
+    sm, bg = up(small), up(big)
+    plan = ops.attention_plan(sm, len(small), ops.attention_chunks_for(len(small), G), d, z["window"], 4, True) if sm is not None else None
+    for name, sinks in (("attention", None), ("attention (gisodra: sink)", torch.zeros(H, device="cuda"))):
+        put(name, lambda: ops.paged_attention_mfma(q, o, kp, vp, bt, sm, bg, H, d ** -0.5, z["window"], plan, exact_weights=True, sinks=sinks),
+            kv_bytes, 4 * pairs * H * d)
+    # ---- between a product and an attention
+    src, bias, hn = f32(rows, (H + 2 * G) * d), f32((H + 2 * G) * d), f32(d)
+    table = ops.rope_table(positions, f32(d // 2).abs())
+    heads = dict(n_q=H, q_col=0, q_width=d, q_out=q, q_out_width=d, n_kv=G, k_col=H * d, k_width=d, v_width=d, slots=slots,
+                 k_pages=kp, v_pages=vp, q_norm=hn, q_norm_dims=d, k_norm=hn, k_norm_dims=d, v_col=(H + G) * d)
+    moved = src.numel() * 4 + rows * (H + 2 * G) * d * 2
+    put("heads_prepare (biases, norms per head, rotation)", lambda: ops.heads_prepare(src, bias, 1e-6, table=table, rotary_dim=d, **heads), moved)
+    put("heads_prepare (gisodra: norms per head)", lambda: ops.heads_prepare(src, None, 1e-6, **heads), moved)
+    # ---- the delta rule with a decay per channel, beside Ropelix's with one per head
+    Hd, Gd, dd, e, r = z["delta_heads"], z["delta_kv"], z["delta_dim"], z["delta_vdim"], z["rank"]
+    C = 2 * Gd * dd + Hd * e
+    raw = f32(rows, C + 2 * r + 2 * Hd)
+    state = torch.zeros(n_seqs + 1, Hd * dd * e + C * (K - 1), device="cuda")
+    dconv = ops.ConvInputs(f32(C, K), state[:, Hd * dd * e :].view(n_seqs + 1, C, K - 1), 0, slot_ids, seq_of_token, q_start, decode)
+    col = -(-(C + Hd) // 4) * 4
+    ready, near = torch.empty(rows, col + Hd * dd, device="cuda"), torch.empty(rows, -(-(C + 2 * Hd) // 4) * 4, device="cuda")
+    gate, rate, dtb, a2, g2 = torch.empty(rows, Hd * e, device="cuda"), f32(Hd).abs(), f32(Hd * dd) - 2.0, rnd(Hd * dd, r), rnd(Hd * e, r)
+    put("delta_prepare (no decays)", lambda: ops.delta_prepare(raw, Gd, dd, Hd, e, dconv, C + 2 * r, -1, None, None, dd ** -0.5, 1e-6, ready),
+        rows * (C + Hd) * 8)
+    put("delta_prepare (ropelix)", lambda: ops.delta_prepare(raw, Gd, dd, Hd, e, dconv, C, C + Hd, rate, dtb[:Hd].contiguous(), dd ** -0.5, 1e-6, near),
+        rows * (C + 2 * Hd) * 8)
+    jobs = [ops.LowRankJob(C, a2, ready[:, col:], dtb, rate, dd), ops.LowRankJob(C + r, g2, gate)]
+    put("low_rank (decays and output gate)", lambda: ops.low_rank(raw, jobs), rows * (2 * r + Hd * (dd + e)) * 4 + (a2.numel() + g2.numel()) * 2,
+        2 * rows * r * Hd * (dd + e))
+    xh, wh, yh = rnd(rows, 2 * r), rnd(2, Hd * max(dd, e), r), torch.empty(rows, 2 * Hd * max(dd, e), device="cuda")
+    put("head_linear (ropelix: two products of that size, fp32 out)", lambda: ops.head_linear(xh, r, wh, yh, Hd * max(dd, e)),
+        rows * (2 * r * 2 + yh.shape[1] * 4) + wh.numel() * 2, 2 * rows * r * yh.shape[1])
+    o32 = torch.empty(rows, Hd * e, device="cuda")
+    S = state[:, : Hd * dd * e].view(n_seqs + 1, Hd, dd, e)
+    scan = lambda h: ops.delta_scan(ready, Gd, dd, Hd, e, S, slot_ids, q_start, n_seqs, o32, h, col)
+    scan1 = lambda h: ops.delta_scan(near, Gd, dd, Hd, e, S, slot_ids, q_start, n_seqs, o32, h)
+    sb = 2 * n_seqs * Hd * dd * e * 4 + rows * (C + Hd + Hd * dd + Hd * e) * 4
+    sb1 = sb - rows * (Hd * dd - Hd) * 4
+    put("delta_scan, decays per channel", lambda: scan(host), sb, 0, 7 * rows * Hd * dd * e)
+    put("delta_scan (ropelix)", lambda: scan1(host), sb1, 0, 7 * rows * Hd * dd * e)
+    if not decode:
+        put("delta_scan, decays per channel, token by token", lambda: scan(None), sb, 0, 7 * rows * Hd * dd * e)
+        put("delta_scan (ropelix), token by token", lambda: scan1(None), sb1, 0, 7 * rows * Hd * dd * e)
+    o16, nw = torch.empty(rows, Hd * e, dtype=torch.bfloat16, device="cuda"), f32(e)
+    put("head_norm_gate (sigmoid)", lambda: ops.head_norm_gate(o32, nw, 1e-6, gate, Hd, o16, sigmoid=True), rows * Hd * e * 10)
+    put("head_norm_gate (ropelix)", lambda: ops.head_norm_gate(o32, nw, 1e-6, gate, Hd, o16), rows * Hd * e * 10)
+    # ---- linear attention with constant decays, beside Gisodra's with decays per channel and token
+    Hl, dl, el = z["lin_heads"], z["lin_dim"], z["lin_vdim"]
+    lrows, ll = f32(rows, 2 * Hl * dl + 2 * Hl * el), torch.full((Hl,), -0.01, device="cuda")
+    lstate, lo = torch.zeros(n_seqs + 1, Hl, dl, el, device="cuda"), torch.empty(rows, Hl * el, device="cuda")
+    light = lambda h: ops.lightning_scan(lrows, 0, Hl * dl, 2 * Hl * dl, ll, lstate, slot_ids, q_start, n_seqs, lo, h)
+    lb = 2 * n_seqs * Hl * dl * el * 4 + rows * (2 * Hl * dl + 2 * Hl * el) * 4
+    put("lightning_scan", lambda: light(host), lb, 0, 5 * rows * Hl * dl * el)
+    rows16, zz, zb = rnd(rows, 2 * Hl * dl + Hl * el), f32(rows, Hl * dl), f32(Hl * dl)
+    gscan = lambda h: ops.decay_scan(rows16, 0, Hl * dl, 2 * Hl * dl, zz, zb, 16.0, dl ** -0.5, lstate, slot_ids, q_start, n_seqs, lo, q_start_host=h)
+    gb = 2 * n_seqs * Hl * dl * el * 4 + rows * (2 * Hl * dl + Hl * el) * 2 + rows * (Hl * dl + Hl * el) * 4
+    put("decay_scan (gisodra)", lambda: gscan(host), gb, 0, 5 * rows * Hl * dl * el)
+    if not decode:
+        put("lightning_scan, token by token", lambda: light(None), lb, 0, 5 * rows * Hl * dl * el)
+        put("decay_scan (gisodra), token by token", lambda: gscan(None), gb, 0, 5 * rows * Hl * dl * el)
+    lo16, lw = torch.empty(rows, Hl * el, dtype=torch.bfloat16, device="cuda"), f32(Hl * el)
+    put("row_norm_gate", lambda: ops.row_norm_gate(lo, lw, 1e-6, lrows[:, 2 * Hl * dl + Hl * el :], lo16), rows * Hl * el * 10)
+    # ---- the stream: three terms (two of them normed) and two norms, beside one scaled term and one norm
+    h, n1, n2, ls = f32(rows, D), torch.empty(rows, D, dtype=torch.bfloat16, device="cuda"), torch.empty(rows, D, dtype=torch.bfloat16, device="cuda"), f32(D)
+    xa, xb, xc, wn = rnd(rows, D), rnd(rows, D), f32(1, rows, D), f32(D)
+    three = ops.StreamTerms([ops.StreamTerm(xa, ls, None, 1e-6), ops.StreamTerm(xb, ls, None, 1e-6), ops.StreamTerm(xc, ls)])
+    two = ops.StreamTerms([ops.StreamTerm(xa, ls), ops.StreamTerm(xb, ls, ls)])
+    put("stream_terms (behind a parallel layer: three terms, two norms)", lambda: ops.stream_terms(h, three, None, [(wn, n1), (wn, n2)], 1e-6), rows * D * 20)
+    put("stream_terms (behind a delta layer: two terms, two norms)", lambda: ops.stream_terms(h, two, None, [(wn, n1), (wn, n2)], 1e-6), rows * D * 16)
+    put("add_rmsnorm (ropelix: scaled per channel)", lambda: ops.add_rmsnorm(h, xa, wn, 1e-6, n1, None, ls), rows * D * 12)
+    # ---- the feed-forwards
+    F = z["ff"]
+    u32, ub, gu = f32(rows, F), f32(F), f32(rows, 2 * F)
+    put("bias_act (square of ReLU)", lambda: ops.bias_act(u32, ub, "relu2", torch.bfloat16), rows * F * 6)
+    put("gated_mul (ropelix: limited)", lambda: ops.gated_mul(gu, None, "limited", torch.bfloat16, None, 7.0, 1.702), rows * F * 10)
+    E, I, top = z["experts"], z["identity"], z["top"]
+    x, router, corr = rnd(rows, D), f32(E + I, D), 0.01 * f32(E + I)
+    put("moe_route (identities, groups by their best)", lambda: ops.moe_route(x, router, None, top, softmax_scores=True, correction=corr,
+        n_groups=z["groups"], keep_groups=z["keep"], group_max=True, raw_weights=True), rows * D * 2 + router.numel() * 4, 0, 2 * rows * D * (E + I))
+    put("moe_route (sodotar: softmax over all)", lambda: ops.moe_route(x, router, None, top, softmax_scores=True, correction=corr),
+        rows * D * 2 + router.numel() * 4, 0, 2 * rows * D * (E + I))
+    choice, weight = ops.moe_route(x, router, None, top, softmax_scores=True)
+    y = f32(rows * top, D)
+    put("moe_combine (identities)", lambda: ops.moe_combine(y, weight, None, None, choice, E, x), rows * D * (4 * top + 4))
+    put("moe_combine (sodotar)", lambda: ops.moe_combine(y, weight), rows * D * (4 * top + 4))
+    return out
+
+
+def poselorn_workload(prefill_tokens: int = 2048, batch: int = 8, context: int = 1024, steps: int = 32, warmup: int = 8) -> int:
+    """Prefill and decode throughput of Poselorn models with random bfloat16 weights beside Ropelix and dense Llama models of
+    equal sizes, and the design's own kernels beside the other models' like ones.  One JSON line."""
+    import torch
+
+    from fastgen_amd.engine import Engine
+
+    results = {}
+    for name, z in POSELORN_SIZES.items():
+        new, near, dense = _poselorn_configs(z)
+        row = {"layers": len(new["layers"])}
+        for label, cfg in (("poselorn", new), ("ropelix", near), ("llama", dense)):
+            engine = Engine.from_config(cfg, seed=5, dtype=torch.bfloat16, page_size=PAGE,
+                                        max_tokens=max(batch * (context + 256), prefill_tokens + PAGE), max_batch=batch,
+                                        max_step_tokens=prefill_tokens)
+            g = torch.Generator().manual_seed(0)
+            prompt = lambda n: torch.randint(0, z["vocab"], (n,), generator=g).tolist()
+            pre = min(engine.time_prefill(prompt(prefill_tokens), repeats=5))
+            dt = engine.time_decode([prompt(context) for _ in range(batch)], steps=steps, warmup=warmup)
+            row[label] = {"prefill_tok_s": round(prefill_tokens / pre, 1), "prefill_ms": round(pre * 1e3, 3),
+                          "decode_tok_s": round(batch * steps / dt, 1), "decode_ms_per_step": round(dt / steps * 1e3, 4),
+                          "weights_gb": round(engine.model.weight_bytes() / 1e9, 3)}
+            print(f"[bench] {name} {label}: {row[label]}", file=sys.stderr, flush=True)
+            del engine
+            torch.cuda.empty_cache()
+        row["kernels_prefill"] = _poselorn_kernels(z, prefill_tokens, context)
+        row["kernels_decode"] = _poselorn_kernels(z, batch, context)
+        print(f"[bench] {name} kernels: {row['kernels_prefill']} {row['kernels_decode']}", file=sys.stderr, flush=True)
+        results[name] = row
+    first = results[next(iter(results))]
+    print(json.dumps({
+        "metric": "Poselorn beside Ropelix and the dense Llama at equal sizes: prefill and decode tok/s", "unit": "tokens/s",
+        "value": first["poselorn"]["decode_tok_s"], "n_gpus": 1, "steps": steps, "warmup": warmup, "higher_is_better": True,
+        "dtype": "bf16", "data": "synthetic",
+        "config": {"prefill_tokens": prefill_tokens, "decode_batch": batch, "decode_context": context, "page_size": PAGE,
+                   "sizes": POSELORN_SIZES},
+        "results": results,
+    }), flush=True)
+    return 0
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -1102,10 +1308,10 @@ def main() -> int:
                          " 2,048); more are fed untimed, in portions")
     ap.add_argument("--dtype", choices=["bf16", "fp32"], default="bf16")
     ap.add_argument("--no-points", action="store_true", help="skip decode at batch 1 and 64")
-    ap.add_argument("--workload", choices=["decode", "serve", "readme", "buderax", "gisodra", "zudisun", "sodotar", "ropelix"],
+    ap.add_argument("--workload", choices=["decode", "serve", "readme", "buderax", "gisodra", "zudisun", "sodotar", "ropelix", "poselorn"],
                     default="decode",
                     help="decode (default): the step benchmark; serve: continuous batching of 256 requests; "
-                         "readme: the load of the reference's README; buderax, gisodra, zudisun, sodotar, ropelix: that design beside the "
+                         "readme: the load of the reference's README; buderax, gisodra, zudisun, sodotar, ropelix, poselorn: that design beside the "
                          "dense Llama at equal sizes")
     ap.add_argument("--step-budget", type=int, default=2048, help="tokens a step of the serve workload")
     ap.add_argument("--show-choices", action="store_true",
@@ -1124,6 +1330,8 @@ def main() -> int:
         return sodotar_workload(prefill_tokens=a.prefill_tokens, batch=a.batch, steps=min(a.steps, 32), warmup=a.warmup)
     if a.workload == "ropelix":
         return ropelix_workload(prefill_tokens=a.prefill_tokens, batch=a.batch, steps=min(a.steps, 32), warmup=a.warmup)
+    if a.workload == "poselorn":
+        return poselorn_workload(prefill_tokens=a.prefill_tokens, batch=a.batch, steps=min(a.steps, 32), warmup=a.warmup)
     if a.workload == "zudisun":
         return zudisun_workload(prefill_tokens=a.prefill_tokens, batch=a.batch, steps=min(a.steps, 32), warmup=a.warmup)
     if a.workload == "buderax":

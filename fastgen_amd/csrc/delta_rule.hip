@@ -291,7 +291,7 @@ extern "C" int fg_delta_scan(const DeltaScanArgs* args, int n_seqs, hipStream_t 
 //   A[t, s] = beta_t sum_c k_t[c] k_s[c] exp(L_t[c] - L_s[c])
 // it is split at the start r of the 16 tokens that hold t: k_t exp(L_t - L_r) meets k_s exp(L_r - L_s).  For s before r
 // both factors are at most one.  Inside the 16 tokens the second one grows; while no channel fades by more than
-// exp(-DC_SAFE) there both stay far inside fp32, else those 16 x 16 sums are taken pair by pair with the difference in the
+// 2^-DC_SAFE there both stay far inside fp32, else those 16 x 16 sums are taken pair by pair with the difference in the
 // exponent.  delta_channel_prepare also leaves the chunk's rows with their decays multiplied in,
 //   Q exp(L), K exp(L), K exp(L_n - L) and exp(L_n),
 // and the scan takes those in place of the rows and the numbers per token.
@@ -307,7 +307,8 @@ struct DeltaChunks {
   float* L;                // [n_chunks, n_v, 64]; decays per channel: exp(L_n), [n_chunks, n_v, d]
   float* Qd; float* Kd; float* Ke;  // decays per channel: [n_chunks, n_v, 64, d]
 };
-#define DC_SAFE 60.f
+#define DC_SAFE 86.f  // in powers of two
+__device__ __forceinline__ float exp2_hw(float x) { return __builtin_amdgcn_exp2f(x); }
 
 __device__ __forceinline__ f32x4 mfma4(const float4& x, const float4& y, f32x4 acc) {
   acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x.x, y.x, acc, 0, 0, 0);
@@ -413,7 +414,7 @@ __global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(const DeltaSca
 }
 
 // Decays per channel: grid (n_chunks, n_v), 4 waves, wave w the tokens 16 w ..; NDM >= d / 16.  LDS: P[t][c] = the sum of
-// log g[c] from the start of t's 16 tokens up to t.
+// log2 g[c] from the start of t's 16 tokens up to t (base 2: the hardware's exponential takes it as it is).
 template <int NDM>
 __global__ __launch_bounds__(256) void delta_channel_prepare_kernel(const DeltaScanArgs a, const DeltaChunks ch) {
   constexpr int LD = 16 * NDM + 4;
@@ -432,7 +433,7 @@ __global__ __launch_bounds__(256) void delta_channel_prepare_kernel(const DeltaS
     for (int t = 0; t < 16; ++t) x[t] = a.rows[(size_t)(t0 + min(16 * j + t, n - 1)) * a.stride + g_col + k];
 #pragma unroll
     for (int t = 0; t < 16; ++t) {
-      sum += 16 * j + t < n ? x[t] : 0.f;
+      sum += 16 * j + t < n ? x[t] * 1.4426950408889634f : 0.f;
       P_s[16 * j + t][k] = sum;
     }
   }
@@ -463,10 +464,10 @@ __global__ __launch_bounds__(256) void delta_channel_prepare_kernel(const DeltaS
           if (m > wave) { behind.x += x.x; behind.y += x.y; behind.z += x.z; behind.w += x.w; }
         }
         safe = safe && fminf(fminf(own.x, own.y), fminf(own.z, own.w)) > -DC_SAFE;
-        const float4 eP = make_float4(expf(P.x), expf(P.y), expf(P.z), expf(P.w));
-        const float4 eb = make_float4(expf(before.x), expf(before.y), expf(before.z), expf(before.w));
-        const float4 ee = make_float4(expf(own.x - P.x + behind.x), expf(own.y - P.y + behind.y), expf(own.z - P.z + behind.z),
-                                      expf(own.w - P.w + behind.w));
+        const float4 eP = make_float4(exp2_hw(P.x), exp2_hw(P.y), exp2_hw(P.z), exp2_hw(P.w));
+        const float4 eb = make_float4(exp2_hw(before.x), exp2_hw(before.y), exp2_hw(before.z), exp2_hw(before.w));
+        const float4 ee = make_float4(exp2_hw(own.x - P.x + behind.x), exp2_hw(own.y - P.y + behind.y), exp2_hw(own.z - P.z + behind.z),
+                                      exp2_hw(own.w - P.w + behind.w));
         qf[j] = make_float4(q.x * eP.x, q.y * eP.y, q.z * eP.z, q.w * eP.w);
         kf[j] = make_float4(k.x * eP.x, k.y * eP.y, k.z * eP.z, k.w * eP.w);
         const float in = t_in ? 1.f : 0.f;
@@ -474,7 +475,7 @@ __global__ __launch_bounds__(256) void delta_channel_prepare_kernel(const DeltaS
         *(float4*)(kd + 16 * j) = make_float4(in * kf[j].x * eb.x, in * kf[j].y * eb.y, in * kf[j].z * eb.z, in * kf[j].w * eb.w);
         *(float4*)(ke + 16 * j) = make_float4(in * k.x * ee.x, in * k.y * ee.y, in * k.z * ee.z, in * k.w * ee.w);
         if (wave == 3 && r16 == 15)
-          *(float4*)(ch.L + at * d + col) = make_float4(eb.x * expf(own.x), eb.y * expf(own.y), eb.z * expf(own.z), eb.w * expf(own.w));
+          *(float4*)(ch.L + at * d + col) = make_float4(eb.x * exp2_hw(own.x), eb.y * exp2_hw(own.y), eb.z * exp2_hw(own.z), eb.w * exp2_hw(own.w));
       }
     }
   }
@@ -494,7 +495,7 @@ __global__ __launch_bounds__(256) void delta_channel_prepare_kernel(const DeltaS
             const float4 y = *(const float4*)&P_s[16 * m + 15][col];
             x.x += y.x; x.y += y.y; x.z += y.z; x.w += y.w;
           }
-          o.x *= expf(x.x); o.y *= expf(x.y); o.z *= expf(x.z); o.w *= expf(x.w);
+          o.x *= exp2_hw(x.x); o.y *= exp2_hw(x.y); o.z *= exp2_hw(x.z); o.w *= exp2_hw(x.w);
           kk = mfma4(kf[j], o, kk);
           qk = mfma4(qf[j], o, qk);
         }
@@ -507,7 +508,7 @@ __global__ __launch_bounds__(256) void delta_channel_prepare_kernel(const DeltaS
         const float ks = row[k], Ps = P_s[16 * wave + r16][k];
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const float f = ks * expf(fminf(P_s[16 * wave + 4 * g + i][k] - Ps, 0.f));  // (pairs with t < s are not used)
+          const float f = ks * exp2_hw(fminf(P_s[16 * wave + 4 * g + i][k] - Ps, 0.f));  // (pairs with t < s are not used)
           kk[i] = fmaf(tr[i][k_col + k], f, kk[i]);
           qk[i] = fmaf(tr[i][k], f, qk[i]);
         }

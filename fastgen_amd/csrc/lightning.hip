@@ -33,7 +33,8 @@ struct LightningChunks {
   float* states;           // [n_chunks, H, d, e]
 };
 
-__device__ __forceinline__ float lt_silu(float x) { return x / (1.f + expf(-x)); }
+// (the hardware's exponential and reciprocal: a few ulp of 32-bit)
+__device__ __forceinline__ float lt_silu(float x) { return x * __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
 __device__ __forceinline__ float4 lt_silu4(const float4& x) { return make_float4(lt_silu(x.x), lt_silu(x.y), lt_silu(x.z), lt_silu(x.w)); }
 __device__ __forceinline__ f32x4 lt_mfma4(const float4& x, const float4& y, f32x4 acc) {
   acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x.x, y.x, acc, 0, 0, 0);
@@ -191,9 +192,17 @@ __global__ __launch_bounds__(256) void lightning_chunk_states_kernel(const Light
           kt[m][j][i] = a.rows[(size_t)(t0 + min(16 * j + 4 * g + i, n - 1)) * a.stride + a.k_col + h * a.d + 16 * (wave + 4 * m) + r16];
     }
   }
-  for (int i = threadIdx.x; i < LC * LC_COLS; i += 256) {
-    const int t = i / LC_COLS, col = i % LC_COLS;
-    V_s[t][col] = lt_silu(a.rows[(size_t)(t0 + min(t, n - 1)) * a.stride + a.v_col + h * a.e + c0 + min(col, cols - 1)]);
+  {
+    const int col = threadIdx.x % LC_COLS, t_own = threadIdx.x / LC_COLS;  // two tokens at a time
+    const float* vp = a.rows + a.v_col + h * a.e + c0 + min(col, cols - 1);
+#pragma unroll
+    for (int u0 = 0; u0 < LC / 2; u0 += 16) {
+      float v[16];
+#pragma unroll
+      for (int u = 0; u < 16; ++u) v[u] = vp[(size_t)(t0 + min(2 * (u0 + u) + t_own, n - 1)) * a.stride];
+#pragma unroll
+      for (int u = 0; u < 16; ++u) V_s[2 * (u0 + u) + t_own][col] = lt_silu(v[u]);
+    }
   }
   float fade[4][4];
 #pragma unroll

@@ -25,14 +25,17 @@ struct LowRankArgs {
   int T;
 };
 
-template <bool FAST>
 __device__ __forceinline__ float low_rank_act(const LowRankJob& j, int n, float y) {
   if (j.bias) y += j.bias[n];
-  if (j.kind == 1) {
-    const float e = expf(-fabsf(y));
-    y = -j.rate[n / j.per] * (fmaxf(y, 0.f) + log1pf(e));
-  }
+  if (j.kind == 1) y = -j.rate[n / j.per] * (fmaxf(y, 0.f) + log1pf(expf(-fabsf(y))));
   return y;
+}
+
+// softplus with the hardware's exponential and logarithm; where 1 + e would lose e's digits, the logarithm's series
+__device__ __forceinline__ float low_rank_softplus(float y) {
+  const float e = __expf(-fabsf(y));
+  const float series = e * (1.f - e * (0.5f - e * (0.33333333f - 0.25f * e)));
+  return fmaxf(y, 0.f) + (e < 0.02f ? series : __logf(1.f + e));
 }
 
 // grid (ceil(T / (16 MB)), ceil(most outputs / (64 NB)), jobs), 4 waves.  A wave holds its tokens' z (KS steps of 32) in
@@ -60,6 +63,14 @@ __global__ __launch_bounds__(256) void low_rank_mfma_kernel(const LowRankArgs a)
   for (int nb = 0; nb < NB; ++nb) {
     const int n0 = first + 16 * nb;
     if (n0 >= j.N) break;  // uniform in the wave
+    const int n = n0 + 4 * g;
+    float bias[4], rate[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int c = min(n + i, j.N - 1);
+      bias[i] = j.bias ? j.bias[c] : 0.f;
+      rate[i] = j.kind == 1 ? j.rate[j.per % 16 == 0 ? n0 / j.per : c / j.per] : 0.f;  // (per is uniform)
+    }
     const bf16_t* wrow = (const bf16_t*)j.w + (size_t)min(n0 + r16, j.N - 1) * j.K;
     bf16x8 w[KS];
 #pragma unroll
@@ -76,12 +87,15 @@ __global__ __launch_bounds__(256) void low_rank_mfma_kernel(const LowRankArgs a)
     }
 #pragma unroll
     for (int mb = 0; mb < MB; ++mb) {
-      const int t = m0 + 16 * mb + r16, n = n0 + 4 * g;
+      const int t = m0 + 16 * mb + r16;
       if (t >= a.T) continue;
       float* y = j.out + (size_t)t * j.out_stride + n;
       float v[4];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) v[i] = n + i < j.N ? low_rank_act<true>(j, n + i, acc[mb][i]) : 0.f;
+      for (int i = 0; i < 4; ++i) {
+        v[i] = acc[mb][i] + bias[i];
+        if (j.kind == 1) v[i] = -rate[i] * low_rank_softplus(v[i]);  // uniform
+      }
       if (n + 3 < j.N && j.out_stride % 4 == 0 && ((uintptr_t)j.out & 15) == 0) {
         *(float4*)y = make_float4(v[0], v[1], v[2], v[3]);
       } else {
@@ -107,7 +121,7 @@ __global__ __launch_bounds__(256) void low_rank_kernel(const LowRankArgs a) {
   const TW* w = (const TW*)j.w + (size_t)n * j.K;
   float acc = 0.f;
   for (int k = 0; k < j.K; ++k) acc = fmaf(to_f<TW>(w[k]), z[k], acc);
-  j.out[(size_t)blockIdx.x * j.out_stride + n] = low_rank_act<false>(j, n, acc);
+  j.out[(size_t)blockIdx.x * j.out_stride + n] = low_rank_act(j, n, acc);
 }
 
 // mfma: bf16 weights, K % 8 == 0 and at most 256, columns and row stride of src in multiples of 8, 16-byte aligned rows
@@ -142,7 +156,9 @@ extern "C" int fg_low_rank(const LowRankArgs* args, int w_dtype, int mfma, hipSt
   } while (0)
     if (a.T <= 16) PICK(1, 1);
     else if (a.T <= 256) PICK(2, 1);
-    else PICK(4, 4);
+    // (a wave converts its tokens' middles for every 16 NB outputs: more of them where that leaves workgroups enough)
+    else if ((long long)((a.T + 63) / 64) * ((n_max + 63) / 64) * a.n_jobs < 2048) PICK(4, 1);
+    else PICK(4, 2);
 #undef PICK
 #undef GO
     return fg_launch_status();

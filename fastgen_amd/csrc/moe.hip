@@ -23,12 +23,13 @@ typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 
 // ------------------------------------------------------------------- route
-// A workgroup a token.  Logits: the WAVES waves take the experts in turns of EPW (a wave reads the row of
-// x once for its EPW experts, eight elements a lane and round; the lanes' partial sums are added by the
-// wave in a fixed order), into LDS.  Few tokens (decode) get 16 waves a token and 2 experts a turn, so that
-// the router's rows are asked for by many waves at once; many tokens 4 waves and 4 experts a turn.  Then the `top` largest (ties: the lower expert) by a
-// wave-wide argmax repeated `top` times, and the softmax over them; every wave does this on the same LDS
-// values, the first one stores.  LDS: n_experts logits, then `top` chosen values, then n_experts scores.
+// A workgroup one token (few tokens: decode) or four.  Logits: the WAVES waves take the experts in turns of EPW (a wave
+// reads the rows of x once for its EPW experts, eight elements a lane and round, and an expert's row of the router once
+// for its tokens; the lanes' partial sums are added by the wave in a fixed order), into LDS.  Few tokens get 16 waves and
+// 2 experts a turn, so that the router's rows are asked for by many waves at once; many tokens 4 waves, 4 experts a turn and
+// 4 tokens, or the router would be read from the L2 once a token.  From there on a wave a token: the `top` largest (ties:
+// the lower expert) by a wave-wide argmax repeated `top` times, and the softmax over them.  LDS, per token: n_experts +
+// n_extra logits, then `top` chosen values, then n_experts scores, then n_groups ranks.
 //
 // A second way of scoring (`sigmoid_scores`): an expert's score is sigmoid(logit); the choice goes by the
 // score plus `correction` (per expert, or null), inside the `keep_groups` best of `n_groups` groups of
@@ -49,91 +50,112 @@ struct RouteMode {
   float* extra;
   int group_max, raw_weights;
 };
-template <class T, int WAVES, int EPW>
+// What a wave's lanes wrote to LDS is there for the wave's other lanes.
+__device__ __forceinline__ void moe_wave_sync() {
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  __builtin_amdgcn_wave_barrier();
+}
+
+template <class T, int WAVES, int EPW, int TOK>
 __global__ __launch_bounds__(64 * WAVES) void moe_route_kernel(
-    const T* __restrict__ x, int ldx, const float* __restrict__ wr, const float* __restrict__ bias,
+    const T* __restrict__ x, int ldx, const float* __restrict__ wr, const float* __restrict__ bias, int n_tokens,
     int dim, int n_experts, int top, int* __restrict__ choice, float* __restrict__ weight, const RouteMode mode) {
+  static_assert(TOK <= WAVES, "a wave a token");
   extern __shared__ float lds[];
-  float* z = lds;
-  float* chosen = lds + n_experts + mode.n_extra;
   const int n_rows = n_experts + mode.n_extra;  // rows of the router matrix
-  float* score = chosen + top;
+  const int per_token = n_rows + top + n_experts + mode.n_groups;
   const int lane = threadIdx.x % FG_WAVE, wave = threadIdx.x / FG_WAVE;
-  const size_t t = blockIdx.x;
-  const T* xr = x + t * ldx;
-  for (int e0 = wave * EPW; e0 < n_rows; e0 += WAVES * EPW) {
-    float s[EPW];
+  const int t0 = blockIdx.x * TOK;
+  const T* xr[TOK];
 #pragma unroll
-    for (int j = 0; j < EPW; ++j) s[j] = 0.f;
+  for (int i = 0; i < TOK; ++i) xr[i] = x + (size_t)min(t0 + i, n_tokens - 1) * ldx;
+  for (int e0 = wave * EPW; e0 < n_rows; e0 += WAVES * EPW) {
+    float s[EPW][TOK];
+#pragma unroll
+    for (int j = 0; j < EPW; ++j)
+#pragma unroll
+      for (int i = 0; i < TOK; ++i) s[j][i] = 0.f;
     if (dim % 8 == 0 && ldx % 8 == 0) {
       for (int k = lane * 8; k < dim; k += FG_WAVE * 8) {
-        float xv[8];
-        load8<T>(xr + k, xv);
+        float xv[TOK][8];
+#pragma unroll
+        for (int i = 0; i < TOK; ++i) load8<T>(xr[i] + k, xv[i]);
 #pragma unroll
         for (int j = 0; j < EPW; ++j) {
           float wv[8];
           load8<float>(wr + (size_t)min(e0 + j, n_rows - 1) * dim + k, wv);
 #pragma unroll
-          for (int i = 0; i < 8; ++i) s[j] = fmaf(xv[i], wv[i], s[j]);
+          for (int i = 0; i < TOK; ++i)
+#pragma unroll
+            for (int u = 0; u < 8; ++u) s[j][i] = fmaf(xv[i][u], wv[u], s[j][i]);
         }
       }
     } else {
       for (int k = lane; k < dim; k += FG_WAVE) {
-        const float xv = to_f<T>(xr[k]);
+        float xv[TOK];
 #pragma unroll
-        for (int j = 0; j < EPW; ++j) s[j] = fmaf(xv, wr[(size_t)min(e0 + j, n_rows - 1) * dim + k], s[j]);
+        for (int i = 0; i < TOK; ++i) xv[i] = to_f<T>(xr[i][k]);
+#pragma unroll
+        for (int j = 0; j < EPW; ++j) {
+          const float wv = wr[(size_t)min(e0 + j, n_rows - 1) * dim + k];
+#pragma unroll
+          for (int i = 0; i < TOK; ++i) s[j][i] = fmaf(xv[i], wv, s[j][i]);
+        }
       }
     }
 #pragma unroll
-    for (int j = 0; j < EPW; ++j) {
-      const float v = wave_sum(s[j]);
-      if (lane == 0 && e0 + j < n_rows) z[e0 + j] = v + (bias && e0 + j < n_experts ? bias[e0 + j] : 0.f);
-    }
+    for (int j = 0; j < EPW; ++j)
+#pragma unroll
+      for (int i = 0; i < TOK; ++i) {
+        const float v = wave_sum(s[j][i]);
+        if (lane == 0 && e0 + j < n_rows) lds[i * per_token + e0 + j] = v + (bias && e0 + j < n_experts ? bias[e0 + j] : 0.f);
+      }
   }
   __syncthreads();
-  for (int e = threadIdx.x; e < mode.n_extra; e += blockDim.x) mode.extra[t * mode.n_extra + e] = z[n_experts + e];
+  const size_t t = t0 + wave;
+  if (wave >= TOK || t >= (size_t)n_tokens) return;  // whole waves; no block barrier below
+  float* z = lds + wave * per_token;
+  float* chosen = z + n_rows;
+  float* score = chosen + top;
+  for (int e = lane; e < mode.n_extra; e += FG_WAVE) mode.extra[t * mode.n_extra + e] = z[n_experts + e];
   if (mode.sigmoid_scores) {  // uniform
     float top_z = 0.f, all = 1.f;
     if (mode.sigmoid_scores == 2) {
-      // every thread takes the maximum and the sum over all experts itself, in the experts' order
       top_z = -INFINITY;
-      for (int e = 0; e < n_experts; ++e) top_z = fmaxf(top_z, z[e]);
+      for (int e = lane; e < n_experts; e += FG_WAVE) top_z = fmaxf(top_z, z[e]);
+      top_z = wave_max(top_z);
       all = 0.f;
-      for (int e = 0; e < n_experts; ++e) all += expf(z[e] - top_z);
-      __syncthreads();  // every thread has read the logits before any of them is overwritten
+      for (int e = lane; e < n_experts; e += FG_WAVE) all += expf(z[e] - top_z);
+      all = wave_sum(all);
     }
-    for (int e = threadIdx.x; e < n_experts; e += blockDim.x) {
+    for (int e = lane; e < n_experts; e += FG_WAVE) {
       const float sc = mode.sigmoid_scores == 2 ? expf(z[e] - top_z) / all : 1.f / (1.f + expf(-z[e]));
       score[e] = sc;
       z[e] = sc + (mode.correction ? mode.correction[e] : 0.f);
     }
-    __syncthreads();
+    moe_wave_sync();
     if (mode.n_groups > 1 && mode.keep_groups < mode.n_groups) {  // uniform
-      // one wave ranks the groups (a lane a group, in turns) and strikes the experts of those that lose
+      // a lane a group, in turns: the groups are ranked and the experts of those that lose are struck
       float* rank = score + n_experts;  // n_groups values
       const int per = n_experts / mode.n_groups;
-      if (wave == 0) {
-        for (int g = lane; g < mode.n_groups; g += FG_WAVE) {
-          float a = -INFINITY, b = -INFINITY;  // the two largest
-          for (int i = 0; i < per; ++i) {
-            const float v = z[g * per + i];
-            if (v > a) { b = a; a = v; } else if (v > b) { b = v; }
-          }
-          rank[g] = per > 1 && !mode.group_max ? a + b : a;
+      for (int g = lane; g < mode.n_groups; g += FG_WAVE) {
+        float a = -INFINITY, b = -INFINITY;  // the two largest
+        for (int i = 0; i < per; ++i) {
+          const float v = z[g * per + i];
+          if (v > a) { b = a; a = v; } else if (v > b) { b = v; }
         }
+        rank[g] = per > 1 && !mode.group_max ? a + b : a;
       }
-      __syncthreads();
-      if (wave == 0) {
-        for (int g = lane; g < mode.n_groups; g += FG_WAVE) {
-          // a group stays if fewer than keep_groups groups rank before it (ties: the lower group first)
-          int before = 0;
-          const float mine = rank[g];
-          for (int o = 0; o < mode.n_groups; ++o) before += (rank[o] > mine || (rank[o] == mine && o < g)) ? 1 : 0;
-          if (before >= mode.keep_groups)
-            for (int i = 0; i < per; ++i) z[g * per + i] = -INFINITY;
-        }
+      moe_wave_sync();
+      for (int g = lane; g < mode.n_groups; g += FG_WAVE) {
+        // a group stays if fewer than keep_groups groups rank before it (ties: the lower group first)
+        int before = 0;
+        const float mine = rank[g];
+        for (int o = 0; o < mode.n_groups; ++o) before += (rank[o] > mine || (rank[o] == mine && o < g)) ? 1 : 0;
+        if (before >= mode.keep_groups)
+          for (int i = 0; i < per; ++i) z[g * per + i] = -INFINITY;
       }
-      __syncthreads();
+      moe_wave_sync();
     }
   }
   for (int j = 0; j < top; ++j) {
@@ -149,20 +171,19 @@ __global__ __launch_bounds__(64 * WAVES) void moe_route_kernel(
       const int oa = __shfl_xor(at, m, FG_WAVE);
       if (ov > best || (ov == best && oa < at)) { best = ov; at = oa; }
     }
-    __syncthreads();  // every wave has read the logits of this turn
-    if (threadIdx.x == 0) {
+    if (lane == 0) {
       at = min(at, n_experts - 1);  // (only if every logit is NaN)
       z[at] = -INFINITY;
       chosen[j] = mode.sigmoid_scores ? score[at] : best;
       choice[t * top + j] = at;
     }
-    __syncthreads();
+    moe_wave_sync();
   }
-  if (threadIdx.x == 0 && mode.sigmoid_scores) {
+  if (lane == 0 && mode.sigmoid_scores) {
     float sum = 0.f;
     for (int j = 0; j < top; ++j) sum += chosen[j];
     for (int j = 0; j < top; ++j) weight[t * top + j] = (mode.raw_weights ? chosen[j] : chosen[j] / (sum + 1e-20f)) * mode.weight_scale;
-  } else if (threadIdx.x == 0) {
+  } else if (lane == 0) {
     const float m = chosen[0];  // the largest
     float sum = 0.f;
     for (int j = 0; j < top; ++j) sum += expf(chosen[j] - m);
@@ -181,16 +202,17 @@ extern "C" int fg_moe_route_mode(const void* x, int ldx, int dtype, const float*
       top > keep_groups * (n_experts / n_groups) || (!sigmoid_scores && (correction || n_groups > 1)))
     return FG_ERR_ARG;
   const RouteMode mode = {sigmoid_scores, correction, n_groups, keep_groups, weight_scale, n_extra, extra, group_max, raw_weights};
-  const size_t lds = (size_t)(2 * n_experts + n_extra + top + n_groups) * sizeof(float);
+  const size_t lds = (size_t)(2 * n_experts + n_extra + top + n_groups) * sizeof(float);  // a token's
   if (lds > 60000) return FG_ERR_ARG;
-#define GO(T, WAVES, EPW)                                                                                        \
-  moe_route_kernel<T, WAVES, EPW><<<n_tokens, 64 * WAVES, lds, stream>>>((const T*)x, ldx, wr, bias, dim, n_experts, \
-                                                                         top, choice, weight, mode)
-  const bool few = n_tokens <= 64;
+#define GO(T, WAVES, EPW, TOK)                                                                                        \
+  moe_route_kernel<T, WAVES, EPW, TOK><<<(n_tokens + TOK - 1) / TOK, 64 * WAVES, TOK * lds, stream>>>(                 \
+      (const T*)x, ldx, wr, bias, n_tokens, dim, n_experts, top, choice, weight, mode)
+  // (many tokens: four a workgroup from where that still leaves a workgroup for every compute unit)
+  const int form = n_tokens <= 64 ? 0 : n_tokens < 1024 || 4 * lds > 60000 ? 1 : 2;
   if (dtype == FG_F32) {
-    if (few) GO(float, 16, 2); else GO(float, 4, 4);
+    if (form == 0) GO(float, 16, 2, 1); else if (form == 1) GO(float, 4, 4, 1); else GO(float, 4, 4, 4);
   } else if (dtype == FG_BF16) {
-    if (few) GO(bf16_t, 16, 2); else GO(bf16_t, 4, 4);
+    if (form == 0) GO(bf16_t, 16, 2, 1); else if (form == 1) GO(bf16_t, 4, 4, 1); else GO(bf16_t, 4, 4, 4);
   } else {
     return FG_ERR_ARG;
   }
@@ -682,27 +704,63 @@ struct CombineIdentity {
   const int* choice; int n_tiled;
   const void* x; int ldx;
 };
-template <class TP, class TX>
+template <int VEC, class T> __device__ __forceinline__ void mc_load(const T* p, float (&v)[VEC]) {
+  if constexpr (VEC == 4 && sizeof(T) == 4) {
+    const float4 a = *(const float4*)p;
+    v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w;
+  } else {
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) v[i] = to_f<T>(p[i]);
+  }
+}
+// grid (n_tokens, ceil(dim / (256 VEC))): a thread VEC neighbouring columns, the outputs of four experts in flight
+template <class TP, class TX, int VEC>
 __global__ __launch_bounds__(256) void moe_combine_kernel(
     const float* __restrict__ y, const float* __restrict__ weight, const TP* __restrict__ plus, int ldp, int n_plus,
     size_t plus_stride, int top, int dim, float* __restrict__ out, const float* __restrict__ plus_gate, int gate_stride,
     const CombineIdentity id) {
-  const int t = blockIdx.x;
+  const int t = blockIdx.x, d = (blockIdx.y * 256 + threadIdx.x) * VEC;
+  if (d >= dim) return;
   const float pg = plus_gate ? 1.f / (1.f + expf(-plus_gate[(size_t)t * gate_stride])) : 1.f;
-  for (int d = threadIdx.x; d < dim; d += 256) {
-    float s = 0.f;
-    for (int j = 0; j < top; ++j) {
-      const size_t p = (size_t)t * top + j;
-      const float o = id.choice && id.choice[p] >= id.n_tiled ? to_f<TX>(((const TX*)id.x)[(size_t)t * id.ldx + d]) : y[p * dim + d];
-      s = fmaf(weight[p], o, s);
+  float own[VEC], s[VEC];
+  if (id.choice) mc_load<VEC, TX>((const TX*)id.x + (size_t)t * id.ldx + d, own);
+#pragma unroll
+  for (int i = 0; i < VEC; ++i) s[i] = 0.f;
+  for (int j0 = 0; j0 < top; j0 += 4) {
+    float o[4][VEC], w[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const size_t p = (size_t)t * top + min(j0 + j, top - 1);
+      w[j] = j0 + j < top ? weight[p] : 0.f;
+      if (id.choice && id.choice[p] >= id.n_tiled) {  // uniform
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) o[j][i] = own[i];
+      } else {
+        mc_load<VEC, float>(y + p * dim + d, o[j]);
+      }
     }
-    if (plus) {
-      float m = to_f<TP>(plus[(size_t)t * ldp + d]);
-      for (int p = 1; p < n_plus; ++p) m += to_f<TP>(plus[p * plus_stride + (size_t)t * ldp + d]);
-      s = (plus_gate ? m * pg : m) + s;
-    }
-    out[(size_t)t * dim + d] = s;
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (j0 + j < top) {  // uniform
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) s[i] = fmaf(w[j], o[j][i], s[i]);
+      }
   }
+  if (plus) {
+    float m[VEC];
+    mc_load<VEC, TP>(plus + (size_t)t * ldp + d, m);
+    for (int p = 1; p < n_plus; ++p) {
+      float more[VEC];
+      mc_load<VEC, TP>(plus + p * plus_stride + (size_t)t * ldp + d, more);
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) m[i] += more[i];
+    }
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) s[i] = (plus_gate ? m[i] * pg : m[i]) + s[i];
+  }
+  float* o = out + (size_t)t * dim + d;
+  if constexpr (VEC == 4) *(float4*)o = make_float4(s[0], s[1], s[2], s[3]);
+  else o[0] = s[0];
 }
 
 extern "C" int fg_moe_combine_identity(const float* y, const float* weight, const void* plus, int ldp, int plus_dtype,
@@ -715,18 +773,26 @@ extern "C" int fg_moe_combine_identity(const float* y, const float* weight, cons
   if (choice && (!x || ldx < dim || n_tiled < 0)) return FG_ERR_ARG;
   const CombineIdentity id = {choice, n_tiled, x, ldx};
   if (x_dtype != FG_F32 && x_dtype != FG_BF16) return FG_ERR_ARG;
-  if (plus_dtype == FG_F32 && x_dtype == FG_F32)
-    moe_combine_kernel<float, float><<<n_tokens, 256, 0, stream>>>(y, weight, (const float*)plus, ldp, n_plus, (size_t)plus_stride,
-                                                                   top, dim, out, plus_gate, gate_stride, id);
-  else if (plus_dtype == FG_F32)
-    moe_combine_kernel<float, bf16_t><<<n_tokens, 256, 0, stream>>>(y, weight, (const float*)plus, ldp, n_plus, (size_t)plus_stride,
-                                                                    top, dim, out, plus_gate, gate_stride, id);
-  else if (plus_dtype == FG_BF16 && x_dtype == FG_BF16)
-    moe_combine_kernel<bf16_t, bf16_t><<<n_tokens, 256, 0, stream>>>(y, weight, (const bf16_t*)plus, ldp, n_plus,
-                                                                     (size_t)plus_stride, top, dim, out, plus_gate, gate_stride, id);
-  else if (plus_dtype == FG_BF16 && !choice)
-    moe_combine_kernel<bf16_t, float><<<n_tokens, 256, 0, stream>>>(y, weight, (const bf16_t*)plus, ldp, n_plus,
-                                                                    (size_t)plus_stride, top, dim, out, plus_gate, gate_stride, id);
+  // (16-byte loads of the fp32 operands)
+  const bool vec = dim % 4 == 0 && !((uintptr_t)y & 15) && !((uintptr_t)out & 15) &&
+                   (!plus || plus_dtype != FG_F32 || (ldp % 4 == 0 && plus_stride % 4 == 0 && !((uintptr_t)plus & 15))) &&
+                   (!choice || x_dtype != FG_F32 || (ldx % 4 == 0 && !((uintptr_t)x & 15)));
+  const dim3 grid(n_tokens, (dim + (vec ? 1023 : 255)) / (vec ? 1024 : 256));
+  if (grid.y > 65535) return FG_ERR_ARG;
+#define GO(TP, TX)                                                                                                         \
+  do {                                                                                                                     \
+    if (vec)                                                                                                               \
+      moe_combine_kernel<TP, TX, 4><<<grid, 256, 0, stream>>>(y, weight, (const TP*)plus, ldp, n_plus, (size_t)plus_stride, \
+                                                              top, dim, out, plus_gate, gate_stride, id);                  \
+    else                                                                                                                   \
+      moe_combine_kernel<TP, TX, 1><<<grid, 256, 0, stream>>>(y, weight, (const TP*)plus, ldp, n_plus, (size_t)plus_stride, \
+                                                              top, dim, out, plus_gate, gate_stride, id);                  \
+  } while (0)
+  if (plus_dtype == FG_F32 && x_dtype == FG_F32) GO(float, float);
+  else if (plus_dtype == FG_F32) GO(float, bf16_t);
+  else if (plus_dtype == FG_BF16 && x_dtype == FG_BF16) GO(bf16_t, bf16_t);
+  else if (plus_dtype == FG_BF16 && !choice) GO(bf16_t, float);
+#undef GO
   else
     return FG_ERR_ARG;
   return fg_launch_status();
