@@ -50,6 +50,31 @@ struct RouteMode {
   float* extra;
   int group_max, raw_weights;
 };
+// A value over the wave's lanes, in every one of them, without a trip through the LDS crossbar: rotations within rows of
+// 16 lanes, then rows and halves exchanged between two registers.
+template <class OP>
+__device__ __forceinline__ uint32_t moe_over_wave(uint32_t v, OP op) {
+  v = op(v, (uint32_t)__builtin_amdgcn_update_dpp(0, (int)v, 0x121 /* row_ror:1 */, 0xf, 0xf, false));
+  v = op(v, (uint32_t)__builtin_amdgcn_update_dpp(0, (int)v, 0x122, 0xf, 0xf, false));
+  v = op(v, (uint32_t)__builtin_amdgcn_update_dpp(0, (int)v, 0x124, 0xf, 0xf, false));
+  v = op(v, (uint32_t)__builtin_amdgcn_update_dpp(0, (int)v, 0x128, 0xf, 0xf, false));
+  const auto a = __builtin_amdgcn_permlane16_swap(v, v, false, false);
+  v = op(a[0], a[1]);
+  const auto b = __builtin_amdgcn_permlane32_swap(v, v, false, false);
+  return op(b[0], b[1]);
+}
+__device__ __forceinline__ float moe_wave_sum(float v) {
+  return __uint_as_float(moe_over_wave(__float_as_uint(v), [](uint32_t a, uint32_t b) {
+    return __float_as_uint(__uint_as_float(a) + __uint_as_float(b)); }));
+}
+__device__ __forceinline__ float moe_wave_max(float v) {
+  return __uint_as_float(moe_over_wave(__float_as_uint(v), [](uint32_t a, uint32_t b) {
+    return __float_as_uint(fmaxf(__uint_as_float(a), __uint_as_float(b))); }));
+}
+__device__ __forceinline__ int moe_wave_min(int v) {
+  return (int)moe_over_wave((uint32_t)v, [](uint32_t a, uint32_t b) { return (uint32_t)min((int)a, (int)b); });
+}
+
 // What a wave's lanes wrote to LDS is there for the wave's other lanes.
 __device__ __forceinline__ void moe_wave_sync() {
   asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
@@ -107,7 +132,7 @@ __global__ __launch_bounds__(64 * WAVES) void moe_route_kernel(
     for (int j = 0; j < EPW; ++j)
 #pragma unroll
       for (int i = 0; i < TOK; ++i) {
-        const float v = wave_sum(s[j][i]);
+        const float v = moe_wave_sum(s[j][i]);
         if (lane == 0 && e0 + j < n_rows) lds[i * per_token + e0 + j] = v + (bias && e0 + j < n_experts ? bias[e0 + j] : 0.f);
       }
   }
@@ -123,10 +148,10 @@ __global__ __launch_bounds__(64 * WAVES) void moe_route_kernel(
     if (mode.sigmoid_scores == 2) {
       top_z = -INFINITY;
       for (int e = lane; e < n_experts; e += FG_WAVE) top_z = fmaxf(top_z, z[e]);
-      top_z = wave_max(top_z);
+      top_z = moe_wave_max(top_z);
       all = 0.f;
       for (int e = lane; e < n_experts; e += FG_WAVE) all += expf(z[e] - top_z);
-      all = wave_sum(all);
+      all = moe_wave_sum(all);
     }
     for (int e = lane; e < n_experts; e += FG_WAVE) {
       const float sc = mode.sigmoid_scores == 2 ? expf(z[e] - top_z) / all : 1.f / (1.f + expf(-z[e]));
@@ -165,12 +190,9 @@ __global__ __launch_bounds__(64 * WAVES) void moe_route_kernel(
       const float v = z[e];
       if (v > best || (v == best && e < at)) { best = v; at = e; }
     }
-#pragma unroll
-    for (int m = FG_WAVE / 2; m > 0; m >>= 1) {
-      const float ov = __shfl_xor(best, m, FG_WAVE);
-      const int oa = __shfl_xor(at, m, FG_WAVE);
-      if (ov > best || (ov == best && oa < at)) { best = ov; at = oa; }
-    }
+    const float all_best = moe_wave_max(best);
+    at = moe_wave_min(best == all_best ? at : 0x7fffffff);  // of equal values the lowest expert
+    best = all_best;
     if (lane == 0) {
       at = min(at, n_experts - 1);  // (only if every logit is NaN)
       z[at] = -INFINITY;
