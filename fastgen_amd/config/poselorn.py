@@ -2,8 +2,8 @@
 
 A Poselorn ``config.json`` is nested: ``width``, ``vocab``, ``embedding.scale``, ``residual_mult``, ``norm.eps``, a list
 ``layers`` whose entries name their mixer (``type``), its sizes (``mixer``) and their feed-forward (``mlp``, or null), and
-optionally ``loop``: layers ``start .. stop-1`` run ``times`` times in a row with the same weights and storage per pass; every
-pass but the first begins by adding the embedding's output.  In a layer both sublayers read the same stream through norms of
+optionally ``loop``, a stretch of layers (``start`` to before ``stop``) that is repeated, ``times`` passes over one set of
+weights, each pass with storage of its own; every pass but the first begins by adding the embedding's output.  In a layer both sublayers read the same stream through norms of
 their own, and their outputs, scaled per channel (``l<i>.ls1`` / ``ls2``) and by ``residual_mult``, are added at once.
 
 * ``channel_delta``: the gated delta rule behind short convolutions (``conv`` taps) with a decay per key channel; the decays and

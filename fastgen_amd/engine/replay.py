@@ -2,8 +2,8 @@
 the logits at the wanted places are written to disk.  Nothing is sampled.
 
 It drives the same model, step function, cache and kernels that generation
-uses (``ModelRunner.step``); it has no forward pass, cache or loader of its
-own.  The reference has no such tool.
+uses (``ModelRunner.step``); it adds only the reading of requests and
+the writing of logits.  The reference has no such tool.
 """
 
 from __future__ import annotations
@@ -79,7 +79,7 @@ def replay(model_dir: str, dtype: str, out_dir: str, max_tokens: int, page_size:
 def main(argv=None) -> int:
     ap = argparse.ArgumentParser(
         prog="trace_run",
-        description="Feed given token ids through a model step by step and write the logits asked for.",
+        description="Replay recorded requests through a model and write the logits they ask for.",
     )
     ap.add_argument("--model", required=True, help="folder with config.json and model.safetensors")
     ap.add_argument("--dtype", required=True, choices=sorted(DTYPES))

@@ -39,7 +39,8 @@ class RMSNorm(Norm):
         """``delta`` may be :class:`~fastgen_amd.kernels.ops.PostNormed`: a sublayer's output that is normed
         itself before it is added (the norm behind a sublayer); one kernel does that norm, the addition and
         this norm.  :class:`~fastgen_amd.kernels.ops.ScaledDelta`: rows times a vector;
-        :class:`~fastgen_amd.kernels.ops.StreamTerms`: several sublayers' outputs.  ``h`` may be several residual streams ``[S, T, dim]`` (``delta``: the
+        :class:`~fastgen_amd.kernels.ops.StreamTerms`: several sublayers' outputs.
+        ``h`` may be several residual streams ``[S, T, dim]`` (``delta``: the
         :class:`~fastgen_amd.kernels.ops.StreamUpdate` still to be applied, or None): their sum is normed."""
         n = h.shape[-2] if rows is None else rows.numel()
         out = torch.empty((n, self.dim), dtype=dtype, device=h.device)

@@ -63,7 +63,7 @@ def mixed(lengths: Dict[str, int], max_live: int = 4, seed: int = 0, prompt_frac
             else:
                 c = min(n_prompt - p, rng.choice([2, 3, 5, 8, 17, 32]))
             if rng.random() < 0.15 and len(order) > 1:
-                continue  # a request may be left out of a step and go on later
+                continue  # skipped in this step
             if c > left:
                 if left < 2:
                     continue
